@@ -10,6 +10,7 @@ model, tp-size, disaggregation-mode, mem-fraction).
 from __future__ import annotations
 
 from dataclasses import dataclass, field
+from typing import Optional
 
 
 @dataclass
@@ -27,6 +28,8 @@ class ModelConfig:
     max_position: int = 16384
     dtype: str = "bfloat16"
     qk_norm: bool = False      # Qwen3-style per-head RMSNorm on q/k
+    architecture: str = "llama"    # key of models/registry.py
+    weights_path: str = ""         # folder with model.safetensors; "": random
 
     @property
     def q_size(self) -> int:
@@ -98,3 +101,8 @@ class EngineConfig:
     enable_prefix_cache: bool = True   # full-page KV reuse (Mooncake analog)
     enforce_eager: bool = False        # False: capture decode in hipGraphs
     seed: int = 0
+    # models with per-sequence state: sequences in flight (0: max_batch_size)
+    state_slots: int = 0
+    # prompt portions and decoded tokens of one step run as one batch
+    # (None: as the model prefers)
+    mixed_steps: Optional[bool] = None

@@ -65,7 +65,8 @@ class LLMEngine:
                  pp=None):
         self.cfg = cfg
         self.runner = ModelRunner(cfg, tp, pp)
-        self.scheduler = Scheduler(cfg, self.runner.cache)
+        self.scheduler = Scheduler(cfg, self.runner.cache,
+                                   self.runner.mixed_steps)
         self.stats = EngineStats()
 
     # ------------------------------------------------------------------
@@ -88,8 +89,10 @@ class LLMEngine:
         mode, seqs = self.scheduler.schedule()
         self.stats.sched_wall_s += time.monotonic() - t0
         t0 = time.monotonic()
-        if mode == "prefill":
-            self.runner.prefill(seqs)
+        if mode in ("prefill", "mixed"):
+            running = list(self.scheduler.running) if mode == "mixed" else []
+            self.runner.mixed(seqs, running)
+            self.stats.decode_tokens += len(running)
             self.stats.prefill_tokens += sum(s.chunk_len for s in seqs)
             self.stats.prefill_steps += 1
             prefix = self.runner.cache.prefix

@@ -34,11 +34,23 @@ class PagedKVCache:
         layers = num_layers or m.num_layers      # PP: only local layers
         self.num_layers = layers
         if num_pages is None:
-            num_pages = self._size_pool(cfg, device, layers)
+            num_pages = self._size_pool(device)
         self.num_pages = num_pages
-        kvh = m.num_kv_heads // max(1, cfg.tp_size)   # TP shards the heads
-        shape = (layers, 2, num_pages, kvh, cfg.page_size, m.head_dim)
         self.ipc_exportable = False
+        self._alloc_storage(device)
+        # page 0 is reserved scratch: hipGraph decode padding rows write
+        # their (dead) KV slot there (model_runner._decode_graph)
+        self._free: List[int] = list(range(num_pages - 1, 0, -1))
+        import threading
+        self._lock = threading.Lock()   # alloc/free may race import threads
+        self.prefix: Optional["PrefixCache"] = (
+            PrefixCache(self) if cfg.enable_prefix_cache else None)
+
+    def _alloc_storage(self, device: torch.device) -> None:
+        m = self.cfg.model
+        kvh = m.num_kv_heads // max(1, self.cfg.tp_size)  # TP shards heads
+        shape = (self.num_layers, 2, self.num_pages, kvh,
+                 self.cfg.page_size, m.head_dim)
         if device.type == "cuda":
             # hipMalloc base allocation (not the caching allocator) so the
             # pool is hipIpc-exportable: prefill engines map it and push
@@ -60,21 +72,15 @@ class PagedKVCache:
                                       device=device)
         else:
             self.kv = torch.zeros(shape, dtype=torch.bfloat16, device=device)
-        # page 0 is reserved scratch: hipGraph decode padding rows write
-        # their (dead) KV slot there (model_runner._decode_graph)
-        self._free: List[int] = list(range(num_pages - 1, 0, -1))
-        import threading
-        self._lock = threading.Lock()   # alloc/free may race import threads
-        self.prefix: Optional["PrefixCache"] = (
-            PrefixCache(self) if cfg.enable_prefix_cache else None)
 
-    @staticmethod
-    def _size_pool(cfg: EngineConfig, device: torch.device,
-                   num_layers: Optional[int] = None) -> int:
-        m = cfg.model
-        kvh = m.num_kv_heads // max(1, cfg.tp_size)
-        page_bytes = ((num_layers or m.num_layers) * 2 * kvh *
-                      cfg.page_size * m.head_dim * 2)
+    def _page_bytes(self) -> int:
+        m = self.cfg.model
+        kvh = m.num_kv_heads // max(1, self.cfg.tp_size)
+        return (self.num_layers * 2 * kvh * self.cfg.page_size *
+                m.head_dim * 2)
+
+    def _size_pool(self, device: torch.device) -> int:
+        cfg = self.cfg
         if device.type == "cuda" and torch.cuda.is_available():
             free, _total = torch.cuda.mem_get_info(device)
             budget = int(free * cfg.gpu_memory_utilization)
@@ -82,7 +88,36 @@ class PagedKVCache:
             budget = 64 << 20     # CPU tests: 64 MB
         if cfg.kv_pool_tokens:
             return max(1, cfg.kv_pool_tokens // cfg.page_size)
-        return max(8, budget // page_bytes)
+        return max(8, budget // self._page_bytes())
+
+    # -- per-sequence state slots (recurrent models override) ---------------
+
+    def has_room(self, num_pages: int) -> bool:
+        """Can a sequence of this many pages be admitted now?"""
+        return num_pages <= self.free_pages_evictable
+
+    def alloc_slot(self) -> int:
+        return 0
+
+    def free_slot(self, slot: int) -> None:
+        pass
+
+    # -- migration ------------------------------------------------------------
+
+    def export_pages(self, pages: List[int], slot: int = 0) -> torch.Tensor:
+        """What a peer needs to continue a sequence, as one tensor."""
+        idx = torch.tensor(pages, dtype=torch.int64, device=self.kv.device)
+        return self.kv.index_select(2, idx).contiguous()
+
+    def export_shape(self, num_pages: int):
+        """(shape, dtype) of export_pages for that many pages."""
+        m = self.kv.shape
+        return (m[0], m[1], num_pages, m[3], m[4], m[5]), self.kv.dtype
+
+    def import_pages(self, pages: List[int], buf: torch.Tensor,
+                     slot: int = 0) -> None:
+        idx = torch.tensor(pages, dtype=torch.int64, device=self.kv.device)
+        self.kv.index_copy_(2, idx, buf.to(self.kv.device))
 
     # -- page accounting ----------------------------------------------------
 
@@ -131,6 +166,7 @@ class BlockTable:
         self.pages: List[int] = []
         self.num_shared = 0
         self.num_tokens = 0
+        self.state_slot = cache.alloc_slot()    # 0: the model keeps no state
 
     def ensure(self, num_tokens: int) -> None:
         need = (num_tokens + self.cache.page_size - 1) // self.cache.page_size
@@ -160,6 +196,9 @@ class BlockTable:
         self.pages = []
         self.num_shared = 0
         self.num_tokens = 0
+        if self.state_slot:
+            self.cache.free_slot(self.state_slot)
+            self.state_slot = 0
 
 
 class PrefixCache:

@@ -13,12 +13,13 @@ from __future__ import annotations
 import logging
 from typing import Dict, List, Optional, Tuple
 
+import numpy as np
 import torch
 
-from ..models.llama import (ForwardBatch, LlamaForCausalLM, PPContext,
-                            TPContext)
+from ..models.llama import PPContext, TPContext
+from ..models.registry import build_model
+from .batch import ForwardBatch, VarlenLayout
 from .config import EngineConfig
-from .kv_cache import PagedKVCache
 from .sequence import Sequence
 
 log = logging.getLogger(__name__)
@@ -33,83 +34,159 @@ class ModelRunner:
         self.device = torch.device(cfg.device)
         torch.manual_seed(cfg.seed)
         self.pp = pp or PPContext()
-        self.model = LlamaForCausalLM(cfg.model, self.device, tp, pp=self.pp)
-        self.cache = PagedKVCache(cfg, self.device,
-                                  num_layers=self.model.num_local_layers)
+        self.model = build_model(cfg.model, self.device, tp, self.pp)
+        self.cache = self.model.make_cache(cfg)
+        self.mixed_steps = (self.model.mixed_steps if cfg.mixed_steps is None
+                            else bool(cfg.mixed_steps))
+        if self.mixed_steps and not self.model.mixed_steps:
+            raise ValueError(f"{cfg.model.name}: mixed steps not supported")
         self.max_pages_per_seq = (cfg.max_seq_len + cfg.page_size - 1) // \
             cfg.page_size
         self._graphs: Dict[int, Tuple] = {}
         self._graph_pool = None
+        # device-resident decode inputs of the last batch composition
+        self._dstate: Optional[dict] = None
         log.info("model %s on %s: %d KV pages (%.1f GB pool)",
                  cfg.model.name, self.device, self.cache.num_pages,
-                 self.cache.kv.numel() * 2 / 1e9)
+                 self.cache.kv.numel() * self.cache.kv.element_size() / 1e9)
 
     # ------------------------------------------------------------------
 
     def _i32(self, data) -> torch.Tensor:
         return torch.tensor(data, dtype=torch.int32, device=self.device)
 
+    # one sequence's part of a varlen step: tokens at [start, start + len)
+    Chunk = Tuple[Sequence, int, List[int]]
+
     @torch.inference_mode()
-    def prefill(self, seqs: List[Sequence]) -> List[int]:
-        """One prefill step: each sequence contributes its current chunk
-        [num_prefilled, num_prefilled + chunk_len) — a full prompt, a
-        cached-prefix suffix, or one piece of a chunked long prompt.  Only
-        sequences whose chunk reaches the prompt end get a token sampled."""
+    def run_chunks(self, chunks: List[Chunk]) -> Tuple[torch.Tensor,
+                                                       List[int]]:
+        """One varlen forward over portions of several sequences — a full
+        prompt, a cached-prefix suffix, a piece of a long prompt or (models
+        with mixed steps) a single decoded token beside them.  Returns the
+        last stage's hidden rows and each chunk's first row; the rows of
+        single-token chunks with a past come first."""
+        order = list(range(len(chunks)))
+        num_decode = 0
+        if self.model.mixed_steps:
+            single = [len(t) == 1 and start > 0 for _, start, t in chunks]
+            num_decode = sum(single)
+            order.sort(key=lambda i: not single[i])
         tokens: List[int] = []
         positions: List[int] = []
         slots: List[int] = []
         gather: List[int] = []
         cu = [0]
         cu_k = [0]
-        completing: List[Sequence] = []
-        last_idx: List[int] = []
-        any_past = any(seq.num_prefilled > 0 for seq in seqs)
-        for seq in seqs:
-            start = seq.num_prefilled
-            end = start + (seq.chunk_len or
-                           (seq.num_prompt_tokens - start))
-            tokens.extend(seq.prompt_tokens[start:end])
+        first_row = [0] * len(chunks)
+        starts, ends, tables = [], [], []
+        any_past = any(start > 0 for _, start, _ in chunks)
+        for i in order:
+            seq, start, toks = chunks[i]
+            end = start + len(toks)
+            tokens.extend(toks)
             positions.extend(range(start, end))
             slots.extend(seq.block_table.slots_for(start, end - start))
+            first_row[i] = cu[-1]
             cu.append(cu[-1] + (end - start))
             cu_k.append(cu_k[-1] + end)
-            if any_past:
+            if any_past and not self.model.stateful:
                 gather.extend(seq.block_table.slots_for(0, end))
-            if end == seq.num_prompt_tokens:
-                completing.append(seq)
-                last_idx.append(cu[-1] - 1)
-            seq.num_prefilled = end
+            starts.append(start)
+            ends.append(end)
+            tables.append(seq.block_table)
         batch = ForwardBatch(
             mode="prefill",
             positions=self._i32(positions),
             slot_mapping=self._i32(slots),
-            cu_seqlens=self._i32(cu),
-            cu_seqlens_k=self._i32(cu_k) if any_past else None,
-            kv_gather_slots=self._i32(gather) if any_past else None)
+            cu_seqlens=self._i32(cu))
+        if self.model.stateful:
+            batch.starts = self._i32(starts)
+            batch.state_slots = self._i32([t.state_slot for t in tables])
+            batch.num_decode = num_decode
+            batch.layout = VarlenLayout(starts, ends, tables, num_decode,
+                                        self.cfg.page_size, self.device)
+            batch.cu_prefill = self._i32([c - num_decode
+                                          for c in cu[num_decode:]])
+            if num_decode:
+                batch.block_tables = torch.from_numpy(self._table_array(
+                    tables[:num_decode])).to(self.device)
+                batch.context_lens = self._i32(ends[:num_decode])
+        elif any_past:
+            batch.cu_seqlens_k = self._i32(cu_k)
+            batch.kv_gather_slots = self._i32(gather)
+        # decode inputs that were left on the device are behind now
+        self._dstate = None
         hidden_in = None
         if not self.pp.first:
             hidden_in = self.pp.recv_prev(
                 (len(tokens), self.cfg.model.hidden_size),
-                self.model.dtype, self.device)
+                self.model.stream_dtype, self.device)
         hidden = self.model.forward(
             torch.tensor(tokens, dtype=torch.int64, device=self.device),
             batch, self.cache, hidden=hidden_in)
         if not self.pp.last:
             self.pp.send_next(hidden)
-        if not completing:
+        return hidden, first_row
+
+    def prefill(self, seqs: List[Sequence]) -> List[int]:
+        """One prefill step: each sequence contributes its current chunk
+        [num_prefilled, num_prefilled + chunk_len).  Only sequences whose
+        chunk reaches the prompt end get a token sampled."""
+        return self.mixed(seqs, [])
+
+    @torch.inference_mode()
+    def mixed(self, prefills: List[Sequence],
+              decodes: List[Sequence]) -> List[int]:
+        """One step of prompt chunks and decoded tokens as one batch."""
+        chunks: List[ModelRunner.Chunk] = []
+        sampled: List[Sequence] = []
+        at: List[int] = []              # chunk of each sampled sequence
+        for seq in decodes:
+            sampled.append(seq)
+            at.append(len(chunks))
+            chunks.append((seq, seq.num_tokens - 1, [seq.last_token]))
+        for seq in prefills:
+            start = seq.num_prefilled
+            end = start + (seq.chunk_len or
+                           (seq.num_prompt_tokens - start))
+            if end == seq.num_prompt_tokens:
+                sampled.append(seq)
+                at.append(len(chunks))
+            chunks.append((seq, start, seq.prompt_tokens[start:end]))
+            seq.num_prefilled = end
+        hidden, first_row = self.run_chunks(chunks)
+        if not sampled:
             return []
         if self.pp.last:
-            logits = self.model.logits(hidden, self._i32(last_idx))
-            next_dev = self.sample_device(logits, completing)[0]
+            last = [first_row[i] + len(chunks[i][2]) - 1 for i in at]
+            logits = self.model.logits(hidden, self._i32(last))
+            next_dev = self.sample_device(logits, sampled)[0]
         else:
-            next_dev = torch.empty(len(completing), dtype=torch.int64,
+            next_dev = torch.empty(len(sampled), dtype=torch.int64,
                                    device=self.device)
         if self.pp.size > 1:
             next_dev = self.pp.broadcast_tokens(next_dev)
         next_tokens = next_dev.tolist()
-        for seq, tok in zip(completing, next_tokens):
+        for seq, tok in zip(sampled, next_tokens):
             seq.append_token(tok)
         return next_tokens
+
+    @torch.inference_mode()
+    def feed(self, chunks: List[Chunk],
+             want: List[List[int]]) -> torch.Tensor:
+        """Teacher-forced step: runs the given tokens as one batch, as
+        generation would (single tokens alone are a decode step), and returns
+        the logits at the wanted places of each chunk, in order."""
+        if all(len(t) == 1 and start > 0 for _, start, t in chunks):
+            self._dstate = None
+            logits = self._decode_logits([seq for seq, _, _ in chunks])
+            rows = [i for i, w in enumerate(want) for _ in w]
+            return logits[torch.tensor(rows, dtype=torch.int64,
+                                       device=self.device)]
+        hidden, first_row = self.run_chunks(chunks)
+        rows = [first_row[i] + p for i, w in enumerate(want) for p in w]
+        return self.model.logits(hidden, self._i32(rows))
 
     # ------------------------------------------------------------------
 
@@ -120,22 +197,30 @@ class ModelRunner:
         admission — engine/scheduler.py), so the only host->device traffic
         per step is nothing at all; sampled tokens stay on-device as the
         next step's input."""
-        import numpy as np
         dev = self.device
         positions = self._i32([seq.num_tokens - 1 for seq in seqs])
         ctx = self._i32([seq.num_tokens for seq in seqs])
         tokens = torch.tensor([seq.last_token for seq in seqs],
                               dtype=torch.int64, device=dev)
-        max_pages = max(len(seq.block_table.pages) for seq in seqs)
+        bt_np = self._table_array([seq.block_table for seq in seqs])
+        state = {"ids": tuple(s.seq_id for s in seqs),
+                 "positions": positions, "ctx": ctx, "tokens": tokens,
+                 "bt": torch.from_numpy(bt_np).to(dev), "fresh": True,
+                 "state_slots": None}
+        if self.model.stateful:
+            state["state_slots"] = self._i32(
+                [seq.block_table.state_slot for seq in seqs])
+        return state
+
+    @staticmethod
+    def _table_array(tables) -> np.ndarray:
         # numpy staging: batch composition churns every step under
         # continuous serving, so the rebuild is on the step critical path
-        bt_np = np.zeros((len(seqs), max_pages), dtype=np.int32)
-        for i, seq in enumerate(seqs):
-            pages = seq.block_table.pages
-            bt_np[i, :len(pages)] = pages
-        return {"ids": tuple(s.seq_id for s in seqs),
-                "positions": positions, "ctx": ctx, "tokens": tokens,
-                "bt": torch.from_numpy(bt_np).to(dev), "fresh": True}
+        out = np.zeros((len(tables), max(len(t.pages) for t in tables)),
+                       dtype=np.int32)
+        for i, t in enumerate(tables):
+            out[i, :len(t.pages)] = t.pages
+        return out
 
     def _decode_slots(self, state: dict) -> torch.Tensor:
         ps = self.cfg.page_size
@@ -144,11 +229,11 @@ class ModelRunner:
                             (pos // ps).unsqueeze(1)).squeeze(1)
         return (page * ps + (pos % ps).to(torch.int32)).to(torch.int32)
 
-    @torch.inference_mode()
-    def decode(self, seqs: List[Sequence]) -> List[int]:
+    def _decode_logits(self, seqs: List[Sequence]) -> Optional[torch.Tensor]:
+        """Forward of one decode step; logits [n, vocab] on the last stage."""
         n = len(seqs)
         ids = tuple(s.seq_id for s in seqs)
-        state = self._dstate if getattr(self, "_dstate", None) else None
+        state = self._dstate
         if state is None or state["ids"] != ids:
             state = self._build_decode_state(seqs)
             self._dstate = state
@@ -163,28 +248,36 @@ class ModelRunner:
                      self.model.tp.graph_safe and    # xGMI AR or no TP
                      n <= GRAPH_BATCH_SIZES[-1])
         if use_graph:
-            logits = self._decode_graph(state, slots, n)
-        else:
-            batch = ForwardBatch(
-                mode="decode",
-                positions=state["positions"],
-                slot_mapping=slots,
-                block_tables=state["bt"],
-                context_lens=state["ctx"],
-                decode_num_splits=self._splits_for(n))
-            hidden_in = None
-            if not self.pp.first:
-                hidden_in = self.pp.recv_prev(
-                    (n, self.cfg.model.hidden_size),
-                    self.model.dtype, self.device)
-            hidden = self.model.forward(state["tokens"], batch, self.cache,
-                                        hidden=hidden_in)
-            if self.pp.last:
-                logits = self.model.logits(hidden)
-            else:
-                self.pp.send_next(hidden)
+            return self._decode_graph(state, slots, n)[:n]
+        batch = self._decode_batch(state, slots, n)
+        hidden_in = None
+        if not self.pp.first:
+            hidden_in = self.pp.recv_prev(
+                (n, self.cfg.model.hidden_size),
+                self.model.stream_dtype, self.device)
+        hidden = self.model.forward(state["tokens"], batch, self.cache,
+                                    hidden=hidden_in)
         if self.pp.last:
-            next_dev, next_tokens = self.sample_device(logits[:n], seqs)
+            return self.model.logits(hidden)
+        self.pp.send_next(hidden)
+        return None
+
+    def _decode_batch(self, inputs: dict, slots: torch.Tensor,
+                      n: int) -> ForwardBatch:
+        return ForwardBatch(
+            mode="decode", positions=inputs["positions"], slot_mapping=slots,
+            block_tables=inputs["bt"], context_lens=inputs["ctx"],
+            starts=inputs["positions"], state_slots=inputs["state_slots"],
+            decode_num_splits=self.model.decode_splits(
+                n, self.cfg.max_seq_len))
+
+    @torch.inference_mode()
+    def decode(self, seqs: List[Sequence]) -> List[int]:
+        n = len(seqs)
+        logits = self._decode_logits(seqs)
+        state = self._dstate
+        if self.pp.last:
+            next_dev, next_tokens = self.sample_device(logits, seqs)
         else:
             next_dev = torch.empty(n, dtype=torch.int64, device=self.device)
         if self.pp.size > 1:
@@ -197,15 +290,6 @@ class ModelRunner:
 
     # ------------------------------------------------------------------
 
-    def _splits_for(self, batch_size: int) -> int:
-        """Sync-free split-KV policy (graph-safe: depends only on the padded
-        batch size and the config's max context)."""
-        from .. import ops as _ops
-        m = self.cfg.model
-        tp = max(1, getattr(self.model.tp, "size", 1))
-        return _ops.pick_decode_splits(batch_size, m.num_kv_heads // tp,
-                                       self.cfg.max_seq_len)
-
     def _graph_bucket(self, n: int) -> int:
         for b in GRAPH_BATCH_SIZES:
             if n <= b:
@@ -214,7 +298,6 @@ class ModelRunner:
 
     def _build_graph(self, bs: int):
         """Capture one decode step at batch size ``bs`` into a hipGraph."""
-        m = self.cfg.model
         static = {
             "tokens": torch.zeros(bs, dtype=torch.int64, device=self.device),
             "positions": torch.zeros(bs, dtype=torch.int32, device=self.device),
@@ -222,12 +305,11 @@ class ModelRunner:
             "ctx": torch.ones(bs, dtype=torch.int32, device=self.device),
             "bt": torch.zeros(bs, self.max_pages_per_seq, dtype=torch.int32,
                               device=self.device),
+            # padding rows use the scratch slot 0
+            "state_slots": torch.zeros(bs, dtype=torch.int32,
+                                       device=self.device),
         }
-        batch = ForwardBatch(mode="decode", positions=static["positions"],
-                             slot_mapping=static["slots"],
-                             block_tables=static["bt"],
-                             context_lens=static["ctx"],
-                             decode_num_splits=self._splits_for(bs))
+        batch = self._decode_batch(static, static["slots"], bs)
         # warm up allocations outside capture
         torch.cuda.synchronize()
         hidden = self.model.forward(static["tokens"], batch, self.cache)
@@ -253,6 +335,8 @@ class ModelRunner:
         static["positions"][:n].copy_(state["positions"])
         static["slots"][:n].copy_(slots)
         static["ctx"][:n].copy_(state["ctx"])
+        if state["state_slots"] is not None:
+            static["state_slots"][:n].copy_(state["state_slots"])
         bt = state["bt"]
         if state.get("graph_bt_loaded") != (state["ids"], bs):
             # block tables are stable for this batch: upload once per batch
@@ -264,6 +348,7 @@ class ModelRunner:
                 static["slots"][n:] = 0
                 static["positions"][n:] = 0
                 static["ctx"][n:] = 1
+                static["state_slots"][n:] = 0
             state["graph_bt_loaded"] = (state["ids"], bs)
         graph.replay()
         return logits

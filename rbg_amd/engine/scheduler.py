@@ -1,8 +1,8 @@
 """Continuous-batching scheduler.
 
 Each engine step is either one prefill batch (as many waiting prompts as fit
-the token budget) or one decode step over every running sequence — the
-standard continuous-batching loop of the engines the reference orchestrates
+the token budget) or one decode step over every running sequence, or both at
+once for models that run mixed steps — the standard continuous-batching loop of the engines the reference orchestrates
 (SURVEY §2.3 decode engine row).  Admission reserves KV pages for prompt +
 max_new_tokens up front, so a running sequence can never hit OutOfPages
 mid-decode (no preemption needed at node scale; revisit for oversubscribed
@@ -19,8 +19,10 @@ from .sequence import FINISHED, RUNNING, Sequence
 
 
 class Scheduler:
-    def __init__(self, cfg: EngineConfig, cache: PagedKVCache):
+    def __init__(self, cfg: EngineConfig, cache: PagedKVCache,
+                 mixed_steps: bool = False):
         self.cfg = cfg
+        self.mixed_steps = mixed_steps
         self.cache = cache
         self.waiting: Deque[Sequence] = deque()
         self.running: List[Sequence] = []
@@ -36,18 +38,22 @@ class Scheduler:
         return (total + self.cfg.page_size - 1) // self.cfg.page_size
 
     def schedule(self) -> Tuple[str, List[Sequence]]:
-        """Returns ("prefill"|"decode"|"idle", sequences)."""
+        """Returns ("prefill"|"mixed"|"decode"|"idle", sequences).  "mixed":
+        the prompt chunks returned and every running sequence's next token
+        are one step."""
         # prefill first: new prompts keep the decode batch full.  A prompt
         # whose remaining suffix exceeds the step budget is CHUNKED: it stays
         # at the head of the queue and prefills budget-sized pieces per step
         # (the attend-over-[past; new] path of the prefill kernel).
         batch: List[Sequence] = []
         budget = self.cfg.max_prefill_tokens
+        if self.mixed_steps:
+            budget = max(1, budget - len(self.running))
         while self.waiting and len(self.running) + len(batch) < \
                 self.cfg.max_batch_size and budget > 0:
             seq = self.waiting[0]
             if seq.block_table is None:
-                if self._pages_needed(seq) > self.cache.free_pages_evictable:
+                if not self.cache.has_room(self._pages_needed(seq)):
                     break
                 seq.block_table = BlockTable(self.cache)
                 if self.cache.prefix is not None and not seq.imported_kv:
@@ -69,7 +75,8 @@ class Scheduler:
             self.waiting.popleft()
             seq.status = RUNNING
         if batch:
-            return "prefill", batch
+            mixed = self.mixed_steps and self.running
+            return ("mixed" if mixed else "prefill"), batch
         if self.running:
             return "decode", list(self.running)
         return "idle", []

@@ -32,7 +32,8 @@ import torch
 from ..api import constants as C
 from ..runtime.worker import WorkerContext, register_runner
 from ..server.rpc import RpcClient, RpcServer
-from .config import EngineConfig, ModelConfig
+from ..models.registry import resolve_model
+from .config import EngineConfig
 from .engine import LLMEngine
 from .sequence import FINISHED, SamplingParams, Sequence
 
@@ -41,11 +42,12 @@ log = logging.getLogger(__name__)
 
 def _engine_cfg(ctx: WorkerContext) -> EngineConfig:
     args = ctx.args
-    model = ModelConfig.preset(args.get("model", "llama-3-8b"))
+    name = args.get("model", "llama-3-8b")
+    model = resolve_model(name)
     device = "cuda" if (torch.cuda.is_available() and ctx.gpu_ids != []) \
         else args.get("device", "cpu")
-    if device == "cpu" and args.get("model", "") not in ("tiny",):
-        model = ModelConfig.preset(args.get("cpu_model", "tiny"))
+    if device == "cpu" and not (name.startswith("tiny") or model.weights_path):
+        model = resolve_model(args.get("cpu_model", "tiny"))
     return EngineConfig(
         model=model, device=device,
         page_size=int(args.get("page_size", 16)),
@@ -56,6 +58,8 @@ def _engine_cfg(ctx: WorkerContext) -> EngineConfig:
         enable_prefix_cache=bool(args.get("enable_prefix_cache", True)),
         max_prefill_tokens=int(args.get("max_prefill_tokens", 8192)),
         enforce_eager=bool(args.get("enforce_eager", device != "cuda")),
+        state_slots=int(args.get("state_slots", 0)),
+        mixed_steps=args.get("mixed_steps"),
     )
 
 
@@ -165,7 +169,8 @@ class ServeWorker:
         # lock otherwise starves waiters indefinitely (lock convoy)
         self._pause = threading.Event()
         self.results: Dict[int, Sequence] = {}
-        self._finished_pages: Dict[int, List[int]] = {}
+        # finished prefills awaiting migration: (pages, shared, state slot)
+        self._finished_pages: Dict[int, tuple] = {}
         self._plan: Optional[_TransferPlan] = None
         self._transfer = None
         # xGMI fast path (parallel/kv_peer.py): direct hipIpc page push for
@@ -243,33 +248,30 @@ class ServeWorker:
             return torch.device("cpu")
         return self.engine.runner.cache.kv.device
 
-    def _send_pages(self, pages: List[int], dst_rank: int) -> None:
+    def _send_pages(self, pages: List[int], dst_rank: int,
+                    slot: int = 0) -> None:
         import torch.distributed as dist
 
         from ..parallel.comm import to_wire
         cache = self.engine.runner.cache
         with self._xfer_lock:
-            idx = torch.tensor(pages, dtype=torch.int64, device=cache.kv.device)
-            buf = cache.kv.index_select(2, idx).contiguous()
+            buf = cache.export_pages(pages, slot)
             if buf.device != self._xfer_buf_device():
                 buf = buf.to(self._xfer_buf_device())
             dist.send(to_wire(buf), dst_rank)
 
-    def _recv_pages(self, pages: List[int], src_rank: int) -> None:
+    def _recv_pages(self, pages: List[int], src_rank: int,
+                    slot: int = 0) -> None:
         import torch.distributed as dist
 
         from ..parallel.comm import from_wire, wire_dtype
         cache = self.engine.runner.cache
         with self._xfer_lock:
-            m = cache.kv.shape
+            shape, dtype = cache.export_shape(len(pages))
             dev = self._xfer_buf_device()
-            buf = torch.empty((m[0], m[1], len(pages), m[3], m[4], m[5]),
-                              dtype=wire_dtype(cache.kv.dtype, dev),
-                              device=dev)
+            buf = torch.empty(shape, dtype=wire_dtype(dtype, dev), device=dev)
             dist.recv(buf, src_rank)
-            buf = from_wire(buf, cache.kv.dtype)
-            idx = torch.tensor(pages, dtype=torch.int64, device=cache.kv.device)
-            cache.kv.index_copy_(2, idx, buf.to(cache.kv.device))
+            cache.import_pages(pages, from_wire(buf, dtype), slot)
 
     def _peer_rank(self, peer_instance: str) -> int:
         """My point-to-point counterpart in `peer_instance`: same position
@@ -318,7 +320,8 @@ class ServeWorker:
             # prefill TP: each rank ships its own KV shard to its decode
             # counterpart; page ids are rank-identical (lockstep allocators)
             parked = self._finished_pages.pop(int(op["seq_id"]))
-            self._send_pages(parked[0], self._peer_rank(op["dst_instance"]))
+            self._send_pages(parked[0], self._peer_rank(op["dst_instance"]),
+                             parked[2])
             self._release_parked(parked)
         elif kind == "import":
             seq = self._import_alloc(op["tokens"], int(op["num_pages"]),
@@ -492,7 +495,7 @@ class ServeWorker:
     # -- prefill role --------------------------------------------------------
 
     def _release_parked(self, parked) -> None:
-        pages, nshared = parked
+        pages, nshared, slot = parked
         cache = self.engine.runner.cache
         if nshared and cache.prefix is not None:
             for pg in pages[:nshared]:
@@ -500,6 +503,8 @@ class ServeWorker:
             cache.free(pages[nshared:])
         else:
             cache.free(pages)
+        if slot:
+            cache.free_slot(slot)
 
     def _rpc_prefill(self, tokens: List[int], max_new_tokens: int,
                      decode_instance: str, temperature: float = 0.0
@@ -521,7 +526,7 @@ class ServeWorker:
             parked = self._finished_pages[seq.seq_id]
         else:
             parked = self._finished_pages.pop(seq.seq_id)
-        pages, nshared = parked
+        pages, _nshared, slot = parked
         first_token = seq.output_tokens[0]
         meta = dict(tokens=tokens, first_token=first_token,
                     num_pages=len(pages), max_new_tokens=max_new_tokens,
@@ -556,7 +561,7 @@ class ServeWorker:
                                         seq_id=res["seq_id"])
                         else:
                             self._send_pages(
-                                pages, self._peer_rank(decode_instance))
+                                pages, self._peer_rank(decode_instance), slot)
                     finally:
                         self._release_parked(parked)
             finally:
@@ -581,7 +586,7 @@ class ServeWorker:
             elif has_group:
                 self.transfer.send_pages(
                     self.engine.runner.cache, pages,
-                    self.plan().rank_of(decode_instance))
+                    self.plan().rank_of(decode_instance), slot)
             else:
                 raise RuntimeError(
                     "decode peer declined the xGMI push and no transfer "
@@ -616,10 +621,12 @@ class ServeWorker:
         """Receive the KV shard into the allocated pages and enqueue as
         running.  Runs inline (lockstep apply) or in a recv thread."""
         if self.gcomm is not None:
-            self._recv_pages(seq.block_table.pages, recv_from)
+            self._recv_pages(seq.block_table.pages, recv_from,
+                             seq.block_table.state_slot)
         else:
             self.transfer.recv_pages(self.engine.runner.cache,
-                                     seq.block_table.pages, recv_from)
+                                     seq.block_table.pages, recv_from,
+                                     seq.block_table.state_slot)
         self._import_enqueue(seq, first_token, max_new_tokens, arrival_time)
 
     def _import_enqueue(self, seq: Sequence, first_token: int,
@@ -734,9 +741,11 @@ class ServeWorker:
                 continue
             seq = entry[0]
             self._pending_imports.pop(sid, None)
-            if seq.block_table is not None and seq.block_table.pages:
-                self.engine.runner.cache.free(seq.block_table.pages)
-                seq.block_table.pages = []
+            bt = seq.block_table
+            if bt is not None and bt.pages:
+                self._release_parked((bt.pages, 0,
+                                      getattr(bt, "state_slot", 0)))
+                bt.pages = []
             self.results.pop(sid, None)
             log.warning("pending KV import %d expired after %.0fs "
                         "(prefill died mid-migration?); pages reclaimed",
@@ -763,9 +772,11 @@ class ServeWorker:
                     if s.should_stop() and s.block_table is not None:
                         self._finished_pages[s.seq_id] = (
                             list(s.block_table.pages),
-                            s.block_table.num_shared)
+                            s.block_table.num_shared,
+                            s.block_table.state_slot)
                         s.block_table.pages = []   # keep pages alive
                         s.block_table.num_shared = 0
+                        s.block_table.state_slot = 0
                 orig()
             sched._retire_finished = retire_keep_pages
         if self.tp is not None:

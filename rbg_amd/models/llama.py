@@ -17,33 +17,15 @@ orchestrates.
 from __future__ import annotations
 
 import math
-from dataclasses import dataclass
 from typing import Optional
 
 import torch
 import torch.nn as nn
 
 from .. import ops
-from ..engine.config import ModelConfig
+from ..engine.batch import ForwardBatch
+from ..engine.config import EngineConfig, ModelConfig
 from ..engine.kv_cache import PagedKVCache
-
-
-@dataclass
-class ForwardBatch:
-    """Everything the kernels need for one step; built by the model runner."""
-    mode: str                       # "prefill" | "decode"
-    positions: torch.Tensor         # [T] int32
-    slot_mapping: torch.Tensor      # [T] int32 (KV write slots)
-    # prefill
-    cu_seqlens: Optional[torch.Tensor] = None   # [B+1] int32 (q rows)
-    cu_seqlens_k: Optional[torch.Tensor] = None  # [B+1] int32 (total KV)
-    kv_gather_slots: Optional[torch.Tensor] = None  # [Tkv] int32 — prefix
-    #   caching / chunked prefill: gather the FULL [past; new] K/V from the
-    #   paged pool (the new tokens' rows were just written by rope_store_kv)
-    # decode
-    block_tables: Optional[torch.Tensor] = None  # [S, max_pages] int32
-    context_lens: Optional[torch.Tensor] = None  # [S] int32
-    decode_num_splits: int = 0      # 0 = pick host-side (sync-free in graphs)
 
 
 def _linear_weight(out_f: int, in_f: int, device, dtype, gen,
@@ -295,6 +277,9 @@ class LlamaLayer(nn.Module):
 
 
 class LlamaForCausalLM(nn.Module):
+    stateful = False        # nothing per sequence beyond its KV pages
+    mixed_steps = False     # a step is prefill or decode
+
     def __init__(self, cfg: ModelConfig, device: torch.device,
                  tp: Optional[TPContext] = None, base_seed: int = 1234,
                  pp: Optional[PPContext] = None):
@@ -305,7 +290,7 @@ class LlamaForCausalLM(nn.Module):
         self.base_seed = base_seed
         self.device = device
         dtype = torch.bfloat16
-        self.dtype = dtype
+        self.dtype = self.stream_dtype = dtype
 
         # Per-tensor generators keyed by (base_seed, tag): weights are
         # identical for every TP degree (full-then-shard) AND every PP
@@ -346,6 +331,16 @@ class LlamaForCausalLM(nn.Module):
     @property
     def num_local_layers(self) -> int:
         return self.layer_end - self.layer_start
+
+    def make_cache(self, cfg: EngineConfig) -> PagedKVCache:
+        return PagedKVCache(cfg, self.device, num_layers=self.num_local_layers)
+
+    def decode_splits(self, batch_size: int, max_seq_len: int) -> int:
+        """Sync-free split-KV policy (graph-safe: depends only on the padded
+        batch size and the config's max context)."""
+        tp = max(1, self.tp.size)
+        return ops.pick_decode_splits(batch_size, self.cfg.num_kv_heads // tp,
+                                      max_seq_len)
 
     @torch.inference_mode()
     def forward(self, tokens: torch.Tensor, batch: ForwardBatch,

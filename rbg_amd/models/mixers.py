@@ -1,0 +1,223 @@
+"""Token mixers and feed-forwards of models with an f32 residual stream.
+
+Each part loads its tensors, declares what it keeps for a sequence
+(``cache_spec``) and computes from the layer's normed input into a column slice
+of the layer's output operand: the layer concatenates the parts' products and
+applies all their output projections as ONE GEMM, which also adds them up.
+The parts that read the same input are one GEMM too (``FusedProjection``).
+
+Work split: library GEMMs for the projections, one hand-written kernel each
+for the recurrence (with decay, gates, unit keys and head norm inside) and for
+the attention (with window, softmax and, in prefill, the output gate inside).
+Tensor parallelism shards heads and feed-forward columns.
+"""
+from __future__ import annotations
+
+import math
+from typing import Any, Dict, List, Tuple
+
+import torch
+import torch.nn as nn
+
+from .. import ops
+from ..engine.batch import ForwardBatch
+from ..engine.state_cache import LayerCacheSpec, StateCache
+from .weights import WeightSource
+
+
+def param(t: torch.Tensor, dtype: torch.dtype) -> nn.Parameter:
+    return nn.Parameter(t.to(dtype).contiguous(), requires_grad=False)
+
+
+def shard(t: torch.Tensor, tp, dim: int = 0) -> torch.Tensor:
+    return t if tp.size == 1 else t.chunk(tp.size, dim=dim)[tp.rank]
+
+
+class FusedProjection(nn.Module):
+    """Several projections of one input as one GEMM.  Segments start at
+    multiples of 8 columns (zero rows between), so that every slice of the
+    result can be read 16 bytes at a time."""
+
+    def __init__(self, parts: List[Tuple[str, torch.Tensor]],
+                 dtype: torch.dtype):
+        super().__init__()
+        rows, at = [], 0
+        self.cols: Dict[str, Tuple[int, int]] = {}
+        for name, w in parts:
+            self.cols[name] = (at, w.shape[0])
+            rows.append(w)
+            pad = -w.shape[0] % 8
+            if pad:
+                rows.append(w.new_zeros(pad, w.shape[1]))
+            at += w.shape[0] + pad
+        self.weight = param(torch.cat(rows), dtype)
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        return ops.linear(x, self.weight)
+
+    def offset(self, name: str) -> int:
+        return self.cols[name][0]
+
+    def slice(self, y: torch.Tensor, name: str) -> torch.Tensor:
+        at, n = self.cols[name]
+        return y[:, at:at + n]
+
+
+class GeneralDelta(nn.Module):
+    """Generalized delta rule with per-channel decay and removal rate."""
+
+    decay_scale = math.exp(-0.5)    # w = exp(-decay_scale * sigmoid(.))
+    unit_eps = 1e-6                 # inside the root of the key's norm
+
+    def __init__(self, spec: Dict[str, Any], width: int, eps: float,
+                 src: WeightSource, prefix: str, tp, dtype: torch.dtype,
+                 decay_rank: int):
+        super().__init__()
+        heads, dim = int(spec["heads"]), int(spec["dim"])
+        assert heads % tp.size == 0, "TP degree must divide head counts"
+        self.heads, self.dim, self.eps, self.dtype = \
+            heads // tp.size, dim, eps, dtype
+        full = heads * dim
+        rank = src.shape(prefix + "w1", (decay_rank, width))[0]
+
+        def lin(name, shape):
+            return src.take(prefix + name, shape)
+        parts = [(n, shard(lin(n, (full, width)), tp))
+                 for n in ("r", "k", "v", "a", "g")]
+        parts.append(("w1", lin("w1", (rank, width))))
+        self.proj = FusedProjection(parts, dtype)
+        self.offs = [self.proj.offset(n)
+                     for n in ("r", "k", "v", "a", "g", "w1")]
+        self.w2 = param(shard(lin("w2", (full, rank)), tp), dtype)
+        f32 = torch.float32
+        self.w0 = param(shard(src.take(prefix + "w0", (full,), "normal"), tp),
+                        f32)
+        self.a_bias = param(shard(src.take(prefix + "a.b", (full,), "normal"),
+                                  tp), f32)
+        self.norm = param(shard(src.take(prefix + "norm", (full,), "ones"),
+                                tp), f32)
+        self.w_out = shard(lin("o", (width, full)), tp, dim=1)
+        self.out_dim = self.heads * dim
+
+    def cache_spec(self) -> LayerCacheSpec:
+        return LayerCacheSpec(state={
+            "delta": ((self.heads, self.dim, self.dim), torch.float32)})
+
+    def forward(self, h: torch.Tensor, out: torch.Tensor, batch: ForwardBatch,
+                cache: StateCache, layer: int) -> None:
+        y = self.proj(h)
+        state = cache.state(layer, "delta")
+
+        def run(rows, z, seqs, cu):
+            ops.delta_rule(y[rows], z, self.w2, self.w0, self.a_bias,
+                           self.norm, state, batch.state_slots[seqs], cu,
+                           batch.starts[seqs], out[rows], self.offs,
+                           self.decay_scale, self.unit_eps, self.eps)
+        every = slice(None)
+        if batch.mode == "decode":
+            run(every, None, every, None)
+            return
+        nd = batch.num_decode
+        if nd:
+            run(slice(0, nd), None, slice(0, nd), None)
+        if nd == y.shape[0]:
+            return
+        low = ops.tanh_rows(self.proj.slice(y[nd:], "w1"))
+        z = ops.linear(low, self.w2)
+        run(slice(nd, None), z, slice(nd, None), batch.cu_prefill)
+
+
+class LatentAttention(nn.Module):
+    """Softmax attention over a cached low-rank latent, without positions,
+    through a sliding window, with an output gate.
+
+    Prefill expands the visible latents to per-head keys and values; decode
+    folds the key expansion into the query and the value expansion into the
+    output, so that it streams only the latents."""
+
+    def __init__(self, spec: Dict[str, Any], width: int, eps: float,
+                 src: WeightSource, prefix: str, tp, dtype: torch.dtype):
+        super().__init__()
+        heads = int(spec["heads"])
+        assert heads % tp.size == 0, "TP degree must divide head counts"
+        self.heads = heads // tp.size
+        self.dim, self.vdim = int(spec["dim"]), int(spec["vdim"])
+        self.rank = int(spec["kv_rank"])
+        self.scale = float(spec["scale"])
+        mask = spec.get("mask") or {}
+        self.window = int(mask.get("size") or 0)     # 0: everything before
+        self.eps, self.dtype = eps, dtype
+        qk, vo = heads * self.dim, heads * self.vdim
+
+        def lin(name, shape):
+            return src.take(prefix + name, shape)
+        self.proj = FusedProjection([
+            ("q", shard(lin("q", (qk, width)), tp)),
+            ("dkv", lin("dkv", (self.rank, width))),
+            ("g", shard(lin("g", (vo, width)), tp))], dtype)
+        self.c_norm = param(src.take(prefix + "dkv.norm", (self.rank,),
+                                     "ones"), torch.float32)
+        uk = shard(lin("uk", (qk, self.rank)), tp)
+        uv = shard(lin("uv", (vo, self.rank)), tp)
+        # prefill: one expansion GEMM.  decode: per-head factors, the value
+        # one stored transposed so that no product has a transposed operand
+        self.expand = FusedProjection([("k", uk), ("v", uv)], dtype)
+        self.uk = param(uk.reshape(self.heads, self.dim, self.rank), dtype)
+        self.uv_t = param(uv.reshape(self.heads, self.vdim, self.rank)
+                          .transpose(1, 2), dtype)
+        self.w_out = shard(lin("o", (width, vo)), tp, dim=1)
+        self.out_dim = self.heads * self.vdim
+
+    def cache_spec(self) -> LayerCacheSpec:
+        return LayerCacheSpec(latent_rank=self.rank)
+
+    def forward(self, h: torch.Tensor, out: torch.Tensor, batch: ForwardBatch,
+                cache: StateCache, layer: int) -> None:
+        y = self.proj(h)
+        latents = cache.latents(layer)
+        c = ops.latent_store(self.proj.slice(y, "dkv"), self.c_norm, latents,
+                             batch.slot_mapping, self.eps)
+        nd = y.shape[0] if batch.mode == "decode" else batch.num_decode
+        if nd:
+            self._decode(y[:nd], out[:nd], batch, latents)
+        if nd < y.shape[0]:
+            self._prefill(y[nd:], c[nd:], out[nd:], batch, latents)
+
+    def _prefill(self, y, c, out, batch, latents) -> None:
+        view = batch.layout.window_view(self.window)
+        if view.slots is not None:
+            c = latents.view(-1, self.rank)[view.slots]
+        kv = self.expand(c)
+        k = self.expand.slice(kv, "k").unflatten(1, (self.heads, self.dim))
+        v = self.expand.slice(kv, "v").unflatten(1, (self.heads, self.vdim))
+        q = self.proj.slice(y, "q").unflatten(1, (self.heads, self.dim))
+        ops.window_attention(q, k, v, self.proj.slice(y, "g"), out, view,
+                             self.scale, self.window)
+
+    def _decode(self, y, out, batch, latents) -> None:
+        q = self.proj.slice(y, "q").unflatten(1, (self.heads, self.dim))
+        q = torch.bmm(q.transpose(0, 1).contiguous(), self.uk)
+        o = ops.latent_decode(q, latents, batch.block_tables,
+                              batch.context_lens, self.scale, self.window)
+        o = torch.bmm(o, self.uv_t)
+        ops.head_gate(o, self.proj.slice(y, "g"), out)
+
+
+class GatedGelu(nn.Module):
+    """down(gelu_tanh(gate x) * up x); the layer applies ``down``."""
+
+    def __init__(self, spec: Dict[str, Any], width: int, src: WeightSource,
+                 prefix: str, tp, dtype: torch.dtype):
+        super().__init__()
+        if spec.get("kind") != "dense":
+            raise ValueError(f"unknown feed-forward kind {spec.get('kind')!r}")
+        ff = int(spec["ff"])
+        assert ff % tp.size == 0, "TP degree must divide the feed-forward"
+        gate = shard(src.take(prefix + "gate", (ff, width)), tp)
+        up = shard(src.take(prefix + "up", (ff, width)), tp)
+        self.gate_up = param(torch.cat([gate, up]), dtype)
+        self.w_out = shard(src.take(prefix + "down", (width, ff)), tp, dim=1)
+        self.out_dim = ff // tp.size
+
+    def forward(self, x: torch.Tensor, out: torch.Tensor) -> None:
+        ops.gelu_mul(ops.linear(x, self.gate_up), out)

@@ -21,35 +21,30 @@ except Exception as e:  # noqa: BLE001
 
 HAVE_HIP = _hip is not None
 
+_mix = None
+_mix_err: Exception | None = None
+try:
+    from . import _hip_mix as _mix   # type: ignore[attr-defined]
+except Exception as e:  # noqa: BLE001
+    _mix_err = e
+
+HAVE_MIX = _mix is not None
+
 
 def _check_stale() -> None:
-    """Fail loudly on a GPU box if the shipped .so predates the kernel
-    sources (stale-binary guard; the stamp is written by
-    __graft_entry__.build())."""
-    import hashlib
-    import os
-    here = os.path.dirname(os.path.abspath(__file__))
-    stamp = os.path.join(here, "_hip_ops.srchash")
-    if not os.path.exists(stamp):
-        return
-    h = hashlib.sha256()
-    hip_dir = os.path.join(here, "hip")
-    for name in sorted(os.listdir(hip_dir)):
-        if name.endswith("_hip.hip"):
-            continue
-        if name.endswith((".hip", ".cpp", ".h")):
-            with open(os.path.join(hip_dir, name), "rb") as f:
-                h.update(name.encode() + b"\0" + f.read() + b"\0")
-    with open(stamp) as f:
-        recorded = f.read().strip()
-    if recorded and recorded != h.hexdigest():
-        raise RuntimeError(
-            "rbg_amd HIP extension is STALE: kernel sources changed after "
-            "the last build.  Rebuild in-tree: PYTORCH_ROCM_ARCH=gfx950 "
-            "python setup.py build_ext --inplace")
+    """Fail loudly on a GPU box if a shipped .so predates its kernel sources
+    (stale-binary guard; the stamps are written by utils/hip_build.py)."""
+    from ..utils import hip_build
+    for name, mod in (("_hip_ops", _hip), ("_hip_mix", _mix)):
+        if mod is not None and hip_build.is_stale(name):
+            raise RuntimeError(
+                f"rbg_amd HIP extension {name} is STALE: kernel sources "
+                "changed after the last build.  Rebuild in-tree: "
+                "PYTORCH_ROCM_ARCH=gfx950 python setup.py build_ext "
+                "--inplace")
 
 
-if HAVE_HIP and torch.cuda.is_available():
+if (HAVE_HIP or HAVE_MIX) and torch.cuda.is_available():
     _check_stale()
 
 
@@ -60,6 +55,15 @@ def _require_hip():
             "Build it in-tree: PYTORCH_ROCM_ARCH=gfx950 python setup.py "
             f"build_ext --inplace (import error: {_hip_err!r})")
     return _hip
+
+
+def _require_mix():
+    if _mix is None:
+        raise RuntimeError(
+            "rbg_amd HIP extension _hip_mix is not built but a GPU tensor was "
+            "passed.  Build it in-tree: PYTORCH_ROCM_ARCH=gfx950 python "
+            f"setup.py build_ext --inplace (import error: {_mix_err!r})")
+    return _mix
 
 
 def _on_gpu(t: torch.Tensor) -> bool:
@@ -83,7 +87,8 @@ def linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
             w.shape[0] % 32 == 0 and x.shape[1] % 512 == 0 and
             (w.shape[0] <= 4608 or
              (x.shape[0] <= 64 and w.shape[0] <= 8192))):
-        return _require_hip().skinny_gemm(
+        # linked into both extensions: a process has the one its model needs
+        return (_hip or _require_mix()).skinny_gemm(
             x if x.is_contiguous() else x.contiguous(), w)
     return torch.nn.functional.linear(x, w)
 
@@ -178,3 +183,132 @@ def prefill_attention(q, k, v, cu_seqlens, scale: float,
 
 
 build_cos_sin_table = reference.build_cos_sin_table
+
+
+# -- f32 residual stream ----------------------------------------------------
+
+
+def embed_stream(tokens, table, scale: float) -> torch.Tensor:
+    """f32 stream [T, W] = table[tokens] * scale."""
+    if _on_gpu(table):
+        return _require_mix().embed_stream(tokens, table, scale)
+    return reference.embed_stream(tokens, table, scale)
+
+
+def stream_norm(x, delta, w1, w2, groups: int, eps: float, dtype):
+    """x += delta (in place, f32); returns the grouped RMS norms of x under
+    w1 and w2 (None without w2) in ``dtype``."""
+    if _on_gpu(x):
+        out = _require_mix().stream_norm(x, delta, w1, w2, groups, eps,
+                                         dtype == torch.float32, None, None,
+                                         None, None)
+        return out[0], (out[1] if w2 is not None else None)
+    return reference.stream_norm(x, delta, w1, w2, groups, eps, dtype)
+
+
+def stream_norm_conv(x, delta, w1, w2, groups: int, eps: float, dtype,
+                     conv_w, conv_state, slots, positions):
+    """Decode form of stream_norm + causal_conv, one token per sequence: the
+    first result is convolved with its slot's history, which moves on."""
+    if _on_gpu(x):
+        out = _require_mix().stream_norm(x, delta, w1, w2, groups, eps,
+                                         dtype == torch.float32, conv_w,
+                                         conv_state, slots, positions)
+        return out[0], (out[1] if w2 is not None else None)
+    n1, n2 = reference.stream_norm(x, delta, w1, w2, groups, eps, dtype)
+    cu = torch.arange(n1.shape[0] + 1, dtype=torch.int32)
+    return reference.causal_conv(n1, conv_w, conv_state, cu, positions,
+                                 slots), n2
+
+
+CONV_TILE = 16
+
+
+def causal_conv(x, conv_w, conv_state, tiles, cu_seqlens, starts, slots):
+    """x + causal depthwise convolution over varlen sequences; conv_w is
+    [taps, W], conv_state [slots, taps-1, W] (advanced in place)."""
+    if _on_gpu(x):
+        return _require_mix().causal_conv(x, conv_w, conv_state, tiles,
+                                          cu_seqlens, starts, slots,
+                                          max(CONV_TILE, conv_w.shape[0]))
+    return reference.causal_conv(x, conv_w, conv_state, cu_seqlens, starts,
+                                 slots)
+
+
+# -- gates ------------------------------------------------------------------
+
+
+def gelu_mul(x, out) -> None:
+    """out (may be a column slice) = gelu_tanh(x[:, :F]) * x[:, F:]."""
+    if _on_gpu(x):
+        _require_mix().gelu_mul(x, out)
+        return
+    reference.gelu_mul(x, out)
+
+
+def tanh_rows(x) -> torch.Tensor:
+    if _on_gpu(x):
+        return _require_mix().tanh_rows(x)
+    return torch.tanh(x.float()).to(x.dtype)
+
+
+def head_gate(o, g, out) -> None:
+    """out[row, h*D+d] = o[h, row, d] * sigmoid(g[row, h*D+d])."""
+    if _on_gpu(o):
+        _require_mix().head_gate(o, g, out)
+        return
+    reference.head_gate(o, g, out)
+
+
+# -- generalized delta rule ---------------------------------------------------
+
+
+def delta_rule(proj, z, w2, w0, a_bias, norm_w, state, slots, cu_seqlens,
+               starts, out, offs, decay_scale: float, unit_eps: float,
+               norm_eps: float) -> None:
+    """Gated delta rule over varlen rows (cu_seqlens None: one row per
+    sequence), with the head norm and the output gate; ``offs`` are the
+    columns of r, k, v, a, g and the low-rank decay input in ``proj``.  The
+    decay logit is ``z``, or W2 tanh(low) formed in the kernel when None."""
+    if _on_gpu(proj):
+        _require_mix().delta_step(proj, z, w2, w0, a_bias, norm_w, state,
+                                  slots, cu_seqlens, starts, out, offs,
+                                  decay_scale, unit_eps, norm_eps)
+        return
+    reference.delta_rule(proj, z, w2, w0, a_bias, norm_w, state, slots,
+                         cu_seqlens, starts, out, offs, decay_scale, unit_eps,
+                         norm_eps)
+
+
+# -- latent attention -----------------------------------------------------------
+
+
+def latent_store(x, w, cache, slots, eps: float) -> torch.Tensor:
+    """c = rms_norm(x) * w, written to the paged latents; returns c."""
+    if _on_gpu(x):
+        return _require_mix().latent_store(x, w, cache, slots, eps)
+    return reference.latent_store(x, w, cache, slots, eps)
+
+
+def window_attention(q, k, v, gate, out, view, scale: float,
+                     window: int) -> None:
+    """Causal attention over the last ``window`` positions (0: all), q/k
+    [T, H, D], v [T, H, Dv]; ``view`` locates each query among the keys
+    (engine/batch.py WindowView).  out = o * sigmoid(gate)."""
+    if _on_gpu(q):
+        _require_mix().attn_rows(q, k, v, gate, out, view.row_info, scale,
+                                 window)
+        return
+    reference.window_attention(q, k, v, gate, out, view.row_info, scale,
+                               window)
+
+
+def latent_decode(q, cache, block_tables, context_lens, scale: float,
+                  window: int) -> torch.Tensor:
+    """q [H, S, rank] absorbed queries against the paged latents (key and
+    value at once); returns [H, S, rank]."""
+    if _on_gpu(q):
+        return _require_mix().latent_decode_rows(q, cache, block_tables,
+                                                 context_lens, scale, window)
+    return reference.latent_decode(q, cache, block_tables, context_lens,
+                                   scale, window)

@@ -1,0 +1,35 @@
+// Argument blocks shared by the token-mixer kernels and their bindings.
+#pragma once
+
+struct DeltaArgs {
+  const void* proj;       // [rows, proj_stride]; column offsets below
+  const void* z;          // [rows, heads*dim] or null: from low/w2
+  const void* w2;         // [heads*dim, rank]
+  const float* w0;        // [heads*dim]
+  const float* a_bias;    // [heads*dim]
+  const float* norm_w;    // [heads*dim]
+  float* state;           // [slots, heads, dim, dim]
+  const int* slots;       // [seqs]
+  const int* cu;          // [seqs+1] rows, or null: one row per sequence
+  const int* starts;      // [seqs] position of the first row
+  void* out;              // [rows, out_stride]
+  long proj_stride, out_stride;
+  int off_r, off_k, off_v, off_a, off_g, off_low;
+  int heads, dim, rank;
+  float decay_scale, unit_eps, norm_eps;
+};
+
+struct AttnRowsArgs {
+  const void* q;          // + row*q_row + head*q_head
+  const void* k;          // + key_row*k_row + head*k_head
+  const void* v;          // + key_row*v_row + head*v_head
+  const void* gate;       // null, or + row*g_row + head*dv: times sigmoid
+  void* out;              // + row*o_row + head*o_head
+  const int* row_info;    // contiguous: [rows, 2] = key row of position
+                          //   offset 0, offset of the query
+  const int* tables;      // paged: [rows, max_pages]
+  const int* ctx;         // paged: [rows] tokens visible incl. this one
+  long q_row, q_head, k_row, k_head, v_row, v_head, g_row, o_row, o_head;
+  int rows, heads, d, dv, window, page_size, max_pages;
+  float scale;
+};

@@ -1,0 +1,360 @@
+// PyTorch bindings for the f32-stream and token-mixer kernels (bf16 or f32
+// activations).  Shapes, strides and dtypes are checked here, before launch.
+#include <torch/extension.h>
+#include <ATen/hip/HIPContext.h>
+
+#include <hip/hip_runtime.h>
+
+#include "gemm_bindings.h"
+#include "mix_args.h"
+
+extern "C" {
+void launch_embed_stream(float*, const void*, const long*, float, int, int,
+                         int, hipStream_t);
+void launch_stream_norm(float*, const void*, const float*, const float*, void*,
+                        void*, int, int, int, float, const float*, void*,
+                        const int*, const int*, int, int, hipStream_t);
+void launch_causal_conv(void*, const void*, const float*, void*, const int*,
+                        const int*, const int*, const int*, int, int, int, int,
+                        int, hipStream_t);
+void launch_gelu_mul(void*, long, const void*, long, int, int, hipStream_t);
+void launch_tanh_rows(void*, const void*, long, long, int, int, hipStream_t);
+void launch_head_gate(void*, long, const void*, const void*, long, int, int,
+                      int, int, hipStream_t);
+void launch_delta_step(const DeltaArgs*, int, int, hipStream_t);
+void launch_latent_store(void*, void*, const void*, long, const float*,
+                         const int*, int, int, float, int, hipStream_t);
+void launch_attn_rows(const AttnRowsArgs*, int, hipStream_t);
+}
+
+namespace {
+
+using torch::Tensor;
+using OptTensor = c10::optional<torch::Tensor>;
+
+hipStream_t current_stream() {
+  return at::hip::getCurrentHIPStream().stream();
+}
+
+bool is_f32(const Tensor& t) { return t.scalar_type() == torch::kFloat32; }
+
+// activation: bf16 or f32 on the GPU, 2-D rows with a contiguous inner dim
+void check_rows(const Tensor& t, const char* name) {
+  TORCH_CHECK(t.is_cuda(), name, " must be on GPU");
+  TORCH_CHECK(t.scalar_type() == torch::kBFloat16 || is_f32(t), name,
+              " must be bf16 or f32");
+  TORCH_CHECK(t.dim() == 2 && (t.stride(1) == 1 || t.size(1) == 1), name,
+              " must be 2-D with contiguous rows");
+}
+
+void check_f32(const Tensor& t, const char* name, int64_t numel) {
+  TORCH_CHECK(t.is_cuda() && is_f32(t) && t.is_contiguous(), name,
+              " must be contiguous f32 on GPU");
+  TORCH_CHECK(t.numel() == numel, name, " has ", t.numel(), " elements, not ",
+              numel);
+}
+
+const int* i32(const Tensor& t, const char* name, int64_t at_least) {
+  TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kInt32 &&
+              t.is_contiguous(), name, " must be contiguous int32 on GPU");
+  TORCH_CHECK(t.numel() >= at_least, name, " is too short");
+  return t.data_ptr<int>();
+}
+
+void same_dtype(const Tensor& a, const Tensor& b, const char* name) {
+  TORCH_CHECK(a.scalar_type() == b.scalar_type(), name, ": dtype mismatch");
+}
+
+Tensor embed_stream(Tensor tokens, Tensor table, double scale) {
+  check_rows(table, "table");
+  TORCH_CHECK(table.is_contiguous() && tokens.is_cuda() &&
+              tokens.scalar_type() == torch::kInt64 && tokens.is_contiguous(),
+              "tokens must be int64 on GPU, table contiguous");
+  auto x = torch::empty({tokens.numel(), table.size(1)},
+                        table.options().dtype(torch::kFloat32));
+  if (tokens.numel())
+    launch_embed_stream(x.data_ptr<float>(), table.data_ptr(),
+                        (const long*)tokens.data_ptr<int64_t>(), (float)scale,
+                        (int)tokens.numel(), (int)table.size(1),
+                        is_f32(table), current_stream());
+  return x;
+}
+
+// x += delta; n1, n2 = grouped norms of x under w1, w2 (w2 optional).  With
+// conv arguments n1 becomes the convolved mixer input of a decode step.
+std::vector<Tensor> stream_norm(Tensor x, OptTensor delta, Tensor w1,
+                                OptTensor w2, int64_t groups, double eps,
+                                bool f32, OptTensor conv_w,
+                                OptTensor conv_state, OptTensor slots,
+                                OptTensor positions) {
+  TORCH_CHECK(x.is_cuda() && x.dim() == 2 && is_f32(x) && x.is_contiguous(),
+              "x must be a contiguous f32 [T, W] stream");
+  const int64_t T = x.size(0), W = x.size(1);
+  TORCH_CHECK(groups > 0 && W % groups == 0, "groups must divide the width");
+  TORCH_CHECK((W + 3 * groups + 16) * 4 <= 65536, "width too large");
+  check_f32(w1, "w1", W);
+  if (w2) check_f32(*w2, "w2", W);
+  auto opts = x.options().dtype(f32 ? torch::kFloat32 : torch::kBFloat16);
+  if (delta) {
+    check_rows(*delta, "delta");
+    TORCH_CHECK(delta->is_contiguous() && delta->size(0) == T &&
+                delta->size(1) == W && is_f32(*delta) == f32, "bad delta");
+  }
+  const float* cw = nullptr;
+  void* cs = nullptr;
+  const int *sl = nullptr, *po = nullptr;
+  int taps = 0;
+  if (conv_w) {
+    TORCH_CHECK(conv_state && slots && positions, "conv needs its state");
+    taps = (int)conv_w->size(0);
+    check_f32(*conv_w, "conv_w", taps * W);
+    TORCH_CHECK(conv_state->is_contiguous() && conv_state->dim() == 3 &&
+                conv_state->size(1) == taps - 1 && conv_state->size(2) == W &&
+                is_f32(*conv_state) == f32, "bad conv_state");
+    cw = conv_w->data_ptr<float>();
+    cs = conv_state->data_ptr();
+    sl = i32(*slots, "slots", T);
+    po = i32(*positions, "positions", T);
+  }
+  auto n1 = torch::empty({T, W}, opts);
+  Tensor n2;
+  if (w2) n2 = torch::empty({T, W}, opts);
+  if (T)
+    launch_stream_norm(x.data_ptr<float>(),
+                       delta ? delta->data_ptr() : nullptr,
+                       w1.data_ptr<float>(),
+                       w2 ? w2->data_ptr<float>() : nullptr, n1.data_ptr(),
+                       w2 ? n2.data_ptr() : nullptr, (int)T, (int)W,
+                       (int)groups, (float)eps, cw, cs, sl, po, taps, f32,
+                       current_stream());
+  return w2 ? std::vector<Tensor>{n1, n2} : std::vector<Tensor>{n1};
+}
+
+Tensor causal_conv(Tensor x, Tensor conv_w, Tensor state, Tensor tiles,
+                   Tensor cu, Tensor starts, Tensor slots, int64_t tile) {
+  check_rows(x, "x");
+  const int64_t W = x.size(1), taps = conv_w.size(0);
+  TORCH_CHECK(x.is_contiguous() && state.is_contiguous(), "contiguous only");
+  same_dtype(x, state, "conv state");
+  check_f32(conv_w, "conv_w", taps * W);
+  TORCH_CHECK(state.dim() == 3 && state.size(1) == taps - 1 &&
+              state.size(2) == W, "bad conv state");
+  TORCH_CHECK(tile >= taps - 1, "tile must cover the history");
+  TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 2, "tiles [n, 2]");
+  const int64_t B = slots.numel();
+  auto out = torch::empty_like(x);
+  if (x.size(0))
+    launch_causal_conv(out.data_ptr(), x.data_ptr(), conv_w.data_ptr<float>(),
+                       state.data_ptr(), i32(tiles, "tiles", 2),
+                       i32(cu, "cu", B + 1), i32(starts, "starts", B),
+                       i32(slots, "slots", B), (int)tiles.size(0), (int)tile,
+                       (int)W, (int)taps, is_f32(x), current_stream());
+  return out;
+}
+
+void gelu_mul(Tensor x, Tensor out) {
+  check_rows(x, "x");
+  check_rows(out, "out");
+  same_dtype(x, out, "gelu_mul");
+  TORCH_CHECK(x.is_contiguous() && x.size(1) == 2 * out.size(1) &&
+              x.size(0) == out.size(0), "x must be [T, 2*ff] of out's rows");
+  if (x.size(0))
+    launch_gelu_mul(out.data_ptr(), out.stride(0), x.data_ptr(), x.size(0),
+                    (int)out.size(1), is_f32(x), current_stream());
+}
+
+Tensor tanh_rows(Tensor x) {
+  check_rows(x, "x");
+  auto out = torch::empty({x.size(0), x.size(1)}, x.options());
+  if (x.numel())
+    launch_tanh_rows(out.data_ptr(), x.data_ptr(), x.stride(0), x.size(0),
+                     (int)x.size(1), is_f32(x), current_stream());
+  return out;
+}
+
+void head_gate(Tensor o, Tensor g, Tensor out) {
+  TORCH_CHECK(o.dim() == 3 && o.is_contiguous(), "o must be [H, rows, D]");
+  check_rows(g, "g");
+  check_rows(out, "out");
+  same_dtype(o, out, "head_gate");
+  same_dtype(g, out, "head_gate");
+  const int64_t H = o.size(0), R = o.size(1), D = o.size(2);
+  TORCH_CHECK(g.size(0) == R && g.size(1) == H * D && out.size(0) == R &&
+              out.size(1) == H * D, "head_gate shapes");
+  if (R)
+    launch_head_gate(out.data_ptr(), out.stride(0), o.data_ptr(), g.data_ptr(),
+                     g.stride(0), (int)R, (int)H, (int)D, is_f32(out),
+                     current_stream());
+}
+
+// offs: columns of r, k, v, a, g, low in proj
+DeltaArgs delta_args(const Tensor& proj, const OptTensor& z, const Tensor& w2,
+                     const Tensor& w0, const Tensor& a_bias,
+                     const Tensor& norm_w, const Tensor& state,
+                     const Tensor& slots, const OptTensor& cu,
+                     const Tensor& starts, const Tensor& out,
+                     const std::vector<int64_t>& offs, double decay_scale,
+                     double unit_eps, double norm_eps) {
+  check_rows(proj, "proj");
+  check_rows(out, "out");
+  same_dtype(proj, out, "delta");
+  TORCH_CHECK(state.dim() == 4 && state.is_cuda() && is_f32(state) &&
+              state.is_contiguous() && state.size(2) == state.size(3),
+              "state must be f32 [slots, heads, dim, dim]");
+  const int64_t H = state.size(1), D = state.size(2), HD = H * D;
+  TORCH_CHECK(D <= 256, "head dim above 256");
+  TORCH_CHECK(w2.dim() == 2 && w2.is_contiguous() && w2.size(0) == HD,
+              "w2 must be [heads*dim, rank]");
+  same_dtype(proj, w2, "delta w2");
+  const int64_t rank = w2.size(1), rows = proj.size(0), B = slots.numel();
+  TORCH_CHECK(rank <= 4096, "decay rank above 4096");
+  check_f32(w0, "w0", HD);
+  check_f32(a_bias, "a_bias", HD);
+  check_f32(norm_w, "norm_w", HD);
+  TORCH_CHECK(out.size(0) == rows && out.size(1) == HD, "out shape");
+  TORCH_CHECK(offs.size() == 6, "six column offsets");
+  for (int i = 0; i < 6; ++i)
+    TORCH_CHECK(offs[i] >= 0 &&
+                offs[i] + (i < 5 ? HD : rank) <= proj.size(1),
+                "column offset outside proj");
+  if (z) {
+    check_rows(*z, "z");
+    same_dtype(proj, *z, "delta z");
+    TORCH_CHECK(z->is_contiguous() && z->size(0) == rows && z->size(1) == HD,
+                "z shape");
+  }
+  if (!cu) TORCH_CHECK(B == rows, "one row per sequence without cu");
+  DeltaArgs p{};
+  p.proj = proj.data_ptr();
+  p.z = z ? z->data_ptr() : nullptr;
+  p.w2 = w2.data_ptr();
+  p.w0 = w0.data_ptr<float>();
+  p.a_bias = a_bias.data_ptr<float>();
+  p.norm_w = norm_w.data_ptr<float>();
+  p.state = state.data_ptr<float>();
+  p.slots = i32(slots, "slots", B);
+  p.cu = cu ? i32(*cu, "cu", B + 1) : nullptr;
+  p.starts = i32(starts, "starts", B);
+  p.out = out.data_ptr();
+  p.proj_stride = proj.stride(0);
+  p.out_stride = out.stride(0);
+  p.off_r = (int)offs[0]; p.off_k = (int)offs[1]; p.off_v = (int)offs[2];
+  p.off_a = (int)offs[3]; p.off_g = (int)offs[4]; p.off_low = (int)offs[5];
+  p.heads = (int)H; p.dim = (int)D; p.rank = (int)rank;
+  p.decay_scale = (float)decay_scale;
+  p.unit_eps = (float)unit_eps;
+  p.norm_eps = (float)norm_eps;
+  return p;
+}
+
+void delta_step(Tensor proj, OptTensor z, Tensor w2, Tensor w0, Tensor a_bias,
+                Tensor norm_w, Tensor state, Tensor slots, OptTensor cu,
+                Tensor starts, Tensor out, std::vector<int64_t> offs,
+                double decay_scale, double unit_eps, double norm_eps) {
+  const DeltaArgs p = delta_args(proj, z, w2, w0, a_bias, norm_w, state, slots,
+                                 cu, starts, out, offs, decay_scale, unit_eps,
+                                 norm_eps);
+  if (slots.numel() && proj.size(0))
+    launch_delta_step(&p, (int)slots.numel(), is_f32(proj), current_stream());
+}
+
+Tensor latent_store(Tensor x, Tensor w, Tensor cache, Tensor slots,
+                    double eps) {
+  check_rows(x, "x");
+  const int64_t T = x.size(0), R = x.size(1);
+  same_dtype(x, cache, "latent cache");
+  TORCH_CHECK(cache.is_cuda() && cache.is_contiguous() && cache.dim() == 3 &&
+              cache.size(2) == R, "cache must be [pages, page_size, rank]");
+  check_f32(w, "w", R);
+  auto c = torch::empty({T, R}, x.options());
+  if (T)
+    launch_latent_store(c.data_ptr(), cache.data_ptr(), x.data_ptr(),
+                        x.stride(0), w.data_ptr<float>(),
+                        i32(slots, "slots", T), (int)T, (int)R, (float)eps,
+                        is_f32(x), current_stream());
+  return c;
+}
+
+void check_heads(const Tensor& t, const char* name) {
+  TORCH_CHECK(t.is_cuda() && t.dim() == 3 &&
+              (t.stride(2) == 1 || t.size(2) == 1), name,
+              " must be 3-D with a contiguous inner dim");
+}
+
+// q [rows, H, D], k [keys, H, D], v [keys, H, Dv] (any row/head strides);
+// out [rows, H*Dv] (row stride free), times sigmoid(gate) when given
+void attn_rows(Tensor q, Tensor k, Tensor v, OptTensor gate, Tensor out,
+               Tensor row_info, double scale, int64_t window) {
+  check_heads(q, "q"); check_heads(k, "k"); check_heads(v, "v");
+  check_rows(out, "out");
+  same_dtype(q, k, "attn k"); same_dtype(q, v, "attn v");
+  same_dtype(q, out, "attn out");
+  const int64_t R = q.size(0), H = q.size(1), D = q.size(2), DV = v.size(2);
+  TORCH_CHECK(k.size(1) == H && k.size(2) == D && v.size(1) == H &&
+              v.size(0) == k.size(0), "k/v shapes");
+  TORCH_CHECK(out.size(0) == R && out.size(1) == H * DV, "out shape");
+  TORCH_CHECK(D <= 1024 && DV <= 1024, "head size above 1024");
+  AttnRowsArgs p{};
+  if (gate) {
+    check_rows(*gate, "gate");
+    same_dtype(q, *gate, "attn gate");
+    TORCH_CHECK(gate->size(0) == R && gate->size(1) == H * DV, "gate shape");
+    p.gate = gate->data_ptr();
+    p.g_row = gate->stride(0);
+  }
+  p.q = q.data_ptr(); p.k = k.data_ptr(); p.v = v.data_ptr();
+  p.out = out.data_ptr();
+  p.row_info = i32(row_info, "row_info", 2 * R);
+  p.q_row = q.stride(0); p.q_head = q.stride(1);
+  p.k_row = k.stride(0); p.k_head = k.stride(1);
+  p.v_row = v.stride(0); p.v_head = v.stride(1);
+  p.o_row = out.stride(0); p.o_head = DV;
+  p.rows = (int)R; p.heads = (int)H; p.d = (int)D; p.dv = (int)DV;
+  p.window = (int)window; p.scale = (float)scale;
+  if (R) launch_attn_rows(&p, is_f32(q), current_stream());
+}
+
+// q [H, rows, rank] absorbed queries over the paged latents; out the same
+Tensor latent_decode_rows(Tensor q, Tensor cache, Tensor tables, Tensor ctx,
+                          double scale, int64_t window) {
+  check_heads(q, "q");
+  same_dtype(q, cache, "latent cache");
+  const int64_t H = q.size(0), R = q.size(1), K = q.size(2);
+  TORCH_CHECK(cache.dim() == 3 && cache.is_contiguous() && cache.size(2) == K,
+              "cache must be [pages, page_size, rank]");
+  TORCH_CHECK(K <= 1024, "rank above 1024");
+  TORCH_CHECK(tables.dim() == 2 && tables.size(0) == R, "tables [rows, pages]");
+  auto out = torch::empty({H, R, K}, q.options());
+  AttnRowsArgs p{};
+  p.q = q.data_ptr(); p.k = cache.data_ptr(); p.v = cache.data_ptr();
+  p.out = out.data_ptr();
+  p.tables = i32(tables, "tables", 1);
+  p.ctx = i32(ctx, "ctx", R);
+  p.q_row = q.stride(1); p.q_head = q.stride(0);
+  p.k_row = K; p.v_row = K;
+  p.o_row = K; p.o_head = R * K;
+  p.rows = (int)R; p.heads = (int)H; p.d = (int)K; p.dv = (int)K;
+  p.window = (int)window; p.page_size = (int)cache.size(1);
+  p.max_pages = (int)tables.size(1); p.scale = (float)scale;
+  if (R) launch_attn_rows(&p, is_f32(q), current_stream());
+  return out;
+}
+
+}  // namespace
+
+PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
+  m.def("embed_stream", &embed_stream, "f32 stream = embed[token] * scale");
+  m.def("stream_norm", &stream_norm,
+        "stream += delta; grouped RMS norms (+ decode input convolution)");
+  m.def("causal_conv", &causal_conv, "x + causal depthwise conv, varlen");
+  m.def("gelu_mul", &gelu_mul, "gelu_tanh(gate) * up");
+  m.def("tanh_rows", &tanh_rows, "tanh of a column slice");
+  m.def("head_gate", &head_gate, "head-major o * sigmoid(g), row-major");
+  m.def("delta_step", &delta_step, "generalized delta rule, token by token");
+  m.def("latent_store", &latent_store, "normed latent into the paged pool");
+  m.def("attn_rows", &attn_rows, "window attention, one wave per row and head");
+  m.def("skinny_gemm", &skinny_gemm, "decode-shape GEMM (M<=128)",
+        py::arg("a"), py::arg("w"), py::arg("force_splits") = 0);
+  m.def("latent_decode_rows", &latent_decode_rows,
+        "absorbed decode attention over paged latents");
+}

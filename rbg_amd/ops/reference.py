@@ -159,3 +159,113 @@ def prefill_block_info(cu_seqlens: torch.Tensor, qtile: int = 64,
     device = cu_seqlens.device
     return (torch.tensor(infos, dtype=torch.int32, device=device).view(-1, 4),
             torch.tensor(lens, dtype=torch.int32, device=device))
+
+
+# -- f32 residual stream, delta rule, latent attention ------------------------
+
+
+def embed_stream(tokens, table, scale):
+    return table[tokens.long()].float() * scale
+
+
+def stream_norm(x, delta, w1, w2, groups, eps, dtype):
+    if delta is not None:
+        x += delta.float()
+    g = x.view(x.shape[0], groups, -1)
+    y = (g / torch.sqrt(g.pow(2).mean(-1, keepdim=True) + eps)).view_as(x)
+    return ((y * w1).to(dtype),
+            (y * w2).to(dtype) if w2 is not None else None)
+
+
+def causal_conv(x, conv_w, conv_state, cu_seqlens, starts, slots):
+    taps = conv_w.shape[0]
+    out = torch.empty_like(x)
+    cu = cu_seqlens.tolist()
+    for b, slot in enumerate(slots.tolist()):
+        rows = x[cu[b]:cu[b + 1]].float()
+        hist = conv_state[slot].float()
+        if int(starts[b]) == 0:
+            hist = torch.zeros_like(hist)
+        ext = torch.cat([hist, rows])
+        y = rows.clone()
+        for j in range(taps):
+            y += conv_w[j] * ext[j:j + rows.shape[0]]
+        out[cu[b]:cu[b + 1]] = y.to(x.dtype)
+        conv_state[slot] = ext[ext.shape[0] - (taps - 1):].to(x.dtype)
+    return out
+
+
+def gelu_mul(x, out):
+    gate, up = x.float().chunk(2, dim=-1)
+    act = torch.nn.functional.gelu(gate, approximate="tanh")
+    out.copy_((act * up).to(x.dtype))
+
+
+def head_gate(o, g, out):
+    rows = o.transpose(0, 1).reshape(g.shape).float()
+    out.copy_((rows * torch.sigmoid(g.float())).to(out.dtype))
+
+
+def delta_rule(proj, z, w2, w0, a_bias, norm_w, state, slots, cu_seqlens,
+               starts, out, offs, decay_scale, unit_eps, norm_eps):
+    H, D = state.shape[1:3]
+    r, k, v, a, g = (proj[:, o:o + H * D].float().view(-1, H, D)
+                     for o in offs[:5])
+    if z is None:
+        low = torch.tanh(proj[:, offs[5]:offs[5] + w2.shape[1]].float())
+        z = torch.nn.functional.linear(low.to(proj.dtype), w2)
+    w = torch.exp(-decay_scale * torch.sigmoid(z.float() + w0)).view(-1, H, D)
+    a = torch.sigmoid(a + a_bias.view(H, D))
+    u = k * torch.rsqrt(k.pow(2).sum(-1, keepdim=True) + unit_eps)
+    B = slots.numel()
+    cu = (cu_seqlens.tolist() if cu_seqlens is not None
+          else list(range(B + 1)))
+    for b, slot in enumerate(slots.tolist()):
+        S = state[slot]
+        if int(starts[b]) == 0:
+            S.zero_()
+        for t in range(cu[b], cu[b + 1]):
+            proj_u = torch.einsum("hk,hkv->hv", u[t], S)
+            S.mul_(w[t].unsqueeze(-1))
+            S.sub_((a[t] * u[t]).unsqueeze(-1) * proj_u.unsqueeze(1))
+            S.add_(k[t].unsqueeze(-1) * v[t].unsqueeze(1))
+            o = torch.einsum("hk,hkv->hv", r[t], S)
+            o = o / torch.sqrt(o.pow(2).mean(-1, keepdim=True) + norm_eps)
+            o = o.reshape(-1) * norm_w * torch.sigmoid(g[t].reshape(-1))
+            out[t] = o.to(out.dtype)
+
+
+def latent_store(x, w, cache, slots, eps):
+    xf = x.float()
+    c = (xf / torch.sqrt(xf.pow(2).mean(-1, keepdim=True) + eps) * w)
+    c = c.to(x.dtype)
+    cache.view(-1, cache.shape[-1])[slots.long()] = c
+    return c
+
+
+def window_attention(q, k, v, gate, out, row_info, scale, window):
+    T, H, _ = q.shape
+    for t, (base, pos) in enumerate(row_info.tolist()):
+        lo = max(0, pos - window + 1) if window > 0 else 0
+        ks = k[base + lo:base + pos + 1].float()
+        s = torch.einsum("hd,khd->hk", q[t].float(), ks) * scale
+        o = torch.einsum("hk,khd->hd", torch.softmax(s, dim=-1),
+                         v[base + lo:base + pos + 1].float()).reshape(-1)
+        if gate is not None:
+            o = o * torch.sigmoid(gate[t].float())
+        out[t] = o.to(out.dtype)
+
+
+def latent_decode(q, cache, block_tables, context_lens, scale, window):
+    H, S, R = q.shape
+    out = torch.empty_like(q)
+    ps = cache.shape[1]
+    flat = cache.view(-1, R)
+    for s in range(S):
+        ctx = int(context_lens[s])
+        lo = max(0, ctx - window) if window > 0 else 0
+        j = torch.arange(lo, ctx)
+        c = flat[block_tables[s].long()[j // ps] * ps + j % ps].float()
+        p = torch.softmax(q[:, s].float() @ c.T * scale, dim=-1)
+        out[:, s] = (p @ c).to(q.dtype)
+    return out

@@ -84,13 +84,11 @@ class TransferEngine:
                             if self.backend == "nccl" else "cpu")
 
     def send_pages(self, cache: PagedKVCache, pages: List[int],
-                   dst_rank: int) -> None:
+                   dst_rank: int, slot: int = 0) -> None:
         from .comm import to_wire
         self.connect()
         with self._lock:
-            idx = torch.tensor(pages, dtype=torch.int64,
-                               device=cache.kv.device)
-            buf = cache.kv.index_select(2, idx).contiguous()
+            buf = cache.export_pages(pages, slot)
             if self.backend == "gloo" and buf.is_cuda:
                 buf = buf.cpu()
             buf = to_wire(buf)
@@ -103,15 +101,14 @@ class TransferEngine:
                 dist.send(buf, dst_rank)
 
     def recv_pages(self, cache: PagedKVCache, pages: List[int],
-                   src_rank: int) -> None:
+                   src_rank: int, slot: int = 0) -> None:
         from .comm import from_wire, wire_dtype
         self.connect()
         with self._lock:
-            m = cache.kv.shape
-            shape = (m[0], m[1], len(pages), m[3], m[4], m[5])
+            shape, dtype = cache.export_shape(len(pages))
             dev = (cache.kv.device if self.backend == "nccl"
                    else torch.device("cpu"))
-            buf = torch.empty(shape, dtype=wire_dtype(cache.kv.dtype, dev),
+            buf = torch.empty(shape, dtype=wire_dtype(dtype, dev),
                               device=dev)
             if self._stream is not None:
                 with torch.cuda.stream(self._stream):
@@ -119,7 +116,4 @@ class TransferEngine:
                 self._stream.synchronize()
             else:
                 dist.recv(buf, src_rank)
-            buf = from_wire(buf, cache.kv.dtype)
-            idx = torch.tensor(pages, dtype=torch.int64,
-                               device=cache.kv.device)
-            cache.kv.index_copy_(2, idx, buf.to(cache.kv.device))
+            cache.import_pages(pages, from_wire(buf, dtype), slot)

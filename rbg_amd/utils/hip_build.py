@@ -1,0 +1,105 @@
+"""In-tree build of the HIP extensions (gfx950) and their freshness stamps.
+
+Each extension carries a stamp: a hash over its sources and the shared headers
+at build time.  A process on a GPU box refuses an extension whose sources have
+changed since (ops/__init__.py), and ``ensure`` builds a missing or stale one,
+so that a fresh checkout compiles only what its model runs on.
+"""
+from __future__ import annotations
+
+import fcntl
+import glob
+import hashlib
+import os
+import shutil
+import subprocess
+import sys
+from typing import Iterable, Optional
+
+ROOT = os.path.dirname(os.path.dirname(os.path.dirname(
+    os.path.abspath(__file__))))
+OPS_DIR = os.path.join(ROOT, "rbg_amd", "ops")
+HIP_DIR = os.path.join(OPS_DIR, "hip")
+
+# Canonical sources, listed explicitly: a glob would also pick up hipify
+# build artifacts (*_hip.hip) that torch's cpp_extension emits next to
+# the originals, risking duplicate extern-C symbols from drifted copies.
+HIP_SOURCES = {
+    # bf16 attention/norm/GEMM kernels, KV push, xGMI all-reduce
+    "_hip_ops": [
+        "attn_decode.hip",
+        "attn_prefill.hip",
+        "mfma_probe.hip",
+        "rmsnorm.hip",
+        "rope_kv.hip",
+        "silu_mul.hip",
+        "skinny_gemm.hip",
+        "kv_peer_copy.hip",
+        "allreduce.hip",
+        "bindings.cpp",
+    ],
+    # f32-stream norms and the token mixers (delta rule, latents)
+    "_hip_mix": [
+        "stream_norm.hip",
+        "gated_act.hip",
+        "delta_rule.hip",
+        "latent_attn.hip",
+        "skinny_gemm.hip",
+        "mix_bindings.cpp",
+    ],
+}
+
+# model architecture -> the extension with its kernels (default: _hip_ops)
+EXTENSION_OF = {"Bitatar": "_hip_mix"}
+
+
+def source_hash(name: str) -> str:
+    headers = [f for f in os.listdir(HIP_DIR) if f.endswith(".h")]
+    h = hashlib.sha256()
+    for f in sorted(HIP_SOURCES[name] + headers):
+        with open(os.path.join(HIP_DIR, f), "rb") as fh:
+            h.update(f.encode() + b"\0" + fh.read() + b"\0")
+    return h.hexdigest()
+
+
+def stamp_path(name: str) -> str:
+    return os.path.join(OPS_DIR, f"{name}.srchash")
+
+
+def is_stale(name: str) -> bool:
+    """The stamp disagrees with the sources (no stamp: cannot tell)."""
+    try:
+        with open(stamp_path(name)) as f:
+            recorded = f.read().strip()
+    except FileNotFoundError:
+        return False
+    return bool(recorded) and recorded != source_hash(name)
+
+
+def is_built(name: str) -> bool:
+    return bool(glob.glob(os.path.join(OPS_DIR, f"{name}.*.so")))
+
+
+def build(names: Optional[Iterable[str]] = None, clean: bool = False) -> None:
+    """Compile extensions in-tree; ``clean`` recompiles every object."""
+    names = list(names or HIP_SOURCES)
+    if clean:
+        shutil.rmtree(os.path.join(ROOT, "build"), ignore_errors=True)
+    env = dict(os.environ, PYTORCH_ROCM_ARCH="gfx950",
+               RBG_BUILD_EXT=",".join(names))
+    # compiler output goes to stderr: a caller's stdout may be a protocol
+    subprocess.run([sys.executable, "setup.py", "build_ext", "--inplace"],
+                   cwd=ROOT, env=env, check=True, stdout=sys.stderr)
+    for name in names:
+        with open(stamp_path(name), "w") as f:
+            f.write(source_hash(name))
+
+
+def ensure(name: str) -> None:
+    """Build one extension if it is missing or stale (one builder at a time)."""
+    if is_built(name) and not is_stale(name):
+        return
+    with open(os.path.join(ROOT, ".build.lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        if not is_built(name) or is_stale(name):
+            build([name])

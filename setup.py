@@ -1,8 +1,11 @@
-"""In-tree build of the rbg_amd HIP extension for gfx950 (MI355X).
+"""In-tree build of the rbg_amd HIP extensions for gfx950 (MI355X).
 
 Usage: PYTORCH_ROCM_ARCH=gfx950 python setup.py build_ext --inplace
-The resulting rbg_amd/ops/_hip_ops*.so travels with the repo snapshot to GPU
+The resulting rbg_amd/ops/_hip_*.so travel with the repo snapshot to GPU
 boxes (no JIT cache involved).
+
+The extensions and their sources are listed in rbg_amd/utils/hip_build.py;
+RBG_BUILD_EXT=<name>[,<name>] restricts the build to some of them.
 """
 import os
 import sys
@@ -13,39 +16,28 @@ os.environ.setdefault("PYTORCH_ROCM_ARCH", "gfx950")
 
 from torch.utils.cpp_extension import BuildExtension, CUDAExtension  # noqa: E402
 
-ROOT = os.path.dirname(os.path.abspath(__file__))
-HIP_DIR = os.path.join(ROOT, "rbg_amd", "ops", "hip")
+sys.path.insert(0, os.path.dirname(os.path.abspath(__file__)))
+from rbg_amd.utils.hip_build import HIP_SOURCES  # noqa: E402
 
-# Canonical sources, listed explicitly: the glob previously also picked up
-# hipify build artifacts (*_hip.hip) that torch's cpp_extension emits next to
-# the originals, risking duplicate extern-C symbols from drifted copies.
-HIP_SOURCES = [
-    "attn_decode.hip",
-    "attn_prefill.hip",
-    "mfma_probe.hip",
-    "rmsnorm.hip",
-    "rope_kv.hip",
-    "silu_mul.hip",
-    "skinny_gemm.hip",
-    "kv_peer_copy.hip",
-    "allreduce.hip",
-    "bindings.cpp",
-]
-sources = [os.path.join(HIP_DIR, f) for f in HIP_SOURCES]
+HIP_DIR = os.path.join("rbg_amd", "ops", "hip")
 
-ext = CUDAExtension(
-    name="rbg_amd.ops._hip_ops",
-    sources=sources,
-    extra_compile_args={
-        "cxx": ["-O3", "-std=c++17"],
-        "nvcc": ["-O3", "-std=c++17", "--offload-arch=gfx950"],
-    },
-)
+# no packed-f32 VALU instructions: some of their forms are unreliable here
+NVCC_ARGS = ["-O3", "-std=c++17", "--offload-arch=gfx950",
+             "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+
+only = [n for n in os.environ.get("RBG_BUILD_EXT", "").split(",") if n]
+ext_modules = [
+    CUDAExtension(
+        name=f"rbg_amd.ops.{name}",
+        sources=[os.path.join(HIP_DIR, f) for f in files],
+        extra_compile_args={"cxx": ["-O3", "-std=c++17"], "nvcc": NVCC_ARGS},
+    )
+    for name, files in HIP_SOURCES.items() if not only or name in only]
 
 setup(
     name="rbg-mi355x",
     version="0.1.0",
     packages=["rbg_amd"],
-    ext_modules=[ext],
+    ext_modules=ext_modules,
     cmdclass={"build_ext": BuildExtension.with_options(use_ninja=True)},
 )
