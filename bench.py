@@ -50,6 +50,12 @@ def parse_args():
                         "tp/pp: all ranks form one sharded engine")
     p.add_argument("--eager", action="store_true",
                    help="disable hipGraph capture")
+    p.add_argument("--compare", choices=["bitatar"], default=None,
+                   help="instead: prefill/decode throughput of this family "
+                        "beside Llama at equal size, one GPU, one JSON line "
+                        "per workload (--sizes, --batches, --seq-len)")
+    p.add_argument("--sizes", default="2k,4k", help="with --compare")
+    p.add_argument("--batches", default="1,32", help="with --compare")
     return p.parse_args()
 
 
@@ -95,6 +101,16 @@ def main() -> int:
         return 1
     if device == "cuda" and not distributed:
         torch.cuda.set_device(local_rank)
+
+    if args.compare:
+        from rbg_amd.engine.model_bench import run_compare
+        for row in run_compare(device, args.steps, args.warmup,
+                               sizes=args.sizes.split(","),
+                               batches=[int(b) for b in
+                                        args.batches.split(",")],
+                               prompt=args.seq_len, eager=args.eager):
+            print(json.dumps(row), flush=True)
+        return 0
 
     if args.parallel == "pd":
         from rbg_amd.engine.pd_bench import run_pd

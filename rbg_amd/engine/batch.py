@@ -50,7 +50,11 @@ class WindowView:
     #                                 sequence, the query's offset among them
     seq_info: torch.Tensor          # [seqs, 4] int32: first query row, rows,
     #                                 first key row, first query's offset
-    lens: List[int]                 # query rows per sequence
+    blocks: torch.Tensor            # [n, 2] int32: (sequence, first query)
+    #                                 of every 128 query rows
+
+
+QUERY_BLOCK = 128       # query rows per workgroup of the window attention
 
 
 class VarlenLayout:
@@ -64,7 +68,7 @@ class VarlenLayout:
         self.page_size = page_size
         self.device = device
         self._views: Dict[int, WindowView] = {}
-        self._tiles: Dict[int, torch.Tensor] = {}
+        self._tiles: Dict[object, torch.Tensor] = {}
 
     def _dev(self, a: np.ndarray) -> torch.Tensor:
         return torch.from_numpy(np.ascontiguousarray(a)).to(self.device)
@@ -81,7 +85,7 @@ class VarlenLayout:
     def prefill_tiles(self, tile: int) -> torch.Tensor:
         """Like tiles(), over the sequences after the decode rows, with
         sequence numbers counted from there."""
-        key = -tile
+        key = ("prefill", tile)
         if key not in self._tiles:
             out = [(b, t) for b in range(len(self.starts) - self.num_decode)
                    for t in range(0, self.ends[b + self.num_decode] -
@@ -90,12 +94,22 @@ class VarlenLayout:
                 np.array(out, dtype=np.int32).reshape(-1, 2))
         return self._tiles[key]
 
+    def prefill_tile_cu(self, tile: int) -> torch.Tensor:
+        """[seqs + 1] int32: where each sequence's prefill_tiles begin."""
+        key = ("cu", tile)
+        if key not in self._tiles:
+            n = [0] + [(e - s + tile - 1) // tile
+                       for s, e in zip(self.starts[self.num_decode:],
+                                       self.ends[self.num_decode:])]
+            self._tiles[key] = self._dev(np.cumsum(n).astype(np.int32))
+        return self._tiles[key]
+
     def window_view(self, window: int) -> WindowView:
         """Of the prefill sequences; rows are counted after the decode rows."""
         if window in self._views:
             return self._views[window]
         ps = self.page_size
-        slots, info, seqs, lens = [], [], [], []
+        slots, info, seqs = [], [], []
         base = row = 0
         past = False
         for s, e, table in list(zip(self.starts, self.ends,
@@ -108,13 +122,12 @@ class VarlenLayout:
             off = np.arange(s - k0, e - k0)
             info.append(np.stack([np.full_like(off, base), off], axis=1))
             seqs.append((row, e - s, base, s - k0))
-            lens.append(e - s)
             base += e - k0
             row += e - s
         view = WindowView(
             slots=self._dev(np.concatenate(slots)) if past else None,
             row_info=self._dev(np.concatenate(info).astype(np.int32)),
             seq_info=self._dev(np.array(seqs, dtype=np.int32)),
-            lens=lens)
+            blocks=self.prefill_tiles(QUERY_BLOCK))
         self._views[window] = view
         return view

@@ -108,11 +108,11 @@ class GeneralDelta(nn.Module):
         y = self.proj(h)
         state = cache.state(layer, "delta")
 
-        def run(rows, z, seqs, cu):
+        def run(rows, z, seqs, cu, chunks=None):
             ops.delta_rule(y[rows], z, self.w2, self.w0, self.a_bias,
                            self.norm, state, batch.state_slots[seqs], cu,
                            batch.starts[seqs], out[rows], self.offs,
-                           self.decay_scale, self.unit_eps, self.eps)
+                           self.decay_scale, self.unit_eps, self.eps, chunks)
         every = slice(None)
         if batch.mode == "decode":
             run(every, None, every, None)
@@ -124,7 +124,10 @@ class GeneralDelta(nn.Module):
             return
         low = ops.tanh_rows(self.proj.slice(y[nd:], "w1"))
         z = ops.linear(low, self.w2)
-        run(slice(nd, None), z, slice(nd, None), batch.cu_prefill)
+        layout = batch.layout
+        run(slice(nd, None), z, slice(nd, None), batch.cu_prefill,
+            (layout.prefill_tiles(ops.DELTA_CHUNK),
+             layout.prefill_tile_cu(ops.DELTA_CHUNK)))
 
 
 class LatentAttention(nn.Module):
@@ -159,12 +162,11 @@ class LatentAttention(nn.Module):
                                      "ones"), torch.float32)
         uk = shard(lin("uk", (qk, self.rank)), tp)
         uv = shard(lin("uv", (vo, self.rank)), tp)
-        # prefill: one expansion GEMM.  decode: per-head factors, the value
-        # one stored transposed so that no product has a transposed operand
+        # prefill: one expansion GEMM.  decode: per-head maps [n, k]
         self.expand = FusedProjection([("k", uk), ("v", uv)], dtype)
-        self.uk = param(uk.reshape(self.heads, self.dim, self.rank), dtype)
-        self.uv_t = param(uv.reshape(self.heads, self.vdim, self.rank)
+        self.uk_t = param(uk.reshape(self.heads, self.dim, self.rank)
                           .transpose(1, 2), dtype)
+        self.uv = param(uv.reshape(self.heads, self.vdim, self.rank), dtype)
         self.w_out = shard(lin("o", (width, vo)), tp, dim=1)
         self.out_dim = self.heads * self.vdim
 
@@ -196,11 +198,10 @@ class LatentAttention(nn.Module):
 
     def _decode(self, y, out, batch, latents) -> None:
         q = self.proj.slice(y, "q").unflatten(1, (self.heads, self.dim))
-        q = torch.bmm(q.transpose(0, 1).contiguous(), self.uk)
+        q = ops.head_linear(q, self.uk_t).unflatten(1, (self.heads, self.rank))
         o = ops.latent_decode(q, latents, batch.block_tables,
                               batch.context_lens, self.scale, self.window)
-        o = torch.bmm(o, self.uv_t)
-        ops.head_gate(o, self.proj.slice(y, "g"), out)
+        ops.head_linear(o, self.uv, gate=self.proj.slice(y, "g"), out=out)
 
 
 class GatedGelu(nn.Module):

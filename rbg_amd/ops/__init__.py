@@ -252,28 +252,31 @@ def tanh_rows(x) -> torch.Tensor:
     return torch.tanh(x.float()).to(x.dtype)
 
 
-def head_gate(o, g, out) -> None:
-    """out[row, h*D+d] = o[h, row, d] * sigmoid(g[row, h*D+d])."""
-    if _on_gpu(o):
-        _require_mix().head_gate(o, g, out)
-        return
-    reference.head_gate(o, g, out)
-
-
 # -- generalized delta rule ---------------------------------------------------
+
+
+DELTA_CHUNK = 16        # tokens per chunk of the prompt kernels
 
 
 def delta_rule(proj, z, w2, w0, a_bias, norm_w, state, slots, cu_seqlens,
                starts, out, offs, decay_scale: float, unit_eps: float,
-               norm_eps: float) -> None:
+               norm_eps: float, chunks=None) -> None:
     """Gated delta rule over varlen rows (cu_seqlens None: one row per
     sequence), with the head norm and the output gate; ``offs`` are the
     columns of r, k, v, a, g and the low-rank decay input in ``proj``.  The
-    decay logit is ``z``, or W2 tanh(low) formed in the kernel when None."""
+    decay logit is ``z``, or W2 tanh(low) formed in the kernel when None.
+    With ``chunks`` = (tiles, chunk_cu) of DELTA_CHUNK tokens and a ``z``, the
+    rows go through the matrix cores a chunk at a time."""
     if _on_gpu(proj):
-        _require_mix().delta_step(proj, z, w2, w0, a_bias, norm_w, state,
-                                  slots, cu_seqlens, starts, out, offs,
-                                  decay_scale, unit_eps, norm_eps)
+        mix = _require_mix()
+        args = (proj, z, w2, w0, a_bias, norm_w, state, slots, cu_seqlens,
+                starts, out, offs, decay_scale, unit_eps, norm_eps)
+        # the chunk form scales by e^(DELTA_CHUNK * decay_scale)
+        if (chunks is not None and z is not None and state.shape[-1] <= 128
+                and decay_scale * DELTA_CHUNK <= 60.0):
+            mix.delta_chunk(*args, *chunks)
+        else:
+            mix.delta_step(*args)
         return
     reference.delta_rule(proj, z, w2, w0, a_bias, norm_w, state, slots,
                          cu_seqlens, starts, out, offs, decay_scale, unit_eps,
@@ -296,19 +299,45 @@ def window_attention(q, k, v, gate, out, view, scale: float,
     [T, H, D], v [T, H, Dv]; ``view`` locates each query among the keys
     (engine/batch.py WindowView).  out = o * sigmoid(gate)."""
     if _on_gpu(q):
-        _require_mix().attn_rows(q, k, v, gate, out, view.row_info, scale,
-                                 window)
+        _require_mix().window_attention(q, k, v, gate, out, view.row_info,
+                                        view.seq_info, view.blocks, scale,
+                                        window)
         return
     reference.window_attention(q, k, v, gate, out, view.row_info, scale,
                                window)
 
 
+def pick_latent_splits(num_seqs: int, num_heads: int, max_keys: int) -> int:
+    """Key splits of latent_decode: about two workgroups per CU, at least one
+    16-key chunk for each of a workgroup's four waves.  Depends on sizes only,
+    so a captured decode step keeps its value."""
+    base = num_seqs * ((num_heads + 15) // 16)
+    by_keys = max(1, (max_keys + 15) // 64)
+    return int(max(1, min((512 + base - 1) // base, by_keys, 64)))
+
+
 def latent_decode(q, cache, block_tables, context_lens, scale: float,
                   window: int) -> torch.Tensor:
-    """q [H, S, rank] absorbed queries against the paged latents (key and
-    value at once); returns [H, S, rank]."""
+    """q [S, H, rank] absorbed queries against the paged latents (key and
+    value at once); returns [S, H, rank]."""
     if _on_gpu(q):
-        return _require_mix().latent_decode_rows(q, cache, block_tables,
-                                                 context_lens, scale, window)
+        keys = block_tables.shape[1] * cache.shape[1]
+        splits = pick_latent_splits(q.shape[0], q.shape[1],
+                                    min(keys, window) if window else keys)
+        return _require_mix().latent_decode(q, cache, block_tables,
+                                            context_lens, scale, window,
+                                            splits)
     return reference.latent_decode(q, cache, block_tables, context_lens,
                                    scale, window)
+
+
+def head_linear(x, w, gate=None, out=None) -> torch.Tensor:
+    """out[s, h*n + j] = sum_k x[s, h, k] w[h, j, k], times sigmoid(gate);
+    ``out`` [S, H*n] may be a column slice."""
+    if out is None:
+        out = x.new_empty((x.shape[0], w.shape[0] * w.shape[1]))
+    if _on_gpu(x):
+        _require_mix().head_linear(x, w, gate, out)
+    else:
+        reference.head_linear(x, w, gate, out)
+    return out

@@ -1,5 +1,5 @@
-// Elementwise gates in bf16 or f32: gelu_tanh(gate) * up, tanh of a low-rank
-// projection, and o * sigmoid(g).  Inputs and outputs are column slices of the
+// Elementwise gates in bf16 or f32: gelu_tanh(gate) * up, and tanh of a low-rank
+// projection.  Inputs and outputs are column slices of the
 // fused projection buffers (row strides), so no copy stands between a GEMM and
 // its gate, and the products land in the operand of the layer's output GEMM.
 #include "vec_io.h"
@@ -39,27 +39,6 @@ __global__ void tanh_rows_kernel(T* __restrict__ out, const T* __restrict__ x,
   out[i] = from_f<T>(tanhf(to_f(x[(i / width) * stride + i % width])));
 }
 
-// o [H, rows, D] head-major -> out[row, h*D + d] * sigmoid(g[row, h*D + d])
-template <typename T, int V>
-__global__ void head_gate_kernel(T* __restrict__ out, const long out_stride,
-                                 const T* __restrict__ o,
-                                 const T* __restrict__ g, const long g_stride,
-                                 const int rows, const int heads,
-                                 const int dim, const long total) {
-  const long i = blockIdx.x * (long)blockDim.x + threadIdx.x;
-  if (i >= total) return;
-  const int nv = heads * dim / V;
-  const long row = i / nv;
-  const int c = (int)(i % nv) * V;
-  const int h = c / dim, d = c % dim;
-  float ov[V], gv[V];
-  load_vec<V>(o + ((long)h * rows + row) * dim + d, ov);
-  load_vec<V>(g + row * g_stride + c, gv);
-#pragma unroll
-  for (int j = 0; j < V; ++j) ov[j] *= sigmoid_f(gv[j]);
-  store_vec<V>(out + row * out_stride + c, ov);
-}
-
 int blocks_for(long total) {
   long b = (total + 255) / 256;
   return (int)(b < 1 ? 1 : b);
@@ -82,20 +61,6 @@ void gelu_mul_t(void* out, long os, const void* x, long rows, int inter,
                                             total);
 }
 
-template <typename T>
-void head_gate_t(void* out, long os, const void* o, const void* g, long gs,
-                 int rows, int heads, int dim, hipStream_t s) {
-  const bool vec = dim % 8 == 0 && os % 8 == 0 && gs % 8 == 0 &&
-                   aligned16(out) && aligned16(g);
-  const long total = (long)rows * heads * dim / (vec ? 8 : 1);
-  if (vec)
-    head_gate_kernel<T, 8><<<blocks_for(total), 256, 0, s>>>(
-        (T*)out, os, (const T*)o, (const T*)g, gs, rows, heads, dim, total);
-  else
-    head_gate_kernel<T, 1><<<blocks_for(total), 256, 0, s>>>(
-        (T*)out, os, (const T*)o, (const T*)g, gs, rows, heads, dim, total);
-}
-
 }  // namespace
 
 extern "C" {
@@ -115,16 +80,6 @@ void launch_tanh_rows(void* out, const void* x, long stride, long rows,
   else
     tanh_rows_kernel<__hip_bfloat16><<<blocks_for(total), 256, 0, s>>>(
         (__hip_bfloat16*)out, (const __hip_bfloat16*)x, stride, width, total);
-}
-
-void launch_head_gate(void* out, long out_stride, const void* o, const void* g,
-                      long g_stride, int rows, int heads, int dim, int f32,
-                      hipStream_t s) {
-  if (f32)
-    head_gate_t<float>(out, out_stride, o, g, g_stride, rows, heads, dim, s);
-  else
-    head_gate_t<__hip_bfloat16>(out, out_stride, o, g, g_stride, rows, heads,
-                                dim, s);
 }
 
 }  // extern "C"

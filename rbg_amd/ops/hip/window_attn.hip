@@ -1,0 +1,251 @@
+// Causal window attention over contiguous keys and values (gfx950, bf16):
+// varlen prefill of any head sizes up to 256, with an optional sigmoid output
+// gate.  A query at position i sees keys j with 0 <= i - j < window.
+//
+// A workgroup takes 128 query rows of one head (NW waves x QT x 16) and walks the
+// 64-key tiles between its first row's window edge and its last row.  Per tile
+//   S^T = K Q^T      A = K rows from LDS, B = Q rows held in registers
+//   softmax          a query is a lane column: row max and sum are in-lane
+//                    plus two shuffles, and the rescale is one scalar
+//   O^T += V^T P^T   B = the softmax registers themselves (see mfma_util.h),
+//                    split in two bf16 so the weights keep 16 bits; A = V read
+//                    from row-major LDS through the transposing read
+// so the weights never touch LDS.  The next tile's global loads fly under the
+// current tile's MFMAs.  Row pitch is dim + 16 elements: 8 banks per row, which
+// keeps both read patterns conflict-free.
+#include "mfma_util.h"
+#include "mix_args.h"
+#include "vec_io.h"
+
+namespace {
+
+constexpr int KT = 64;
+
+template <int DK, int DV, int NW, int QT>
+__global__ __launch_bounds__(NW * 64, (DK + DV) > 256 ? 1 : 2)
+void window_attn_kernel(const WindowAttnArgs p) {
+  constexpr int KP = DK + 16, VP = DV + 16;
+  constexpr int ROWS = NW * QT * 16;          // 128
+  constexpr int NT = NW * 64;
+  constexpr int KPC = KT * DK / 8 / NT, VPC = KT * DV / 8 / NT;
+  __shared__ __hip_bfloat16 ks[KT * KP];
+  __shared__ __hip_bfloat16 vs[KT * VP];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int gl = lane & 15, gs = lane >> 4;
+
+  // workgroups go round the 8 XCDs: give each XCD whole heads, so that the
+  // query tiles of a head share its keys and values in one L2
+  const int items = p.n_blocks * p.heads, per = (items + 7) / 8;
+  const int work = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+  if ((blockIdx.x >> 3) >= per || work >= items) return;
+  const int head = work / p.n_blocks;
+  const int* bi = p.blocks + (p.n_blocks - 1 - work % p.n_blocks) * 2;
+  const int* si = p.seq_info + bi[0] * 4;
+  const int qrow0 = si[0], qlen = si[1], krow0 = si[2], qoff = si[3];
+  const int t0 = bi[1];                       // first query of the block
+  const int klen = qoff + qlen;
+
+  const __hip_bfloat16* q = (const __hip_bfloat16*)p.q + head * p.q_head;
+  const __hip_bfloat16* k = (const __hip_bfloat16*)p.k + head * p.k_head;
+  const __hip_bfloat16* v = (const __hip_bfloat16*)p.v + head * p.v_head;
+
+  // Q as B operand: column = query, 8 dims per lane
+  mf_bf8 qf[QT][DK / 32];
+  int qpos[QT];
+#pragma unroll
+  for (int t = 0; t < QT; ++t) {
+    const int r = t0 + (wave * QT + t) * 16 + gl;
+    qpos[t] = qoff + r;                       // may lie past the end: unused
+    const __hip_bfloat16* qr = q + (size_t)(qrow0 + min(r, qlen - 1)) * p.q_row;
+#pragma unroll
+    for (int s = 0; s < DK / 32; ++s) {
+      const int d = s * 32 + gs * 8;
+      mf_bf8 z = {};
+      qf[t][s] = d < p.d ? frag8(qr + d) : z;
+    }
+  }
+
+  const int last = min(qoff + t0 + ROWS - 1, klen - 1);
+  const int first = p.window > 0 ? max(0, qoff + t0 - p.window + 1) : 0;
+  const int wlo = p.window > 0
+      ? max(0, qoff + t0 + wave * QT * 16 - p.window + 1) : 0;
+  const int whi = min(qoff + t0 + (wave + 1) * QT * 16 - 1, klen - 1);
+
+  u32x4 kr[KPC], vr[VPC];
+  const u32x4 zero4 = {0, 0, 0, 0};
+  auto fetch = [&](int kt) {
+#pragma unroll
+    for (int i = 0; i < KPC; ++i) {
+      const int e = tid + i * NT, key = e / (DK / 8), c = (e % (DK / 8)) * 8;
+      const size_t row = krow0 + min(kt * KT + key, klen - 1);
+      kr[i] = c < p.d ? *reinterpret_cast<const u32x4*>(k + row * p.k_row + c)
+                      : zero4;
+    }
+#pragma unroll
+    for (int i = 0; i < VPC; ++i) {
+      const int e = tid + i * NT, key = e / (DV / 8), c = (e % (DV / 8)) * 8;
+      const size_t row = krow0 + min(kt * KT + key, klen - 1);
+      vr[i] = c < p.dv ? *reinterpret_cast<const u32x4*>(v + row * p.v_row + c)
+                       : zero4;
+    }
+  };
+  auto land = [&]() {
+#pragma unroll
+    for (int i = 0; i < KPC; ++i) {
+      const int e = tid + i * NT, key = e / (DK / 8), c = (e % (DK / 8)) * 8;
+      *reinterpret_cast<u32x4*>(&ks[key * KP + c]) = kr[i];
+    }
+#pragma unroll
+    for (int i = 0; i < VPC; ++i) {
+      const int e = tid + i * NT, key = e / (DV / 8), c = (e % (DV / 8)) * 8;
+      *reinterpret_cast<u32x4*>(&vs[key * VP + c]) = vr[i];
+    }
+  };
+
+  float m[QT], l[QT];
+  f32x4 acc[QT][DV / 16];
+#pragma unroll
+  for (int t = 0; t < QT; ++t) {
+    m[t] = MASKED;
+    l[t] = 0.f;
+#pragma unroll
+    for (int d = 0; d < DV / 16; ++d) acc[t][d] = {0.f, 0.f, 0.f, 0.f};
+  }
+  const float sl2 = p.scale * LOG2E;
+  const int kt1 = last / KT;
+  fetch(first / KT);
+  for (int kt = first / KT; kt <= kt1; ++kt) {
+    __syncthreads();                          // the tile before is read
+    land();
+    __syncthreads();
+    if (kt < kt1) fetch(kt + 1);
+    const int k0 = kt * KT;
+    if (k0 > whi || k0 + KT <= wlo) continue;  // barriers stay uniform
+
+    f32x4 s[QT][4];
+#pragma unroll
+    for (int t = 0; t < QT; ++t)
+#pragma unroll
+      for (int c = 0; c < 4; ++c) s[t][c] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int c = 0; c < 4; ++c)
+#pragma unroll
+      for (int st = 0; st < DK / 32; ++st) {
+        const mf_bf8 kf = frag8(&ks[(c * 16 + gl) * KP + st * 32 + gs * 8]);
+#pragma unroll
+        for (int t = 0; t < QT; ++t)
+          s[t][c] = mfma_bf16_k32(kf, qf[t][st], s[t][c]);
+      }
+    mf_bf8 ph[QT][2], pl[QT][2];
+#pragma unroll
+    for (int t = 0; t < QT; ++t) {
+      const int hi = qpos[t], lo = p.window > 0 ? hi - p.window + 1 : 0;
+      float mx = MASKED;
+#pragma unroll
+      for (int c = 0; c < 4; ++c)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int j = k0 + c * 16 + gs * 4 + r;
+          const float x = j <= hi && j >= lo ? s[t][c][r] * sl2 : MASKED;
+          s[t][c][r] = x;
+          mx = fmaxf(mx, x);
+        }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      const float mn = fmaxf(m[t], mx);
+      const float corr = exp2_fast(m[t] - mn);
+      m[t] = mn;
+      float sum = 0.f;
+#pragma unroll
+      for (int c = 0; c < 4; ++c)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float x = s[t][c][r];
+          const float e = x > MASKED ? exp2_fast(x - mn) : 0.f;
+          sum += e;
+          __bf16 h, lw;
+          split_bf16(e, h, lw);
+          ph[t][c >> 1][(c & 1) * 4 + r] = h;
+          pl[t][c >> 1][(c & 1) * 4 + r] = lw;
+        }
+      l[t] = l[t] * corr + sum;               // per lane; summed at the end
+#pragma unroll
+      for (int d = 0; d < DV / 16; ++d) acc[t][d] *= corr;
+    }
+#pragma unroll
+    for (int st = 0; st < 2; ++st)
+#pragma unroll
+      for (int d = 0; d < DV / 16; ++d) {
+        const __hip_bfloat16* b =
+            &vs[(st * 32 + gs * 4 + (gl >> 2)) * VP + d * 16 + (gl & 3) * 4];
+        const mf_bf4 v0 = tr_read4(b), v1 = tr_read4(b + 16 * VP);
+        const mf_bf8 vf = {v0[0], v0[1], v0[2], v0[3],
+                           v1[0], v1[1], v1[2], v1[3]};
+#pragma unroll
+        for (int t = 0; t < QT; ++t) {
+          acc[t][d] = mfma_bf16_k32(vf, ph[t][st], acc[t][d]);
+          acc[t][d] = mfma_bf16_k32(vf, pl[t][st], acc[t][d]);
+        }
+      }
+  }
+
+#pragma unroll
+  for (int t = 0; t < QT; ++t) {
+    float sum = l[t];
+    sum += __shfl_xor(sum, 16, 64);
+    sum += __shfl_xor(sum, 32, 64);
+    const int r = t0 + (wave * QT + t) * 16 + gl;
+    if (r >= qlen) continue;
+    const float inv = 1.f / sum;
+    const size_t row = qrow0 + r;
+    __hip_bfloat16* o = (__hip_bfloat16*)p.out + row * p.o_row +
+                        (size_t)head * p.dv;
+    const __hip_bfloat16* g =
+        p.gate ? (const __hip_bfloat16*)p.gate + row * p.g_row +
+                     (size_t)head * p.dv
+               : nullptr;
+#pragma unroll
+    for (int d = 0; d < DV / 16; ++d) {
+      const int c = d * 16 + gs * 4;
+      if (c >= p.dv) continue;
+      union { uint2 u; __hip_bfloat16 e[4]; } ov, gv;
+      if (g) gv.u = *reinterpret_cast<const uint2*>(g + c);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        float x = acc[t][d][e] * inv;
+        if (g) x *= sigmoid_f(bf2f(gv.e[e]));
+        ov.e[e] = f2bf(x);
+      }
+      *reinterpret_cast<uint2*>(o + c) = ov.u;
+    }
+  }
+}
+
+template <int DK>
+void go_dv(const WindowAttnArgs& p, hipStream_t s) {
+  const int grid = 8 * ((p.n_blocks * p.heads + 7) / 8);
+#define WA_GO(DV, NW, QT)                                                     \
+  window_attn_kernel<DK, DV, NW, QT><<<grid, NW * 64, 0, s>>>(p)
+  if (p.dv <= 64) {
+    WA_GO(64, 4, 2);
+  } else if (p.dv <= 128) {
+    WA_GO(128, 4, 2);
+  } else {
+    WA_GO(256, 8, 1);
+  }
+#undef WA_GO
+}
+
+}  // namespace
+
+extern "C" {
+
+int window_attn_rows() { return 128; }        // query rows per block
+
+void launch_window_attn(const WindowAttnArgs* p, hipStream_t s) {
+  if (p->d <= 64) go_dv<64>(*p, s);
+  else if (p->d <= 128) go_dv<128>(*p, s);
+  else go_dv<256>(*p, s);
+}
+
+}  // extern "C"

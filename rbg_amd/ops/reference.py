@@ -201,11 +201,6 @@ def gelu_mul(x, out):
     out.copy_((act * up).to(x.dtype))
 
 
-def head_gate(o, g, out):
-    rows = o.transpose(0, 1).reshape(g.shape).float()
-    out.copy_((rows * torch.sigmoid(g.float())).to(out.dtype))
-
-
 def delta_rule(proj, z, w2, w0, a_bias, norm_w, state, slots, cu_seqlens,
                starts, out, offs, decay_scale, unit_eps, norm_eps):
     H, D = state.shape[1:3]
@@ -257,7 +252,7 @@ def window_attention(q, k, v, gate, out, row_info, scale, window):
 
 
 def latent_decode(q, cache, block_tables, context_lens, scale, window):
-    H, S, R = q.shape
+    S, H, R = q.shape
     out = torch.empty_like(q)
     ps = cache.shape[1]
     flat = cache.view(-1, R)
@@ -266,6 +261,14 @@ def latent_decode(q, cache, block_tables, context_lens, scale, window):
         lo = max(0, ctx - window) if window > 0 else 0
         j = torch.arange(lo, ctx)
         c = flat[block_tables[s].long()[j // ps] * ps + j % ps].float()
-        p = torch.softmax(q[:, s].float() @ c.T * scale, dim=-1)
-        out[:, s] = (p @ c).to(q.dtype)
+        p = torch.softmax(q[s].float() @ c.T * scale, dim=-1)
+        out[s] = (p @ c).to(q.dtype)
     return out
+
+
+def head_linear(x, w, gate, out):
+    y = torch.einsum("shk,hjk->shj", x.float(), w.float())
+    y = y.reshape(out.shape)
+    if gate is not None:
+        y = y * torch.sigmoid(gate.float())
+    out.copy_(y.to(out.dtype))

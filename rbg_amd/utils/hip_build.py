@@ -1,6 +1,6 @@
 """In-tree build of the HIP extensions (gfx950) and their freshness stamps.
 
-Each extension carries a stamp: a hash over its sources and the shared headers
+Each extension carries a stamp: a hash over its sources and headers
 at build time.  A process on a GPU box refuses an extension whose sources have
 changed since (ops/__init__.py), and ``ensure`` builds a missing or stale one,
 so that a fresh checkout compiles only what its model runs on.
@@ -43,10 +43,20 @@ HIP_SOURCES = {
         "stream_norm.hip",
         "gated_act.hip",
         "delta_rule.hip",
+        "delta_chunk.hip",
         "latent_attn.hip",
+        "latent_decode.hip",
+        "window_attn.hip",
+        "head_linear.hip",
         "skinny_gemm.hip",
         "mix_bindings.cpp",
     ],
+}
+
+HIP_HEADERS = {
+    "_hip_ops": ["common.h", "gemm_bindings.h"],
+    "_hip_mix": ["common.h", "gemm_bindings.h", "mfma_util.h", "mix_args.h",
+                 "vec_io.h"],
 }
 
 # model architecture -> the extension with its kernels (default: _hip_ops)
@@ -54,9 +64,8 @@ EXTENSION_OF = {"Bitatar": "_hip_mix"}
 
 
 def source_hash(name: str) -> str:
-    headers = [f for f in os.listdir(HIP_DIR) if f.endswith(".h")]
     h = hashlib.sha256()
-    for f in sorted(HIP_SOURCES[name] + headers):
+    for f in sorted(HIP_SOURCES[name] + HIP_HEADERS[name]):
         with open(os.path.join(HIP_DIR, f), "rb") as fh:
             h.update(f.encode() + b"\0" + fh.read() + b"\0")
     return h.hexdigest()
