@@ -56,6 +56,9 @@ def parse_args():
                         "per workload (--sizes, --batches, --seq-len)")
     p.add_argument("--sizes", default="2k,4k", help="with --compare")
     p.add_argument("--batches", default="1,32", help="with --compare")
+    p.add_argument("--kernels", action="store_true",
+                   help="with --compare: each kernel's time beside its "
+                        "roofline instead")
     return p.parse_args()
 
 
@@ -103,7 +106,12 @@ def main() -> int:
         torch.cuda.set_device(local_rank)
 
     if args.compare:
-        from rbg_amd.engine.model_bench import run_compare
+        from rbg_amd.engine.model_bench import run_compare, run_kernels
+        if args.kernels:
+            for size in args.sizes.split(","):
+                for row in run_kernels(size):
+                    print(json.dumps(dict(row, size=size)), flush=True)
+            return 0
         for row in run_compare(device, args.steps, args.warmup,
                                sizes=args.sizes.split(","),
                                batches=[int(b) for b in

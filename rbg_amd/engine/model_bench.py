@@ -88,3 +88,180 @@ def run_compare(device: str, steps: int, warmup: int,
     return [run_one(model, device, b, prompt, steps, warmup, eager)
             for size in (sizes or SIZES) for b in batches
             for model in pair(size)]
+
+
+# -- kernels against their rooflines -------------------------------------------
+
+HBM_TB_S, BF16_TF, F32_TF = 8.0, 2500.0, 157.0
+
+
+def _time(fn, n: int = 12) -> float:
+    """Median-free mean over calls fn(i), microseconds on the GPU."""
+    for i in range(3):
+        fn(i)
+    torch.cuda.synchronize()
+    a, b = (torch.cuda.Event(enable_timing=True) for _ in range(2))
+    # a captured graph keeps launch gaps out of short kernels' times
+    g = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(g):
+        for i in range(n):
+            fn(i)
+    g.replay()
+    torch.cuda.synchronize()
+    a.record()
+    g.replay()
+    b.record()
+    torch.cuda.synchronize()
+    return a.elapsed_time(b) * 1e3 / n
+
+
+def _row(name: str, us: float, nbytes: float = 0.0, bf16: float = 0.0,
+         f32: float = 0.0) -> Dict[str, Any]:
+    bound = max(nbytes / HBM_TB_S / 1e6, bf16 / BF16_TF / 1e6,
+                f32 / F32_TF / 1e6)
+    return {"kernel": name, "us": round(us, 1),
+            "roofline_us": round(bound, 1),
+            "times_roofline": round(us / bound, 2)}
+
+
+def run_kernels(size: str, batches=(1, 8, 32, 128), ctx: int = 2048,
+                prompts: int = 4) -> List[Dict[str, Any]]:
+    """The mixers' kernels and the like kernels of Llama, one layer's shapes
+    of ``size``; decode inputs rotate through buffers larger than the caches.
+    Rooflines: bytes that must move, or the operations the algorithm has to
+    do (causal halves counted once, the 32-bit recurrence at the f32 rate)."""
+    import math
+
+    from .. import ops
+    from .batch import VarlenLayout
+    w, ff, heads, kvh, _, rank, window, dh, dd = SIZES[size]
+    dev, bf = torch.device("cuda"), torch.bfloat16
+    out: List[Dict[str, Any]] = []
+
+    def rnd(*shape, dtype=bf):
+        return torch.randn(*shape, device=dev, dtype=torch.float32).to(dtype)
+
+    def copies(nbytes: int) -> int:
+        return max(1, min(12, int(600e6 // max(nbytes, 1)) + 1))
+
+    def i32(x):
+        return torch.tensor(x, dtype=torch.int32, device=dev)
+    ps = 16
+    ones, conv_w = torch.ones(w, device=dev), torch.randn(4, w, device=dev)
+    hd = dh * dd
+    offs = [hd * i for i in range(6)]
+    dargs = (rnd(hd, 64), torch.randn(hd, device=dev),
+             torch.randn(hd, device=dev), torch.ones(hd, device=dev))
+    for b in batches:
+        tag = f"B={b}"
+        pages = b * ctx // ps + 1
+        bt = (torch.arange(b * (ctx // ps), device=dev, dtype=torch.int32)
+              .view(b, -1) + 1)
+        cl = i32([ctx] * b)
+        keys = min(window, ctx)
+        n = copies(pages * ps * rank * 2)
+        lat = [rnd(pages, ps, rank) for _ in range(n)]
+        q = rnd(b, heads, rank)
+        us = _time(lambda i: ops.latent_decode(q, lat[i % n], bt, cl, 0.05,
+                                               window))
+        out.append(_row(f"latent_decode {tag}", us,
+                        b * keys * rank * 2 + 2 * b * heads * rank * 2,
+                        bf16=b * heads * keys * rank * 4))
+        del lat
+        n = copies(pages * ps * kvh * 128 * 4)
+        kv = [(rnd(pages, kvh, ps, 128), rnd(pages, kvh, ps, 128))
+              for _ in range(n)]
+        q = rnd(b, heads, 128)
+        sp = ops.pick_decode_splits(b, kvh, ctx + 128)
+        us = _time(lambda i: ops.decode_attention(q, *kv[i % n], bt, cl, 0.05,
+                                                  num_splits=sp))
+        out.append(_row(f"llama decode_attention {tag}", us,
+                        b * ctx * kvh * 128 * 4 + 2 * b * heads * 128 * 2))
+        del kv
+        q, uk = rnd(b, heads, 128), rnd(heads, rank, 128)
+        us = _time(lambda i: ops.head_linear(q, uk))
+        out.append(_row(f"head_linear {tag}", us, uk.numel() * 2 +
+                        b * heads * (128 + rank) * 2))
+        slots = i32(range(1, b + 1))
+        sbytes = b * dh * dd * dd * 8
+        n = copies(sbytes)
+        st = [torch.randn(b + 1, dh, dd, dd, device=dev) for _ in range(n)]
+        proj = rnd(b, hd * 5 + 64)
+        o = rnd(b, hd)
+        us = _time(lambda i: ops.delta_rule(
+            proj, None, *dargs, st[i % n], slots, None, cl, o, offs,
+            math.exp(-0.5), 1e-6, 1e-5))
+        out.append(_row(f"delta_step {tag}", us, sbytes + dargs[0].numel() * 2
+                        + b * hd * 12))
+        del st
+        x, d = rnd(b, w, dtype=torch.float32), rnd(b, w)
+        hist = rnd(b + 1, 3, w)
+        us = _time(lambda i: ops.stream_norm_conv(
+            x, d, ones, ones, 8, 1e-5, bf, conv_w, hist, slots, cl))
+        out.append(_row(f"stream_norm_conv {tag}", us,
+                        b * w * (8 + 2 + 4 + 12) + w * 4 * 6))
+        r, wn = rnd(b, w), rnd(w)
+        us = _time(lambda i: ops.fused_add_rmsnorm(d, r, wn, 1e-5))
+        out.append(_row(f"llama fused_add_rmsnorm {tag}", us, b * w * 8))
+        gu, act = rnd(b, 2 * ff), rnd(b, ff)
+        us = _time(lambda i: ops.gelu_mul(gu, act))
+        out.append(_row(f"gelu_mul {tag}", us, b * ff * 6))
+        us = _time(lambda i: ops.silu_mul(gu))
+        out.append(_row(f"llama silu_mul {tag}", us, b * ff * 6))
+    # prefill: `prompts` prompts of ctx tokens
+    T = prompts * ctx
+
+    class Table:
+        pages = list(range(1, ctx // ps + 1))
+    lay = VarlenLayout([0] * prompts, [ctx] * prompts, [Table()] * prompts, 0,
+                       ps, dev)
+    cu = i32([i * ctx for i in range(prompts + 1)])
+    q, k, v, g = (rnd(T, heads, 128) for _ in range(4))
+    act = rnd(T, heads * 128)
+    view = lay.window_view(window)
+    pairs = prompts * sum(min(i + 1, window) for i in range(ctx))
+    tag = f"{prompts}x{ctx}"
+    us = _time(lambda i: ops.window_attention(
+        q, k, v, g.flatten(1), act, view, 0.05, window))
+    out.append(_row(f"window_attention {tag}", us, T * heads * 128 * 10,
+                    bf16=pairs * heads * 4 * 128))
+    bi, sl = ops.reference.prefill_block_info(cu.cpu(), qtile=128)
+    bi, sl = bi.to(dev), sl.to(dev)
+    kk, vv = k[:, :kvh].contiguous(), v[:, :kvh].contiguous()
+    us = _time(lambda i: ops._require_hip().prefill_attention(
+        q, kk, vv, bi, sl, 0.05, ops.PREFILL_SWZ))
+    out.append(_row(f"llama prefill_attention {tag}", us, T * heads * 128 * 6,
+                    bf16=prompts * ctx * (ctx + 1) // 2 * heads * 4 * 128))
+    proj, z, o = rnd(T, hd * 5 + 64), rnd(T, hd), rnd(T, hd)
+    st = torch.zeros(prompts + 1, dh, dd, dd, device=dev)
+    slots, starts = i32(range(1, prompts + 1)), i32([0] * prompts)
+    chunks = (lay.prefill_tiles(ops.DELTA_CHUNK),
+              lay.prefill_tile_cu(ops.DELTA_CHUNK))
+    us = _time(lambda i: ops.delta_rule(
+        proj, z, *dargs, st, slots, cu, starts, o, offs, math.exp(-0.5), 1e-6,
+        1e-5, chunks), 4)
+    out.append(_row(f"delta_chunk (3 kernels) {tag}", us, T * hd * 14,
+                    f32=T * dh * 8 * dd * dd))
+    x, d = rnd(T, w, dtype=torch.float32), rnd(T, w)
+    us = _time(lambda i: ops.stream_norm(x, d, ones, ones, 8, 1e-5, bf))
+    out.append(_row(f"stream_norm {tag}", us, T * w * 14))
+    hist = rnd(prompts + 1, 3, w)
+    tiles = lay.tiles(ops.CONV_TILE)
+    us = _time(lambda i: ops.causal_conv(d, conv_w, hist, tiles, cu, starts,
+                                         slots))
+    out.append(_row(f"causal_conv {tag}", us, T * w * 4))
+    r, wn = rnd(T, w), rnd(w)
+    us = _time(lambda i: ops.fused_add_rmsnorm(d, r, wn, 1e-5))
+    out.append(_row(f"llama fused_add_rmsnorm {tag}", us, T * w * 8))
+    gu, act = rnd(T, 2 * ff), rnd(T, ff)
+    us = _time(lambda i: ops.gelu_mul(gu, act))
+    out.append(_row(f"gelu_mul {tag}", us, T * ff * 6))
+    us = _time(lambda i: ops.silu_mul(gu))
+    out.append(_row(f"llama silu_mul {tag}", us, T * ff * 6))
+    x = rnd(T, rank + 8)
+    cache = rnd(T // ps + 1, ps, rank)
+    sl = torch.arange(ps, T + ps, device=dev, dtype=torch.int32)
+    us = _time(lambda i: ops.latent_store(
+        x[:, :rank], torch.ones(rank, device=dev), cache, sl, 1e-5))
+    out.append(_row(f"latent_store {tag}", us, T * rank * 6))
+    return out

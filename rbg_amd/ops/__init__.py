@@ -308,12 +308,14 @@ def window_attention(q, k, v, gate, out, view, scale: float,
 
 
 def pick_latent_splits(num_seqs: int, num_heads: int, max_keys: int) -> int:
-    """Key splits of latent_decode: about two workgroups per CU, at least one
-    16-key chunk for each of a workgroup's four waves.  Depends on sizes only,
-    so a captured decode step keeps its value."""
+    """Key splits of latent_decode: two workgroups per CU, one for small
+    batches (the splits' sums cost more than they hide there), at least one
+    64-key step each.  Depends on sizes only, so a captured decode step keeps
+    its value."""
     base = num_seqs * ((num_heads + 15) // 16)
-    by_keys = max(1, (max_keys + 15) // 64)
-    return int(max(1, min((512 + base - 1) // base, by_keys, 64)))
+    want = 512 if base >= 64 else 256
+    steps = (max_keys + 63) // 64
+    return int(max(1, min((want + base - 1) // base, steps, 64)))
 
 
 def latent_decode(q, cache, block_tables, context_lens, scale: float,

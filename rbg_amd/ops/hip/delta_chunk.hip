@@ -24,16 +24,18 @@ namespace {
 constexpr int C = 16;                   // tokens per chunk
 constexpr int SP = C + 4;               // row pitch of [.][16] arrays
 
-// one chunk-head's record in the workspace, in floats
+// one chunk-head's record in the workspace, in floats: the image that the scan
+// keeps in LDS, row pitches included
 template <int DP> struct Rec {
+  static constexpr int PP = DP + 4;               // pitch of [16][DP] arrays
   static constexpr int TU = 0;                    // [16][DP]
-  static constexpr int R = TU + C * DP;           // [16][DP]
-  static constexpr int KT = R + C * DP;           // [DP][16]
-  static constexpr int BT = KT + C * DP;          // [DP][16], negated
-  static constexpr int TM = BT + C * DP;          // [16][16]
-  static constexpr int QK = TM + C * C;           // [16][16]
-  static constexpr int QB = QK + C * C;           // [16][16], negated
-  static constexpr int DC = QB + C * C;           // [DP]
+  static constexpr int R = TU + C * PP;           // [16][DP]
+  static constexpr int KT = R + C * PP;           // [DP][16]
+  static constexpr int BT = KT + DP * SP;         // [DP][16], negated
+  static constexpr int TM = BT + DP * SP;         // [16][16]
+  static constexpr int QK = TM + C * SP;          // [16][16]
+  static constexpr int QB = QK + C * SP;          // [16][16], negated
+  static constexpr int DC = QB + C * SP;          // [DP]
   static constexpr int SIZE = DC + DP;
 };
 
@@ -41,12 +43,14 @@ template <typename T, int DP>
 __global__ __launch_bounds__(256) void delta_prep_kernel(
     const DeltaArgs p, const int* __restrict__ tiles, float* __restrict__ ws) {
   typedef Rec<DP> W;
-  constexpr int PP = DP + 4;            // pitch of [16][DP] arrays
+  constexpr int PP = W::PP;
   constexpr int GR = 256 / DP;          // token groups in the staging step
   constexpr int TPG = C / GR;           // tokens per group
   constexpr int NWV = (DP + 63) / 64;   // waves that share a token's channels
-  __shared__ float us[C * PP], rs[C * PP], ksh[C * PP], bs[C * PP];
-  __shared__ float ls[C * SP], ms[C * SP], qk[C * SP], qb[C * SP], ts[C * SP];
+  __shared__ __attribute__((aligned(16))) float us[C * PP], rs[C * PP],
+      ksh[C * PP], bs[C * PP];
+  __shared__ __attribute__((aligned(16))) float ls[C * SP], ms[C * SP],
+      ts[C * SP];
   __shared__ float csum[GR][DP], nrm[C][NWV == 1 ? 1 : NWV];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int gl = lane & 15, gs = lane >> 4;
@@ -99,15 +103,15 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(
     float ss = 0.f;
 #pragma unroll
     for (int w = 0; w < NWV; ++w) ss += nrm[t][w];
-    const float u = kv[i] / sqrtf(ss + p.unit_eps);
+    const float u = kv[i] * rcp_f(sqrtf(ss + p.unit_eps));
     const float c1 = base + lw[i], c0 = i ? base + lw[i - 1] : base;
-    const float e1 = expf(-c1);
-    us[t * PP + ch] = u * expf(c0);
-    rs[t * PP + ch] = rv[i] * expf(c1);
+    const float e1 = __expf(-c1);
+    us[t * PP + ch] = u * __expf(c0);
+    rs[t * PP + ch] = rv[i] * __expf(c1);
     ksh[t * PP + ch] = kv[i] * e1;
     bs[t * PP + ch] = av[i] * u * e1;
   }
-  if (grp == 0) rec[W::DC + ch] = expf(tot);
+  if (grp == 0) rec[W::DC + ch] = __expf(tot);
   __syncthreads();
 
   // ---- the four token x token products, one per wave --------------------
@@ -129,7 +133,8 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(
       }
     }
     acc += acc2;
-    float* o = wave == 0 ? ls : wave == 1 ? ms : wave == 2 ? qb : qk;
+    float* o = wave == 0 ? ls : wave == 1 ? ms
+               : rec + (wave == 2 ? W::QB : W::QK);
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int t = gs * 4 + r;                     // row; column gl
@@ -154,20 +159,25 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(
       }
     }
   } else {
-    for (int i = tid - 64; i < C * DP; i += 192)
-      rec[W::R + i] = rs[(i / DP) * PP + i % DP];
-    for (int i = tid - 64; i < C * DP; i += 192) {
-      const int d = i >> 4, t = i & 15;
+    for (int i = (tid - 64) * 4; i < C * DP; i += 192 * 4) {
+      const int at = (i / DP) * PP + i % DP;
+      *reinterpret_cast<f32x4*>(rec + W::R + at) =
+          *reinterpret_cast<const f32x4*>(rs + at);
+    }
+    for (int i = tid - 64; i < DP * 4; i += 192) {
+      const int d = i >> 2, t = (i & 3) * 4;        // 4 tokens of a channel
       float dc = 0.f;
 #pragma unroll
       for (int g = 0; g < GR; ++g) dc += csum[g][d];
-      dc = expf(dc);
-      rec[W::KT + i] = ksh[t * PP + d] * dc;
-      rec[W::BT + i] = -bs[t * PP + d] * dc;
-    }
-    for (int i = tid - 64; i < C * C; i += 192) {
-      rec[W::QK + i] = qk[(i >> 4) * SP + (i & 15)];
-      rec[W::QB + i] = qb[(i >> 4) * SP + (i & 15)];
+      dc = __expf(dc);
+      f32x4 kx, bx;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        kx[r] = ksh[(t + r) * PP + d] * dc;
+        bx[r] = -bs[(t + r) * PP + d] * dc;
+      }
+      *reinterpret_cast<f32x4*>(rec + W::KT + d * SP + t) = kx;
+      *reinterpret_cast<f32x4*>(rec + W::BT + d * SP + t) = bx;
     }
   }
   __syncthreads();
@@ -182,7 +192,7 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(
       acc = mfma_f32_k4(tf[r], us[(gs * 4 + r) * PP + d + gl], acc);
 #pragma unroll
     for (int r = 0; r < 4; ++r)
-      rec[W::TU + (gs * 4 + r) * DP + d + gl] = acc[r];
+      rec[W::TU + (gs * 4 + r) * PP + d + gl] = acc[r];
   }
   if (wave == 3) {
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
@@ -191,90 +201,89 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(
       acc = mfma_f32_k4(tf[r], ms[(gs * 4 + r) * SP + gl], acc);
 #pragma unroll
     for (int r = 0; r < 4; ++r)
-      rec[W::TM + (gs * 4 + r) * C + gl] = acc[r];
+      rec[W::TM + (gs * 4 + r) * SP + gl] = acc[r];
   }
 }
 
-// grid (heads, seqs, column groups); NW waves of 16 value columns
-template <typename T, int DP, int NW>
-__global__ __launch_bounds__(NW * 64) void delta_scan_kernel(
+// grid (heads, seqs, column groups).  A workgroup is NC column groups of 16
+// value columns by KS parts of the key rows: wave (kp, cg) keeps its rows of
+// its columns of S.  With KS = 2 the parts' shares of P and O meet in LDS.
+// A record's loads fly under two chunks' MFMAs and land in the other half of
+// LDS.
+template <typename T, int DP, int KS, int NC>
+__global__ __launch_bounds__(KS * NC * 64) void delta_scan_kernel(
     const DeltaArgs p, const int* __restrict__ chunk_cu,
     const float* __restrict__ ws, float* __restrict__ o) {
   typedef Rec<DP> W;
-  constexpr int PP = DP + 4, NT = NW * 64, TT = DP / 16;
-  // the record's arrays, repitched; staged through registers
+  constexpr int PP = W::PP, NT = KS * NC * 64, TT = DP / 16 / KS;
   constexpr int V4 = W::SIZE / 4, PER = (V4 + NT - 1) / NT;
-  __shared__ __attribute__((aligned(16))) float tu[C * PP], rsm[C * PP];
-  __shared__ __attribute__((aligned(16))) float kt[DP * SP], bt[DP * SP];
-  __shared__ __attribute__((aligned(16))) float tm[C * SP], qk[C * SP],
-      qb[C * SP], dc[DP];
+  extern __shared__ __attribute__((aligned(16))) float smem[];
+  f32x4* xch = reinterpret_cast<f32x4*>(smem + 2 * W::SIZE);  // [2][KS*NC*64]
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int gl = lane & 15, gs = lane >> 4;
+  const int cg = wave % NC, kp = wave / NC;
   const int head = blockIdx.x, seq = blockIdx.y;
   const int D = p.dim, HD = p.heads * D;
-  const int vcol = (blockIdx.z * NW + wave) * 16 + gl;
+  const int vcol = (blockIdx.z * NC + cg) * 16 + gl;
   const bool vlive = vcol < D;
   const int vc = min(vcol, D - 1);
   const int row0 = p.cu[seq], len = p.cu[seq + 1] - row0;
   const int ch0 = chunk_cu[seq], nch = chunk_cu[seq + 1] - ch0;
   const bool fresh = p.starts[seq] == 0;
   float* S = p.state + ((size_t)p.slots[seq] * p.heads + head) * D * D;
+  const int k0 = kp * TT * 16;                  // this wave's key rows
 
   f32x4 s[TT];
 #pragma unroll
   for (int t = 0; t < TT; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int kr = t * 16 + gs * 4 + r;
+      const int kr = k0 + t * 16 + gs * 4 + r;
       s[t][r] = !fresh && vlive && kr < D ? S[(size_t)kr * D + vcol] : 0.f;
     }
 
-  f32x4 stage[PER];
-  float v[4], vn[4];
-  auto fetch = [&](int c) {
-    const f32x4* src = reinterpret_cast<const f32x4*>(
-        ws + ((size_t)(ch0 + c) * p.heads + head) * W::SIZE);
+  f32x4 stage[2][PER];
+  float v[4], vn[2][4];
+#define DC_FETCH(c, h)                                                        \
+  do {                                                                        \
+    const f32x4* src = reinterpret_cast<const f32x4*>(                        \
+        ws + ((size_t)(ch0 + (c)) * p.heads + head) * W::SIZE);               \
+    _Pragma("unroll") for (int i = 0; i < PER; ++i)                           \
+      stage[h][i] = src[min(tid + i * NT, V4 - 1)];                           \
+    _Pragma("unroll") for (int r = 0; r < 4; ++r) {                           \
+      const int t = (c) * C + gs * 4 + r;                                     \
+      vn[h][r] = to_f(((const T*)p.proj)[                                     \
+          (size_t)(row0 + min(t, len - 1)) * p.proj_stride + p.off_v +        \
+          head * D + vc]);                                                    \
+      if (t >= len || !vlive) vn[h][r] = 0.f;                                 \
+    }                                                                         \
+  } while (0)
+#define DC_LAND(half)                                                         \
+  do {                                                                        \
+    f32x4* dst = reinterpret_cast<f32x4*>(smem + (half) * W::SIZE);           \
+    _Pragma("unroll") for (int i = 0; i < PER; ++i)                           \
+      if (tid + i * NT < V4) dst[tid + i * NT] = stage[half][i];              \
+    _Pragma("unroll") for (int r = 0; r < 4; ++r) v[r] = vn[half][r];         \
+  } while (0)
+  DC_FETCH(0, 0);
+  DC_LAND(0);
+  DC_FETCH(min(1, nch - 1), 1);
+  __syncthreads();
+  for (int cc = 0; cc < nch; cc += 2)
 #pragma unroll
-    for (int i = 0; i < PER; ++i) stage[i] = src[min(tid + i * NT, V4 - 1)];
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = c * C + gs * 4 + r;
-      vn[r] = to_f(((const T*)p.proj)[
-          (size_t)(row0 + min(t, len - 1)) * p.proj_stride + p.off_v +
-          head * D + vc]);
-      if (t >= len || !vlive) vn[r] = 0.f;
-    }
-  };
-  fetch(0);
-  for (int c = 0; c < nch; ++c) {
-    __syncthreads();
-#pragma unroll
-    for (int i = 0; i < PER; ++i) {
-      const int e = (tid + i * NT) * 4;
-      if (e < W::SIZE) {
-        float* dst;
-        if (e < W::R) dst = tu + (e / DP) * PP + e % DP;
-        else if (e < W::KT) dst = rsm + ((e - W::R) / DP) * PP + e % DP;
-        else if (e < W::BT) dst = kt + ((e - W::KT) >> 4) * SP + (e & 15);
-        else if (e < W::TM) dst = bt + ((e - W::BT) >> 4) * SP + (e & 15);
-        else if (e < W::QK) dst = tm + ((e - W::TM) >> 4) * SP + (e & 15);
-        else if (e < W::QB) dst = qk + ((e - W::QK) >> 4) * SP + (e & 15);
-        else if (e < W::DC) dst = qb + ((e - W::QB) >> 4) * SP + (e & 15);
-        else dst = dc + (e - W::DC);
-        *reinterpret_cast<f32x4*>(dst) = stage[i];
-      }
-    }
-#pragma unroll
-    for (int r = 0; r < 4; ++r) v[r] = vn[r];
-    __syncthreads();
-    if (c + 1 < nch) fetch(c + 1);
+  for (int h = 0; h < 2; ++h) {
+    const int c = cc + h;
+    if (c >= nch) break;
+    const float* rec = smem + h * W::SIZE;
+    // always: a skipped load would make the waits below drain every load
+    DC_FETCH(min(c + 2, nch - 1), h);
 
     // P and O over the old state, two products side by side
     f32x4 pa = {0.f, 0.f, 0.f, 0.f}, oa = pa;
-    {
+    if (kp == 0) {
       float x[4], y[4];
-      load_vec<4>(tm + gl * SP + gs * 4, x);
-      load_vec<4>(qk + gl * SP + gs * 4, y);
+      load_vec<4>(rec + W::TM + gl * SP + gs * 4, x);
+      load_vec<4>(rec + W::QK + gl * SP + gs * 4, y);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         pa = mfma_f32_k4(x[r], v[r], pa);
@@ -284,51 +293,109 @@ __global__ __launch_bounds__(NW * 64) void delta_scan_kernel(
 #pragma unroll
     for (int t = 0; t < TT; ++t) {
       float x[4], y[4];
-      load_vec<4>(tu + gl * PP + t * 16 + gs * 4, x);
-      load_vec<4>(rsm + gl * PP + t * 16 + gs * 4, y);
+      load_vec<4>(rec + W::TU + gl * PP + k0 + t * 16 + gs * 4, x);
+      load_vec<4>(rec + W::R + gl * PP + k0 + t * 16 + gs * 4, y);
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         pa = mfma_f32_k4(x[r], s[t][r], pa);
         oa = mfma_f32_k4(y[r], s[t][r], oa);
       }
     }
-    {
-      float y[4];
-      load_vec<4>(qb + gl * SP + gs * 4, y);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) oa = mfma_f32_k4(y[r], pa[r], oa);
+    if constexpr (KS == 2) {
+      xch[wave * 64 + lane] = pa;
+      if (kp == 1) xch[(KS * NC + cg) * 64 + lane] = oa;
     }
-    // the state moves on
+    // the decay and k v^T parts do not wait for P
 #pragma unroll
     for (int t = 0; t < TT; ++t) {
-      float x[4], y[4], d[4];
-      load_vec<4>(dc + t * 16 + gs * 4, d);
-      load_vec<4>(kt + (t * 16 + gl) * SP + gs * 4, x);
-      load_vec<4>(bt + (t * 16 + gl) * SP + gs * 4, y);
+      float x[4], d[4];
+      load_vec<4>(rec + W::DC + k0 + t * 16 + gs * 4, d);
+      load_vec<4>(rec + W::KT + (k0 + t * 16 + gl) * SP + gs * 4, x);
 #pragma unroll
       for (int r = 0; r < 4; ++r) s[t][r] *= d[r];
 #pragma unroll
       for (int r = 0; r < 4; ++r) s[t] = mfma_f32_k4(x[r], v[r], s[t]);
+    }
+    if constexpr (KS == 2) {
+      __syncthreads();
+      const f32x4 p0 = xch[cg * 64 + lane], p1 = xch[(NC + cg) * 64 + lane];
+      pa = p0 + p1;
+      if (kp == 0) oa += xch[(KS * NC + cg) * 64 + lane];
+    }
+#pragma unroll
+    for (int t = 0; t < TT; ++t) {
+      float y[4];
+      load_vec<4>(rec + W::BT + (k0 + t * 16 + gl) * SP + gs * 4, y);
 #pragma unroll
       for (int r = 0; r < 4; ++r) s[t] = mfma_f32_k4(y[r], pa[r], s[t]);
     }
+    if (kp == 0) {
+      float y[4];
+      load_vec<4>(rec + W::QB + gl * SP + gs * 4, y);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = c * C + gs * 4 + r;
-      if (t < len && vlive)
-        o[(size_t)(row0 + t) * HD + head * D + vcol] = oa[r];
+      for (int r = 0; r < 4; ++r) oa = mfma_f32_k4(y[r], pa[r], oa);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int t = c * C + gs * 4 + r;
+        if (t < len && vlive)
+          o[(size_t)(row0 + t) * HD + head * D + vcol] = oa[r];
+      }
     }
+    DC_LAND(1 - h);
+    __syncthreads();
   }
+#undef DC_FETCH
+#undef DC_LAND
 #pragma unroll
   for (int t = 0; t < TT; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int kr = t * 16 + gs * 4 + r;
+      const int kr = k0 + t * 16 + gs * 4 + r;
       if (vlive && kr < D) S[(size_t)kr * D + vcol] = s[t][r];
     }
 }
 
-// out = o / rms(o) * norm_w * sigmoid(g), one wave per row and head
+// out = o / rms(o) * norm_w * sigmoid(g).  VEC: dim is 4 * LPI for a power of
+// two LPI, and LPI lanes take a row of a head; else one wave does.
+template <typename T, int LPI>
+__global__ __launch_bounds__(256) void delta_out_vec_kernel(
+    const DeltaArgs p, const float* __restrict__ o, const long items) {
+  const int lane = threadIdx.x & 63;
+  const long item = (blockIdx.x * 4L + (threadIdx.x >> 6)) * (64 / LPI) +
+                    lane / LPI;
+  const int d = (lane % LPI) * 4;
+  const long it = item < items ? item : items - 1;
+  const int head = (int)(it % p.heads);
+  const long row = it / p.heads;
+  float x[4], w[4];
+  load_vec<4>(o + it * (LPI * 4) + d, x);
+  float ss = 0.f;
+#pragma unroll
+  for (int r = 0; r < 4; ++r) ss += x[r] * x[r];
+#pragma unroll
+  for (int off = LPI / 2; off >= 1; off >>= 1) ss += __shfl_xor(ss, off, 64);
+  const float inv = 1.f / sqrtf(ss / (LPI * 4) + p.norm_eps);
+  const int col = head * LPI * 4 + d;
+  load_vec<4>(p.norm_w + col, w);
+  if (item >= items) return;
+  const T* g = (const T*)p.proj + row * p.proj_stride + p.off_g + col;
+  T* out = (T*)p.out + row * p.out_stride + col;
+  if constexpr (sizeof(T) == 2) {
+    union { uint2 u; __hip_bfloat16 e[4]; } gv, ov;
+    gv.u = *reinterpret_cast<const uint2*>(g);
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      ov.e[r] = f2bf(x[r] * inv * w[r] * sigmoid_f(bf2f(gv.e[r])));
+    *reinterpret_cast<uint2*>(out) = ov.u;
+  } else {
+    float gv[4];
+    load_vec<4>((const float*)g, gv);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) gv[r] = x[r] * inv * w[r] * sigmoid_f(gv[r]);
+    store_vec<4>((float*)out, gv);
+  }
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void delta_out_kernel(
     const DeltaArgs p, const float* __restrict__ o, const long items) {
@@ -349,18 +416,37 @@ __global__ __launch_bounds__(256) void delta_out_kernel(
                        sigmoid_f(to_f(g[d])));
 }
 
-template <typename T, int DP>
+template <typename T, int DP, int KS, int NC>
 void delta_chunk_t(const DeltaArgs& p, const int* tiles, const int* chunk_cu,
                    float* ws, float* o, int n_tiles, int seqs, long rows,
                    hipStream_t s) {
-  constexpr int NW = DP / 16 < 4 ? DP / 16 : 4;
-  const int zs = (p.dim + NW * 16 - 1) / (NW * 16);
+  constexpr int NT = KS * NC * 64;
+  const int zs = (p.dim + NC * 16 - 1) / (NC * 16);
+  const size_t lds = 2 * Rec<DP>::SIZE * sizeof(float) +
+                     (KS == 2 ? (size_t)(KS + 1) * NC * 64 * 16 : 0);
+  static bool once = false;
+  if (!once) {
+    (void)hipFuncSetAttribute((const void*)delta_scan_kernel<T, DP, KS, NC>,
+                              hipFuncAttributeMaxDynamicSharedMemorySize,
+                              (int)lds);
+    once = true;
+  }
   delta_prep_kernel<T, DP><<<dim3(n_tiles, p.heads), 256, 0, s>>>(p, tiles,
                                                                   ws);
-  delta_scan_kernel<T, DP, NW><<<dim3(p.heads, seqs, zs), NW * 64, 0, s>>>(
+  delta_scan_kernel<T, DP, KS, NC><<<dim3(p.heads, seqs, zs), NT, lds, s>>>(
       p, chunk_cu, ws, o);
   const long items = rows * p.heads;
-  delta_out_kernel<T><<<(int)((items + 3) / 4), 256, 0, s>>>(p, o, items);
+  const bool vec = p.dim == DP && p.proj_stride % 4 == 0 &&
+                   p.out_stride % 4 == 0 && p.off_g % 4 == 0 &&
+                   ((uintptr_t)p.proj & 15) == 0 &&
+                   ((uintptr_t)p.out & 15) == 0;
+  if (vec) {
+    const long per = 4L * (64 / (DP / 4));
+    delta_out_vec_kernel<T, DP / 4>
+        <<<(int)((items + per - 1) / per), 256, 0, s>>>(p, o, items);
+  } else {
+    delta_out_kernel<T><<<(int)((items + 3) / 4), 256, 0, s>>>(p, o, items);
+  }
 }
 
 template <typename T>
@@ -368,11 +454,11 @@ void delta_chunk_d(const DeltaArgs& p, const int* tiles, const int* chunk_cu,
                    float* ws, float* o, int n_tiles, int seqs, long rows,
                    hipStream_t s) {
   if (p.dim <= 32) {
-    delta_chunk_t<T, 32>(p, tiles, chunk_cu, ws, o, n_tiles, seqs, rows, s);
+    delta_chunk_t<T, 32, 1, 2>(p, tiles, chunk_cu, ws, o, n_tiles, seqs, rows, s);
   } else if (p.dim <= 64) {
-    delta_chunk_t<T, 64>(p, tiles, chunk_cu, ws, o, n_tiles, seqs, rows, s);
+    delta_chunk_t<T, 64, 2, 2>(p, tiles, chunk_cu, ws, o, n_tiles, seqs, rows, s);
   } else {
-    delta_chunk_t<T, 128>(p, tiles, chunk_cu, ws, o, n_tiles, seqs, rows, s);
+    delta_chunk_t<T, 128, 2, 4>(p, tiles, chunk_cu, ws, o, n_tiles, seqs, rows, s);
   }
 }
 

@@ -18,8 +18,10 @@
 
 namespace {
 
-template <typename T, int DP, int NT>
-__global__ __launch_bounds__(NT) void delta_step_kernel(const DeltaArgs p) {
+// MINW: waves per SIMD the registers must allow (the loads of one workgroup
+// hide behind the others' work)
+template <typename T, int DP, int NT, int MINW>
+__global__ __launch_bounds__(NT, MINW) void delta_step_kernel(const DeltaArgs p) {
   constexpr int CG = DP / 4;              // column groups of 4
   constexpr int RP = NT / CG;             // key rows per pass
   constexpr int IT = DP / RP;             // passes = rows per thread
@@ -82,6 +84,7 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(const DeltaArgs p) {
         } else {
           const T* w2 = (const T*)p.w2 + (size_t)ch * p.rank;
           if ((p.rank & 7) == 0) {
+#pragma unroll 2
             for (int j = 0; j < p.rank; j += 8) {
               float wv[8];
               load_vec<8>(w2 + j, wv);
@@ -89,6 +92,7 @@ __global__ __launch_bounds__(NT) void delta_step_kernel(const DeltaArgs p) {
               for (int e = 0; e < 8; ++e) zz += wv[e] * low_s[j + e];
             }
           } else {
+#pragma unroll 2
             for (int j = 0; j < p.rank; ++j) zz += to_f(w2[j]) * low_s[j];
           }
         }
@@ -194,11 +198,19 @@ template <typename T>
 void delta_step_t(const DeltaArgs& p, int seqs, hipStream_t s) {
   const dim3 grid(p.heads, seqs);
   const size_t lds = sizeof(float) * (p.z ? 0 : p.rank);
-#define DS_GO(DP, NT) delta_step_kernel<T, DP, NT><<<grid, NT, lds, s>>>(p)
-  if (p.dim <= 32) DS_GO(32, 64);
-  else if (p.dim <= 64) DS_GO(64, 256);
-  else if (p.dim <= 128) DS_GO(128, 256);
-  else DS_GO(256, 1024);
+#define DS_GO(DP, NT, MW)                                                     \
+  delta_step_kernel<T, DP, NT, MW><<<grid, NT, lds, s>>>(p)
+  if (p.dim <= 32) {
+    DS_GO(32, 64, 4);
+  } else if (p.dim <= 64) {
+    DS_GO(64, 256, 5);
+  } else if (p.dim <= 128) {
+    // few heads: more threads shorten each one's walk
+    if (p.heads * seqs <= 512) { DS_GO(128, 512, 2); }
+    else { DS_GO(128, 256, 3); }
+  } else {
+    DS_GO(256, 1024, 4);
+  }
 #undef DS_GO
 }
 

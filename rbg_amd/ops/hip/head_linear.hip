@@ -52,6 +52,23 @@ __global__ __launch_bounds__(256) void head_linear_kernel(
   for (int t = 0; t < MT; ++t) {
     const int s = s0 + t * 16 + gl;
     if (s >= p.rows) continue;
+    if (p.pack) {                       // four columns as one 8-byte access
+      const int n = n0 + gs * 4;
+      if (n >= p.n) continue;
+      const size_t col = (size_t)head * p.n + n;
+      union { uint2 u; __hip_bfloat16 e[4]; } ov, gv;
+      if (p.gate != nullptr)
+        gv.u = *reinterpret_cast<const uint2*>(
+            (const __hip_bfloat16*)p.gate + (size_t)s * p.g_row + col);
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        ov.e[r] = f2bf(p.gate != nullptr
+                           ? acc[t][r] * sigmoid_f(bf2f(gv.e[r]))
+                           : acc[t][r]);
+      *reinterpret_cast<uint2*>((__hip_bfloat16*)p.out + (size_t)s * p.o_row +
+                                col) = ov.u;
+      continue;
+    }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int n = n0 + gs * 4 + r;

@@ -1,17 +1,18 @@
 // Decode attention over paged latents (gfx950, bf16): absorbed queries, one
 // token per sequence, the latent as key and value at once, window-limited.
 //
-// A workgroup takes one sequence, 16 heads and one split of the visible keys;
-// its 4 waves walk 16-key chunks (a part of one page: contiguous memory)
-// independently of each other:
-//   global -> registers, two chunks ahead -> wave-private LDS
-//   S^T = C Q^T    A = latent rows, B = the 16 heads' queries in registers
-//   softmax        a head is a lane column; max and sum take two shuffles
-//   O^T += C^T P^T B = the weights' registers, split in two bf16 so that they
-//                  keep 16 bits; A = the same LDS rows read transposed
-// No barrier inside the loop.  The waves' (m, l, O) merge through LDS, the
-// splits' in latent_combine.  Latents are read once per 16 heads, which the
-// second head tile finds in L2.
+// A workgroup takes one sequence, 16 heads and one split of the visible keys,
+// 64 keys a step (4 chunks of 16: a chunk is part of one page, so contiguous):
+//   stage    wave w brings chunk w: global -> registers, a step ahead -> LDS
+//   S^T = C Q^T    wave w scores its chunk: A = latent rows, B = the heads'
+//            queries in registers; a head is a lane column
+//   softmax  running max shared through LDS; the weights go to LDS as two bf16
+//            (hi + lo), so that they keep 16 bits
+//   O^T += C^T P^T wave w owns a quarter of the rank for all 64 keys: A = the
+//            same LDS rows read transposed, B = the weights
+// The accumulators are split over the waves, so nothing is merged at the end
+// but the sum of the weights.  Splits of the keys meet in latent_combine.  The
+// second tile of 16 heads finds the latents in L2.
 #include "mfma_util.h"
 #include "mix_args.h"
 
@@ -20,22 +21,27 @@ namespace {
 constexpr int NW = 4;
 
 template <int RK>
-__global__ __launch_bounds__(NW * 64, 1) void latent_decode_kernel(
+__global__ __launch_bounds__(NW * 64, 2) void latent_decode_kernel(
     const LatentDecodeArgs p) {
   constexpr int PITCH = RK + 16;              // 8 banks per row
   constexpr int LPC = 16 * RK / 8 / 64;       // 16-byte loads per chunk
-  constexpr int DT = RK / 16;
+  constexpr int DT = RK / 16 / NW;            // 16-column tiles per wave
+  static_assert(DT >= 1 && LPC >= 1, "rank tile too small");
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  __hip_bfloat16* cs = (__hip_bfloat16*)smem +
-                       (threadIdx.x >> 6) * 16 * PITCH;
+  __hip_bfloat16* cs = (__hip_bfloat16*)smem; // [64][PITCH]
+  // weights by chunk, lane group and head: 4 keys each
+  mf_bf4* ph = (mf_bf4*)(cs + 64 * PITCH);    // [4][4][16]
+  mf_bf4* pl = ph + 256;
+  float* mx_s = (float*)(pl + 256);           // [NW][16]
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int gl = lane & 15, gs = lane >> 4;
   const int split = blockIdx.x, seq = blockIdx.y, h0 = blockIdx.z * 16;
   const int pos = p.ctx[seq] - 1;
   const int lo = p.window > 0 ? max(0, pos - p.window + 1) : 0;
   const int c_lo = lo >> 4, c_n = (pos >> 4) - c_lo + 1;
-  // this split's chunks; the waves take every NW-th
-  const int per = (c_n + p.splits - 1) / p.splits;
+  // this split's chunks, whole steps of NW
+  const int steps = (c_n + NW - 1) / NW;
+  const int per = (steps + p.splits - 1) / p.splits * NW;
   const int c_beg = c_lo + split * per;
   const int c_end = min(c_beg + per, c_lo + c_n);
   const int* table = p.tables + (size_t)seq * p.max_pages;
@@ -60,10 +66,10 @@ __global__ __launch_bounds__(NW * 64, 1) void latent_decode_kernel(
   for (int d = 0; d < DT; ++d) acc[d] = {0.f, 0.f, 0.f, 0.f};
   const float sl2 = p.scale * LOG2E;
 
-  u32x4 ra[LPC], rb[LPC];
+  u32x4 reg[LPC];
   const u32x4 zero4 = {0, 0, 0, 0};
-  // a chunk past the end re-reads the last one; it is never used
-#define LD_FETCH(reg, c)                                                      \
+  // a chunk past the end re-reads the last one, as zeros
+#define LD_FETCH(c)                                                           \
   do {                                                                        \
     const int cc = min((c), c_end - 1);                                       \
     const __hip_bfloat16* src =                                               \
@@ -75,163 +81,159 @@ __global__ __launch_bounds__(NW * 64, 1) void latent_decode_kernel(
           ? *reinterpret_cast<const u32x4*>(src + key * p.rank + d) : zero4;  \
     }                                                                         \
   } while (0)
-  // rows outside the window are stored as zeros: their weight is zero, but a
-  // row nobody has written yet may hold anything
-#define LD_LAND(reg, c)                                                       \
-  do {                                                                        \
-    _Pragma("unroll") for (int i = 0; i < LPC; ++i) {                         \
-      const int e = i * 64 + lane, key = e / (RK / 8), d = (e % (RK / 8)) * 8;\
-      const int j = (c) * 16 + key;                                           \
-      *reinterpret_cast<u32x4*>(&cs[key * PITCH + d]) =                       \
-          j >= lo && j <= pos ? reg[i] : zero4;                               \
-    }                                                                         \
-  } while (0)
 
-  auto chunk = [&](int c) {
-    f32x4 s = {0.f, 0.f, 0.f, 0.f}, s2 = {0.f, 0.f, 0.f, 0.f};
+  if (c_beg < c_end) LD_FETCH(c_beg + wave);
+  for (int c0 = c_beg; c0 < c_end; c0 += NW) {
+    const int c = c0 + wave;
+    __hip_bfloat16* mine = cs + wave * 16 * PITCH;
+    // rows outside the window are stored as zeros: their weight is zero, but
+    // a row nobody has written yet may hold anything
+    const int c_hi = min(pos, c_end * 16 - 1);
+#pragma unroll
+    for (int i = 0; i < LPC; ++i) {
+      const int e = i * 64 + lane, key = e / (RK / 8), d = (e % (RK / 8)) * 8;
+      const int j = c * 16 + key;
+      *reinterpret_cast<u32x4*>(&mine[key * PITCH + d]) =
+          j >= lo && j <= c_hi ? reg[i] : zero4;
+    }
+    if (c0 + NW < c_end) LD_FETCH(c + NW);
+    f32x4 s = {0.f, 0.f, 0.f, 0.f}, s2 = s;
 #pragma unroll
     for (int st = 0; st < RK / 32; st += 2) {
-      s = mfma_bf16_k32(frag8(&cs[gl * PITCH + st * 32 + gs * 8]), qf[st], s);
-      if (st + 1 < RK / 32)
-        s2 = mfma_bf16_k32(frag8(&cs[gl * PITCH + st * 32 + 32 + gs * 8]),
-                           qf[st + 1], s2);
+      s = mfma_bf16_k32(frag8(&mine[gl * PITCH + st * 32 + gs * 8]), qf[st],
+                        s);
+      s2 = mfma_bf16_k32(frag8(&mine[gl * PITCH + st * 32 + 32 + gs * 8]),
+                         qf[st + 1], s2);
     }
     s += s2;
     float x[4], mx = MASKED;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int j = c * 16 + gs * 4 + r;
-      x[r] = j >= lo && j <= pos ? s[r] * sl2 : MASKED;
+      x[r] = j >= lo && j <= c_hi ? s[r] * sl2 : MASKED;
       mx = fmaxf(mx, x[r]);
     }
     mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-    const float mn = fmaxf(m, mx), corr = exp2_fast(m - mn);
+    if (gs == 0) mx_s[wave * 16 + gl] = mx;
+    __syncthreads();
+    float mn = m;
+#pragma unroll
+    for (int w = 0; w < NW; ++w) mn = fmaxf(mn, mx_s[w * 16 + gl]);
+    const float corr = exp2_fast(m - mn);
     m = mn;
-    mf_bf4 ph, pl;
     float sum = 0.f;
+    mf_bf4 hi, lw;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const float e = x[r] > MASKED ? exp2_fast(x[r] - mn) : 0.f;
       sum += e;
-      __bf16 h, w;
-      split_bf16(e, h, w);
-      ph[r] = h;
-      pl[r] = w;
+      __bf16 a, b;
+      split_bf16(e, a, b);
+      hi[r] = a;
+      lw[r] = b;
     }
-    l = l * corr + sum;
-    const bool rescale = __any(corr != 1.f);
+    ph[(wave * 4 + gs) * 16 + gl] = hi;
+    pl[(wave * 4 + gs) * 16 + gl] = lw;
+    l = l * corr + sum;                       // this wave's keys
 #pragma unroll
-    for (int d = 0; d < DT; ++d) {
-      const mf_bf4 vf =
-          tr_read4(&cs[(gs * 4 + (gl >> 2)) * PITCH + d * 16 + (gl & 3) * 4]);
-      if (rescale) acc[d] *= corr;
-      acc[d] = mfma_bf16_k16(vf, ph, acc[d]);
-      acc[d] = mfma_bf16_k16(vf, pl, acc[d]);
+    for (int d = 0; d < DT; ++d) acc[d] *= corr;
+    __syncthreads();
+#pragma unroll
+    for (int st = 0; st < 2; ++st) {
+      const mf_bf4 h0v = ph[(st * 8 + gs) * 16 + gl];
+      const mf_bf4 h1v = ph[(st * 8 + 4 + gs) * 16 + gl];
+      const mf_bf4 l0v = pl[(st * 8 + gs) * 16 + gl];
+      const mf_bf4 l1v = pl[(st * 8 + 4 + gs) * 16 + gl];
+      const mf_bf8 hv = {h0v[0], h0v[1], h0v[2], h0v[3],
+                         h1v[0], h1v[1], h1v[2], h1v[3]};
+      const mf_bf8 lv = {l0v[0], l0v[1], l0v[2], l0v[3],
+                         l1v[0], l1v[1], l1v[2], l1v[3]};
+#pragma unroll
+      for (int d = 0; d < DT; ++d) {
+        const __hip_bfloat16* b = &cs[(st * 32 + gs * 4 + (gl >> 2)) * PITCH +
+                                      (wave * DT + d) * 16 + (gl & 3) * 4];
+        const mf_bf4 v0 = tr_read4(b), v1 = tr_read4(b + 16 * PITCH);
+        const mf_bf8 vf = {v0[0], v0[1], v0[2], v0[3],
+                           v1[0], v1[1], v1[2], v1[3]};
+        acc[d] = mfma_bf16_k32(vf, hv, acc[d]);
+        acc[d] = mfma_bf16_k32(vf, lv, acc[d]);
+      }
     }
-  };
-
-  int c = c_beg + wave;
-  if (c < c_end) {
-    LD_FETCH(ra, c);
-    LD_FETCH(rb, c + NW);
-    for (; c < c_end; c += 2 * NW) {
-      LD_LAND(ra, c);
-      LD_FETCH(ra, c + 2 * NW);
-      __builtin_amdgcn_wave_barrier();
-      chunk(c);
-      __builtin_amdgcn_wave_barrier();
-      if (c + NW >= c_end) break;
-      LD_LAND(rb, c + NW);
-      LD_FETCH(rb, c + 3 * NW);
-      __builtin_amdgcn_wave_barrier();
-      chunk(c + NW);
-      __builtin_amdgcn_wave_barrier();
-    }
+    __syncthreads();                          // LDS is free again
   }
 #undef LD_FETCH
-#undef LD_LAND
 
-  // merge the waves: [RK][17] sums and [NW][16] (m, l) in LDS
+  // sum of the weights over lane groups and waves
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
-  __syncthreads();                            // staging is free now
-  float* osum = (float*)smem;
-  float* ml = osum + RK * 17;
-  if (gs == 0) {
-    ml[(wave * 16 + gl) * 2] = m;
-    ml[(wave * 16 + gl) * 2 + 1] = l;
-  }
+  if (gs == 0) mx_s[wave * 16 + gl] = l;
   __syncthreads();
-  float M = MASKED, L = 0.f;
+  float L = 0.f;
 #pragma unroll
-  for (int w = 0; w < NW; ++w) M = fmaxf(M, ml[(w * 16 + gl) * 2]);
-#pragma unroll
-  for (int w = 0; w < NW; ++w)
-    L += ml[(w * 16 + gl) * 2 + 1] * exp2_fast(ml[(w * 16 + gl) * 2] - M);
-  const float f = exp2_fast(m - M);
-  for (int w = 0; w < NW; ++w) {
-    if (wave == w) {
-#pragma unroll
-      for (int d = 0; d < DT; ++d)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          float* o = &osum[(d * 16 + gs * 4 + r) * 17 + gl];
-          *o = (w == 0 ? 0.f : *o) + acc[d][r] * f;
-        }
+  for (int w = 0; w < NW; ++w) L += mx_s[w * 16 + gl];
+  if (h0 + gl >= p.heads) return;
+  const size_t row = (size_t)seq * p.heads + h0 + gl;
+  if (p.splits > 1) {
+    const size_t part = (size_t)split * p.seqs * p.heads + row;
+    if (wave == 0 && gs == 0) {
+      p.part_ml[part * 2] = m;
+      p.part_ml[part * 2 + 1] = L;
     }
-    __syncthreads();
-  }
-  float* lm = ml + NW * 32;                   // [16] L for the writers below
-  if (tid < 16) {
-    lm[tid] = L;
-    if (p.splits > 1 && h0 + tid < p.heads) {
-      float* o = p.part_ml +
-                 (((size_t)split * p.seqs + seq) * p.heads + h0 + tid) * 2;
-      o[0] = M;
-      o[1] = L;
+#pragma unroll
+    for (int d = 0; d < DT; ++d) {
+      const int c = (wave * DT + d) * 16 + gs * 4;
+      if (c < p.rank)
+        *reinterpret_cast<f32x4*>(&p.part_o[part * p.rank + c]) = acc[d];
     }
-  }
-  __syncthreads();
-  for (int i = tid; i < 16 * p.rank; i += NW * 64) {
-    const int h = i / p.rank, d = i % p.rank;
-    if (h0 + h >= p.heads) break;
-    const float o = osum[d * 17 + h];
-    if (p.splits > 1)
-      p.part_o[(((size_t)split * p.seqs + seq) * p.heads + h0 + h) * p.rank +
-               d] = o;
-    else
-      ((__hip_bfloat16*)p.out)[((size_t)seq * p.heads + h0 + h) * p.rank + d] =
-          f2bf(o / lm[h]);
+  } else {
+    const float inv = 1.f / L;
+#pragma unroll
+    for (int d = 0; d < DT; ++d) {
+      const int c = (wave * DT + d) * 16 + gs * 4;
+      if (c >= p.rank) continue;
+      union { uint2 u; __hip_bfloat16 e[4]; } o;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o.e[r] = f2bf(acc[d][r] * inv);
+      *reinterpret_cast<uint2*>(
+          &((__hip_bfloat16*)p.out)[row * p.rank + c]) = o.u;
+    }
   }
 }
 
 // one workgroup per (sequence, head): sum of the splits' partials
-__global__ __launch_bounds__(256) void latent_combine_kernel(
+__global__ __launch_bounds__(128) void latent_combine_kernel(
     const LatentDecodeArgs p) {
+  __shared__ float f[64];                     // splits <= 64
   const size_t row = blockIdx.x;              // seq * heads + head
   const size_t rows = (size_t)p.seqs * p.heads;
-  float M = MASKED, L = 0.f;
-  for (int s = 0; s < p.splits; ++s)
-    M = fmaxf(M, p.part_ml[(s * rows + row) * 2]);
-  for (int s = 0; s < p.splits; ++s)
-    L += p.part_ml[(s * rows + row) * 2 + 1] *
-         exp2_fast(p.part_ml[(s * rows + row) * 2] - M);
-  const float inv = 1.f / L;
-  for (int d = threadIdx.x; d < p.rank; d += 256) {
-    float o = 0.f;
+  const int tid = threadIdx.x;
+  if (tid < 64) {
+    const bool on = tid < p.splits;
+    const float m = on ? p.part_ml[(tid * rows + row) * 2] : MASKED;
+    const float l = on ? p.part_ml[(tid * rows + row) * 2 + 1] : 0.f;
+    const float M = wave_max(m);
+    const float w = on ? exp2_fast(m - M) : 0.f;
+    f[tid] = w / wave_sum(l * w);
+  }
+  __syncthreads();
+  for (int d = tid * 4; d < p.rank; d += 512) {
+    f32x4 o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 8
     for (int s = 0; s < p.splits; ++s)
-      o += p.part_o[(s * rows + row) * p.rank + d] *
-           exp2_fast(p.part_ml[(s * rows + row) * 2] - M);
-    ((__hip_bfloat16*)p.out)[row * p.rank + d] = f2bf(o * inv);
+      o += *reinterpret_cast<const f32x4*>(
+               &p.part_o[(s * rows + row) * p.rank + d]) * f[s];
+    union { uint2 u; __hip_bfloat16 e[4]; } ov;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) ov.e[r] = f2bf(o[r]);
+    *reinterpret_cast<uint2*>(&((__hip_bfloat16*)p.out)[row * p.rank + d]) =
+        ov.u;
   }
 }
 
 template <int RK>
 void latent_decode_t(const LatentDecodeArgs& p, hipStream_t s) {
-  const size_t stage = (size_t)NW * 16 * (RK + 16) * 2;
-  const size_t merge = (size_t)(RK * 17 + NW * 32 + 16) * 4;
-  const size_t lds = stage > merge ? stage : merge;
+  const size_t lds = (size_t)64 * (RK + 16) * 2 + 2 * 256 * 8 + NW * 16 * 4;
   static bool once = false;
   if (!once) {
     (void)hipFuncSetAttribute((const void*)latent_decode_kernel<RK>,
@@ -257,5 +259,5 @@ extern "C" void launch_latent_decode(const LatentDecodeArgs* p,
     latent_decode_t<512>(*p, s);
   }
   if (p->splits > 1)
-    latent_combine_kernel<<<p->seqs * p->heads, 256, 0, s>>>(*p);
+    latent_combine_kernel<<<p->seqs * p->heads, 128, 0, s>>>(*p);
 }

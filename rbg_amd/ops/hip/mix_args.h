@@ -71,4 +71,5 @@ struct HeadLinearArgs {
   void* out;              // + s*o_row + h*n
   long x_row, x_head, g_row, o_row;
   int rows, heads, n, k;
+  int pack;               // out (and gate) allow 8-byte accesses
 };

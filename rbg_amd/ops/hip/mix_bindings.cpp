@@ -392,7 +392,7 @@ Tensor latent_decode(Tensor q, Tensor cache, Tensor tables, Tensor ctx,
     p.seqs = (int)R; p.heads = (int)H; p.rank = (int)K;
     p.window = (int)window; p.page_size = (int)cache.size(1);
     p.max_pages = (int)tables.size(1); p.scale = (float)scale;
-    p.splits = (int)(splits < 1 ? 1 : splits);
+    p.splits = (int)(splits < 1 ? 1 : splits > 64 ? 64 : splits);
     Tensor po, pml;
     if (p.splits > 1) {
       auto f32 = q.options().dtype(torch::kFloat32);
@@ -441,6 +441,8 @@ void head_linear(Tensor x, Tensor w, OptTensor gate, Tensor out) {
   p.x = x.data_ptr(); p.w = w.data_ptr(); p.out = out.data_ptr();
   p.x_row = x.stride(0); p.x_head = x.stride(1); p.o_row = out.stride(0);
   p.rows = (int)R; p.heads = (int)H; p.n = (int)N; p.k = (int)K;
+  p.pack = N % 4 == 0 && p.o_row % 4 == 0 && aligned(out, 8) &&
+           (!gate || (p.g_row % 4 == 0 && aligned(*gate, 8)));
   const bool vec = mult8({K, p.x_row, p.x_head}) && aligned(x, 16) &&
                    aligned(w, 16);
   if (R) launch_head_linear(&p, is_f32(x), vec, current_stream());

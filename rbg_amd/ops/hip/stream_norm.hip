@@ -14,7 +14,6 @@
 namespace {
 
 constexpr int NT = 256;
-constexpr int NW = NT / 64;
 
 template <typename T, int V>
 __global__ __launch_bounds__(NT) void embed_stream_kernel(
@@ -33,7 +32,7 @@ __global__ __launch_bounds__(NT) void embed_stream_kernel(
 
 // CONV: n1 becomes n1 + conv(n1) with the history of state slot slots[row]
 // (all zeros at position 0), and the history moves on by one token.
-template <typename T, int V, bool CONV>
+template <typename T, int V, bool CONV, int NT>
 __global__ __launch_bounds__(NT) void stream_norm_kernel(
     float* __restrict__ x, const T* __restrict__ delta,
     const float* __restrict__ w1, const float* __restrict__ w2,
@@ -41,6 +40,7 @@ __global__ __launch_bounds__(NT) void stream_norm_kernel(
     const float eps, const float* __restrict__ conv_w,
     T* __restrict__ conv_state, const int* __restrict__ slots,
     const int* __restrict__ positions, const int taps) {
+  constexpr int NW = NT / 64;
   extern __shared__ float smem[];
   const int sub = groups >= NW ? 1 : (NW + groups - 1) / groups;
   float* row = smem;                    // [width]
@@ -130,7 +130,9 @@ __global__ __launch_bounds__(NT) void stream_norm_kernel(
 // token of the tile inside the sequence's rows).  Only a sequence's first
 // tile reads its history (the host keeps tile >= taps - 1), and that same
 // thread writes the new history afterwards, so no other workgroup races it.
-template <typename T, int V>
+// TAPS > 0: the taps' weights and the last inputs live in registers, so that a
+// row is read once; 0: any number of taps.
+template <typename T, int V, int TAPS>
 __global__ __launch_bounds__(NT) void causal_conv_kernel(
     T* __restrict__ out, const T* __restrict__ x,
     const float* __restrict__ w, T* __restrict__ state,
@@ -145,37 +147,58 @@ __global__ __launch_bounds__(NT) void causal_conv_kernel(
   T* hist = state + (size_t)slots[seq] * (taps - 1) * width + i;
   const T* xs = x + (size_t)row0 * width + i;
   const int t1 = min(t0 + tile, len);
-  for (int t = t0; t < t1; ++t) {
-    float h[V], cw[V], v[V];
-    load_vec<V>(xs + (size_t)t * width, h);
-    for (int p = 0; p < taps; ++p) {
-      const int src = t - taps + 1 + p;       // row in this step, < 0: history
-      if (src >= 0) {
-        load_vec<V>(xs + (size_t)src * width, v);
-      } else if (fresh) {
-        continue;
-      } else {
-        load_vec<V>(hist + (size_t)(src + taps - 1) * width, v);
-      }
-      load_vec<V>(w + (size_t)p * width + i, cw);
+  // input at row src of this step; before it the history, or zeros
+  auto past = [&](int src, float* v) {
+    if (src >= 0) {
+      load_vec<V>(xs + (size_t)src * width, v);
+    } else if (fresh) {
 #pragma unroll
-      for (int j = 0; j < V; ++j) h[j] += cw[j] * v[j];
+      for (int j = 0; j < V; ++j) v[j] = 0.f;
+    } else {
+      load_vec<V>(hist + (size_t)(src + taps - 1) * width, v);
     }
-    store_vec<V>(out + ((size_t)row0 + t) * width + i, h);
+  };
+  if constexpr (TAPS > 0) {
+    float cw[TAPS][V], win[TAPS][V];
+#pragma unroll
+    for (int p = 0; p < TAPS; ++p)
+      load_vec<V>(w + (size_t)p * width + i, cw[p]);
+#pragma unroll
+    for (int p = 1; p < TAPS; ++p) past(t0 - TAPS + p, win[p]);
+#pragma unroll 4
+    for (int t = t0; t < t1; ++t) {
+#pragma unroll
+      for (int p = 1; p < TAPS; ++p)
+#pragma unroll
+        for (int j = 0; j < V; ++j) win[p - 1][j] = win[p][j];
+      load_vec<V>(xs + (size_t)t * width, win[TAPS - 1]);
+      float h[V];
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        h[j] = win[TAPS - 1][j];
+#pragma unroll
+        for (int p = 0; p < TAPS; ++p) h[j] += cw[p][j] * win[p][j];
+      }
+      store_vec<V>(out + ((size_t)row0 + t) * width + i, h);
+    }
+  } else {
+    for (int t = t0; t < t1; ++t) {
+      float h[V], cw[V], v[V];
+      load_vec<V>(xs + (size_t)t * width, h);
+      for (int p = 0; p < taps; ++p) {
+        past(t - taps + 1 + p, v);
+        load_vec<V>(w + (size_t)p * width + i, cw);
+#pragma unroll
+        for (int j = 0; j < V; ++j) h[j] += cw[j] * v[j];
+      }
+      store_vec<V>(out + ((size_t)row0 + t) * width + i, h);
+    }
   }
   if (t0 == 0) {
     // ascending order: entry p is read (as p + len) no later than overwritten
     for (int p = 0; p < taps - 1; ++p) {
-      const int src = len - (taps - 1) + p;
       float v[V];
-      if (src >= 0) {
-        load_vec<V>(xs + (size_t)src * width, v);
-      } else if (fresh) {
-#pragma unroll
-        for (int j = 0; j < V; ++j) v[j] = 0.f;
-      } else {
-        load_vec<V>(hist + (size_t)(src + taps - 1) * width, v);
-      }
+      past(len - (taps - 1) + p, v);
       store_vec<V>(hist + (size_t)p * width, v);
     }
   }
@@ -187,19 +210,25 @@ void stream_norm_t(float* x, const void* delta, const float* w1,
                    int groups, float eps, const float* conv_w, void* state,
                    const int* slots, const int* positions, int taps,
                    hipStream_t s) {
-  const int sub = groups >= NW ? 1 : (NW + groups - 1) / groups;
+  const int nt = width >= 4096 ? 512 : 256, nw = nt / 64;
+  const int sub = groups >= nw ? 1 : (nw + groups - 1) / groups;
   const size_t lds = sizeof(float) * (width + groups * sub + groups);
   const bool vec = (width / groups) % 8 == 0;
-#define SN_GO(V, C)                                                           \
-  stream_norm_kernel<T, V, C><<<tokens, NT, lds, s>>>(                        \
+#define SN_GO(V, C, N)                                                        \
+  stream_norm_kernel<T, V, C, N><<<tokens, N, lds, s>>>(                      \
       x, (const T*)delta, w1, w2, (T*)n1, (T*)n2, width, groups, eps, conv_w, \
       (T*)state, slots, positions, taps)
+#define SN_VC(V, C)                                                           \
+  do {                                                                        \
+    if (nt == 512) { SN_GO(V, C, 512); } else { SN_GO(V, C, 256); }           \
+  } while (0)
   if (conv_w != nullptr) {
-    if (vec) SN_GO(8, true); else SN_GO(1, true);
+    if (vec) SN_VC(8, true); else SN_VC(1, true);
   } else {
-    if (vec) SN_GO(8, false); else SN_GO(1, false);
+    if (vec) SN_VC(8, false); else SN_VC(1, false);
   }
 #undef SN_GO
+#undef SN_VC
 }
 
 }  // namespace
@@ -237,11 +266,19 @@ void launch_causal_conv(void* out, const void* x, const float* w, void* state,
                         int taps, int f32, hipStream_t s) {
   const int v = width % 8 == 0 ? 8 : 1;
   const dim3 grid(n_tiles, (width / v + NT - 1) / NT);
-#define CC_GO(T, V) causal_conv_kernel<T, V><<<grid, NT, 0, s>>>(             \
+#define CC_GO(T, V, N) causal_conv_kernel<T, V, N><<<grid, NT, 0, s>>>(       \
       (T*)out, (const T*)x, w, (T*)state, tiles, cu, starts, slots, tile,     \
       width, taps)
-  if (f32) { if (v == 8) CC_GO(float, 8); else CC_GO(float, 1); }
-  else { if (v == 8) CC_GO(__hip_bfloat16, 8); else CC_GO(__hip_bfloat16, 1); }
+#define CC_V(T)                                                               \
+  do {                                                                        \
+    if (v == 1) { CC_GO(T, 1, 0); }                                           \
+    else if (taps == 2) { CC_GO(T, 8, 2); }                                   \
+    else if (taps == 3) { CC_GO(T, 8, 3); }                                   \
+    else if (taps == 4) { CC_GO(T, 8, 4); }                                   \
+    else { CC_GO(T, 8, 0); }                                                  \
+  } while (0)
+  if (f32) { CC_V(float); } else { CC_V(__hip_bfloat16); }
+#undef CC_V
 #undef CC_GO
 }
 

@@ -68,4 +68,6 @@ DEV_INLINE void store_vec(float* p, const float* o) {
   }
 }
 
-DEV_INLINE float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
+// f32 to about two units in the last place: hardware exp2 and reciprocal
+DEV_INLINE float rcp_f(float x) { return __builtin_amdgcn_rcpf(x); }
+DEV_INLINE float sigmoid_f(float z) { return rcp_f(1.f + __expf(-z)); }
