@@ -109,7 +109,11 @@ def prompt(n, vocab=101, seed=0):
     return torch.randint(0, vocab, (n,), generator=gen).tolist()
 
 
+def row_errs(got, want):
+    """Per row: RMS of the difference over the RMS of all answers."""
+    d = (got.double().cpu() - want).pow(2).mean(-1).sqrt()
+    return d / want.pow(2).mean().sqrt()
+
+
 def rel_err(got, want):
-    """Worst row: RMS of the difference over the RMS of the answers."""
-    d = (got.double().cpu() - want).pow(2).mean(-1).sqrt().max()
-    return (d / want.pow(2).mean().sqrt()).item()
+    return row_errs(got, want).max().item()
