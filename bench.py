@@ -40,7 +40,8 @@ def parse_args():
                    help="decode batch per GPU")
     p.add_argument("--seq-len", type=int, default=2048,
                    help="synthetic prompt length")
-    p.add_argument("--model", default="llama-3-8b")
+    p.add_argument("--model", default="llama-3-8b",
+                   help="preset name or model folder")
     p.add_argument("--device", default="cuda")
     p.add_argument("--parallel", choices=["pd", "dp", "tp", "pp"],
                    default="pd",
@@ -156,14 +157,15 @@ def main() -> int:
             dist.destroy_process_group()
         return 0
 
-    from rbg_amd.engine.config import EngineConfig, ModelConfig
+    from rbg_amd.engine.config import EngineConfig
     from rbg_amd.engine.engine import LLMEngine
     from rbg_amd.engine.sequence import SamplingParams
+    from rbg_amd.models.registry import resolve_model
     from rbg_amd.models.llama import PPContext, TPContext
 
     tp_mode = args.parallel == "tp" and world > 1
     pp_mode = args.parallel == "pp" and world > 1
-    model_cfg = ModelConfig.preset(args.model)
+    model_cfg = resolve_model(args.model)
     cfg = EngineConfig(
         model=model_cfg, device=device,
         max_batch_size=max(args.batch, 8),

@@ -88,7 +88,11 @@ class PagedKVCache:
             budget = 64 << 20     # CPU tests: 64 MB
         if cfg.kv_pool_tokens:
             return max(1, cfg.kv_pool_tokens // cfg.page_size)
-        return max(8, budget // self._page_bytes())
+        return max(8, (budget - self._fixed_bytes()) // self._page_bytes())
+
+    def _fixed_bytes(self) -> int:
+        """What the cache takes beside its pages."""
+        return 0
 
     # -- per-sequence state slots (recurrent models override) ---------------
 

@@ -27,7 +27,8 @@ from typing import Any, Dict, List, Optional
 
 import torch
 
-from .config import EngineConfig, ModelConfig
+from ..models.registry import resolve_model
+from .config import EngineConfig
 from .engine import LLMEngine
 from .kv_cache import BlockTable
 from .sequence import SamplingParams, Sequence
@@ -51,7 +52,10 @@ def _park_finished_pages(engine: LLMEngine, parked: Dict[int, List[int]]):
 
 def _make_engine(args, device: str, role: str,
                  max_new: int) -> LLMEngine:
-    model_cfg = ModelConfig.preset(args.model)
+    model_cfg = resolve_model(args.model)
+    if model_cfg.architecture != "llama":
+        raise SystemExit(f"{args.model}: the pd benchmark pushes plain KV "
+                         "pages; use --parallel dp for this family")
     horizon = args.seq_len + max_new + 64
     cfg = EngineConfig(
         model=model_cfg, device=device,

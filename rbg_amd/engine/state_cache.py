@@ -51,6 +51,11 @@ class StateCache(PagedKVCache):
         rows = sum(s.latent_rank for s in self.specs) * self.cfg.page_size
         return max(1, rows * self.dtype.itemsize)
 
+    def _fixed_bytes(self) -> int:
+        return self.num_slots * sum(
+            math.prod(shape) * dt.itemsize for spec in self.specs
+            for shape, dt in spec.state.values())
+
     def _size_pool(self, device: torch.device) -> int:
         pages = super()._size_pool(device)
         # a model without paged layers has pages of no size: bound their number

@@ -69,8 +69,8 @@ def main():
     ap.add_argument("--model", default="llama-3-8b")
     ap.add_argument("--device", default="cuda")
     args = ap.parse_args()
-    from rbg_amd.engine.config import ModelConfig
-    model_cfg = ModelConfig.preset(args.model)
+    from rbg_amd.models.registry import resolve_model
+    model_cfg = resolve_model(args.model)
     report = {
         "config": {"model": model_cfg.name, "batch": args.batch,
                    "seq_len": args.seq_len, "out_len": args.out_len},

@@ -102,8 +102,8 @@ def main() -> int:
                          "oversubscribed CPU test boxes where a collective "
                          "world bounce restarts the whole pool")
     args = ap.parse_args()
-    from rbg_amd.engine.config import ModelConfig
-    model_cfg = ModelConfig.preset(args.model)
+    from rbg_amd.models.registry import resolve_model
+    model_cfg = resolve_model(args.model)
     args.vocab = min(model_cfg.vocab_size, 128000)
 
     engine_args = {"model": args.model, "device": args.device,
