@@ -96,7 +96,7 @@ HBM_TB_S, BF16_TF, F32_TF = 8.0, 2500.0, 157.0
 
 
 def _time(fn, n: int = 12) -> float:
-    """Median-free mean over calls fn(i), microseconds on the GPU."""
+    """Mean microseconds on the GPU of fn(0), fn(1), ... in one graph."""
     for i in range(3):
         fn(i)
     torch.cuda.synchronize()
