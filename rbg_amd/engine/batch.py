@@ -30,6 +30,8 @@ class ForwardBatch:
     block_tables: Optional[torch.Tensor] = None  # [S, max_pages] int32
     context_lens: Optional[torch.Tensor] = None  # [S] int32
     decode_num_splits: int = 0      # 0 = pick host-side (sync-free in graphs)
+    # models that look at pairs of tokens: [T] int64, -1 before the first
+    prev_tokens: Optional[torch.Tensor] = None
     # models with per-sequence state
     starts: Optional[torch.Tensor] = None       # [B] int32 first row's position
     state_slots: Optional[torch.Tensor] = None  # [B] int32
@@ -54,7 +56,29 @@ class WindowView:
     #                                 of every 128 query rows
 
 
-QUERY_BLOCK = 128       # query rows per workgroup of the window attention
+@dataclass
+class PagedView:
+    """The prefill rows of a step whose keys are read from the pages."""
+    tables: torch.Tensor            # [seqs, pages] int32
+    seq_info: torch.Tensor          # [seqs, 3] int32: first query row, rows,
+    #                                 position of the first
+    row_info: torch.Tensor          # [rows, 2] int32: (sequence, position)
+    blocks: torch.Tensor            # [n, 2] int32: (sequence, first query)
+    #                                 of every QUERY_BLOCK query rows
+
+
+QUERY_BLOCK = 128       # query rows per workgroup of the prompt attentions
+
+
+def table_array(tables) -> np.ndarray:
+    """Block tables as one array [n, pages], padded with the scratch page."""
+    # numpy staging: batch composition churns every step under continuous
+    # serving, so the rebuild is on the step critical path
+    out = np.zeros((len(tables), max(len(t.pages) for t in tables)),
+                   dtype=np.int32)
+    for i, t in enumerate(tables):
+        out[i, :len(t.pages)] = t.pages
+    return out
 
 
 class VarlenLayout:
@@ -68,6 +92,7 @@ class VarlenLayout:
         self.page_size = page_size
         self.device = device
         self._views: Dict[int, WindowView] = {}
+        self._paged: Optional[PagedView] = None
         self._tiles: Dict[object, torch.Tensor] = {}
 
     def _dev(self, a: np.ndarray) -> torch.Tensor:
@@ -131,3 +156,21 @@ class VarlenLayout:
             blocks=self.prefill_tiles(QUERY_BLOCK))
         self._views[window] = view
         return view
+
+    def paged_view(self) -> PagedView:
+        """Of the prefill sequences; rows are counted after the decode rows."""
+        if self._paged is None:
+            nd = self.num_decode
+            starts, ends = self.starts[nd:], self.ends[nd:]
+            info, rows, row = [], [], 0
+            for b, (s, e) in enumerate(zip(starts, ends)):
+                info.append((row, e - s, s))
+                pos = np.arange(s, e)
+                rows.append(np.stack([np.full_like(pos, b), pos], axis=1))
+                row += e - s
+            self._paged = PagedView(
+                tables=self._dev(table_array(self.tables[nd:])),
+                seq_info=self._dev(np.array(info, dtype=np.int32)),
+                row_info=self._dev(np.concatenate(rows).astype(np.int32)),
+                blocks=self.prefill_tiles(QUERY_BLOCK))
+        return self._paged

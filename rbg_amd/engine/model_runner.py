@@ -18,7 +18,7 @@ import torch
 
 from ..models.llama import PPContext, TPContext
 from ..models.registry import build_model
-from .batch import ForwardBatch, VarlenLayout
+from .batch import ForwardBatch, VarlenLayout, table_array
 from .config import EngineConfig
 from .sequence import Sequence
 
@@ -73,6 +73,7 @@ class ModelRunner:
             num_decode = sum(single)
             order.sort(key=lambda i: not single[i])
         tokens: List[int] = []
+        prev: List[int] = []
         positions: List[int] = []
         slots: List[int] = []
         gather: List[int] = []
@@ -85,12 +86,15 @@ class ModelRunner:
             seq, start, toks = chunks[i]
             end = start + len(toks)
             tokens.extend(toks)
+            if self.model.needs_prev:
+                prev.append(seq.token_at(start - 1))
+                prev.extend(toks[:-1])
             positions.extend(range(start, end))
             slots.extend(seq.block_table.slots_for(start, end - start))
             first_row[i] = cu[-1]
             cu.append(cu[-1] + (end - start))
             cu_k.append(cu_k[-1] + end)
-            if any_past and not self.model.stateful:
+            if any_past and not self.model.varlen:
                 gather.extend(seq.block_table.slots_for(0, end))
             starts.append(start)
             ends.append(end)
@@ -100,7 +104,10 @@ class ModelRunner:
             positions=self._i32(positions),
             slot_mapping=self._i32(slots),
             cu_seqlens=self._i32(cu))
-        if self.model.stateful:
+        if self.model.needs_prev:
+            batch.prev_tokens = torch.tensor(prev, dtype=torch.int64,
+                                             device=self.device)
+        if self.model.varlen:
             batch.starts = self._i32(starts)
             batch.state_slots = self._i32([t.state_slot for t in tables])
             batch.num_decode = num_decode
@@ -109,7 +116,7 @@ class ModelRunner:
             batch.cu_prefill = self._i32([c - num_decode
                                           for c in cu[num_decode:]])
             if num_decode:
-                batch.block_tables = torch.from_numpy(self._table_array(
+                batch.block_tables = torch.from_numpy(table_array(
                     tables[:num_decode])).to(self.device)
                 batch.context_lens = self._i32(ends[:num_decode])
         elif any_past:
@@ -202,25 +209,19 @@ class ModelRunner:
         ctx = self._i32([seq.num_tokens for seq in seqs])
         tokens = torch.tensor([seq.last_token for seq in seqs],
                               dtype=torch.int64, device=dev)
-        bt_np = self._table_array([seq.block_table for seq in seqs])
+        bt_np = table_array([seq.block_table for seq in seqs])
         state = {"ids": tuple(s.seq_id for s in seqs),
                  "positions": positions, "ctx": ctx, "tokens": tokens,
                  "bt": torch.from_numpy(bt_np).to(dev), "fresh": True,
-                 "state_slots": None}
+                 "state_slots": None, "prev": None}
+        if self.model.needs_prev:
+            state["prev"] = torch.tensor(
+                [seq.token_at(seq.num_tokens - 2) for seq in seqs],
+                dtype=torch.int64, device=dev)
         if self.model.stateful:
             state["state_slots"] = self._i32(
                 [seq.block_table.state_slot for seq in seqs])
         return state
-
-    @staticmethod
-    def _table_array(tables) -> np.ndarray:
-        # numpy staging: batch composition churns every step under
-        # continuous serving, so the rebuild is on the step critical path
-        out = np.zeros((len(tables), max(len(t.pages) for t in tables)),
-                       dtype=np.int32)
-        for i, t in enumerate(tables):
-            out[i, :len(t.pages)] = t.pages
-        return out
 
     def _decode_slots(self, state: dict) -> torch.Tensor:
         ps = self.cfg.page_size
@@ -268,6 +269,7 @@ class ModelRunner:
             mode="decode", positions=inputs["positions"], slot_mapping=slots,
             block_tables=inputs["bt"], context_lens=inputs["ctx"],
             starts=inputs["positions"], state_slots=inputs["state_slots"],
+            prev_tokens=inputs["prev"],
             decode_num_splits=self.model.decode_splits(
                 n, self.cfg.max_seq_len))
 
@@ -283,6 +285,8 @@ class ModelRunner:
         if self.pp.size > 1:
             next_dev = self.pp.broadcast_tokens(next_dev)
             next_tokens = next_dev.tolist()
+        if state["prev"] is not None:
+            state["prev"] = state["tokens"]
         state["tokens"] = next_dev
         for seq, tok in zip(seqs, next_tokens):
             seq.append_token(tok)
@@ -300,6 +304,7 @@ class ModelRunner:
         """Capture one decode step at batch size ``bs`` into a hipGraph."""
         static = {
             "tokens": torch.zeros(bs, dtype=torch.int64, device=self.device),
+            "prev": torch.zeros(bs, dtype=torch.int64, device=self.device),
             "positions": torch.zeros(bs, dtype=torch.int32, device=self.device),
             "slots": torch.zeros(bs, dtype=torch.int32, device=self.device),
             "ctx": torch.ones(bs, dtype=torch.int32, device=self.device),
@@ -337,6 +342,8 @@ class ModelRunner:
         static["ctx"][:n].copy_(state["ctx"])
         if state["state_slots"] is not None:
             static["state_slots"][:n].copy_(state["state_slots"])
+        if state["prev"] is not None:
+            static["prev"][:n].copy_(state["prev"])
         bt = state["bt"]
         if state.get("graph_bt_loaded") != (state["ids"], bs):
             # block tables are stable for this batch: upload once per batch

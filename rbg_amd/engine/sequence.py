@@ -67,6 +67,14 @@ class Sequence:
         return (self.output_tokens[-1] if self.output_tokens
                 else self.prompt_tokens[-1])
 
+    def token_at(self, position: int) -> int:
+        """Prompt or output token; -1 before the first."""
+        if position < 0:
+            return -1
+        n = len(self.prompt_tokens)
+        return (self.prompt_tokens[position] if position < n
+                else self.output_tokens[position - n])
+
     def append_token(self, tok: int) -> None:
         if self.first_token_time is None:
             self.first_token_time = time.monotonic()

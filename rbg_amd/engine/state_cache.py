@@ -1,19 +1,20 @@
-"""Cache of models whose layers keep latents or recurrent state.
+"""Cache of models whose layers keep different things of a sequence.
 
 Two kinds of memory per sequence, both carved at start-up:
 
-* pages of latents: attention layers that cache one low-rank row per token.
-  Page accounting, block tables and slot mapping are PagedKVCache's; the pool
-  is one allocation with a view [pages, page_size, rank] per layer (the ranks
-  may differ between layers).
+* pages: attention layers that cache one low-rank latent per token, or keys and
+  values of a layer's own head counts and sizes.  Page accounting, block tables
+  and slot mapping are PagedKVCache's; the pool is one allocation with views per
+  layer: latents [pages, page_size, rank], keys and values [pages, heads,
+  page_size, size].  A layer that reads another's pages has none of its own.
 * one state slot: fixed-size tensors that a token rewrites in place (the past
   inputs of a short convolution, a recurrence's matrix).  Slot 0 is scratch for
   the padding rows of captured decode batches, like page 0.
 
 A slot is handed out dirty: the kernels take a sequence's state as zero at
-position 0 instead of reading it.  Pages of such a model cannot be shared by
-prompt prefix (the state at the page's end is not kept), so there is no prefix
-cache.
+position 0 instead of reading it.  Pages of a model with state cannot be shared
+by prompt prefix (the state at the page's end is not kept), so it has no prefix
+cache.  A model without state has pages only: no slots limit its sequences.
 """
 from __future__ import annotations
 
@@ -31,9 +32,23 @@ from .kv_cache import OutOfPages, PagedKVCache
 class LayerCacheSpec:
     """What one layer keeps for a sequence."""
     latent_rank: int = 0            # row per token in the paged pool, 0: none
+    # (heads, key size, value size) of keys and values in the paged pool
+    kv: Optional[Tuple[int, int, int]] = None
     # name -> (shape without the slot dim, dtype)
     state: Dict[str, Tuple[Tuple[int, ...], torch.dtype]] = \
         field(default_factory=dict)
+
+    def paged_shapes(self) -> List[Tuple[int, int]]:
+        """(heads, size) of each paged tensor; a latent has one head."""
+        out = [(1, self.latent_rank)] if self.latent_rank else []
+        if self.kv is not None:
+            heads, dim, vdim = self.kv
+            out += [(heads, dim), (heads, vdim)]
+        return out
+
+    def row_elements(self) -> int:
+        """Paged elements per token."""
+        return sum(heads * size for heads, size in self.paged_shapes())
 
 
 class StateCache(PagedKVCache):
@@ -42,13 +57,16 @@ class StateCache(PagedKVCache):
                  num_pages: Optional[int] = None):
         self.specs = specs
         self.dtype = dtype
-        self.num_slots = (cfg.state_slots or cfg.max_batch_size) + 1
+        self.has_state = any(s.state for s in specs)
+        self.num_slots = ((cfg.state_slots or cfg.max_batch_size) + 1
+                          if self.has_state else 1)
         super().__init__(cfg, device, num_pages, num_layers=len(specs))
-        self.prefix = None
+        if self.has_state:
+            self.prefix = None
         self._free_slots: List[int] = list(range(self.num_slots - 1, 0, -1))
 
     def _page_bytes(self) -> int:
-        rows = sum(s.latent_rank for s in self.specs) * self.cfg.page_size
+        rows = sum(s.row_elements() for s in self.specs) * self.cfg.page_size
         return max(1, rows * self.dtype.itemsize)
 
     def _fixed_bytes(self) -> int:
@@ -63,19 +81,19 @@ class StateCache(PagedKVCache):
 
     def _alloc_storage(self, device: torch.device) -> None:
         rows = self.num_pages * self.page_size
-        total = sum(s.latent_rank for s in self.specs) * rows
+        total = sum(s.row_elements() for s in self.specs) * rows
         self.kv = torch.zeros(total, dtype=self.dtype, device=device)
-        self._latents: List[Optional[torch.Tensor]] = []
+        self._pages: List[List[torch.Tensor]] = []  # [pages, heads, rows, size]
         self.states: List[Dict[str, torch.Tensor]] = []
         at = 0
         for spec in self.specs:
-            view = None
-            if spec.latent_rank:
-                n = rows * spec.latent_rank
-                view = self.kv[at:at + n].view(
-                    self.num_pages, self.page_size, spec.latent_rank)
+            views = []
+            for heads, size in spec.paged_shapes():
+                n = rows * heads * size
+                views.append(self.kv[at:at + n].view(
+                    self.num_pages, heads, self.page_size, size))
                 at += n
-            self._latents.append(view)
+            self._pages.append(views)
             self.states.append({
                 name: torch.zeros((self.num_slots,) + tuple(shape),
                                   dtype=dt, device=device)
@@ -84,9 +102,13 @@ class StateCache(PagedKVCache):
     # -- views ------------------------------------------------------------------
 
     def latents(self, layer: int) -> torch.Tensor:
-        view = self._latents[layer]
-        assert view is not None, f"layer {layer} caches no latents"
-        return view
+        assert self.specs[layer].latent_rank, f"layer {layer}: no latents"
+        return self._pages[layer][0].squeeze(1)
+
+    def kv_pages(self, layer: int) -> Tuple[torch.Tensor, torch.Tensor]:
+        """Keys and values, [pages, heads, page_size, size] each."""
+        assert self.specs[layer].kv is not None, f"layer {layer}: no keys"
+        return self._pages[layer][-2], self._pages[layer][-1]
 
     def state(self, layer: int, name: str) -> torch.Tensor:
         return self.states[layer][name]
@@ -98,9 +120,12 @@ class StateCache(PagedKVCache):
         return len(self._free_slots)
 
     def has_room(self, num_pages: int) -> bool:
-        return bool(self._free_slots) and super().has_room(num_pages)
+        return (bool(self._free_slots) or not self.has_state) and \
+            super().has_room(num_pages)
 
     def alloc_slot(self) -> int:
+        if not self.has_state:
+            return 0
         with self._lock:
             if not self._free_slots:
                 raise OutOfPages("no free state slot")
@@ -110,14 +135,13 @@ class StateCache(PagedKVCache):
         with self._lock:
             self._free_slots.append(slot)
 
-    # -- migration: latents of the pages, then the slot's state, as bytes -----------
+    # -- migration: a layer's pages, then the slot's state, as bytes -----------
 
     def export_pages(self, pages: List[int], slot: int = 0) -> torch.Tensor:
         idx = torch.tensor(pages, dtype=torch.int64, device=self.kv.device)
         parts = []
-        for view, states in zip(self._latents, self.states):
-            if view is not None:
-                parts.append(view.index_select(0, idx))
+        for views, states in zip(self._pages, self.states):
+            parts.extend(view.index_select(0, idx) for view in views)
             parts.extend(t[slot] for t in states.values())
         return torch.cat([p.contiguous().view(-1).view(torch.uint8)
                           for p in parts])
@@ -125,7 +149,7 @@ class StateCache(PagedKVCache):
     def _export_bytes(self, num_pages: int) -> int:
         n = 0
         for spec in self.specs:
-            n += (spec.latent_rank * self.page_size * num_pages *
+            n += (spec.row_elements() * self.page_size * num_pages *
                   self.dtype.itemsize)
             n += sum(math.prod(shape) * dt.itemsize
                      for shape, dt in spec.state.values())
@@ -148,8 +172,8 @@ class StateCache(PagedKVCache):
             part = buf[at:at + n].clone().view(dtype).view(shape)
             at += n
             return part
-        for view, states in zip(self._latents, self.states):
-            if view is not None:
+        for views, states in zip(self._pages, self.states):
+            for view in views:
                 view.index_copy_(0, idx, take((len(pages),) + view.shape[1:],
                                               view.dtype))
             for t in states.values():

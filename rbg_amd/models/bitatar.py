@@ -22,13 +22,12 @@ import torch.nn as nn
 
 from .. import ops
 from ..engine.batch import ForwardBatch
-from ..engine.config import EngineConfig, ModelConfig
+from ..engine.config import ModelConfig
 from ..engine.state_cache import StateCache
-from .llama import PPContext, TPContext
+from .llama import TPContext
 from .mixers import GatedGelu, GeneralDelta, LatentAttention, param
-from .weights import WeightSource, open_weights
-
-DTYPES = {"bfloat16": torch.bfloat16, "float32": torch.float32}
+from .stream_model import StreamForCausalLM
+from .weights import WeightSource
 
 
 @dataclass
@@ -163,94 +162,23 @@ class BitatarLayer(nn.Module):
         return self.tp.all_reduce(ops.linear(act, self.w_out))
 
 
-class BitatarForCausalLM(nn.Module):
-    """Same surface as LlamaForCausalLM (engine/model_runner.py drives it)."""
+class BitatarForCausalLM(StreamForCausalLM):
+    def build_layer(self, index: int, src: WeightSource) -> BitatarLayer:
+        return BitatarLayer(self.cfg, self.cfg.layers[index], index,
+                            index - self.layer_start, self.tp, src,
+                            self.dtype)
 
-    stateful = True                     # step batches carry slots and starts
-    mixed_steps = True                  # portions and decoded tokens together
+    def spare_tensors(self):
+        return {f"l{i}.norm2" for i in range(self.cfg.num_layers)}
 
-    def __init__(self, cfg: BitatarConfig, device: torch.device,
-                 tp: Optional[TPContext] = None, base_seed: int = 1234,
-                 pp: Optional[PPContext] = None):
-        super().__init__()
-        self.cfg, self.device = cfg, device
-        self.tp = tp or TPContext()
-        self.pp = pp or PPContext()
-        self.dtype = DTYPES[cfg.dtype]
-        self.stream_dtype = torch.float32
-        src = open_weights(cfg.weights_path, base_seed, device)
-        L = cfg.num_layers
-        assert L % self.pp.size == 0, "PP degree must divide layer count"
-        per = L // self.pp.size
-        self.layer_start = self.pp.stage * per
-        self.layer_end = self.layer_start + per
-        self.embed = self.final_norm = self.lm_head = None
-        w = cfg.hidden_size
-        if self.pp.first:
-            self.embed = param(src.take("embed", (cfg.vocab_size, w),
-                                        "linear"), self.dtype)
-        self.layers = nn.ModuleList([
-            BitatarLayer(cfg, cfg.layers[i], i, i - self.layer_start, self.tp,
-                         src, self.dtype)
-            for i in range(self.layer_start, self.layer_end)])
-        if self.pp.last:
-            self.final_norm = param(src.take("final.norm", (w,), "ones"),
-                                    torch.float32)
-            self.lm_head = param(src.take("head", (cfg.vocab_size, w)),
-                                 self.dtype)
-        if self.pp.size == 1:
-            src.finish(optional={f"l{i}.norm2" for i in range(L)})
+    def embed_rows(self, tokens: torch.Tensor,
+                   batch: ForwardBatch) -> torch.Tensor:
+        return ops.embed_stream(tokens, self.embed, self.cfg.embed_scale)
 
-    @property
-    def num_local_layers(self) -> int:
-        return self.layer_end - self.layer_start
+    def add(self, x: torch.Tensor, pending: torch.Tensor) -> torch.Tensor:
+        return x + pending.float()
 
-    def make_cache(self, cfg: EngineConfig) -> StateCache:
-        return StateCache(cfg, self.device,
-                          [layer.cache_spec() for layer in self.layers],
-                          self.dtype)
-
-    def decode_splits(self, batch_size: int, max_seq_len: int) -> int:
-        return 0                        # per layer, from its window
-
-    @torch.inference_mode()
-    def forward(self, tokens: torch.Tensor, batch: ForwardBatch,
-                cache: StateCache,
-                hidden: Optional[torch.Tensor] = None) -> torch.Tensor:
-        """First PP stage embeds `tokens`, later stages take the stream from
-        the one before; the last returns normed rows ready for logits()."""
-        if self.pp.first:
-            x = ops.embed_stream(tokens, self.embed, self.cfg.embed_scale)
-        else:
-            assert hidden is not None, "non-first PP stage needs hidden"
-            x = hidden
-        delta = None
-        for layer in self.layers:
-            delta = layer(x, delta, batch, cache)
-        if not self.pp.last:
-            return x + delta.float()
-        return ops.stream_norm(x, delta, self.final_norm, None,
+    def final(self, x: torch.Tensor, pending: torch.Tensor) -> torch.Tensor:
+        return ops.stream_norm(x, pending, self.final_norm, None,
                                self.cfg.norm_groups, self.cfg.rms_eps,
                                self.dtype)[0]
-
-    @torch.inference_mode()
-    def logits(self, hidden: torch.Tensor,
-               gather_idx: Optional[torch.Tensor] = None) -> torch.Tensor:
-        if gather_idx is not None:
-            hidden = hidden[gather_idx.long()]
-        return torch.nn.functional.linear(hidden, self.lm_head).float()
-
-    def reload_weights(self, seed: int) -> None:
-        """In-place refresh from the weights' file, or from a new seed when
-        the model is random (the cache and captured graphs keep their
-        addresses)."""
-        fresh = BitatarForCausalLM(self.cfg, self.device, self.tp,
-                                   base_seed=seed, pp=self.pp)
-        with torch.no_grad():
-            for p, q in zip(self.parameters(), fresh.parameters()):
-                p.copy_(q)
-        del fresh
-        if self.device.type == "cuda":
-            torch.cuda.empty_cache()
-        if self.tp.size > 1:
-            torch.distributed.barrier(group=self.tp.group)

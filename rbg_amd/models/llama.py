@@ -278,7 +278,9 @@ class LlamaLayer(nn.Module):
 
 class LlamaForCausalLM(nn.Module):
     stateful = False        # nothing per sequence beyond its KV pages
+    varlen = False          # batches need no VarlenLayout
     mixed_steps = False     # a step is prefill or decode
+    needs_prev = False      # nor each token's predecessor
 
     def __init__(self, cfg: ModelConfig, device: torch.device,
                  tp: Optional[TPContext] = None, base_seed: int = 1234,

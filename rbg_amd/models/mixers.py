@@ -10,11 +10,14 @@ Work split: library GEMMs for the projections, one hand-written kernel each
 for the recurrence (with decay, gates, unit keys and head norm inside) and for
 the attention (with window, softmax and, in prefill, the output gate inside).
 Tensor parallelism shards heads and feed-forward columns.
+
+Parts of a design that norms each branch before adding it (``PagedAttention``,
+``SparseExperts``) apply their own output projection instead.
 """
 from __future__ import annotations
 
 import math
-from typing import Any, Dict, List, Tuple
+from typing import Any, Dict, List, Optional, Tuple
 
 import torch
 import torch.nn as nn
@@ -222,3 +225,116 @@ class GatedGelu(nn.Module):
 
     def forward(self, x: torch.Tensor, out: torch.Tensor) -> None:
         ops.gelu_mul(ops.linear(x, self.gate_up), out)
+
+
+class PagedAttention(nn.Module):
+    """Causal softmax attention over paged keys and values of any sizes:
+    grouped heads, biases, partial rotary positions, scores squashed by a soft
+    cap, a silent key of score zero (a sink), and, with ``kv_from``, another
+    layer's keys and values.
+
+    One GEMM projects queries (and keys and values); one kernel adds the
+    biases, rotates, and writes keys and values to the pages; the attention
+    kernels read pages only, so that a layer's own tokens and another layer's
+    are found in the same place."""
+
+    def __init__(self, spec: Dict[str, Any], width: int, src: WeightSource,
+                 prefix: str, tp, dtype: torch.dtype, sink: bool):
+        super().__init__()
+        heads, kv_heads = int(spec["heads"]), int(spec["kv_heads"])
+        if heads % kv_heads:
+            raise ValueError(f"{heads} heads over {kv_heads} key heads")
+        assert heads % tp.size == 0 and kv_heads % tp.size == 0, \
+            "TP degree must divide head counts"
+        self.heads, self.kv_heads = heads // tp.size, kv_heads // tp.size
+        self.dim, self.vdim = int(spec["dim"]), int(spec["vdim"])
+        self.scale = float(spec["scale"])
+        self.softcap = float(spec.get("softcap") or 0.0)    # 0: none
+        self.sink = sink
+        self.rot = spec["rot"]
+        if int(self.rot["dims"]) > self.dim:
+            raise ValueError("more rotated dimensions than a head has")
+        self.kv_from: Optional[int] = spec.get("kv_from")   # global layer
+        self.cos_sin: Optional[torch.Tensor] = None         # set with the cache
+        outs = {"q": heads * self.dim}
+        if self.kv_from is None:
+            outs.update(k=kv_heads * self.dim, v=kv_heads * self.vdim)
+        parts, biases = [], []
+        for name, n in outs.items():
+            parts.append((name, shard(src.take(prefix + name, (n, width)),
+                                      tp)))
+            bias = shard(src.take(prefix + name + ".b", (n,)), tp)
+            biases += [bias, bias.new_zeros(-bias.numel() % 8)]
+        self.proj = FusedProjection(parts, dtype)
+        self.bias = param(torch.cat(biases), torch.float32)
+        self.w_out = param(shard(src.take(prefix + "o",
+                                          (width, heads * self.vdim)),
+                                 tp, dim=1), dtype)
+
+    def cache_spec(self) -> LayerCacheSpec:
+        if self.kv_from is not None:
+            return LayerCacheSpec()
+        return LayerCacheSpec(kv=(self.kv_heads, self.dim, self.vdim))
+
+    def forward(self, h: torch.Tensor, batch: ForwardBatch, cache: StateCache,
+                kv_layer: int) -> torch.Tensor:
+        y = self.proj(h)
+        k, v = cache.kv_pages(kv_layer)
+        offs = [self.proj.offset(n) for n in self.proj.cols]
+        ops.rope_store_paged(y, self.bias, self.cos_sin, batch.positions,
+                             batch.slot_mapping, self.heads, self.dim, k, v,
+                             offs)
+        q = self.proj.slice(y, "q").unflatten(1, (self.heads, self.dim))
+        out = y.new_empty((y.shape[0], self.heads * self.vdim))
+        score = (self.scale, self.softcap, self.sink)
+        nd = y.shape[0] if batch.mode == "decode" else batch.num_decode
+        if nd:
+            ops.paged_decode(q[:nd], k, v, batch.block_tables,
+                             batch.context_lens, out[:nd], *score)
+        if nd < y.shape[0]:
+            ops.paged_prefill(q[nd:], k, v, batch.layout.paged_view(),
+                              out[nd:], *score)
+        return ops.linear(out, self.w_out)
+
+
+class SparseExperts(nn.Module):
+    """Mixture of small feed-forwards down(relu(up x)^2): sigmoid router
+    scores, a correction that only the choice sees, a choice limited to the
+    best groups of neighbouring experts, unnormalized weights.
+
+    Tensor parallelism shards every expert's inner columns."""
+
+    def __init__(self, spec: Dict[str, Any], width: int, src: WeightSource,
+                 prefix: str, tp, dtype: torch.dtype):
+        super().__init__()
+        if spec.get("kind") != "moe":
+            raise ValueError(f"unknown feed-forward kind {spec.get('kind')!r}")
+        r, ff = spec["router"], int(spec["expert"]["ff"])
+        assert ff % tp.size == 0, "TP degree must divide the feed-forward"
+        n, self.top = int(r["experts"]), int(r["top"])
+        groups = r.get("groups") or {}
+        self.groups = int(groups.get("count", 1))
+        self.keep = int(groups.get("keep", self.groups))
+        if n % self.groups or not 1 <= self.keep <= self.groups or not \
+                1 <= self.top <= self.keep * (n // self.groups):
+            raise ValueError(f"router: {n} experts, {self.groups} groups, "
+                             f"{self.keep} kept, {self.top} chosen")
+
+        def stack(name, shape, dim):
+            return param(torch.stack([
+                shard(src.take(f"{prefix}e{e}.{name}", shape), tp, dim)
+                for e in range(n)]), dtype)
+        self.up = stack("up", (ff, width), 0)
+        self.down = stack("down", (width, ff), 1)
+        self.router = param(src.take(prefix + "router", (n, width)), dtype)
+        self.correction = param(src.take(prefix + "correction", (n,)),
+                                torch.float32)
+
+    def forward(self, x: torch.Tensor):
+        """Outputs of the chosen experts, one row per (token, choice) in
+        expert order, and the routing that weighs and finds them."""
+        logits = ops.router_logits(x, self.router)
+        route = ops.moe_route(logits, self.correction, self.groups, self.keep,
+                              self.top, ops.expert_tile(x, self.up, self.top))
+        h = ops.expert_linear(x, self.up, route, gather=True, relu2=True)
+        return ops.expert_linear(h, self.down, route), route

@@ -6,17 +6,19 @@ import os
 from typing import Callable, Dict
 
 from ..engine.config import ModelConfig
-from . import bitatar, llama
+from . import bitatar, llama, notadra
 
 # architecture -> model class
 MODELS: Dict[str, type] = {
     "llama": llama.LlamaForCausalLM,        # Llama and Qwen3 shapes
     "Bitatar": bitatar.BitatarForCausalLM,
+    "Notadra": notadra.NotadraForCausalLM,
 }
 
 # architecture of a config.json -> its reader
 CONFIG_READERS: Dict[str, Callable[..., ModelConfig]] = {
     "Bitatar": bitatar.BitatarConfig.from_json,
+    "Notadra": notadra.NotadraConfig.from_json,
 }
 
 
@@ -37,7 +39,7 @@ def resolve_model(name: str) -> ModelConfig:
     """A preset's name, or a model folder."""
     if os.path.isdir(name):
         return load_config(name)
-    cfg = bitatar.preset(name)
+    cfg = bitatar.preset(name) or notadra.preset(name)
     return cfg if cfg is not None else ModelConfig.preset(name)
 
 

@@ -98,6 +98,8 @@ class RandomSource(WeightSource):
         t = torch.empty(shape, device=self.device, dtype=self.dtype)
         if init == "ones":
             return t.fill_(1.0)
+        if init == "zeros":
+            return t.zero_()
         scale = 1.0
         if init == "linear":
             scale = 1.0 / math.sqrt(shape[-1])

@@ -8,6 +8,9 @@ as the implementation.
 """
 from __future__ import annotations
 
+from dataclasses import dataclass
+from typing import Optional
+
 import torch
 
 from . import reference
@@ -30,12 +33,22 @@ except Exception as e:  # noqa: BLE001
 
 HAVE_MIX = _mix is not None
 
+_moe = None
+_moe_err: Exception | None = None
+try:
+    from . import _hip_moe as _moe   # type: ignore[attr-defined]
+except Exception as e:  # noqa: BLE001
+    _moe_err = e
+
+HAVE_MOE = _moe is not None
+
 
 def _check_stale() -> None:
     """Fail loudly on a GPU box if a shipped .so predates its kernel sources
     (stale-binary guard; the stamps are written by utils/hip_build.py)."""
     from ..utils import hip_build
-    for name, mod in (("_hip_ops", _hip), ("_hip_mix", _mix)):
+    for name, mod in (("_hip_ops", _hip), ("_hip_mix", _mix),
+                      ("_hip_moe", _moe)):
         if mod is not None and hip_build.is_stale(name):
             raise RuntimeError(
                 f"rbg_amd HIP extension {name} is STALE: kernel sources "
@@ -44,7 +57,7 @@ def _check_stale() -> None:
                 "--inplace")
 
 
-if (HAVE_HIP or HAVE_MIX) and torch.cuda.is_available():
+if (HAVE_HIP or HAVE_MIX or HAVE_MOE) and torch.cuda.is_available():
     _check_stale()
 
 
@@ -64,6 +77,15 @@ def _require_mix():
             "passed.  Build it in-tree: PYTORCH_ROCM_ARCH=gfx950 python "
             f"setup.py build_ext --inplace (import error: {_mix_err!r})")
     return _mix
+
+
+def _require_moe():
+    if _moe is None:
+        raise RuntimeError(
+            "rbg_amd HIP extension _hip_moe is not built but a GPU tensor was "
+            "passed.  Build it in-tree: PYTORCH_ROCM_ARCH=gfx950 python "
+            f"setup.py build_ext --inplace (import error: {_moe_err!r})")
+    return _moe
 
 
 def _on_gpu(t: torch.Tensor) -> bool:
@@ -87,8 +109,8 @@ def linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
             w.shape[0] % 32 == 0 and x.shape[1] % 512 == 0 and
             (w.shape[0] <= 4608 or
              (x.shape[0] <= 64 and w.shape[0] <= 8192))):
-        # linked into both extensions: a process has the one its model needs
-        return (_hip or _require_mix()).skinny_gemm(
+        # linked into every extension: a process has the one its model needs
+        return (_hip or _mix or _require_moe()).skinny_gemm(
             x if x.is_contiguous() else x.contiguous(), w)
     return torch.nn.functional.linear(x, w)
 
@@ -343,3 +365,147 @@ def head_linear(x, w, gate=None, out=None) -> torch.Tensor:
     else:
         reference.head_linear(x, w, gate, out)
     return out
+
+
+# -- sandwich norms, paged attention, sparse experts ---------------------------
+
+
+@dataclass
+class Routing:
+    """Which experts a step's tokens go to: T * top (token, choice) pairs,
+    stored in expert order and cut into tiles of one expert each."""
+    top: int
+    tile: int                   # most rows of a tile
+    weights: torch.Tensor       # [T, top] f32
+    inv: torch.Tensor           # [T * top] int32: a pair's row
+    rows: torch.Tensor          # [T * top] int32: a row's token
+    tiles: torch.Tensor         # [n, 3] int32: expert, first row, rows
+    count: Optional[torch.Tensor] = None    # GPU: how many tiles are used
+
+
+def embed_pairs(tokens, prev, table, pairs, mul_prev: int,
+                mul_cur: int) -> torch.Tensor:
+    """f32 stream: table[token] + pairs[(prev * mul_prev + token * mul_cur) mod
+    buckets], the last row of ``pairs`` where prev is -1."""
+    if _on_gpu(table):
+        return _require_moe().embed_pairs(tokens, prev, table, pairs, mul_prev,
+                                          mul_cur)
+    return reference.embed_pairs(tokens, prev, table, pairs, mul_prev, mul_cur)
+
+
+def sandwich_norm(x, pending, w, eps: float, dtype):
+    """x += RMS norm of what is pending under its weight (in place, f32; None:
+    nothing); returns the RMS norm of x under w in ``dtype`` (None without w).
+    ``pending`` = (rows, routing or None, weight); rows with a routing are
+    weighed and summed first."""
+    rows = route = wb = None
+    if pending is not None:
+        rows, route, wb = pending
+    if _on_gpu(x):
+        return _require_moe().sandwich_norm(
+            x, rows, route.inv if route else None,
+            route.weights if route else None, wb, w, eps,
+            dtype == torch.float32)
+    return reference.sandwich_norm(x, rows, route, wb, w, eps, dtype)
+
+
+def moe_combine(y, route) -> torch.Tensor:
+    """Weighed sums of each token's expert rows, in y's dtype."""
+    if _on_gpu(y):
+        return _require_moe().moe_combine(y, route.inv, route.weights)
+    return reference.moe_combine(y, route).to(y.dtype)
+
+
+def rope_store_paged(proj, bias, cos_sin, positions, slots, heads: int,
+                     dim: int, k, v, offs) -> None:
+    """Adds the biases of a fused projection, rotates the leading dimensions of
+    its queries (in place) and keys by cos_sin [positions, dims] = [cos | sin],
+    and writes keys and values to the pages [pages, kv heads, page_size, size].
+    ``offs`` are the columns of q, k, v; of q alone when the keys are another
+    layer's."""
+    if _on_gpu(proj):
+        _require_moe().rope_store_paged(proj, bias, cos_sin, positions, slots,
+                                        heads, dim, k, v, offs)
+        return
+    reference.rope_store_paged(proj, bias, cos_sin, positions, slots, heads,
+                               dim, k, v, offs)
+
+
+def paged_prefill(q, k, v, view, out, scale: float, softcap: float,
+                  sink: bool) -> None:
+    """Causal attention of portions [R, H, D] over the pages; ``view`` is the
+    step's engine/batch.py PagedView.  Scores are scale * q.k, then softcap *
+    tanh(score / softcap) (0: as they are); ``sink`` adds a key of score 0 and
+    no value."""
+    if _on_gpu(q):
+        _require_moe().paged_prefill(q, k, v, view.tables, view.seq_info,
+                                     view.row_info, view.blocks, out, scale,
+                                     softcap, sink)
+        return
+    reference.paged_rows(q, k, v, view.tables, view.row_info, out, scale,
+                         softcap, sink)
+
+
+def pick_paged_splits(num_seqs: int, kv_heads: int, max_keys: int) -> int:
+    """Key splits of paged_decode: two workgroups per CU, at least one
+    128-key step each.  Depends on sizes only, so that a captured decode step
+    keeps its value."""
+    base = max(1, num_seqs * kv_heads)
+    steps = (max_keys + 127) // 128
+    return int(max(1, min((512 + base - 1) // base, steps, 64)))
+
+
+def paged_decode(q, k, v, tables, context_lens, out, scale: float,
+                 softcap: float, sink: bool, splits: int = 0) -> None:
+    """One query row per sequence, [S, H, D]; scores as in paged_prefill."""
+    if _on_gpu(q):
+        if splits <= 0:
+            splits = pick_paged_splits(q.shape[0], k.shape[1],
+                                       tables.shape[1] * k.shape[2])
+        _require_moe().paged_decode(q, k, v, tables, context_lens, out, scale,
+                                    softcap, sink, splits)
+        return
+    info = torch.stack([torch.arange(q.shape[0], dtype=torch.int32),
+                        context_lens - 1], dim=1)
+    reference.paged_rows(q, k, v, tables, info, out, scale, softcap, sink)
+
+
+def router_logits(x, w) -> torch.Tensor:
+    """x W^T in 32-bit, [T, experts] f32."""
+    if _on_gpu(x):
+        return _require_moe().router_logits(x, w)
+    return x.float() @ w.float().T
+
+
+def expert_tile(x, w, top: int) -> int:
+    """Rows per tile that suit x [T, K] through experts w [E, N, K]."""
+    rows = x.shape[0] * top / w.shape[0]        # per expert, on average
+    if (not _on_gpu(x) or x.dtype == torch.float32 or w.shape[1] % 8 or
+            w.shape[2] % 8 or rows <= 16):
+        return 16
+    return 32 if rows <= 32 else 128
+
+
+def moe_route(logits, correction, groups: int, keep: int, top: int,
+              tile: int) -> Routing:
+    """Chooses the ``top`` experts of each token by sigmoid(logit) + correction
+    among the ``keep`` groups with the largest sums of their two best, and lays
+    the pairs out by expert.  Weights are the sigmoids."""
+    if _on_gpu(logits):
+        weights, inv, rows, tiles, count = _require_moe().moe_route(
+            logits, correction, groups, keep, top, tile)
+        return Routing(top, tile, weights, inv, rows, tiles, count)
+    ids, weights = reference.moe_choose(logits, correction, groups, keep, top)
+    return Routing(top, tile, weights,
+                   *reference.moe_tiles(ids, logits.shape[1], tile))
+
+
+def expert_linear(x, w, route, gather: bool = False,
+                  relu2: bool = False) -> torch.Tensor:
+    """Rows in expert order times their expert's w [E, N, K]; ``gather`` takes
+    x's rows by token, ``relu2`` applies max(0, .)^2."""
+    if _on_gpu(x):
+        return _require_moe().expert_linear(
+            x, w, route.rows if gather else None, route.tiles, route.count,
+            route.rows.numel(), route.tile, relu2)
+    return reference.expert_linear(x, w, route, gather, relu2)

@@ -1,10 +1,6 @@
 // PyTorch bindings for the f32-stream and token-mixer kernels (bf16 or f32
 // activations).  Shapes, strides and dtypes are checked here, before launch.
-#include <torch/extension.h>
-#include <ATen/hip/HIPContext.h>
-
-#include <hip/hip_runtime.h>
-
+#include "bind_util.h"
 #include "gemm_bindings.h"
 #include "mix_args.h"
 
@@ -34,42 +30,6 @@ void launch_delta_chunk(const DeltaArgs*, const int*, const int*, float*,
 }
 
 namespace {
-
-using torch::Tensor;
-using OptTensor = c10::optional<torch::Tensor>;
-
-hipStream_t current_stream() {
-  return at::hip::getCurrentHIPStream().stream();
-}
-
-bool is_f32(const Tensor& t) { return t.scalar_type() == torch::kFloat32; }
-
-// activation: bf16 or f32 on the GPU, 2-D rows with a contiguous inner dim
-void check_rows(const Tensor& t, const char* name) {
-  TORCH_CHECK(t.is_cuda(), name, " must be on GPU");
-  TORCH_CHECK(t.scalar_type() == torch::kBFloat16 || is_f32(t), name,
-              " must be bf16 or f32");
-  TORCH_CHECK(t.dim() == 2 && (t.stride(1) == 1 || t.size(1) == 1), name,
-              " must be 2-D with contiguous rows");
-}
-
-void check_f32(const Tensor& t, const char* name, int64_t numel) {
-  TORCH_CHECK(t.is_cuda() && is_f32(t) && t.is_contiguous(), name,
-              " must be contiguous f32 on GPU");
-  TORCH_CHECK(t.numel() == numel, name, " has ", t.numel(), " elements, not ",
-              numel);
-}
-
-const int* i32(const Tensor& t, const char* name, int64_t at_least) {
-  TORCH_CHECK(t.is_cuda() && t.scalar_type() == torch::kInt32 &&
-              t.is_contiguous(), name, " must be contiguous int32 on GPU");
-  TORCH_CHECK(t.numel() >= at_least, name, " is too short");
-  return t.data_ptr<int>();
-}
-
-void same_dtype(const Tensor& a, const Tensor& b, const char* name) {
-  TORCH_CHECK(a.scalar_type() == b.scalar_type(), name, ": dtype mismatch");
-}
 
 Tensor embed_stream(Tensor tokens, Tensor table, double scale) {
   check_rows(table, "table");
@@ -289,22 +249,6 @@ Tensor latent_store(Tensor x, Tensor w, Tensor cache, Tensor slots,
                         i32(slots, "slots", T), (int)T, (int)R, (float)eps,
                         is_f32(x), current_stream());
   return c;
-}
-
-void check_heads(const Tensor& t, const char* name) {
-  TORCH_CHECK(t.is_cuda() && t.dim() == 3 &&
-              (t.stride(2) == 1 || t.size(2) == 1), name,
-              " must be 3-D with a contiguous inner dim");
-}
-
-bool mult8(std::initializer_list<int64_t> xs) {
-  for (auto x : xs)
-    if (x % 8) return false;
-  return true;
-}
-
-bool aligned(const Tensor& t, int bytes) {
-  return ((uintptr_t)t.data_ptr() % bytes) == 0;
 }
 
 // q [rows, H, D], k [keys, H, D], v [keys, H, Dv] (any row/head strides);

@@ -1,0 +1,58 @@
+// Argument blocks shared by the paged-attention and expert kernels and their
+// bindings.
+#pragma once
+
+struct PagedAttnArgs {
+  const void* q;          // + row*q_row + head*q_head
+  const void* k;          // [pages, kv_heads, page_size, d]
+  const void* v;          // [pages, kv_heads, page_size, dv]
+  void* out;              // + row*o_row + head*dv
+  const int* tables;      // [seqs, max_pages]
+  const int* ctx;         // decode: [seqs] tokens visible incl. this one
+  const int* seq_info;    // prompts: [seqs, 3] = first row, rows, position of
+                          //   the first
+  const int* row_info;    // prompts: [rows, 2] = sequence, position
+  const int* blocks;      // prompts: [n_blocks, 2] = sequence, first query
+  float* part_o;          // decode: [splits, seqs, heads, dv]  (splits > 1)
+  float* part_ml;         //         [splits, seqs, heads, 2]
+  long q_row, q_head, o_row;
+  int rows, heads, kv_heads, d, dv, page_size, max_pages, n_blocks, splits;
+  int page_shift;         // log2(page_size); prompt and decode forms only
+  float scale, softcap;   // softcap 0: none
+  int sink;               // one key of score 0 without a value
+};
+
+struct RopePagedArgs {
+  void* proj;             // [rows, stride]
+  const float* bias;      // [width]
+  const float* cos_sin;   // [positions, rot] = [cos | sin]
+  const int* positions;   // [rows]
+  const int* slots;       // [rows]
+  void* k;                // [pages, kv_heads, page_size, d], or null
+  void* v;                // [pages, kv_heads, page_size, dv]
+  long stride;
+  int off_q, off_k, off_v;
+  int rows, heads, kv_heads, d, dv, rot, page_size, table_rows;
+};
+
+struct MoeRouteArgs {
+  const float* logits;    // [tokens, experts]
+  const float* correction;
+  float* weights;         // [tokens, top]
+  int* ids;               // [tokens, top]
+  int* inv;               // [tokens * top] pair -> row
+  int* rows;              // [tokens * top] row -> token
+  int* tiles;             // [.., 3] = expert, first row, rows
+  int* count;             // [1] tiles used
+  int tokens, experts, groups, keep, top, tile;
+};
+
+struct MoeGemmArgs {
+  const void* x;          // [.., k] rows
+  const void* w;          // [experts, n, k]
+  void* out;              // [pairs, n]
+  const int* rows;        // gather: row -> row of x; null: the same
+  const int* tiles;
+  const int* count;
+  int max_tiles, tile, n, k, relu2;
+};

@@ -272,3 +272,110 @@ def head_linear(x, w, gate, out):
     if gate is not None:
         y = y * torch.sigmoid(gate.float())
     out.copy_(y.to(out.dtype))
+
+
+# -- sandwich norms, paged attention, sparse experts ---------------------------
+
+
+def embed_pairs(tokens, prev, table, pairs, mul_prev, mul_cur):
+    buckets = pairs.shape[0] - 1
+    row = (prev * mul_prev + tokens * mul_cur) % buckets
+    row = torch.where(prev < 0, torch.full_like(row, buckets), row)
+    return table[tokens].float() + pairs[row].float()
+
+
+def _rms(x, w, eps):
+    return x / torch.sqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w
+
+
+def moe_combine(y, route):
+    """f32 sums of each token's weighed expert rows."""
+    rows = y.float()[route.inv.long()].view(-1, route.top, y.shape[1])
+    return (rows * route.weights.unsqueeze(-1)).sum(1)
+
+
+def sandwich_norm(x, rows, route, wb, w, eps, dtype):
+    if rows is not None:
+        y = rows.float() if route is None else moe_combine(rows, route)
+        x += _rms(y, wb, eps)
+    return None if w is None else _rms(x, w, eps).to(dtype)
+
+
+def rope_store_paged(proj, bias, cos_sin, positions, slots, heads, dim, k, v,
+                     offs):
+    y = proj.float() + bias
+    half = cos_sin.shape[1] // 2
+    cs = cos_sin[positions.long()].unsqueeze(1)
+    cos, sin = cs[..., :half], cs[..., half:]
+
+    def turn(at, n):
+        t = y[:, at:at + n * dim].view(-1, n, dim)
+        a, b = t[..., :half], t[..., half:2 * half]
+        return torch.cat([a * cos - b * sin, b * cos + a * sin,
+                          t[..., 2 * half:]], dim=-1)
+    proj[:, offs[0]:offs[0] + heads * dim] = \
+        turn(offs[0], heads).flatten(1).to(proj.dtype)
+    if len(offs) == 1:
+        return
+    ps, kvh, vdim = k.shape[2], k.shape[1], v.shape[3]
+    pages, at = slots.long() // ps, slots.long() % ps
+    k[pages, :, at] = turn(offs[1], kvh).to(k.dtype)
+    v[pages, :, at] = y[:, offs[2]:offs[2] + kvh * vdim].view(
+        -1, kvh, vdim).to(v.dtype)
+
+
+def paged_rows(q, k, v, tables, row_info, out, scale, softcap, sink):
+    """Each row of q [R, H, D] against the keys of its sequence up to its
+    position; row_info [R, 2] = (row of tables, position)."""
+    ps, kvh = k.shape[2], k.shape[1]
+    per = q.shape[1] // kvh
+    for r, (seq, pos) in enumerate(row_info.tolist()):
+        j = torch.arange(pos + 1)
+        pages, at = tables[seq].long()[j // ps], j % ps
+        ks = k[pages, :, at].float()                # [keys, kvh, D]
+        qs = q[r].float().view(kvh, per, -1)
+        s = torch.einsum("gpd,kgd->gpk", qs, ks) * scale
+        if softcap > 0:
+            s = softcap * torch.tanh(s / softcap)
+        if sink:                                    # a key without a value
+            s = torch.cat([s, torch.zeros_like(s[..., :1])], dim=-1)
+        p = torch.softmax(s, dim=-1)[..., :pos + 1]
+        o = torch.einsum("gpk,kgd->gpd", p, v[pages, :, at].float())
+        out[r] = o.reshape(-1).to(out.dtype)
+
+
+def moe_choose(logits, correction, groups, keep, top):
+    """(experts, weights) of each token, [T, top]."""
+    T, E = logits.shape
+    s = torch.sigmoid(logits)
+    choice = (s + correction).view(T, groups, E // groups)
+    best = choice.topk(min(2, E // groups), dim=-1).values.sum(-1)
+    kept = torch.zeros(T, groups, dtype=torch.bool)
+    kept.scatter_(1, best.topk(keep, dim=-1).indices, True)
+    choice = choice.masked_fill(~kept.unsqueeze(-1), float("-inf"))
+    ids = choice.view(T, E).topk(top, dim=-1).indices
+    return ids, s.gather(1, ids)
+
+
+def moe_tiles(ids, experts, tile):
+    """Pairs in expert order: (inverse permutation, their tokens, tiles [n, 3]
+    = (expert, first row, rows))."""
+    flat = ids.reshape(-1)
+    order = torch.sort(flat, stable=True).indices
+    inv = torch.empty_like(order)
+    inv[order] = torch.arange(order.numel())
+    tiles, at = [], 0
+    for e, n in enumerate(torch.bincount(flat, minlength=experts).tolist()):
+        tiles += [(e, at + i, min(tile, n - i)) for i in range(0, n, tile)]
+        at += n
+    return (inv.int(), (order // ids.shape[1]).int(),
+            torch.tensor(tiles, dtype=torch.int32).view(-1, 3))
+
+
+def expert_linear(x, w, route, gather, relu2):
+    out = x.new_empty((route.rows.numel(), w.shape[1]))
+    for e, at, n in route.tiles.tolist():
+        rows = x[route.rows[at:at + n].long()] if gather else x[at:at + n]
+        y = rows.float() @ w[e].float().T
+        out[at:at + n] = (torch.relu(y).pow(2) if relu2 else y).to(x.dtype)
+    return out

@@ -51,16 +51,28 @@ HIP_SOURCES = {
         "skinny_gemm.hip",
         "mix_bindings.cpp",
     ],
+    # sandwich norms, paged attention of any sizes, sparse experts
+    "_hip_moe": [
+        "sandwich_norm.hip",
+        "rope_paged.hip",
+        "paged_attn.hip",
+        "moe_route.hip",
+        "moe_gemm.hip",
+        "skinny_gemm.hip",
+        "moe_bindings.cpp",
+    ],
 }
 
 HIP_HEADERS = {
     "_hip_ops": ["common.h", "gemm_bindings.h"],
-    "_hip_mix": ["common.h", "gemm_bindings.h", "mfma_util.h", "mix_args.h",
-                 "vec_io.h"],
+    "_hip_mix": ["bind_util.h", "common.h", "gemm_bindings.h", "mfma_util.h",
+                 "mix_args.h", "vec_io.h"],
+    "_hip_moe": ["bind_util.h", "common.h", "gemm_bindings.h", "mfma_util.h",
+                 "moe_args.h", "vec_io.h"],
 }
 
 # model architecture -> the extension with its kernels (default: _hip_ops)
-EXTENSION_OF = {"Bitatar": "_hip_mix"}
+EXTENSION_OF = {"Bitatar": "_hip_mix", "Notadra": "_hip_moe"}
 
 
 def source_hash(name: str) -> str:
