@@ -51,7 +51,7 @@ def parse_args():
                         "tp/pp: all ranks form one sharded engine")
     p.add_argument("--eager", action="store_true",
                    help="disable hipGraph capture")
-    p.add_argument("--compare", choices=["bitatar"], default=None,
+    p.add_argument("--compare", choices=["bitatar", "notadra"], default=None,
                    help="instead: prefill/decode throughput of this family "
                         "beside Llama at equal size, one GPU, one JSON line "
                         "per workload (--sizes, --batches, --seq-len)")
@@ -110,14 +110,15 @@ def main() -> int:
         from rbg_amd.engine.model_bench import run_compare, run_kernels
         if args.kernels:
             for size in args.sizes.split(","):
-                for row in run_kernels(size):
+                for row in run_kernels(size, family=args.compare):
                     print(json.dumps(dict(row, size=size)), flush=True)
             return 0
         for row in run_compare(device, args.steps, args.warmup,
                                sizes=args.sizes.split(","),
                                batches=[int(b) for b in
                                         args.batches.split(",")],
-                               prompt=args.seq_len, eager=args.eager):
+                               prompt=args.seq_len, eager=args.eager,
+                               family=args.compare):
             print(json.dumps(row), flush=True)
         return 0
 

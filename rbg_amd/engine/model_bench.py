@@ -2,7 +2,7 @@
 
 Random weights, a few layers of a real model's widths, one GPU, bf16.  Each
 workload runs through the engine (scheduler, cache, captured decode steps), so
-the numbers are those of serving.  ``bench.py --compare bitatar`` prints them.
+the numbers are those of serving.  ``bench.py --compare <family>`` prints them.
 """
 from __future__ import annotations
 
@@ -26,7 +26,11 @@ SIZES = {
 }
 
 
-def pair(size: str) -> List[ModelConfig]:
+def pair(size: str, family: str = "bitatar") -> List[ModelConfig]:
+    """The family's model and the Llama of equal size."""
+    if family == "notadra":
+        from .notadra_bench import notadra_pair
+        return notadra_pair(size)
     w, ff, heads, kvh, layers, rank, window, dh, dd = SIZES[size]
     return [
         BitatarConfig.stacked(
@@ -84,10 +88,11 @@ def run_one(model: ModelConfig, device: str, batch: int, prompt: int,
 def run_compare(device: str, steps: int, warmup: int,
                 sizes: Optional[List[str]] = None,
                 batches=(1, 32), prompt: int = 2048,
-                eager: bool = False) -> List[Dict[str, Any]]:
+                eager: bool = False,
+                family: str = "bitatar") -> List[Dict[str, Any]]:
     return [run_one(model, device, b, prompt, steps, warmup, eager)
             for size in (sizes or SIZES) for b in batches
-            for model in pair(size)]
+            for model in pair(size, family)]
 
 
 # -- kernels against their rooflines -------------------------------------------
@@ -125,11 +130,15 @@ def _row(name: str, us: float, nbytes: float = 0.0, bf16: float = 0.0,
 
 
 def run_kernels(size: str, batches=(1, 8, 32, 128), ctx: int = 2048,
-                prompts: int = 4) -> List[Dict[str, Any]]:
+                prompts: int = 4,
+                family: str = "bitatar") -> List[Dict[str, Any]]:
     """The mixers' kernels and the like kernels of Llama, one layer's shapes
     of ``size``; decode inputs rotate through buffers larger than the caches.
     Rooflines: bytes that must move, or the operations the algorithm has to
     do (causal halves counted once, the 32-bit recurrence at the f32 rate)."""
+    if family == "notadra":
+        from .notadra_bench import notadra_kernels
+        return notadra_kernels(size, batches, ctx, prompts)
     import math
 
     from .. import ops
