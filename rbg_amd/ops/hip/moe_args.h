@@ -44,6 +44,7 @@ struct MoeRouteArgs {
   int* rows;              // [tokens * top] row -> token
   int* tiles;             // [.., 3] = expert, first row, rows
   int* count;             // [1] tiles used
+  int* part;              // [blocks, experts] of moe_route_blocks
   int tokens, experts, groups, keep, top, tile;
 };
 

@@ -23,6 +23,7 @@ void launch_paged_rows(const PagedAttnArgs*, int, hipStream_t);
 void launch_router_logits(float*, const void*, const void*, int, int, int, int,
                           int, hipStream_t);
 int moe_max_experts();
+int moe_route_blocks(int, int);
 void launch_moe_route(const MoeRouteArgs*, hipStream_t);
 void launch_moe_gemm(const MoeGemmArgs*, int, int, hipStream_t);
 }
@@ -292,6 +293,12 @@ std::vector<Tensor> moe_route(Tensor logits, Tensor correction, int64_t groups,
   p.ids = ids.data_ptr<int>(); p.inv = inv.data_ptr<int>();
   p.rows = rows.data_ptr<int>(); p.tiles = tiles.data_ptr<int>();
   p.count = count.data_ptr<int>();
+  const int blocks = moe_route_blocks((int)T, (int)E);
+  Tensor part;
+  if (blocks) {
+    part = torch::empty({blocks, E}, i);
+    p.part = part.data_ptr<int>();
+  }
   p.tokens = (int)T; p.experts = (int)E; p.groups = (int)groups;
   p.keep = (int)keep; p.top = (int)top; p.tile = (int)tile;
   if (T) launch_moe_route(&p, current_stream());
@@ -321,6 +328,8 @@ Tensor expert_linear(Tensor x, Tensor w, OptTensor rows, Tensor tiles,
                    aligned(w, 16);
   TORCH_CHECK(tile <= (vec ? 128 : 16), "tile too large for these sizes");
   TORCH_CHECK(p.max_tiles <= 65535, "too many tiles");
+  // the tiled form counts bytes of x and of one expert's weights in 32 bits
+  TORCH_CHECK(x.numel() < (1ll << 31) && N * K < (1ll << 31), "x or w too large");
   if (pairs) launch_moe_gemm(&p, is_f32(x), vec, current_stream());
   return out;
 }

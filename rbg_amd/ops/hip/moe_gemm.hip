@@ -3,10 +3,12 @@
 // a tile of rows per expert (moe_route.hip).  The number of tiles is on the
 // device; launches cover the most there can be and the rest leaves at once.
 //
-//   tiled   128 rows x 128 columns, 64 k a step, both operands straight from
-//           global memory into double-buffered LDS (rows may be gathered: every
-//           lane brings its own address).  16-byte pieces of a row are stored
-//           swizzled by the row, which keeps fragment reads free of conflicts.
+//   tiled   128 rows x 128 or 192 columns, 64 k a step, both operands straight
+//           from global memory into LDS (rows may be gathered: every lane brings
+//           its own address).  One buffer: the other workgroups of the CU, three
+//           or four of them, compute while one waits, which measured better than
+//           two buffers with half the workgroups.  16-byte pieces of a row are
+//           stored swizzled by the row: fragment reads are free of conflicts.
 //   skinny  decode: 16 * MT rows against 16 * NN weight rows, whose fragments go
 //           from global memory into the MFMAs; waves split K and meet in LDS.
 //   rows    any sizes, bf16 or f32: a thread per column, up to 16 rows at once.
@@ -30,19 +32,29 @@ DEV_INLINE void put4(const MoeGemmArgs& p, const size_t row, const int n,
   *reinterpret_cast<uint2*>((__hip_bfloat16*)p.out + row * p.n + n) = o.u;
 }
 
-constexpr int BM = 128, BN = 128, BK = 64, GT = 256;
-constexpr int STAGE = (BM + BN) * BK;           // elements of one buffer
+constexpr int BM = 128, BK = 64, GT = 256;
 
-DEV_INLINE void load_lds16(const __hip_bfloat16* g, __hip_bfloat16* l) {
-  typedef __attribute__((address_space(1))) const void gvoid;
-  typedef __attribute__((address_space(3))) void lvoid;
-  __builtin_amdgcn_global_load_lds((gvoid*)(uintptr_t)g,
-                                   (lvoid*)(uint32_t)(uintptr_t)l, 16, 0, 0);
+// 16 bytes per lane from base + off to 16 * lane past the wave's LDS address.
+// Not the compiler's builtin: it would wait for the data before any LDS read.
+DEV_INLINE void load_lds16(const uint32_t off, const void* base,
+                           const uint32_t lds) {
+  asm volatile("s_mov_b32 m0, %2\n\ts_nop 0\n\t"
+               "global_load_lds_dwordx4 %0, %1"
+               :: "v"(off), "s"(base), "s"(lds) : "memory", "m0");
 }
 
-__global__ __launch_bounds__(GT, 2) void moe_tiled_kernel(const MoeGemmArgs p) {
-  extern __shared__ __attribute__((aligned(16))) char gemm_smem[];
-  __hip_bfloat16* lds = (__hip_bfloat16*)gemm_smem;
+// what this wave asked for is in LDS, and every wave is here
+DEV_INLINE void landed_barrier() {
+  asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
+}
+
+// 4 waves of 64 rows x BN / 2 columns
+template <int BN, int OCC>
+__global__ __launch_bounds__(GT, OCC)
+void moe_tiled_kernel(const MoeGemmArgs p) {
+  constexpr int TN = BN / 32, XI = BM / 32, WI = BN / 32;
+  __shared__ __attribute__((aligned(16)))
+  __hip_bfloat16 lds[(BM + BN) * BK];
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int gl = lane & 15, gs = lane >> 4;
@@ -60,82 +72,98 @@ __global__ __launch_bounds__(GT, 2) void moe_tiled_kernel(const MoeGemmArgs p) {
   const int expert = tile[0], row0 = tile[1], rows = tile[2];
 
   // wave-instruction c brings rows c*32 + wave*8 .. +7, 8 pieces of 16 bytes
-  // each; lane's row is fixed modulo 8, so its piece number is too
+  // each; a lane's row is fixed modulo 8, so its piece number is too
   const int lr = lane >> 3, piece = (lane & 7) ^ lr;
-  const __hip_bfloat16* xp[4];
-  const __hip_bfloat16* wp[4];
+  uint32_t xo[XI], wo[WI];                      // bytes; the host checks sizes
 #pragma unroll
-  for (int c = 0; c < 4; ++c) {
-    const int r = c * 32 + wave * 8 + lr;
-    const int xr = row0 + min(r, rows - 1);
-    xp[c] = (const __hip_bfloat16*)p.x +
-            (size_t)(p.rows != nullptr ? p.rows[xr] : xr) * p.k;
-    wp[c] = (const __hip_bfloat16*)p.w +
-            ((size_t)expert * p.n + min(n0 + r, p.n - 1)) * p.k;
+  for (int c = 0; c < XI; ++c) {
+    const int at = row0 + min(c * 32 + wave * 8 + lr, rows - 1);
+    xo[c] = ((uint32_t)(p.rows != nullptr ? p.rows[at] : at) * p.k +
+             piece * 8) * 2;
   }
-  auto issue = [&](int kt, int buf) {
-    // columns past the end repeat the last ones; compute() masks them
-    const int col = min(kt * BK + piece * 8, p.k - 8);
-    __hip_bfloat16* to = lds + buf * STAGE + wave * 8 * BK;
 #pragma unroll
-    for (int c = 0; c < 4; ++c) {
-      load_lds16(xp[c] + col, to + c * 32 * BK);
-      load_lds16(wp[c] + col, to + BM * BK + c * 32 * BK);
-    }
+  for (int c = 0; c < WI; ++c)
+    wo[c] = ((uint32_t)min(n0 + c * 32 + wave * 8 + lr, p.n - 1) * p.k +
+             piece * 8) * 2;
+  const char* xb = (const char*)p.x;
+  const char* wb = (const char*)p.w + (size_t)expert * p.n * p.k * 2;
+  const uint32_t to = __builtin_amdgcn_readfirstlane(
+      (uint32_t)(uintptr_t)lds + wave * 1024);
+  auto issue = [&](int kt) {
+#pragma unroll
+    for (int c = 0; c < XI; ++c)
+      load_lds16(xo[c], xb + kt * BK * 2, to + c * 4096);
+#pragma unroll
+    for (int c = 0; c < WI; ++c)
+      load_lds16(wo[c], wb + kt * BK * 2, to + BM * BK * 2 + c * 4096);
   };
-  const int wm = (wave >> 1) * 64, wn = (wave & 1) * 64;
-  f32x4 acc[4][4];
+  const int wm = (wave >> 1) * 64, wn = (wave & 1) * (BN / 2);
+  f32x4 acc[TN][4];
 #pragma unroll
-  for (int i = 0; i < 4; ++i)
+  for (int i = 0; i < TN; ++i)
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[i][j] = {0.f, 0.f, 0.f, 0.f};
-  auto compute = [&](int buf, int k_left) {
-    const __hip_bfloat16* xs = lds + buf * STAGE;
-    const __hip_bfloat16* ws = xs + BM * BK;
+  const __hip_bfloat16* xs = lds + (wm + gl) * BK;
+  const __hip_bfloat16* ws = lds + (BM + wn + gl) * BK;
+  auto compute = [&](int k_left) {
     const mf_bf8 z = {};
 #pragma unroll
     for (int h = 0; h < 2; ++h) {
       const int at = ((h * 4 + gs) ^ (gl & 7)) * 8;
-      const bool on = h * 32 + gs * 8 < k_left;
-      mf_bf8 a[4], b[4];
+      mf_bf8 a[TN], b[4];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        a[i] = frag8(ws + (wn + i * 16 + gl) * BK + at);
-        b[i] = frag8(xs + (wm + i * 16 + gl) * BK + at);
-      }
+      for (int i = 0; i < TN; ++i) a[i] = frag8(ws + i * 16 * BK + at);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) b[j] = frag8(xs + j * 16 * BK + at);
       if (k_left < BK) {
+        const bool on = h * 32 + gs * 8 < k_left;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          a[i] = on ? a[i] : z;
-          b[i] = on ? b[i] : z;
-        }
+        for (int i = 0; i < TN; ++i) a[i] = on ? a[i] : z;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) b[j] = on ? b[j] : z;
       }
+      __builtin_amdgcn_s_setprio(1);
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
+      for (int i = 0; i < TN; ++i)
 #pragma unroll
         for (int j = 0; j < 4; ++j)
           acc[i][j] = mfma_bf16_k32(a[i], b[j], acc[i][j]);
+      __builtin_amdgcn_s_setprio(0);
     }
   };
-  const int nk = (p.k + BK - 1) / BK;
-  issue(0, 0);
+  const int nk = p.k / BK, rest = p.k % BK;
   for (int kt = 0; kt < nk; ++kt) {
-    // this step's pieces have landed, and the other buffer is read
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    __syncthreads();
-    if (kt + 1 < nk) issue(kt + 1, (kt + 1) & 1);
-    compute(kt & 1, p.k - kt * BK);
+    issue(kt);
+    landed_barrier();
+    compute(BK);
+    landed_barrier();                           // everyone has read
+  }
+  if (rest) {                                   // pieces past the end: the last
+    const int back = max(piece * 8 - (rest - 8), 0) * 2;
+#pragma unroll
+    for (int c = 0; c < XI; ++c) xo[c] -= back;
+#pragma unroll
+    for (int c = 0; c < WI; ++c) wo[c] -= back;
+    issue(nk);
+    landed_barrier();
+    compute(rest);
   }
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
     const int r = wm + j * 16 + gl;
     if (r >= rows) continue;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
+    for (int i = 0; i < TN; ++i) {
       const int n = n0 + wn + i * 16 + gs * 4;
       if (n < p.n) put4(p, row0 + r, n, acc[i][j]);
     }
   }
+}
+
+template <int BN, int OCC>
+void moe_tiled(const MoeGemmArgs& p, hipStream_t s) {
+  const int nb = (p.n + BN - 1) / BN;
+  moe_tiled_kernel<BN, OCC><<<8 * ((p.max_tiles * nb + 7) / 8), GT, 0, s>>>(p);
 }
 
 constexpr int SW = 4;                           // waves of a skinny workgroup
@@ -263,15 +291,9 @@ extern "C" void launch_moe_gemm(const MoeGemmArgs* p, int f32, int vec,
     moe_skinny_kernel<2, 2><<<dim3((p->n + 31) / 32, p->max_tiles), SW * 64, 0,
                               s>>>(*p);
   } else {
-    static bool once = false;
-    if (!once) {
-      (void)hipFuncSetAttribute((const void*)moe_tiled_kernel,
-                                hipFuncAttributeMaxDynamicSharedMemorySize,
-                                2 * STAGE * 2);
-      once = true;
-    }
-    const int nb = (p->n + BN - 1) / BN;
-    moe_tiled_kernel<<<8 * ((p->max_tiles * nb + 7) / 8), GT, 2 * STAGE * 2,
-                       s>>>(*p);
+    // the wide form is 1.08 times as fast per column
+    const long wide = (p->n + 191) / 192 * 192L, slim = (p->n + 127) / 128 * 128L;
+    if (wide * 100 <= slim * 108) moe_tiled<192, 3>(*p, s);
+    else moe_tiled<128, 4>(*p, s);
   }
 }

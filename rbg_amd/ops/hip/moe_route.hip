@@ -1,15 +1,17 @@
 // Routing of tokens to experts (gfx950).
 //
-//   logits   x W^T with f32 sums: a workgroup takes 16 experts and 16 * MT
-//            tokens, its waves split K and meet in LDS.  W rows are MFMA A
-//            fragments, so lanes are tokens and registers experts.
+//   logits   x W^T with f32 sums: a workgroup takes 16 * MT tokens and one or
+//            four tiles of 16 experts, its waves split K and meet in LDS.  W
+//            rows are MFMA A fragments: lanes are tokens, registers experts.
 //   choose   one wave per token: sigmoid, correction, the two best of each group
 //            of neighbours, the best groups, the best experts of those.  Ranks
 //            are counted, not sorted: an expert's rank is the number of experts
 //            ahead of it in the order (score, index), which is total, so every
 //            place is filled exactly once whatever the scores are.
-//   lay out  one workgroup: pairs (token, choice) counted per expert, offsets
-//            by a scan, tiles of one expert each, and the permutation.
+//   lay out  pairs (token, choice) counted per expert, offsets by a scan, tiles
+//            of one expert each, and the permutation: one workgroup, together
+//            with the choice for decode batches; for prompts the counting and
+//            the permutation are spread over blocks of 64 tokens.
 #include "mfma_util.h"
 #include "moe_args.h"
 #include "vec_io.h"
@@ -18,15 +20,18 @@ namespace {
 
 constexpr int UN = 4;                           // 32-k steps in flight
 
-template <int MT, int NW>
-__global__ __launch_bounds__(NW * 64) void router_logits_kernel(
+// EW * KW waves: EW tiles of 16 experts (which find the tokens' rows in L1), KW
+// slices of K
+template <int MT, int EW, int KW>
+__global__ __launch_bounds__(EW * KW * 64) void router_logits_kernel(
     float* __restrict__ out, const __hip_bfloat16* __restrict__ x,
     const __hip_bfloat16* __restrict__ w, const int tokens, const int experts,
     const int k_len) {
-  __shared__ f32x4 red[NW][MT][64];
+  __shared__ f32x4 red[KW][EW][MT][64];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int gl = lane & 15, gs = lane >> 4;
-  const int e0 = blockIdx.x * 16, t0 = blockIdx.y * 16 * MT;
+  const int ew = wave % EW, kw = wave / EW;
+  const int e0 = (blockIdx.x * EW + ew) * 16, t0 = blockIdx.y * 16 * MT;
   const __hip_bfloat16* wr = w + (size_t)min(e0 + gl, experts - 1) * k_len;
   const __hip_bfloat16* xr[MT];
 #pragma unroll
@@ -35,8 +40,8 @@ __global__ __launch_bounds__(NW * 64) void router_logits_kernel(
   f32x4 acc[MT];
 #pragma unroll
   for (int t = 0; t < MT; ++t) acc[t] = {0.f, 0.f, 0.f, 0.f};
-  const int per = ((k_len + NW * 32 - 1) / (NW * 32)) * 32;
-  const int kb = wave * per, ke = min(kb + per, k_len);
+  const int per = ((k_len + KW * 32 - 1) / (KW * 32)) * 32;
+  const int kb = kw * per, ke = min(kb + per, k_len);
   for (int k0 = kb; k0 < ke; k0 += 32 * UN) {
     // unconditional clamped loads, all before the first product
     mf_bf8 wf[UN], xf[UN][MT];
@@ -57,14 +62,15 @@ __global__ __launch_bounds__(NW * 64) void router_logits_kernel(
     }
   }
 #pragma unroll
-  for (int t = 0; t < MT; ++t) red[wave][t][lane] = acc[t];
+  for (int t = 0; t < MT; ++t) red[kw][ew][t][lane] = acc[t];
   __syncthreads();
-  for (int i = threadIdx.x; i < MT * 64; i += NW * 64) {
-    const int t = i >> 6, ln = i & 63;
+  for (int i = threadIdx.x; i < EW * MT * 64; i += EW * KW * 64) {
+    const int ln = i & 63, t = (i >> 6) % MT, we = (i >> 6) / MT;
     f32x4 s = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int wv = 0; wv < NW; ++wv) s += red[wv][t][ln];
-    const int tok = t0 + t * 16 + (ln & 15), e = e0 + (ln >> 4) * 4;
+    for (int kk = 0; kk < KW; ++kk) s += red[kk][we][t][ln];
+    const int tok = t0 + t * 16 + (ln & 15);
+    const int e = (blockIdx.x * EW + we) * 16 + (ln >> 4) * 4;
     if (tok >= tokens) continue;
 #pragma unroll
     for (int r = 0; r < 4; ++r)
@@ -95,47 +101,61 @@ DEV_INLINE void wave_fence() {
 
 DEV_INLINE float sigmoid_exact(float z) { return 1.f / (1.f + expf(-z)); }
 
-// One wave, one token.  choice [experts], group [groups]: its own LDS.
+// LDS floats of one wave's choice: experts and groups, padded to whole quads
+__host__ __device__ inline int choice_floats(int experts, int groups) {
+  return ((experts + 3) & ~3) + ((groups + 3) & ~3);
+}
+
+// how many of the n values (padded with -inf) are ahead of value `mine` at `at`
+DEV_INLINE int rank_of(const float* v, const int n, const float mine,
+                       const int at) {
+  int rank = 0;
+#pragma unroll 4
+  for (int o = 0; o < n; o += 4) {
+    const float4 c = *reinterpret_cast<const float4*>(v + o);
+    rank += c.x > mine || (c.x == mine && o < at);
+    rank += c.y > mine || (c.y == mine && o + 1 < at);
+    rank += c.z > mine || (c.z == mine && o + 2 < at);
+    rank += c.w > mine || (c.w == mine && o + 3 < at);
+  }
+  return rank;
+}
+
+// One wave, one token; `choice` is its own LDS.
 DEV_INLINE void choose(const MoeRouteArgs& p, const int token, float* choice,
-                       float* group, const int lane) {
+                       const int lane) {
   const float* z = p.logits + (size_t)token * p.experts;
-  for (int e = lane; e < p.experts; e += 64)    // NaN becomes the least score
-    choice[e] = fmaxf(sigmoid_exact(z[e]) + p.correction[e], -3e38f);
+  const int ep = (p.experts + 3) & ~3, gp = (p.groups + 3) & ~3;
+  float* group = choice + ep;
+  for (int e = lane; e < ep; e += 64)           // NaN becomes the least score
+    choice[e] = e < p.experts
+        ? fmaxf(sigmoid_exact(z[e]) + p.correction[e], -3e38f) : -INFINITY;
   wave_fence();
   const int size = p.experts / p.groups;
   if (p.keep < p.groups) {
-    for (int g = lane; g < p.groups; g += 64) {
+    for (int g = lane; g < gp; g += 64) {
       float a = -INFINITY, b = -INFINITY;
-      for (int i = 0; i < size; ++i) {
-        const float c = choice[g * size + i];
-        b = fmaxf(b, fminf(a, c));
-        a = fmaxf(a, c);
+      if (g < p.groups) {
+#pragma unroll 4
+        for (int i = 0; i < size; ++i) {
+          const float c = choice[g * size + i];
+          b = fmaxf(b, fminf(a, c));
+          a = fmaxf(a, c);
+        }
+        if (size > 1) a += b;
       }
-      group[g] = size > 1 ? a + b : a;
+      group[g] = a;
     }
     wave_fence();
-    // groups beyond 64 keep their scores in LDS until every rank is known
-    for (int g0 = 0; g0 < p.groups; g0 += 64) {
-      const int g = g0 + lane;
-      if (g < p.groups) {
-        int rank = 0;
-        const float mine = group[g];
-        for (int o = 0; o < p.groups; ++o)
-          rank += group[o] > mine || (group[o] == mine && o < g);
-        if (rank >= p.keep)
-          for (int i = 0; i < size; ++i) choice[g * size + i] = -INFINITY;
-      }
-    }
+    for (int g = lane; g < p.groups; g += 64)
+      if (rank_of(group, gp, group[g], g) >= p.keep)
+        for (int i = 0; i < size; ++i) choice[g * size + i] = -INFINITY;
     wave_fence();
   }
   for (int e = lane; e < p.experts; e += 64) {
     const float mine = choice[e];
     if (mine == -INFINITY) continue;
-    int rank = 0;
-    for (int o = 0; o < p.experts; ++o) {
-      const float c = choice[o];
-      rank += c > mine || (c == mine && o < e);
-    }
+    const int rank = rank_of(choice, ep, mine, e);
     if (rank < p.top) {
       p.ids[(size_t)token * p.top + rank] = e;
       p.weights[(size_t)token * p.top + rank] = sigmoid_exact(z[e]);
@@ -144,18 +164,12 @@ DEV_INLINE void choose(const MoeRouteArgs& p, const int token, float* choice,
   wave_fence();
 }
 
-// One workgroup of NT threads.  count [experts], cursor [experts], scan
-// [2 * waves]: LDS.
+// From each expert's count (LDS) its first row (LDS, cursor) and its tiles.  One
+// workgroup of NT threads; scan [2 * waves]: LDS.
 template <int NT>
-DEV_INLINE void lay_out(const MoeRouteArgs& p, int* count, int* cursor,
+DEV_INLINE void offsets(const MoeRouteArgs& p, const int* count, int* cursor,
                         int* scan) {
-  const int tid = threadIdx.x, pairs = p.tokens * p.top;
-  for (int e = tid; e < p.experts; e += NT) count[e] = 0;
-  __syncthreads();
-#pragma unroll 4
-  for (int i = tid; i < pairs; i += NT) atomicAdd(&count[p.ids[i]], 1);
-  __syncthreads();
-  // exclusive sums of rows (low half) and tiles (high half), NT experts a round
+  const int tid = threadIdx.x;
   int rows0 = 0, tiles0 = 0;
   for (int e0 = 0; e0 < p.experts; e0 += NT) {
     const int e = e0 + tid, n = e < p.experts ? count[e] : 0;
@@ -176,13 +190,15 @@ DEV_INLINE void lay_out(const MoeRouteArgs& p, int* count, int* cursor,
     }
     __syncthreads();
     int ra = rows0, ta = tiles0;
+#pragma unroll
     for (int wv = 0; wv < NT / 64; ++wv) {
+      const int a = scan[wv * 2], b = scan[wv * 2 + 1];
       if (wv < (tid >> 6)) {
-        ra += scan[wv * 2];
-        ta += scan[wv * 2 + 1];
+        ra += a;
+        ta += b;
       }
-      rows0 += scan[wv * 2];
-      tiles0 += scan[wv * 2 + 1];
+      rows0 += a;
+      tiles0 += b;
     }
     if (e < p.experts) {
       const int first = ra + r - n;
@@ -197,41 +213,114 @@ DEV_INLINE void lay_out(const MoeRouteArgs& p, int* count, int* cursor,
     __syncthreads();
   }
   if (tid == 0) *p.count = tiles0;
+}
+
+// Pairs [lo, hi) counted into, or placed by, an LDS array over the experts.
+template <int NT>
+DEV_INLINE void count_pairs(const MoeRouteArgs& p, int* count, int lo, int hi) {
+  for (int e = threadIdx.x; e < p.experts; e += NT) count[e] = 0;
+  __syncthreads();
 #pragma unroll 4
-  for (int i = tid; i < pairs; i += NT) {
+  for (int i = lo + threadIdx.x; i < hi; i += NT)
+    atomicAdd(&count[p.ids[i]], 1);
+  __syncthreads();
+}
+
+template <int NT>
+DEV_INLINE void place_pairs(const MoeRouteArgs& p, int* cursor, int lo,
+                            int hi) {
+#pragma unroll 4
+  for (int i = lo + threadIdx.x; i < hi; i += NT) {
     const int at = atomicAdd(&cursor[p.ids[i]], 1);
     p.inv[i] = at;
     p.rows[at] = i / p.top;
   }
 }
 
-__global__ __launch_bounds__(256) void choose_kernel(const MoeRouteArgs p) {
+// decode batches: choice and layout in one workgroup
+template <int NT>
+__global__ __launch_bounds__(NT) void route_small_kernel(const MoeRouteArgs p) {
   extern __shared__ float route_smem[];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int token = blockIdx.x * 4 + wave;
-  if (token >= p.tokens) return;                // whole wave leaves
-  float* mine = route_smem + wave * (p.experts + p.groups);
-  choose(p, token, mine, mine + p.experts, lane);
-}
-
-constexpr int LN = 1024;
-
-__global__ __launch_bounds__(LN) void lay_out_kernel(const MoeRouteArgs p) {
-  extern __shared__ int lay_smem[];
-  lay_out<LN>(p, lay_smem, lay_smem + p.experts, lay_smem + 2 * p.experts);
-}
-
-// decode batches: both in one workgroup
-__global__ __launch_bounds__(LN) void route_small_kernel(const MoeRouteArgs p) {
-  extern __shared__ float route_smem[];
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  float* mine = route_smem + wave * (p.experts + p.groups);
-  for (int t = wave; t < p.tokens; t += LN / 64)
-    choose(p, t, mine, mine + p.experts, lane);
+  float* mine = route_smem + wave * choice_floats(p.experts, p.groups);
+  for (int t = wave; t < p.tokens; t += NT / 64) choose(p, t, mine, lane);
   __threadfence_block();
   __syncthreads();
-  int* lay = (int*)route_smem;
-  lay_out<LN>(p, lay, lay + p.experts, lay + 2 * p.experts);
+  int* count = (int*)route_smem;
+  int* cursor = count + p.experts;
+  count_pairs<NT>(p, count, 0, p.tokens * p.top);
+  offsets<NT>(p, count, cursor, cursor + p.experts);
+  place_pairs<NT>(p, cursor, 0, p.tokens * p.top);
+}
+
+// 64 tokens' choice, and how often it took each expert: part [blocks, experts]
+constexpr int BT = 64, CN = 1024;
+
+template <int NT>
+__global__ __launch_bounds__(NT) void choose_kernel(const MoeRouteArgs p) {
+  extern __shared__ float route_smem[];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  float* mine = route_smem + wave * choice_floats(p.experts, p.groups);
+  const int lo = blockIdx.x * BT, hi = min(lo + BT, p.tokens);
+  for (int t = lo + wave; t < hi; t += NT / 64) choose(p, t, mine, lane);
+  __threadfence_block();
+  __syncthreads();
+  int* count = (int*)route_smem;
+  count_pairs<NT>(p, count, lo * p.top, hi * p.top);
+  for (int e = threadIdx.x; e < p.experts; e += NT)
+    p.part[(size_t)blockIdx.x * p.experts + e] = count[e];
+}
+
+// part becomes the first row of each block's pairs of each expert.  A thread
+// takes a run of blocks of one expert.
+__global__ __launch_bounds__(CN) void offsets_kernel(const MoeRouteArgs p,
+                                                     const int blocks) {
+  extern __shared__ int lay_smem[];
+  int* count = lay_smem;                        // [experts]
+  int* cursor = count + p.experts;              // [experts]
+  int* scan = cursor + p.experts;               // [2 * waves]
+  int* run = scan + 2 * CN / 64;                // [CN]
+  const int lanes = min(max(CN / p.experts, 1), 32);    // runs per expert
+  const int len = (blocks + lanes - 1) / lanes;
+  const int e = threadIdx.x % p.experts, r = threadIdx.x / p.experts;
+  const bool on = p.experts <= CN && r < lanes;
+  const int b0 = min(r * len, blocks), b1 = min(b0 + len, blocks);
+  int n = 0;
+  if (on) {
+#pragma unroll 4
+    for (int b = b0; b < b1; ++b) n += p.part[(size_t)b * p.experts + e];
+    run[r * p.experts + e] = n;
+  }
+  __syncthreads();
+  if (threadIdx.x < p.experts) {
+    int total = 0;
+    for (int i = 0; i < lanes; ++i) {
+      const int v = run[i * p.experts + threadIdx.x];
+      run[i * p.experts + threadIdx.x] = total;
+      total += v;
+    }
+    count[threadIdx.x] = total;
+  }
+  __syncthreads();
+  offsets<CN>(p, count, cursor, scan);
+  if (on) {
+    int at = cursor[e] + run[r * p.experts + e];
+#pragma unroll 4
+    for (int b = b0; b < b1; ++b) {
+      const int v = p.part[(size_t)b * p.experts + e];
+      p.part[(size_t)b * p.experts + e] = at;
+      at += v;
+    }
+  }
+}
+
+__global__ __launch_bounds__(256) void place_kernel(const MoeRouteArgs p) {
+  extern __shared__ int lay_smem[];
+  for (int e = threadIdx.x; e < p.experts; e += 256)
+    lay_smem[e] = p.part[(size_t)blockIdx.x * p.experts + e];
+  __syncthreads();
+  const int lo = blockIdx.x * BT, hi = min(lo + BT, p.tokens);
+  place_pairs<256>(p, lay_smem, lo * p.top, hi * p.top);
 }
 
 }  // namespace
@@ -244,13 +333,14 @@ void launch_router_logits(float* out, const void* x, const void* w, int tokens,
   if (vec) {
     const __hip_bfloat16 *xb = (const __hip_bfloat16*)x,
                          *wb = (const __hip_bfloat16*)w;
-    const int eb = (experts + 15) / 16;
     if (tokens <= 512) {
-      router_logits_kernel<1, 8><<<dim3(eb, (tokens + 15) / 16), 512, 0, s>>>(
-          out, xb, wb, tokens, experts, k);
+      router_logits_kernel<1, 1, 8>
+          <<<dim3((experts + 15) / 16, (tokens + 15) / 16), 512, 0, s>>>(
+              out, xb, wb, tokens, experts, k);
     } else {
-      router_logits_kernel<4, 4><<<dim3(eb, (tokens + 63) / 64), 256, 0, s>>>(
-          out, xb, wb, tokens, experts, k);
+      router_logits_kernel<2, 4, 4>
+          <<<dim3((experts + 63) / 64, (tokens + 31) / 32), 1024, 0, s>>>(
+              out, xb, wb, tokens, experts, k);
     }
     return;
   }
@@ -268,16 +358,32 @@ void launch_router_logits(float* out, const void* x, const void* w, int tokens,
 
 int moe_max_experts() { return 1024; }
 
+// blocks of tokens that count on their own; 0: one workgroup does everything
+int moe_route_blocks(int tokens, int experts) {
+  return tokens <= 64 && experts <= 512 ? 0 : (tokens + BT - 1) / BT;
+}
+
 void launch_moe_route(const MoeRouteArgs* p, hipStream_t s) {
-  const size_t lay = sizeof(int) * (2 * p->experts + 2 * LN / 64);
-  if (p->tokens <= 64 && p->experts <= 512) {
-    const size_t own = sizeof(float) * 16 * (p->experts + p->groups);
-    route_small_kernel<<<1, LN, own > lay ? own : lay, s>>>(*p);
+  const int blocks = moe_route_blocks(p->tokens, p->experts);
+  const size_t own = sizeof(float) * choice_floats(p->experts, p->groups);
+  if (blocks == 0) {
+    const size_t lay = sizeof(int) * (2 * p->experts + 32);
+    if (p->tokens <= 4) {
+      route_small_kernel<256><<<1, 256, own * 4 > lay ? own * 4 : lay, s>>>(*p);
+    } else {
+      route_small_kernel<1024><<<1, 1024, own * 16 > lay ? own * 16 : lay,
+                                 s>>>(*p);
+    }
     return;
   }
-  choose_kernel<<<(p->tokens + 3) / 4, 256,
-                  sizeof(float) * 4 * (p->experts + p->groups), s>>>(*p);
-  lay_out_kernel<<<1, LN, lay, s>>>(*p);
+  if (own * 16 <= 65536) {
+    choose_kernel<1024><<<blocks, 1024, own * 16, s>>>(*p);
+  } else {
+    choose_kernel<256><<<blocks, 256, own * 4, s>>>(*p);
+  }
+  offsets_kernel<<<1, CN, sizeof(int) * (2 * p->experts + 2 * CN / 64 + CN),
+                   s>>>(*p, blocks);
+  place_kernel<<<blocks, 256, sizeof(int) * p->experts, s>>>(*p);
 }
 
 }  // extern "C"

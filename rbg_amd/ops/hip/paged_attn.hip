@@ -15,6 +15,9 @@
 //            strip.  The waves meet at the end, the splits in a second kernel.
 //   rows     one wave per (query row, head), any sizes, bf16 or f32.
 //
+// A soft cap bounds the scores; when its exponentials fit f32 with room (BOUND),
+// nothing has to be subtracted, and the running maximum and every rescaling go.
+//
 // Scores and weights are f32.  Weights enter the second product as two bf16
 // (hi + lo), which keeps 16 bits of them.  The sink is the running maximum's
 // first value (zero) and one more term of the final sum.
@@ -44,9 +47,12 @@ struct ScoreMap {
   }
 };
 
+// largest |score| * log2(e) whose exponential may be summed as it is
+constexpr float BOUND_LOG2 = 100.f;
+
 constexpr int KT = 64;
 
-template <int DK, int DV, int NW, int QT>
+template <int DK, int DV, int NW, int QT, bool BOUND>
 __global__ __launch_bounds__(NW * 64, (DK + DV) > 256 ? 1 : 2)
 void paged_prefill_kernel(const PagedAttnArgs p) {
   constexpr int KP = DK + 16, VP = DV + 16;   // 8 banks per row
@@ -147,7 +153,7 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
   f32x4 acc[QT][DV / 16];
 #pragma unroll
   for (int t = 0; t < QT; ++t) {
-    m[t] = p.sink ? 0.f : MASKED;
+    m[t] = BOUND || p.sink ? 0.f : MASKED;
     l[t] = 0.f;
 #pragma unroll
     for (int d = 0; d < DV / 16; ++d) acc[t][d] = {0.f, 0.f, 0.f, 0.f};
@@ -185,37 +191,42 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
 #pragma unroll
     for (int t = 0; t < QT; ++t) {
       const int hi = qpos[t];
-      float mx = MASKED;
+      float mn = 0.f;
+      if (!BOUND) {
+        float mx = MASKED;
 #pragma unroll
-      for (int c = 0; c < 4; ++c)
+        for (int c = 0; c < 4; ++c)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int j = k0 + c * 16 + gs * 4 + r;
-          const float x = j <= hi ? score(s[t][c][r]) : MASKED;
-          s[t][c][r] = x;
-          mx = fmaxf(mx, x);
-        }
-      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-      const float mn = fmaxf(m[t], mx);
-      const float corr = exp2_fast(m[t] - mn);
-      m[t] = mn;
+          for (int r = 0; r < 4; ++r) {
+            const int j = k0 + c * 16 + gs * 4 + r;
+            const float x = j <= hi ? score(s[t][c][r]) : MASKED;
+            s[t][c][r] = x;
+            mx = fmaxf(mx, x);
+          }
+        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+        mn = fmaxf(m[t], mx);
+        const float corr = exp2_fast(m[t] - mn);
+        m[t] = mn;
+        l[t] *= corr;
+#pragma unroll
+        for (int d = 0; d < DV / 16; ++d) acc[t][d] *= corr;
+      }
       float sum = 0.f;
 #pragma unroll
       for (int c = 0; c < 4; ++c)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const float x = s[t][c][r];
-          const float e = x > MASKED ? exp2_fast(x - mn) : 0.f;
+          const int j = k0 + c * 16 + gs * 4 + r;
+          const float x = BOUND ? score(s[t][c][r]) : s[t][c][r] - mn;
+          const float e = j <= hi ? exp2_fast(x) : 0.f;
           sum += e;
           __bf16 h, lw;
           split_bf16(e, h, lw);
           ph[t][c >> 1][(c & 1) * 4 + r] = h;
           pl[t][c >> 1][(c & 1) * 4 + r] = lw;
         }
-      l[t] = l[t] * corr + sum;               // per lane; summed at the end
-#pragma unroll
-      for (int d = 0; d < DV / 16; ++d) acc[t][d] *= corr;
+      l[t] += sum;                            // per lane; summed at the end
     }
 #pragma unroll
     for (int st = 0; st < 2; ++st)
@@ -259,7 +270,7 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
 
 constexpr int DW = 4;                         // waves of a decode workgroup
 
-template <int DK, int DV>
+template <int DK, int DV, bool BOUND>
 __global__ __launch_bounds__(DW * 64, (DK + DV) > 256 ? 1 : 2)
 void paged_decode_kernel(const PagedAttnArgs p) {
   constexpr int VP = DV + 16, VL = DV / 16;   // VL 16-byte loads of 32 rows
@@ -297,7 +308,7 @@ void paged_decode_kernel(const PagedAttnArgs p) {
     mf_bf8 z = {};
     qf[s] = d < p.d ? frag8(q + d) : z;
   }
-  float m = p.sink ? 0.f : MASKED, l = 0.f;
+  float m = BOUND || p.sink ? 0.f : MASKED, l = 0.f;
   f32x4 acc[DV / 16];
 #pragma unroll
   for (int d = 0; d < DV / 16; ++d) acc[d] = {0.f, 0.f, 0.f, 0.f};
@@ -364,36 +375,41 @@ void paged_decode_kernel(const PagedAttnArgs p) {
       fetch();
       pages(min(step + 2, s_end - 1));
     }
-    float mx = MASKED;
+    float mn = 0.f;
+    if (!BOUND) {
+      float mx = MASKED;
 #pragma unroll
-    for (int c = 0; c < 2; ++c)
+      for (int c = 0; c < 2; ++c)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int j = j0 + c * 16 + gs * 4 + r;
-        const float x = j <= pos ? score(s[c][r]) : MASKED;
-        s[c][r] = x;
-        mx = fmaxf(mx, x);
-      }
-    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-    const float mn = fmaxf(m, mx);
-    const float corr = exp2_fast(m - mn);
-    m = mn;
-    float sum = 0.f;
+        for (int r = 0; r < 4; ++r) {
+          const int j = j0 + c * 16 + gs * 4 + r;
+          const float x = j <= pos ? score(s[c][r]) : MASKED;
+          s[c][r] = x;
+          mx = fmaxf(mx, x);
+        }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      mn = fmaxf(m, mx);
+      const float corr = exp2_fast(m - mn);
+      m = mn;
+      l *= corr;
+#pragma unroll
+      for (int d = 0; d < DV / 16; ++d) acc[d] *= corr;
+    }
     mf_bf8 ph, pl;
 #pragma unroll
     for (int c = 0; c < 2; ++c)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const float x = s[c][r];
-        const float e = x > MASKED ? exp2_fast(x - mn) : 0.f;
-        sum += e;
+        const int j = j0 + c * 16 + gs * 4 + r;
+        const float x = BOUND ? score(s[c][r]) : s[c][r] - mn;
+        const float e = j <= pos ? exp2_fast(x) : 0.f;
+        l += e;
         __bf16 h, lw;
         split_bf16(e, h, lw);
         ph[c * 4 + r] = h;
         pl[c * 4 + r] = lw;
       }
-    l = l * corr + sum;
 #pragma unroll
     for (int d = 0; d < DV / 16; ++d) {
       const __hip_bfloat16* b =
@@ -401,7 +417,7 @@ void paged_decode_kernel(const PagedAttnArgs p) {
       const mf_bf4 v0 = tr_read4(b), v1 = tr_read4(b + 16 * VP);
       const mf_bf8 vf = {v0[0], v0[1], v0[2], v0[3],
                          v1[0], v1[1], v1[2], v1[3]};
-      acc[d] = mfma_bf16_k32(vf, ph, acc[d] * corr);
+      acc[d] = mfma_bf16_k32(vf, ph, acc[d]);
       acc[d] = mfma_bf16_k32(vf, pl, acc[d]);
     }
   }
@@ -549,11 +565,20 @@ __global__ __launch_bounds__(256) void paged_rows_kernel(
   }
 }
 
+bool bounded(const PagedAttnArgs& p) {
+  return p.softcap > 0.f && p.softcap * LOG2E <= BOUND_LOG2;
+}
+
 template <int DK>
 void prefill_dv(const PagedAttnArgs& p, hipStream_t s) {
   const int grid = 8 * ((p.n_blocks * p.heads + 7) / 8);
 #define PP_GO(DV, NW, QT)                                                     \
-  paged_prefill_kernel<DK, DV, NW, QT><<<grid, NW * 64, 0, s>>>(p)
+  do {                                                                        \
+    if (bounded(p))                                                           \
+      paged_prefill_kernel<DK, DV, NW, QT, true><<<grid, NW * 64, 0, s>>>(p); \
+    else                                                                      \
+      paged_prefill_kernel<DK, DV, NW, QT, false><<<grid, NW * 64, 0, s>>>(p);\
+  } while (0)
   if (p.dv <= 64) PP_GO(64, 4, 2);
   else if (p.dv <= 96) PP_GO(96, 4, 2);
   else if (p.dv <= 128) PP_GO(128, 4, 2);
@@ -565,7 +590,13 @@ template <int DK>
 void decode_dv(const PagedAttnArgs& p, hipStream_t s) {
   const int tiles = (p.heads / p.kv_heads + 15) / 16;
   const dim3 grid(p.splits, p.rows, p.kv_heads * tiles);
-#define PD_GO(DV) paged_decode_kernel<DK, DV><<<grid, DW * 64, 0, s>>>(p)
+#define PD_GO(DV)                                                             \
+  do {                                                                        \
+    if (bounded(p))                                                           \
+      paged_decode_kernel<DK, DV, true><<<grid, DW * 64, 0, s>>>(p);          \
+    else                                                                      \
+      paged_decode_kernel<DK, DV, false><<<grid, DW * 64, 0, s>>>(p);         \
+  } while (0)
   if (p.dv <= 64) PD_GO(64);
   else if (p.dv <= 96) PD_GO(96);
   else if (p.dv <= 128) PD_GO(128);

@@ -9,12 +9,7 @@
 namespace {
 
 template <typename T, int V>
-__global__ __launch_bounds__(256) void rope_paged_kernel(
-    const RopePagedArgs p, const long total, const int units) {
-  const long i = blockIdx.x * 256L + threadIdx.x;
-  if (i >= total) return;
-  const int row = (int)(i / units);
-  int u = (int)(i % units);
+DEV_INLINE void rope_unit(const RopePagedArgs& p, const int row, int u) {
   const int half = p.rot / 2;
   const int pair_u = half / V, per_head = pair_u + (p.d - p.rot) / V;
   const int slot = p.k != nullptr ? p.slots[row] : -1;
@@ -77,15 +72,28 @@ __global__ __launch_bounds__(256) void rope_paged_kernel(
   }
 }
 
+// TPR threads per row
+template <typename T, int V, int TPR>
+__global__ __launch_bounds__(256) void rope_paged_kernel(
+    const RopePagedArgs p, const int units) {
+  const int row = blockIdx.x * (256 / TPR) + threadIdx.x / TPR;
+  if (row >= p.rows) return;
+  for (int u = threadIdx.x % TPR; u < units; u += TPR)
+    rope_unit<T, V>(p, row, u);
+}
+
 template <typename T, int V>
 void rope_paged_t(const RopePagedArgs& p, hipStream_t s) {
   const int per_head = p.rot / 2 / V + (p.d - p.rot) / V;
   const int units = p.k != nullptr
       ? (p.heads + p.kv_heads) * per_head + p.kv_heads * (p.dv / V)
       : p.heads * per_head;
-  const long total = (long)p.rows * units;
-  rope_paged_kernel<T, V><<<(int)((total + 255) / 256), 256, 0, s>>>(p, total,
-                                                                     units);
+  // long prompts: a wave per row; short steps: more waves, to hide latency
+  if (p.rows >= 1024) {
+    rope_paged_kernel<T, V, 64><<<(p.rows + 3) / 4, 256, 0, s>>>(p, units);
+  } else {
+    rope_paged_kernel<T, V, 256><<<p.rows, 256, 0, s>>>(p, units);
+  }
 }
 
 }  // namespace

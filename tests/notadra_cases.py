@@ -74,21 +74,27 @@ def shapes(cfg):
 
 def weights(cfg, seed=0, sharpen=2.5):
     """bf16 values.  Queries are sharpened so that single keys stand out.
-    Router rows of one length and wide corrections keep the choices apart:
-    rounding must not change who is chosen."""
+    Tokens are of two kinds, far apart along one direction that the routers
+    look at: each kind has its experts, and rounding does not change who is
+    chosen."""
     gen = torch.Generator().manual_seed(seed)
+    kind = torch.randn(cfg["width"], generator=gen).sign()
     out = {}
     for name, shape in shapes(cfg).items():
         t = torch.randn(shape, generator=gen)
         if "norm" in name.split(".")[-1]:
             t = 0.3 * t
+        elif name == "embed":
+            t += 3.0 * kind * (torch.arange(shape[0]) % 2 * 2 - 1).view(-1, 1)
         elif name.endswith("correction"):
-            t = 0.4 * t - 0.8               # choice scores of both signs
+            t = 0.2 * t - 0.7               # choice scores of both signs
         elif name.endswith(".b"):
             t = 0.3 * t
         elif name.endswith("router"):
-            t = 6.0 * t / math.sqrt(shape[1])
-        elif len(shape) == 2 and name not in ("embed", "bigram"):
+            side = (torch.arange(shape[0]) // 2 % 2 * 2 - 1).view(-1, 1)
+            t = (0.1 * t + 4.0 * side * kind / math.sqrt(shape[1])) / \
+                math.sqrt(shape[1])
+        elif len(shape) == 2 and name != "bigram":
             t = t / math.sqrt(shape[1])
             if name.endswith("mix.q"):
                 t = t * sharpen

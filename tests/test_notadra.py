@@ -24,8 +24,7 @@ GPU = pytest.mark.gpu
 WHERE = [pytest.param(("cpu", "float32"), id="cpu-f32"),
          pytest.param(("cuda", "float32"), id="gpu-f32", marks=GPU),
          pytest.param(("cuda", "bfloat16"), id="gpu-bf16", marks=GPU)]
-# relative to the answers' RMS; in bf16 a near tie between two experts may be
-# decided otherwise, which a few positions are allowed to show
+# relative to the answers' RMS
 TOL = {"float32": 3e-5, "bfloat16": 5e-2}
 
 MODELS = {
@@ -55,6 +54,8 @@ MODELS = {
                         scale=0.1), experts(ff=32, n=16, top=3))],
         width=64, buckets=997, mul_prev=101, mul_cur=1),
 }
+# weights whose routers leave a margin between chosen and left out
+SEEDS = {"mix": 3, "odd": 3, "wide": 6}
 
 
 @pytest.fixture(scope="module")
@@ -65,7 +66,7 @@ def model(tmp_path_factory):
     def get(name):
         if name not in made:
             cfg = MODELS[name]
-            w = cases.weights(cfg, seed=len(name))
+            w = cases.weights(cfg, seed=SEEDS[name])
             folder = cases.save(tmp_path_factory.mktemp(name), cfg, w)
             made[name] = (folder, cfg, w)
         return made[name]
@@ -96,12 +97,8 @@ def feed(rid, toks, want=True):
 
 
 def check(got, want, where):
-    err = row_errs(got, want).sort().values
-    tol = TOL[where[1]]
-    if where[1] == "float32":
-        assert err[-1] < tol, err[-1]
-    else:
-        assert err[int(0.9 * (len(err) - 1))] < tol and err[-1] < 1.0, err
+    err = row_errs(got, want)
+    assert err.max() < TOL[where[1]], err
 
 
 @pytest.mark.parametrize("where", WHERE)

@@ -195,7 +195,7 @@ def attn_case(H, G, D, DV, n, scale, seed=0):
 
 @pytest.mark.parametrize("where", WHERE)
 @pytest.mark.parametrize("H,G,D,DV", ATTN_SIZES)
-@pytest.mark.parametrize("softcap", [6.0, 50.0])
+@pytest.mark.parametrize("softcap", [6.0, 50.0, 300.0])
 def test_paged_prefill_portions(where, H, G, D, DV, softcap):
     """Portions cut anywhere, over keys in shuffled pages."""
     n, scale = 150, 0.7 / math.sqrt(D)
@@ -242,7 +242,7 @@ def test_paged_prefill_batch_after_decode_rows(where):
 def test_paged_decode(where, H, G, D, DV):
     """Contexts around page and step borders, the last rows of pages
     poisoned."""
-    scale, cap = 0.7 / math.sqrt(D), 12.0
+    scale = 0.7 / math.sqrt(D)
     ctxs = [1, 15, 16, 17, 31, 32, 33, 127, 128, 129, 161, 290]
     parts = [tuple(seen(t, where)
                    for t in attn_case(H, G, D, DV, c, scale, seed=c))
@@ -253,7 +253,7 @@ def test_paged_decode(where, H, G, D, DV):
     bt = i32([t.pages + [0] * (wide - len(t.pages)) for t in tables], where)
     picks = [(c - 1) // 7 * 7 for c in ctxs]    # a query with a key of its own
     q = torch.stack([p[0][i] for p, i in zip(parts, picks)])
-    for splits in (0, 1, 3):
+    for splits, cap in ((0, 12.0), (1, 50.0), (3, 300.0)):
         out = torch.zeros(len(ctxs), H * DV, device=where[0], dtype=where[1])
         ops.paged_decode(put(q, where), kp, vp, bt, i32(ctxs, where), out,
                          scale, cap, True, splits)
