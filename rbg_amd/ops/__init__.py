@@ -479,11 +479,14 @@ def router_logits(x, w) -> torch.Tensor:
 
 def expert_tile(x, w, top: int) -> int:
     """Rows per tile that suit x [T, K] through experts w [E, N, K]."""
-    rows = x.shape[0] * top / w.shape[0]        # per expert, on average
+    pairs = x.shape[0] * top
+    rows = pairs / w.shape[0]                   # per expert, on average
     if (not _on_gpu(x) or x.dtype == torch.float32 or w.shape[1] % 8 or
-            w.shape[2] % 8 or rows <= 16):
+            w.shape[2] % 8 or
+            # the chip would not be full of 64-column pieces
+            pairs * ((w.shape[1] + 63) // 64) < 256):
         return 16
-    return 32 if rows <= 32 else 128
+    return 32 if rows <= 20 else 64 if rows <= 40 else 128
 
 
 def moe_route(logits, correction, groups: int, keep: int, top: int,

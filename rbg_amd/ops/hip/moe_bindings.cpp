@@ -23,7 +23,7 @@ void launch_paged_rows(const PagedAttnArgs*, int, hipStream_t);
 void launch_router_logits(float*, const void*, const void*, int, int, int, int,
                           int, hipStream_t);
 int moe_max_experts();
-int moe_route_blocks(int, int);
+int moe_route_blocks(int);
 void launch_moe_route(const MoeRouteArgs*, hipStream_t);
 void launch_moe_gemm(const MoeGemmArgs*, int, int, hipStream_t);
 }
@@ -293,7 +293,7 @@ std::vector<Tensor> moe_route(Tensor logits, Tensor correction, int64_t groups,
   p.ids = ids.data_ptr<int>(); p.inv = inv.data_ptr<int>();
   p.rows = rows.data_ptr<int>(); p.tiles = tiles.data_ptr<int>();
   p.count = count.data_ptr<int>();
-  const int blocks = moe_route_blocks((int)T, (int)E);
+  const int blocks = moe_route_blocks((int)T);
   Tensor part;
   if (blocks) {
     part = torch::empty({blocks, E}, i);

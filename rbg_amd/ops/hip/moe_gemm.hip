@@ -7,12 +7,14 @@
 //           from global memory into LDS (rows may be gathered: every lane brings
 //           its own address).  One buffer: the other workgroups of the CU, three
 //           or four of them, compute while one waits, which measured better than
-//           two buffers with half the workgroups.  16-byte pieces of a row are
-//           stored swizzled by the row: fragment reads are free of conflicts.
-//   skinny  decode: 16 * MT rows against 16 * NN weight rows, whose fragments go
-//           from global memory into the MFMAs; waves split K and meet in LDS.
+//           two buffers with half the workgroups.
+//   stream  32 or 64 rows x 64 columns, several stages of LDS deep: decode
+//           batches, whose time is the weights' way from memory.
+//   skinny  up to 16 rows x 16 columns, weight fragments from global memory into
+//           the MFMAs, waves split K and meet in LDS: batches whose experts do
+//           not fill the chip otherwise.
 //   rows    any sizes, bf16 or f32: a thread per column, up to 16 rows at once.
-#include "mfma_util.h"
+#include "lds_stream.h"
 #include "moe_args.h"
 #include "vec_io.h"
 
@@ -32,21 +34,7 @@ DEV_INLINE void put4(const MoeGemmArgs& p, const size_t row, const int n,
   *reinterpret_cast<uint2*>((__hip_bfloat16*)p.out + row * p.n + n) = o.u;
 }
 
-constexpr int BM = 128, BK = 64, GT = 256;
-
-// 16 bytes per lane from base + off to 16 * lane past the wave's LDS address.
-// Not the compiler's builtin: it would wait for the data before any LDS read.
-DEV_INLINE void load_lds16(const uint32_t off, const void* base,
-                           const uint32_t lds) {
-  asm volatile("s_mov_b32 m0, %2\n\ts_nop 0\n\t"
-               "global_load_lds_dwordx4 %0, %1"
-               :: "v"(off), "s"(base), "s"(lds) : "memory", "m0");
-}
-
-// what this wave asked for is in LDS, and every wave is here
-DEV_INLINE void landed_barrier() {
-  asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
-}
+constexpr int BM = 128, GT = 256;
 
 // 4 waves of 64 rows x BN / 2 columns
 template <int BN, int OCC>
@@ -71,9 +59,8 @@ void moe_tiled_kernel(const MoeGemmArgs p) {
   const int n0 = in / gn * BN;
   const int expert = tile[0], row0 = tile[1], rows = tile[2];
 
-  // wave-instruction c brings rows c*32 + wave*8 .. +7, 8 pieces of 16 bytes
-  // each; a lane's row is fixed modulo 8, so its piece number is too
-  const int lr = lane >> 3, piece = (lane & 7) ^ lr;
+  // wave instruction c brings rows c*32 + wave*8 .. +7
+  const int lr = lane >> 3, piece = stage_piece();
   uint32_t xo[XI], wo[WI];                      // bytes; the host checks sizes
 #pragma unroll
   for (int c = 0; c < XI; ++c) {
@@ -109,7 +96,7 @@ void moe_tiled_kernel(const MoeGemmArgs p) {
     const mf_bf8 z = {};
 #pragma unroll
     for (int h = 0; h < 2; ++h) {
-      const int at = ((h * 4 + gs) ^ (gl & 7)) * 8;
+      const int at = stage_at(h);
       mf_bf8 a[TN], b[4];
 #pragma unroll
       for (int i = 0; i < TN; ++i) a[i] = frag8(ws + i * 16 * BK + at);
@@ -134,18 +121,18 @@ void moe_tiled_kernel(const MoeGemmArgs p) {
   const int nk = p.k / BK, rest = p.k % BK;
   for (int kt = 0; kt < nk; ++kt) {
     issue(kt);
-    landed_barrier();
+    landed_barrier<0>();
     compute(BK);
-    landed_barrier();                           // everyone has read
+    landed_barrier<0>();                           // everyone has read
   }
   if (rest) {                                   // pieces past the end: the last
-    const int back = max(piece * 8 - (rest - 8), 0) * 2;
+    const uint32_t back = tail_back(rest);
 #pragma unroll
     for (int c = 0; c < XI; ++c) xo[c] -= back;
 #pragma unroll
     for (int c = 0; c < WI; ++c) wo[c] -= back;
     issue(nk);
-    landed_barrier();
+    landed_barrier<0>();
     compute(rest);
   }
 #pragma unroll
@@ -166,77 +153,91 @@ void moe_tiled(const MoeGemmArgs& p, hipStream_t s) {
   moe_tiled_kernel<BN, OCC><<<8 * ((p.max_tiles * nb + 7) / 8), GT, 0, s>>>(p);
 }
 
+template <int SM, int NB>
+__global__ __launch_bounds__(256) void moe_stream_kernel(const MoeGemmArgs p) {
+  using Stream = LdsStream<SM, NB>;
+  extern __shared__ __attribute__((aligned(16))) char stream_smem[];
+  if ((int)blockIdx.y >= *p.count) return;
+  const int* tile = p.tiles + (size_t)blockIdx.y * 3;
+  const int expert = tile[0], row0 = tile[1], rows = tile[2];
+  const int n0 = blockIdx.x * 64, piece = stage_piece();
+  uint32_t xo[Stream::XI], wo[2];
+#pragma unroll
+  for (int c = 0; c < Stream::XI; ++c) {
+    const int at = row0 + min(c * 32 + Stream::row(), rows - 1);
+    xo[c] = ((uint32_t)(p.rows != nullptr ? p.rows[at] : at) * p.k +
+             piece * 8) * 2;
+  }
+#pragma unroll
+  for (int c = 0; c < 2; ++c)
+    wo[c] = ((uint32_t)min(n0 + c * 32 + Stream::row(), p.n - 1) * p.k +
+             piece * 8) * 2;
+  f32x4 acc[Stream::TM];
+  Stream::run(p.x, xo, (const char*)p.w + (size_t)expert * p.n * p.k * 2, wo,
+              p.k, (blockIdx.x + 5 * blockIdx.y) % ((p.k + BK - 1) / BK),
+              (rows + 15) / 16, stream_smem, acc);
+  const int n = n0 + (threadIdx.x >> 6) * 16 + ((threadIdx.x & 63) >> 4) * 4;
+#pragma unroll
+  for (int j = 0; j < Stream::TM; ++j) {
+    const int r = j * 16 + (threadIdx.x & 15);
+    if (r < rows && n < p.n) put4(p, row0 + r, n, acc[j]);
+  }
+}
+
+template <int SM, int NB>
+void moe_stream(const MoeGemmArgs& p, hipStream_t s) {
+  constexpr int lds = LdsStream<SM, NB>::BYTES;
+  static bool once = false;
+  if (!once) {
+    (void)hipFuncSetAttribute((const void*)moe_stream_kernel<SM, NB>,
+                              hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    once = true;
+  }
+  const dim3 grid((p.n + 63) / 64, p.max_tiles);
+  moe_stream_kernel<SM, NB><<<grid, 256, lds, s>>>(p);
+}
+
 constexpr int SW = 4;                           // waves of a skinny workgroup
 constexpr int UN = 4;                           // 32-k steps in flight
 
-template <int MT, int NN>
 __global__ __launch_bounds__(SW * 64) void moe_skinny_kernel(
     const MoeGemmArgs p) {
-  __shared__ f32x4 red[SW][NN * MT][64];
+  __shared__ f32x4 red[SW][64];
   if ((int)blockIdx.y >= *p.count) return;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int gl = lane & 15, gs = lane >> 4;
   const int* tile = p.tiles + (size_t)blockIdx.y * 3;
   const int expert = tile[0], row0 = tile[1], rows = tile[2];
-  const int n0 = blockIdx.x * 16 * NN;
-  const __hip_bfloat16* wr[NN];
-#pragma unroll
-  for (int n = 0; n < NN; ++n)
-    wr[n] = (const __hip_bfloat16*)p.w +
-            ((size_t)expert * p.n + min(n0 + n * 16 + gl, p.n - 1)) * p.k;
-  const __hip_bfloat16* xr[MT];
-#pragma unroll
-  for (int t = 0; t < MT; ++t) {
-    const int r = row0 + min(t * 16 + gl, rows - 1);
-    xr[t] = (const __hip_bfloat16*)p.x +
-            (size_t)(p.rows != nullptr ? p.rows[r] : r) * p.k;
-  }
-  f32x4 acc[NN][MT];
-#pragma unroll
-  for (int n = 0; n < NN; ++n)
-#pragma unroll
-    for (int t = 0; t < MT; ++t) acc[n][t] = {0.f, 0.f, 0.f, 0.f};
+  const int n0 = blockIdx.x * 16, at = row0 + min(gl, rows - 1);
+  const __hip_bfloat16* wr = (const __hip_bfloat16*)p.w +
+      ((size_t)expert * p.n + min(n0 + gl, p.n - 1)) * p.k;
+  const __hip_bfloat16* xr = (const __hip_bfloat16*)p.x +
+      (size_t)(p.rows != nullptr ? p.rows[at] : at) * p.k;
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
   const int per = ((p.k + SW * 32 - 1) / (SW * 32)) * 32;
   const int kb = wave * per, ke = min(kb + per, p.k);
   for (int k0 = kb; k0 < ke; k0 += 32 * UN) {
     // unconditional clamped loads, all before the first product: a guard would
     // serialise them
-    mf_bf8 wf[UN][NN], xf[UN][MT];
+    mf_bf8 wf[UN], xf[UN];
     const mf_bf8 z = {};
 #pragma unroll
     for (int u = 0; u < UN; ++u) {
       const int kc = min(k0 + u * 32 + gs * 8, p.k - 8);
-#pragma unroll
-      for (int n = 0; n < NN; ++n) wf[u][n] = frag8(wr[n] + kc);
-#pragma unroll
-      for (int t = 0; t < MT; ++t) xf[u][t] = frag8(xr[t] + kc);
+      wf[u] = frag8(wr + kc);
+      xf[u] = frag8(xr + kc);
     }
 #pragma unroll
-    for (int u = 0; u < UN; ++u) {
-      const bool on = k0 + u * 32 + gs * 8 < ke;
-#pragma unroll
-      for (int n = 0; n < NN; ++n) {
-        const mf_bf8 w = on ? wf[u][n] : z;
-#pragma unroll
-        for (int t = 0; t < MT; ++t)
-          acc[n][t] = mfma_bf16_k32(w, xf[u][t], acc[n][t]);
-      }
-    }
+    for (int u = 0; u < UN; ++u)
+      acc = mfma_bf16_k32(k0 + u * 32 + gs * 8 < ke ? wf[u] : z, xf[u], acc);
   }
-#pragma unroll
-  for (int n = 0; n < NN; ++n)
-#pragma unroll
-    for (int t = 0; t < MT; ++t) red[wave][n * MT + t][lane] = acc[n][t];
+  red[wave][lane] = acc;
   __syncthreads();
-  for (int i = threadIdx.x; i < NN * MT * 64; i += SW * 64) {
-    const int u = i >> 6, ln = i & 63;
-    f32x4 s = red[0][u][ln];
+  if (wave > 0) return;
 #pragma unroll
-    for (int wv = 1; wv < SW; ++wv) s += red[wv][u][ln];
-    const int r = (u % MT) * 16 + (ln & 15);
-    const int n = n0 + (u / MT) * 16 + (ln >> 4) * 4;
-    if (r < rows && n < p.n) put4(p, row0 + r, n, s);
-  }
+  for (int wv = 1; wv < SW; ++wv) acc += red[wv][lane];
+  const int n = n0 + gs * 4;
+  if (gl < rows && n < p.n) put4(p, row0 + gl, n, acc);
 }
 
 template <typename T>
@@ -279,17 +280,12 @@ extern "C" void launch_moe_gemm(const MoeGemmArgs* p, int f32, int vec,
       moe_rows_kernel<__hip_bfloat16><<<grid, 256, 0, s>>>(*p);
     }
   } else if (p->tile <= 16) {
-    // wide workgroups once the experts alone fill the chip
-    if (p->max_tiles >= 32) {
-      moe_skinny_kernel<1, 2><<<dim3((p->n + 31) / 32, p->max_tiles), SW * 64,
-                                0, s>>>(*p);
-    } else {
-      moe_skinny_kernel<1, 1><<<dim3((p->n + 15) / 16, p->max_tiles), SW * 64,
-                                0, s>>>(*p);
-    }
+    moe_skinny_kernel<<<dim3((p->n + 15) / 16, p->max_tiles), SW * 64, 0,
+                        s>>>(*p);
   } else if (p->tile <= 32) {
-    moe_skinny_kernel<2, 2><<<dim3((p->n + 31) / 32, p->max_tiles), SW * 64, 0,
-                              s>>>(*p);
+    moe_stream<32, 4>(*p, s);
+  } else if (p->tile <= 64) {
+    moe_stream<64, 4>(*p, s);
   } else {
     // the wide form is 1.08 times as fast per column
     const long wide = (p->n + 191) / 192 * 192L, slim = (p->n + 127) / 128 * 128L;

@@ -1,8 +1,7 @@
 // Routing of tokens to experts (gfx950).
 //
-//   logits   x W^T with f32 sums: a workgroup takes 16 * MT tokens and one or
-//            four tiles of 16 experts, its waves split K and meet in LDS.  W
-//            rows are MFMA A fragments: lanes are tokens, registers experts.
+//   logits   x W^T with f32 sums.  W rows are MFMA A fragments: lanes are tokens,
+//            registers experts.
 //   choose   one wave per token: sigmoid, correction, the two best of each group
 //            of neighbours, the best groups, the best experts of those.  Ranks
 //            are counted, not sorted: an expert's rank is the number of experts
@@ -10,9 +9,9 @@
 //            place is filled exactly once whatever the scores are.
 //   lay out  pairs (token, choice) counted per expert, offsets by a scan, tiles
 //            of one expert each, and the permutation: one workgroup, together
-//            with the choice for decode batches; for prompts the counting and
-//            the permutation are spread over blocks of 64 tokens.
-#include "mfma_util.h"
+//            with the choice for small batches; for prompts the counting and the
+//            permutation are spread over blocks of tokens.
+#include "lds_stream.h"
 #include "moe_args.h"
 #include "vec_io.h"
 
@@ -20,61 +19,73 @@ namespace {
 
 constexpr int UN = 4;                           // 32-k steps in flight
 
-// EW * KW waves: EW tiles of 16 experts (which find the tokens' rows in L1), KW
-// slices of K
-template <int MT, int EW, int KW>
-__global__ __launch_bounds__(EW * KW * 64) void router_logits_kernel(
+// decode batches: 8 waves split K
+__global__ __launch_bounds__(512) void router_skinny_kernel(
     float* __restrict__ out, const __hip_bfloat16* __restrict__ x,
     const __hip_bfloat16* __restrict__ w, const int tokens, const int experts,
     const int k_len) {
-  __shared__ f32x4 red[KW][EW][MT][64];
+  constexpr int KW = 8;
+  __shared__ f32x4 red[KW][64];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int gl = lane & 15, gs = lane >> 4;
-  const int ew = wave % EW, kw = wave / EW;
-  const int e0 = (blockIdx.x * EW + ew) * 16, t0 = blockIdx.y * 16 * MT;
+  const int e0 = blockIdx.x * 16, t0 = blockIdx.y * 16;
   const __hip_bfloat16* wr = w + (size_t)min(e0 + gl, experts - 1) * k_len;
-  const __hip_bfloat16* xr[MT];
-#pragma unroll
-  for (int t = 0; t < MT; ++t)
-    xr[t] = x + (size_t)min(t0 + t * 16 + gl, tokens - 1) * k_len;
-  f32x4 acc[MT];
-#pragma unroll
-  for (int t = 0; t < MT; ++t) acc[t] = {0.f, 0.f, 0.f, 0.f};
+  const __hip_bfloat16* xr = x + (size_t)min(t0 + gl, tokens - 1) * k_len;
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
   const int per = ((k_len + KW * 32 - 1) / (KW * 32)) * 32;
-  const int kb = kw * per, ke = min(kb + per, k_len);
+  const int kb = wave * per, ke = min(kb + per, k_len);
   for (int k0 = kb; k0 < ke; k0 += 32 * UN) {
     // unconditional clamped loads, all before the first product
-    mf_bf8 wf[UN], xf[UN][MT];
+    mf_bf8 wf[UN], xf[UN];
     const mf_bf8 z = {};
 #pragma unroll
     for (int u = 0; u < UN; ++u) {
       const int kc = min(k0 + u * 32 + gs * 8, k_len - 8);
       wf[u] = frag8(wr + kc);
-#pragma unroll
-      for (int t = 0; t < MT; ++t) xf[u][t] = frag8(xr[t] + kc);
+      xf[u] = frag8(xr + kc);
     }
 #pragma unroll
-    for (int u = 0; u < UN; ++u) {
-      const mf_bf8 w1 = k0 + u * 32 + gs * 8 < ke ? wf[u] : z;
-#pragma unroll
-      for (int t = 0; t < MT; ++t)
-        acc[t] = mfma_bf16_k32(w1, xf[u][t], acc[t]);
-    }
+    for (int u = 0; u < UN; ++u)
+      acc = mfma_bf16_k32(k0 + u * 32 + gs * 8 < ke ? wf[u] : z, xf[u], acc);
   }
-#pragma unroll
-  for (int t = 0; t < MT; ++t) red[kw][ew][t][lane] = acc[t];
+  red[wave][lane] = acc;
   __syncthreads();
-  for (int i = threadIdx.x; i < EW * MT * 64; i += EW * KW * 64) {
-    const int ln = i & 63, t = (i >> 6) % MT, we = (i >> 6) / MT;
-    f32x4 s = {0.f, 0.f, 0.f, 0.f};
+  if (wave > 0) return;
 #pragma unroll
-    for (int kk = 0; kk < KW; ++kk) s += red[kk][we][t][ln];
-    const int tok = t0 + t * 16 + (ln & 15);
-    const int e = (blockIdx.x * EW + we) * 16 + (ln >> 4) * 4;
+  for (int kk = 1; kk < KW; ++kk) acc += red[kk][lane];
+  const int e = e0 + gs * 4;
+  if (t0 + gl >= tokens) return;
+#pragma unroll
+  for (int r = 0; r < 4; ++r)
+    if (e + r < experts) out[(size_t)(t0 + gl) * experts + e + r] = acc[r];
+}
+
+// prompts: 32 tokens x 64 experts through LDS
+using RouterStream = LdsStream<32, 4>;
+
+__global__ __launch_bounds__(256) void router_stream_kernel(
+    float* __restrict__ out, const __hip_bfloat16* __restrict__ x,
+    const __hip_bfloat16* __restrict__ w, const int tokens, const int experts,
+    const int k_len) {
+  __shared__ __attribute__((aligned(16))) char smem[RouterStream::BYTES];
+  const int e0 = blockIdx.x * 64, t0 = blockIdx.y * 32;
+  const int piece = stage_piece(), row = RouterStream::row();
+  const uint32_t xo[1] = {
+      ((uint32_t)min(row, tokens - 1 - t0) * k_len + piece * 8) * 2};
+  const uint32_t wo[2] = {
+      ((uint32_t)min(e0 + row, experts - 1) * k_len + piece * 8) * 2,
+      ((uint32_t)min(e0 + 32 + row, experts - 1) * k_len + piece * 8) * 2};
+  f32x4 acc[2];
+  RouterStream::run(x + (size_t)t0 * k_len, xo, w, wo, k_len,
+                    blockIdx.y % ((k_len + BK - 1) / BK), 2, smem, acc);
+  const int e = e0 + (threadIdx.x >> 6) * 16 + ((threadIdx.x & 63) >> 4) * 4;
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    const int tok = t0 + j * 16 + (threadIdx.x & 15);
     if (tok >= tokens) continue;
 #pragma unroll
     for (int r = 0; r < 4; ++r)
-      if (e + r < experts) out[(size_t)tok * experts + e + r] = s[r];
+      if (e + r < experts) out[(size_t)tok * experts + e + r] = acc[j][r];
   }
 }
 
@@ -253,11 +264,32 @@ __global__ __launch_bounds__(NT) void route_small_kernel(const MoeRouteArgs p) {
   place_pairs<NT>(p, cursor, 0, p.tokens * p.top);
 }
 
-// 64 tokens' choice, and how often it took each expert: part [blocks, experts]
-constexpr int BT = 64, CN = 1024;
+// middling batches: the choice, 4 tokens a workgroup, then the layout in one
+__global__ __launch_bounds__(256) void choose_kernel(const MoeRouteArgs p) {
+  extern __shared__ float route_smem[];
+  const int wave = threadIdx.x >> 6, t = blockIdx.x * 4 + wave;
+  if (t < p.tokens)                             // whole waves
+    choose(p, t, route_smem + wave * choice_floats(p.experts, p.groups),
+           threadIdx.x & 63);
+}
+
+constexpr int CN = 1024;
+
+__global__ __launch_bounds__(CN) void lay_out_kernel(const MoeRouteArgs p) {
+  extern __shared__ int lay_smem[];
+  int* cursor = lay_smem + p.experts;
+  count_pairs<CN>(p, lay_smem, 0, p.tokens * p.top);
+  offsets<CN>(p, lay_smem, cursor, cursor + p.experts);
+  place_pairs<CN>(p, cursor, 0, p.tokens * p.top);
+}
+
+// prompts: BT tokens' choice, and how often it took each expert: part [blocks,
+// experts]
+constexpr int BT = 32;
 
 template <int NT>
-__global__ __launch_bounds__(NT) void choose_kernel(const MoeRouteArgs p) {
+__global__ __launch_bounds__(NT) void choose_count_kernel(
+    const MoeRouteArgs p) {
   extern __shared__ float route_smem[];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   float* mine = route_smem + wave * choice_floats(p.experts, p.groups);
@@ -287,7 +319,7 @@ __global__ __launch_bounds__(CN) void offsets_kernel(const MoeRouteArgs p,
   const int b0 = min(r * len, blocks), b1 = min(b0 + len, blocks);
   int n = 0;
   if (on) {
-#pragma unroll 4
+#pragma unroll 8
     for (int b = b0; b < b1; ++b) n += p.part[(size_t)b * p.experts + e];
     run[r * p.experts + e] = n;
   }
@@ -305,7 +337,7 @@ __global__ __launch_bounds__(CN) void offsets_kernel(const MoeRouteArgs p,
   offsets<CN>(p, count, cursor, scan);
   if (on) {
     int at = cursor[e] + run[r * p.experts + e];
-#pragma unroll 4
+#pragma unroll 8
     for (int b = b0; b < b1; ++b) {
       const int v = p.part[(size_t)b * p.experts + e];
       p.part[(size_t)b * p.experts + e] = at;
@@ -334,12 +366,12 @@ void launch_router_logits(float* out, const void* x, const void* w, int tokens,
     const __hip_bfloat16 *xb = (const __hip_bfloat16*)x,
                          *wb = (const __hip_bfloat16*)w;
     if (tokens <= 512) {
-      router_logits_kernel<1, 1, 8>
+      router_skinny_kernel
           <<<dim3((experts + 15) / 16, (tokens + 15) / 16), 512, 0, s>>>(
               out, xb, wb, tokens, experts, k);
     } else {
-      router_logits_kernel<2, 4, 4>
-          <<<dim3((experts + 63) / 64, (tokens + 31) / 32), 1024, 0, s>>>(
+      router_stream_kernel
+          <<<dim3((experts + 63) / 64, (tokens + 31) / 32), 256, 0, s>>>(
               out, xb, wb, tokens, experts, k);
     }
     return;
@@ -358,32 +390,32 @@ void launch_router_logits(float* out, const void* x, const void* w, int tokens,
 
 int moe_max_experts() { return 1024; }
 
-// blocks of tokens that count on their own; 0: one workgroup does everything
-int moe_route_blocks(int tokens, int experts) {
-  return tokens <= 64 && experts <= 512 ? 0 : (tokens + BT - 1) / BT;
+// blocks of tokens that count on their own
+int moe_route_blocks(int tokens) {
+  return tokens <= 512 ? 0 : (tokens + BT - 1) / BT;
 }
 
 void launch_moe_route(const MoeRouteArgs* p, hipStream_t s) {
-  const int blocks = moe_route_blocks(p->tokens, p->experts);
+  const int blocks = moe_route_blocks(p->tokens);
   const size_t own = sizeof(float) * choice_floats(p->experts, p->groups);
-  if (blocks == 0) {
-    const size_t lay = sizeof(int) * (2 * p->experts + 32);
-    if (p->tokens <= 4) {
-      route_small_kernel<256><<<1, 256, own * 4 > lay ? own * 4 : lay, s>>>(*p);
+  const size_t lay = sizeof(int) * (2 * p->experts + 32);
+  if (blocks > 0) {
+    if (own * 16 <= 65536) {
+      choose_count_kernel<1024><<<blocks, 1024, own * 16, s>>>(*p);
     } else {
-      route_small_kernel<1024><<<1, 1024, own * 16 > lay ? own * 16 : lay,
-                                 s>>>(*p);
+      choose_count_kernel<256><<<blocks, 256, own * 4, s>>>(*p);
     }
-    return;
-  }
-  if (own * 16 <= 65536) {
-    choose_kernel<1024><<<blocks, 1024, own * 16, s>>>(*p);
+    offsets_kernel<<<1, CN, lay + sizeof(int) * CN, s>>>(*p, blocks);
+    place_kernel<<<blocks, 256, sizeof(int) * p->experts, s>>>(*p);
+  } else if (p->tokens <= 4) {
+    route_small_kernel<256><<<1, 256, own * 4 > lay ? own * 4 : lay, s>>>(*p);
+  } else if (p->tokens <= 16 && own * 16 <= 65536) {
+    route_small_kernel<1024><<<1, 1024, own * 16 > lay ? own * 16 : lay,
+                               s>>>(*p);
   } else {
-    choose_kernel<256><<<blocks, 256, own * 4, s>>>(*p);
+    choose_kernel<<<(p->tokens + 3) / 4, 256, own * 4, s>>>(*p);
+    lay_out_kernel<<<1, CN, lay, s>>>(*p);
   }
-  offsets_kernel<<<1, CN, sizeof(int) * (2 * p->experts + 2 * CN / 64 + CN),
-                   s>>>(*p, blocks);
-  place_kernel<<<blocks, 256, sizeof(int) * p->experts, s>>>(*p);
 }
 
 }  // extern "C"

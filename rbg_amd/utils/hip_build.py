@@ -67,8 +67,8 @@ HIP_HEADERS = {
     "_hip_ops": ["common.h", "gemm_bindings.h"],
     "_hip_mix": ["bind_util.h", "common.h", "gemm_bindings.h", "mfma_util.h",
                  "mix_args.h", "vec_io.h"],
-    "_hip_moe": ["bind_util.h", "common.h", "gemm_bindings.h", "mfma_util.h",
-                 "moe_args.h", "vec_io.h"],
+    "_hip_moe": ["bind_util.h", "common.h", "gemm_bindings.h", "lds_stream.h",
+                 "mfma_util.h", "moe_args.h", "vec_io.h"],
 }
 
 # model architecture -> the extension with its kernels (default: _hip_ops)

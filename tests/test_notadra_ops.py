@@ -299,7 +299,8 @@ def test_score_options_and_page_sizes(where, sink, cap):
 
 @pytest.mark.parametrize("where", WHERE)
 @pytest.mark.parametrize("T,E,K", [(1, 16, 48), (5, 8, 264), (70, 20, 64),
-                                   (600, 33, 128), (3, 7, 37)])
+                                   (600, 33, 128), (3, 7, 37),
+                                   (1000, 130, 200)])
 def test_router_logits(where, T, E, K):
     x, w = rnd(T, K), rnd(E, K, seed=1)
     out = ops.router_logits(put(x, where), put(w, where))
@@ -363,7 +364,7 @@ def test_route_places_everyone_whatever_the_scores():
     (1, 16, 3, 24, 48), (3, 4, 2, 40, 136), (20, 8, 2, 96, 256),
     (150, 4, 2, 136, 72), (400, 4, 3, 264, 200), (5, 6, 2, 13, 21),
     (130, 3, 3, 8, 8)])
-@pytest.mark.parametrize("tile", [16, 32, 128])
+@pytest.mark.parametrize("tile", [16, 32, 64, 128])
 def test_expert_linear(where, T, E, top, N, K, tile):
     """Gathered rows with the squared relu, then rows in expert order."""
     if tile > 16 and (where[1] == F32 or N % 8 or K % 8):
@@ -396,10 +397,11 @@ def test_tile_choice():
 
 @pytest.mark.gpu
 def test_tile_choice_by_load():
-    w = torch.zeros(64, 32, 32, device="cuda", dtype=BF16)
+    w = torch.zeros(64, 256, 32, device="cuda", dtype=BF16)
     x = torch.zeros(8192, 32, device="cuda", dtype=BF16)
     assert ops.expert_tile(x[:1], w, 8) == 16
-    assert ops.expert_tile(x[:256], w, 8) == 32
+    assert ops.expert_tile(x[:128], w, 8) == 32
+    assert ops.expert_tile(x[:256], w, 8) == 64
     assert ops.expert_tile(x, w, 8) == 128
     assert ops.expert_tile(x.float(), w.float(), 8) == 16
     odd = torch.zeros(64, 31, 32, device="cuda", dtype=BF16)
