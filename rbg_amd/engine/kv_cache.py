@@ -15,6 +15,7 @@ from __future__ import annotations
 
 from typing import Dict, List, Optional, Tuple
 
+import numpy as np
 import torch
 
 from .config import EngineConfig
@@ -182,13 +183,14 @@ class BlockTable:
         self.pages = list(pages)
         self.num_shared = len(pages)
 
-    def slots_for(self, start: int, count: int) -> List[int]:
+    def slots_for(self, start: int, count: int) -> np.ndarray:
         """Global slot ids (page*page_size + offset) for token positions
-        [start, start+count)."""
+        [start, start+count), int32."""
         self.ensure(start + count)
         ps = self.cache.page_size
-        return [self.pages[(start + i) // ps] * ps + (start + i) % ps
-                for i in range(count)]
+        pos = np.arange(start, start + count)
+        return (np.asarray(self.pages, dtype=np.int32)[pos // ps] * ps +
+                pos % ps).astype(np.int32)
 
     def release(self) -> None:
         if self.num_shared and self.cache.prefix is not None:

@@ -60,8 +60,9 @@ def run_one(model: ModelConfig, device: str, batch: int, prompt: int,
     gen = torch.Generator().manual_seed(5)
     prompts = torch.randint(0, model.vocab_size, (batch, prompt),
                             generator=gen).tolist()
-    # one prompt warms kernels and libraries up, then the timed prefill
-    eng.generate(prompts[:1], SamplingParams(max_new_tokens=1))
+    # a full step warms kernels and libraries up, then the timed prefill
+    eng.generate(prompts[:max(1, eng.cfg.max_prefill_tokens // prompt)],
+                 SamplingParams(max_new_tokens=1))
     for p in prompts:
         eng.add_request(p, SamplingParams(max_new_tokens=steps + warmup + 32))
     t0 = _sync(device)

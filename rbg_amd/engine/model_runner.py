@@ -55,6 +55,9 @@ class ModelRunner:
     def _i32(self, data) -> torch.Tensor:
         return torch.tensor(data, dtype=torch.int32, device=self.device)
 
+    def _join(self, parts: List[np.ndarray]) -> torch.Tensor:
+        return torch.from_numpy(np.concatenate(parts)).to(self.device)
+
     # one sequence's part of a varlen step: tokens at [start, start + len)
     Chunk = Tuple[Sequence, int, List[int]]
 
@@ -72,11 +75,12 @@ class ModelRunner:
             single = [len(t) == 1 and start > 0 for _, start, t in chunks]
             num_decode = sum(single)
             order.sort(key=lambda i: not single[i])
-        tokens: List[int] = []
-        prev: List[int] = []
-        positions: List[int] = []
-        slots: List[int] = []
-        gather: List[int] = []
+        # numpy pieces: a step of many tokens is on the GPU's critical path
+        tokens: List[np.ndarray] = []
+        prev: List[np.ndarray] = []
+        positions: List[np.ndarray] = []
+        slots: List[np.ndarray] = []
+        gather: List[np.ndarray] = []
         cu = [0]
         cu_k = [0]
         first_row = [0] * len(chunks)
@@ -85,28 +89,26 @@ class ModelRunner:
         for i in order:
             seq, start, toks = chunks[i]
             end = start + len(toks)
-            tokens.extend(toks)
+            tokens.append(np.asarray(toks, dtype=np.int64))
             if self.model.needs_prev:
-                prev.append(seq.token_at(start - 1))
-                prev.extend(toks[:-1])
-            positions.extend(range(start, end))
-            slots.extend(seq.block_table.slots_for(start, end - start))
+                prev += [np.array([seq.token_at(start - 1)]), tokens[-1][:-1]]
+            positions.append(np.arange(start, end, dtype=np.int32))
+            slots.append(seq.block_table.slots_for(start, end - start))
             first_row[i] = cu[-1]
             cu.append(cu[-1] + (end - start))
             cu_k.append(cu_k[-1] + end)
             if any_past and not self.model.varlen:
-                gather.extend(seq.block_table.slots_for(0, end))
+                gather.append(seq.block_table.slots_for(0, end))
             starts.append(start)
             ends.append(end)
             tables.append(seq.block_table)
         batch = ForwardBatch(
             mode="prefill",
-            positions=self._i32(positions),
-            slot_mapping=self._i32(slots),
+            positions=self._join(positions),
+            slot_mapping=self._join(slots),
             cu_seqlens=self._i32(cu))
         if self.model.needs_prev:
-            batch.prev_tokens = torch.tensor(prev, dtype=torch.int64,
-                                             device=self.device)
+            batch.prev_tokens = self._join(prev)
         if self.model.varlen:
             batch.starts = self._i32(starts)
             batch.state_slots = self._i32([t.state_slot for t in tables])
@@ -121,17 +123,16 @@ class ModelRunner:
                 batch.context_lens = self._i32(ends[:num_decode])
         elif any_past:
             batch.cu_seqlens_k = self._i32(cu_k)
-            batch.kv_gather_slots = self._i32(gather)
+            batch.kv_gather_slots = self._join(gather)
         # decode inputs that were left on the device are behind now
         self._dstate = None
         hidden_in = None
         if not self.pp.first:
             hidden_in = self.pp.recv_prev(
-                (len(tokens), self.cfg.model.hidden_size),
+                (cu[-1], self.cfg.model.hidden_size),
                 self.model.stream_dtype, self.device)
-        hidden = self.model.forward(
-            torch.tensor(tokens, dtype=torch.int64, device=self.device),
-            batch, self.cache, hidden=hidden_in)
+        hidden = self.model.forward(self._join(tokens), batch, self.cache,
+                                    hidden=hidden_in)
         if not self.pp.last:
             self.pp.send_next(hidden)
         return hidden, first_row
