@@ -35,7 +35,7 @@ def main(argv=None) -> int:
     if args.device == "cuda":
         # compile what this family runs on, before anything imports it
         from ..utils import hip_build
-        hip_build.ensure(hip_build.EXTENSION_OF.get(arch, "_hip_ops"))
+        hip_build.ensure(*hip_build.EXTENSIONS_OF.get(arch, ("_hip_ops",)))
     from ..engine.trace import TraceSession
     from ..models.registry import load_config
     import torch

@@ -11,8 +11,11 @@ for the recurrence (with decay, gates, unit keys and head norm inside) and for
 the attention (with window, softmax and, in prefill, the output gate inside).
 Tensor parallelism shards heads and feed-forward columns.
 
-Parts of a design that norms each branch before adding it (``PagedAttention``,
-``SparseExperts``) apply their own output projection instead.
+Parts of a design that norms or gates each branch before adding it
+(``PagedAttention``, ``SparseExperts``, and those after them) apply their own
+output projection instead.  ``GatedDeltaRule``, ``DifferentialAttention`` and
+``GatedSilu`` leave the input projection to the layer as ``parts``: where every
+sublayer reads one norm, a layer has a single input GEMM.
 """
 from __future__ import annotations
 
@@ -64,6 +67,19 @@ class FusedProjection(nn.Module):
     def slice(self, y: torch.Tensor, name: str) -> torch.Tensor:
         at, n = self.cols[name]
         return y[:, at:at + n]
+
+
+Parts = List[Tuple[str, torch.Tensor]]
+
+
+def pad8(t: torch.Tensor, dim: int = 0) -> torch.Tensor:
+    """t with zeros up to a multiple of 8 along ``dim``."""
+    n = -t.shape[dim] % 8
+    if not n:
+        return t
+    shape = list(t.shape)
+    shape[dim] = n
+    return torch.cat([t, t.new_zeros(shape)], dim=dim)
 
 
 class GeneralDelta(nn.Module):
@@ -338,3 +354,245 @@ class SparseExperts(nn.Module):
                               self.top, ops.expert_tile(x, self.up, self.top))
         h = ops.expert_linear(x, self.up, route, gather=True, relu2=True)
         return ops.expert_linear(h, self.down, route), route
+
+
+class GatedDeltaRule(nn.Module):
+    """Gated delta rule behind a short convolution, with one decay per head or
+    (``per_channel``) one per head and key channel from a low-rank map, grouped
+    query/key heads, a head norm and an output gate (silu, or a sigmoid of a
+    low-rank map)."""
+
+    unit_eps = 1e-6                 # inside the root of q's and k's norms
+
+    def __init__(self, spec: Dict[str, Any], width: int, eps: float,
+                 src: WeightSource, prefix: str, tp, dtype: torch.dtype,
+                 per_channel: bool, rank: int):
+        super().__init__()
+        heads, kv_heads = int(spec["heads"]), int(spec["kv_heads"])
+        if heads % kv_heads:
+            raise ValueError(f"{heads} heads over {kv_heads} key heads")
+        assert heads % tp.size == 0 and kv_heads % tp.size == 0, \
+            "TP degree must divide head counts"
+        self.heads, self.kv_heads = heads // tp.size, kv_heads // tp.size
+        self.dim, self.vdim = int(spec["dim"]), int(spec["vdim"])
+        self.taps, self.eps, self.dtype = int(spec["conv"]), eps, dtype
+        self.per_channel = per_channel
+        qk, vo, f32 = kv_heads * self.dim, heads * self.vdim, torch.float32
+
+        def take(name, shape, init="linear"):
+            return src.take(prefix + name, shape, init)
+
+        def mine(t, dim=0):
+            return shard(t, tp, dim)
+        self.parts: Parts = []
+        conv = []
+        for name, n in (("q", qk), ("k", qk), ("v", vo)):
+            self.parts.append((name, mine(take(name, (n, width)))))
+            # [taps, channels]; zero columns where the projection has zero rows
+            conv.append(pad8(mine(take(name + ".conv", (n, self.taps),
+                                       "conv"))).T)
+        self.conv_w = param(torch.cat(conv, dim=1), f32)
+        self.parts.append(("b", mine(take("b", (heads, width)))))
+        self.low: Optional[nn.Parameter] = None
+        if per_channel:
+            # both low-rank maps' second halves as one block-diagonal matrix
+            names = (("a1", "a2", heads * self.dim), ("g1", "g2", vo))
+            second = []
+            for one, two, n in names:
+                r = src.shape(prefix + one, (rank, width))[0]
+                self.parts.append((one, take(one, (r, width))))
+                second.append(pad8(pad8(mine(take(two, (n, r)))), 1))
+            self.low = param(torch.block_diag(*second), dtype)
+            self.gate_at = second[0].shape[0]
+        else:
+            self.parts.append(("a", mine(take("a", (heads, width)))))
+            self.parts.append(("g", mine(take("g", (vo, width)))))
+        bias = heads * self.dim if per_channel else heads
+        self.a_log = param(mine(take("A_log", (heads,), "normal")), f32)
+        self.dt_bias = param(mine(take("dt_bias", (bias,), "rate")), f32)
+        self.norm = param(take("norm", (self.vdim,), "ones"), f32)
+        self.w_out = param(mine(take("o", (width, vo)), 1), dtype)
+
+    def cache_spec(self) -> LayerCacheSpec:
+        state = {"delta": ((self.heads, self.dim, self.vdim), torch.float32)}
+        if self.taps > 1:
+            state["conv"] = ((self.taps, self.conv_w.shape[1]), self.dtype)
+        return LayerCacheSpec(state=state)
+
+    def forward(self, y: torch.Tensor, proj: FusedProjection,
+                batch: ForwardBatch, cache: StateCache,
+                layer: int) -> torch.Tensor:
+        width = self.conv_w.shape[1]
+        at = proj.offset("q")
+        offs = [proj.offset(n) - at for n in ("q", "k", "v")]
+        qkv, beta = y[:, at:at + width], proj.slice(y, "b")
+        if self.per_channel:
+            lo = proj.offset("a1")
+            z = ops.linear(y[:, lo:lo + self.low.shape[1]], self.low)
+            decay = z[:, :self.dt_bias.numel()]
+            gate = z[:, self.gate_at:self.gate_at + self.heads * self.vdim]
+        else:
+            decay, gate = proj.slice(y, "a"), proj.slice(y, "g")
+        p = ops.GatedDelta(self.a_log, self.dt_bias, self.norm, self.kv_heads,
+                           not self.per_channel, self.dim ** -0.5,
+                           self.unit_eps, self.eps)
+        state = cache.state(layer, "delta")
+        # one tap looks at nothing past: the ring is never read
+        ring = (cache.state(layer, "conv") if self.taps > 1 else
+                y.new_empty((cache.num_slots, 1, width)))
+        out = y.new_empty((y.shape[0], self.heads * self.vdim))
+        nd = y.shape[0] if batch.mode == "decode" else batch.num_decode
+        if nd:
+            ops.gated_delta(p, qkv[:nd], offs, beta[:nd], decay[:nd],
+                            gate[:nd], state, batch.state_slots[:nd], None,
+                            batch.starts[:nd], out[:nd],
+                            conv=(self.conv_w, ring))
+        if nd < y.shape[0]:
+            slots, starts = batch.state_slots[nd:], batch.starts[nd:]
+            layout, cu = batch.layout, batch.cu_prefill
+            c = ops.short_conv(
+                qkv[nd:], self.conv_w, ring,
+                layout.prefill_tiles(max(ops.CONV_TILE, self.taps)), cu,
+                starts, slots)
+            ops.gated_delta(p, c, offs, beta[nd:], decay[nd:], gate[nd:],
+                            state, slots, cu, starts, out[nd:],
+                            chunks=(layout.prefill_tiles(ops.DELTA_CHUNK),
+                                    layout.prefill_tile_cu(ops.DELTA_CHUNK)))
+        return ops.linear(out, self.w_out)
+
+
+class DifferentialAttention(nn.Module):
+    """Attention of two maps over paged keys and values, without positions,
+    through a sliding window; a head's output is the maps' weighed difference
+    over its root mean square.  With ``kv_from`` the keys and values are
+    another layer's."""
+
+    def __init__(self, spec: Dict[str, Any], width: int, eps: float,
+                 src: WeightSource, prefix: str, tp, dtype: torch.dtype):
+        super().__init__()
+        heads, kv_heads = int(spec["heads"]), int(spec["kv_heads"])
+        if heads % kv_heads:
+            raise ValueError(f"{heads} heads over {kv_heads} key heads")
+        assert heads % tp.size == 0 and kv_heads % tp.size == 0, \
+            "TP degree must divide head counts"
+        self.heads, self.kv_heads = heads // tp.size, kv_heads // tp.size
+        self.dim, self.vdim = int(spec["dim"]), int(spec["vdim"])
+        self.scale, self.eps = float(spec["scale"]), eps
+        mask = spec.get("mask") or {}
+        self.window = int(mask.get("size") or 0)     # 0: everything before
+        self.kv_from: Optional[int] = spec.get("kv_from")   # global layer
+        outs = {"q": heads * 2 * self.dim}
+        if self.kv_from is None:
+            outs.update(k=kv_heads * 2 * self.dim, v=kv_heads * self.vdim)
+        self.parts: Parts = [
+            (name, shard(src.take(prefix + name, (n, width)), tp))
+            for name, n in outs.items()]
+        self.diff = float(spec["diff"])
+        lq1, lk1, lq2, lk2 = (src.take(prefix + n, (self.dim,)).float()
+                              for n in ("lq1", "lk1", "lq2", "lk2"))
+        lam = (lq1 * lk1).sum().exp() - (lq2 * lk2).sum().exp() + self.diff
+        self.lam = param(lam.view(1), torch.float32)
+        self.w_out = param(shard(src.take(prefix + "o",
+                                          (width, heads * self.vdim)),
+                                 tp, dim=1), dtype)
+
+    def cache_spec(self) -> LayerCacheSpec:
+        if self.kv_from is not None:
+            return LayerCacheSpec()
+        return LayerCacheSpec(kv=(self.kv_heads, 2 * self.dim, self.vdim))
+
+    def forward(self, y: torch.Tensor, proj: FusedProjection,
+                batch: ForwardBatch, cache: StateCache,
+                kv_layer: int) -> torch.Tensor:
+        k, v = cache.kv_pages(kv_layer)
+        if self.kv_from is None:
+            ops.rope_store_paged(
+                y, None, None, batch.positions, batch.slot_mapping,
+                self.heads, 2 * self.dim, k, v,
+                [proj.offset(n) for n in ("q", "k", "v")])
+        q = proj.slice(y, "q").unflatten(1, (self.heads, 2 * self.dim))
+        out = y.new_empty((y.shape[0], self.heads * self.vdim))
+        kw = dict(window=self.window, diff=ops.Difference(
+            self.lam, 1.0 - self.diff, self.eps))
+        nd = y.shape[0] if batch.mode == "decode" else batch.num_decode
+        if nd:
+            ops.paged_decode(q[:nd], k, v, batch.block_tables,
+                             batch.context_lens, out[:nd], self.scale, 0.0,
+                             False, **kw)
+        if nd < y.shape[0]:
+            ops.paged_prefill(q[nd:], k, v, batch.layout.paged_view(),
+                              out[nd:], self.scale, 0.0, False, **kw)
+        return ops.linear(out, self.w_out)
+
+
+class GatedSilu(nn.Module):
+    """down(silu(gate x) * up x), all with biases; the last one is left to the
+    kernel that adds the branch (``bias``)."""
+
+    def __init__(self, spec: Dict[str, Any], width: int, src: WeightSource,
+                 prefix: str, tp, dtype: torch.dtype):
+        super().__init__()
+        ff = int(spec["ff"])
+        assert ff % tp.size == 0, "TP degree must divide the feed-forward"
+        f32 = torch.float32
+        self.parts: Parts = [
+            (n, shard(src.take(prefix + n, (ff, width)), tp))
+            for n in ("gate", "up")]
+        self.gate_b, self.up_b = (
+            param(shard(src.take(prefix + n + ".b", (ff,), "zeros"), tp), f32)
+            for n in ("gate", "up"))
+        self.down = param(shard(src.take(prefix + "down", (width, ff)), tp,
+                                dim=1), dtype)
+        self.bias = param(src.take(prefix + "down.b", (width,), "zeros"), f32)
+
+    def forward(self, h: torch.Tensor, y: torch.Tensor,
+                proj: FusedProjection):
+        act = y.new_empty((y.shape[0], self.down.shape[1]))
+        ops.silu_glu(proj.slice(y, "gate"), proj.slice(y, "up"), self.gate_b,
+                     self.up_b, act)
+        return ops.linear(act, self.down), None
+
+
+class GluExperts(nn.Module):
+    """Mixture of small gated feed-forwards down(silu(gate x) * up x); the
+    largest router logits are chosen and weighed by their softmax.
+
+    Tensor parallelism shards every expert's inner columns."""
+
+    bias = None
+    parts: Parts = []
+
+    def __init__(self, spec: Dict[str, Any], width: int, src: WeightSource,
+                 prefix: str, tp, dtype: torch.dtype):
+        super().__init__()
+        r, ff = spec["router"], int(spec["expert"]["ff"])
+        assert ff % tp.size == 0, "TP degree must divide the feed-forward"
+        n, self.top = int(r["experts"]), int(r["top"])
+        if not 1 <= self.top <= n:
+            raise ValueError(f"router: {n} experts, {self.top} chosen")
+
+        def take(e, name, shape, dim):
+            # columns up to a multiple of 8: silu(0) * 0 meets zeros in down
+            return pad8(shard(src.take(f"{prefix}e{e}.{name}", shape), tp,
+                              dim), dim)
+
+        def glu(e):
+            return ops.interleave_glu(take(e, "gate", (ff, width), 0),
+                                      take(e, "up", (ff, width), 0))
+        self.up = param(torch.stack([glu(e) for e in range(n)]), dtype)
+        self.down = param(torch.stack([take(e, "down", (width, ff), 1)
+                                       for e in range(n)]), dtype)
+        self.router = param(src.take(prefix + "router", (n, width)), dtype)
+        self.router_b = param(src.take(prefix + "router.b", (n,), "zeros"),
+                              torch.float32)
+
+    def forward(self, h: torch.Tensor, y: torch.Tensor,
+                proj: FusedProjection):
+        """Outputs of the chosen experts, one row per (token, choice) in
+        expert order, and the routing that weighs and finds them."""
+        logits = ops.router_logits(h, self.router)
+        route = ops.moe_route(logits, self.router_b, 1, 1, self.top,
+                              ops.expert_tile(h, self.up, self.top),
+                              softmax=True)
+        a = ops.expert_linear(h, self.up, route, gather=True, swiglu=True)
+        return ops.expert_linear(a, self.down, route), route

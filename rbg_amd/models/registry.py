@@ -6,19 +6,21 @@ import os
 from typing import Callable, Dict
 
 from ..engine.config import ModelConfig
-from . import bitatar, llama, notadra
+from . import bitatar, gogalix, llama, notadra
 
 # architecture -> model class
 MODELS: Dict[str, type] = {
     "llama": llama.LlamaForCausalLM,        # Llama and Qwen3 shapes
     "Bitatar": bitatar.BitatarForCausalLM,
     "Notadra": notadra.NotadraForCausalLM,
+    "Gogalix": gogalix.GogalixForCausalLM,
 }
 
 # architecture of a config.json -> its reader
 CONFIG_READERS: Dict[str, Callable[..., ModelConfig]] = {
     "Bitatar": bitatar.BitatarConfig.from_json,
     "Notadra": notadra.NotadraConfig.from_json,
+    "Gogalix": gogalix.GogalixConfig.from_json,
 }
 
 
@@ -39,8 +41,11 @@ def resolve_model(name: str) -> ModelConfig:
     """A preset's name, or a model folder."""
     if os.path.isdir(name):
         return load_config(name)
-    cfg = bitatar.preset(name) or notadra.preset(name)
-    return cfg if cfg is not None else ModelConfig.preset(name)
+    for family in (bitatar, notadra, gogalix):
+        cfg = family.preset(name)
+        if cfg is not None:
+            return cfg
+    return ModelConfig.preset(name)
 
 
 def build_model(cfg: ModelConfig, device, tp=None, pp=None):

@@ -105,6 +105,8 @@ class RandomSource(WeightSource):
             scale = 1.0 / math.sqrt(shape[-1])
         elif init == "conv":
             scale = 0.5 / math.sqrt(shape[-1])
+        elif init == "rate":        # of a decay, before its softplus
+            return t.normal_(-3.0, 1.0, generator=gen)
         return t.normal_(0.0, scale, generator=gen)
 
 

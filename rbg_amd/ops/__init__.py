@@ -42,13 +42,22 @@ except Exception as e:  # noqa: BLE001
 
 HAVE_MOE = _moe is not None
 
+_gated = None
+_gated_err: Exception | None = None
+try:
+    from . import _hip_gated as _gated   # type: ignore[attr-defined]
+except Exception as e:  # noqa: BLE001
+    _gated_err = e
+
+HAVE_GATED = _gated is not None
+
 
 def _check_stale() -> None:
     """Fail loudly on a GPU box if a shipped .so predates its kernel sources
     (stale-binary guard; the stamps are written by utils/hip_build.py)."""
     from ..utils import hip_build
     for name, mod in (("_hip_ops", _hip), ("_hip_mix", _mix),
-                      ("_hip_moe", _moe)):
+                      ("_hip_moe", _moe), ("_hip_gated", _gated)):
         if mod is not None and hip_build.is_stale(name):
             raise RuntimeError(
                 f"rbg_amd HIP extension {name} is STALE: kernel sources "
@@ -57,7 +66,8 @@ def _check_stale() -> None:
                 "--inplace")
 
 
-if (HAVE_HIP or HAVE_MIX or HAVE_MOE) and torch.cuda.is_available():
+if (HAVE_HIP or HAVE_MIX or HAVE_MOE or HAVE_GATED) and \
+        torch.cuda.is_available():
     _check_stale()
 
 
@@ -88,6 +98,15 @@ def _require_moe():
     return _moe
 
 
+def _require_gated():
+    if _gated is None:
+        raise RuntimeError(
+            "rbg_amd HIP extension _hip_gated is not built but a GPU tensor "
+            "was passed.  Build it in-tree: PYTORCH_ROCM_ARCH=gfx950 python "
+            f"setup.py build_ext --inplace (import error: {_gated_err!r})")
+    return _gated
+
+
 def _on_gpu(t: torch.Tensor) -> bool:
     return t.is_cuda
 
@@ -110,7 +129,7 @@ def linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
             (w.shape[0] <= 4608 or
              (x.shape[0] <= 64 and w.shape[0] <= 8192))):
         # linked into every extension: a process has the one its model needs
-        return (_hip or _mix or _require_moe()).skinny_gemm(
+        return (_hip or _mix or _gated or _require_moe()).skinny_gemm(
             x if x.is_contiguous() else x.contiguous(), w)
     return torch.nn.functional.linear(x, w)
 
@@ -213,7 +232,8 @@ build_cos_sin_table = reference.build_cos_sin_table
 def embed_stream(tokens, table, scale: float) -> torch.Tensor:
     """f32 stream [T, W] = table[tokens] * scale."""
     if _on_gpu(table):
-        return _require_mix().embed_stream(tokens, table, scale)
+        # linked into both extensions of designs that scale
+        return (_mix or _require_gated()).embed_stream(tokens, table, scale)
     return reference.embed_stream(tokens, table, scale)
 
 
@@ -418,11 +438,11 @@ def moe_combine(y, route) -> torch.Tensor:
 
 def rope_store_paged(proj, bias, cos_sin, positions, slots, heads: int,
                      dim: int, k, v, offs) -> None:
-    """Adds the biases of a fused projection, rotates the leading dimensions of
-    its queries (in place) and keys by cos_sin [positions, dims] = [cos | sin],
-    and writes keys and values to the pages [pages, kv heads, page_size, size].
-    ``offs`` are the columns of q, k, v; of q alone when the keys are another
-    layer's."""
+    """Adds the biases (None: none) of a fused projection, rotates the leading
+    dimensions of its queries (in place) and keys by cos_sin [positions, dims]
+    = [cos | sin] (None: not), and writes keys and values to the pages [pages,
+    kv heads, page_size, size].  ``offs`` are the columns of q, k, v; of q
+    alone when the keys are another layer's."""
     if _on_gpu(proj):
         _require_moe().rope_store_paged(proj, bias, cos_sin, positions, slots,
                                         heads, dim, k, v, offs)
@@ -431,19 +451,36 @@ def rope_store_paged(proj, bias, cos_sin, positions, slots, heads: int,
                                dim, k, v, offs)
 
 
+@dataclass
+class Difference:
+    """Differential heads: a head's query and key are two, whose softmaxes o1
+    and o2 over the same values become (o1 - lam o2) / rms * scale."""
+    lam: torch.Tensor           # [1] f32
+    scale: float
+    eps: float                  # inside the root
+
+
+def _difference(diff: Optional[Difference]):
+    return (None, 1.0, 0.0) if diff is None else (diff.lam, diff.scale,
+                                                  diff.eps)
+
+
 def paged_prefill(q, k, v, view, out, scale: float, softcap: float,
-                  sink: bool) -> None:
+                  sink: bool, window: int = 0,
+                  diff: Optional[Difference] = None) -> None:
     """Causal attention of portions [R, H, D] over the pages; ``view`` is the
     step's engine/batch.py PagedView.  Scores are scale * q.k, then softcap *
     tanh(score / softcap) (0: as they are); ``sink`` adds a key of score 0 and
-    no value."""
+    no value; ``window`` is how many keys a row sees, itself included (0: all
+    before it).  With ``diff`` q and k hold two maps of half the size."""
     if _on_gpu(q):
         _require_moe().paged_prefill(q, k, v, view.tables, view.seq_info,
                                      view.row_info, view.blocks, out, scale,
-                                     softcap, sink)
+                                     softcap, sink, window,
+                                     *_difference(diff))
         return
     reference.paged_rows(q, k, v, view.tables, view.row_info, out, scale,
-                         softcap, sink)
+                         softcap, sink, window, diff)
 
 
 def pick_paged_splits(num_seqs: int, kv_heads: int, max_keys: int) -> int:
@@ -456,18 +493,24 @@ def pick_paged_splits(num_seqs: int, kv_heads: int, max_keys: int) -> int:
 
 
 def paged_decode(q, k, v, tables, context_lens, out, scale: float,
-                 softcap: float, sink: bool, splits: int = 0) -> None:
+                 softcap: float, sink: bool, splits: int = 0, window: int = 0,
+                 diff: Optional[Difference] = None) -> None:
     """One query row per sequence, [S, H, D]; scores as in paged_prefill."""
     if _on_gpu(q):
         if splits <= 0:
-            splits = pick_paged_splits(q.shape[0], k.shape[1],
-                                       tables.shape[1] * k.shape[2])
+            keys = tables.shape[1] * k.shape[2]
+            # a window may begin anywhere in its first step
+            splits = pick_paged_splits(
+                q.shape[0], k.shape[1],
+                min(keys, window + 127) if window else keys)
         _require_moe().paged_decode(q, k, v, tables, context_lens, out, scale,
-                                    softcap, sink, splits)
+                                    softcap, sink, window,
+                                    *_difference(diff), splits)
         return
     info = torch.stack([torch.arange(q.shape[0], dtype=torch.int32),
                         context_lens - 1], dim=1)
-    reference.paged_rows(q, k, v, tables, info, out, scale, softcap, sink)
+    reference.paged_rows(q, k, v, tables, info, out, scale, softcap, sink,
+                         window, diff)
 
 
 def router_logits(x, w) -> torch.Tensor:
@@ -490,25 +533,132 @@ def expert_tile(x, w, top: int) -> int:
 
 
 def moe_route(logits, correction, groups: int, keep: int, top: int,
-              tile: int) -> Routing:
+              tile: int, softmax: bool = False) -> Routing:
     """Chooses the ``top`` experts of each token by sigmoid(logit) + correction
     among the ``keep`` groups with the largest sums of their two best, and lays
-    the pairs out by expert.  Weights are the sigmoids."""
+    the pairs out by expert.  Weights are the sigmoids.  ``softmax``: the
+    choice is by logit + correction, the weights are the softmax of the
+    chosen."""
     if _on_gpu(logits):
         weights, inv, rows, tiles, count = _require_moe().moe_route(
-            logits, correction, groups, keep, top, tile)
+            logits, correction, groups, keep, top, tile, softmax)
         return Routing(top, tile, weights, inv, rows, tiles, count)
-    ids, weights = reference.moe_choose(logits, correction, groups, keep, top)
+    ids, weights = reference.moe_choose(logits, correction, groups, keep, top,
+                                        softmax)
     return Routing(top, tile, weights,
                    *reference.moe_tiles(ids, logits.shape[1], tile))
 
 
-def expert_linear(x, w, route, gather: bool = False,
-                  relu2: bool = False) -> torch.Tensor:
+def interleave_glu(gate, up) -> torch.Tensor:
+    """Rows of two matrices [.., F, K] (F even) as expert_linear's ``swiglu``
+    reads them: two of the gate, two of the up matrix, and so on."""
+    f, k = gate.shape[-2:]
+    pair = [t.unflatten(-2, (f // 2, 2)) for t in (gate, up)]
+    return torch.cat(pair, dim=-2).flatten(-3, -2)
+
+
+def expert_linear(x, w, route, gather: bool = False, relu2: bool = False,
+                  swiglu: bool = False) -> torch.Tensor:
     """Rows in expert order times their expert's w [E, N, K]; ``gather`` takes
-    x's rows by token, ``relu2`` applies max(0, .)^2."""
+    x's rows by token, ``relu2`` applies max(0, .)^2, ``swiglu`` takes w's rows
+    as interleave_glu lays them and gives silu(gate) * up, [.., N / 2]."""
     if _on_gpu(x):
         return _require_moe().expert_linear(
             x, w, route.rows if gather else None, route.tiles, route.count,
-            route.rows.numel(), route.tile, relu2)
-    return reference.expert_linear(x, w, route, gather, relu2)
+            route.rows.numel(), route.tile, relu2, swiglu)
+    return reference.expert_linear(x, w, route, gather, relu2, swiglu)
+
+
+# -- gated branches, gated delta rule -------------------------------------------
+
+
+@dataclass
+class Branch:
+    """What a layer leaves to be added to the stream: (rows + bias) * scale *
+    sigmoid(logits + gate_bias), rows of tokens or (with a routing) of their
+    chosen experts, weighed and summed."""
+    rows: torch.Tensor          # [T, W], or expert rows
+    logits: torch.Tensor        # [T, W]
+    gate_bias: torch.Tensor     # [W] f32
+    scale: torch.Tensor         # [W] f32
+    bias: Optional[torch.Tensor] = None         # [W] f32
+    route: Optional[Routing] = None
+
+
+def gate_norm(x, branches, w, eps: float, dtype):
+    """x += the branches (in place, f32; at most two); returns the RMS norm of
+    x under w, one number or one per coordinate, in ``dtype`` (None without
+    w)."""
+    if _on_gpu(x):
+        return _require_gated().gate_norm(
+            x, [(b.rows, b.route.inv if b.route else None,
+                 b.route.weights if b.route else None, b.logits, b.gate_bias,
+                 b.scale, b.bias) for b in branches], w, eps,
+            dtype == torch.float32)
+    return reference.gate_norm(x, branches, w, eps, dtype)
+
+
+def silu_glu(gate, up, gate_bias, up_bias, out) -> None:
+    """out = silu(gate + gate_bias) * (up + up_bias); gate and up are column
+    slices of one buffer, the biases may be None."""
+    if _on_gpu(gate):
+        _require_gated().silu_glu(gate, up, gate_bias, up_bias, out)
+        return
+    reference.silu_glu(gate, up, gate_bias, up_bias, out)
+
+
+def short_conv(x, conv_w, ring, tiles, cu_seqlens, starts, slots):
+    """silu of the causal depthwise convolution of varlen rows (a column
+    slice); conv_w [taps, W], the last tap the current token's; ring [slots,
+    taps, W] holds a sequence's last inputs, position p's at p % taps."""
+    if _on_gpu(x):
+        return _require_gated().short_conv(x, conv_w, ring, tiles, cu_seqlens,
+                                           starts, slots,
+                                           max(CONV_TILE, conv_w.shape[0]))
+    return reference.short_conv(x, conv_w, ring, cu_seqlens, starts, slots)
+
+
+@dataclass
+class GatedDelta:
+    """Constants of a gated delta rule (gated_delta)."""
+    a_log: torch.Tensor         # [H] f32
+    dt_bias: torch.Tensor       # [H] f32, or [H*D]: a decay per key channel
+    norm: torch.Tensor          # [E] f32
+    kv_heads: int
+    silu: bool                  # output gate: silu, else sigmoid
+    q_scale: float
+    unit_eps: float             # inside the root of q's and k's norms
+    norm_eps: float             # inside the root of the head norm's
+
+
+def gated_delta(p: GatedDelta, qkv, offs, beta, decay, gate, state, slots,
+                cu_seqlens, starts, out, conv=None, chunks=None) -> None:
+    """Gated delta rule over varlen rows (cu_seqlens None: one row per
+    sequence) with the head norm and the output gate.  ``offs`` are the columns
+    of q, k [kv_heads, D], v [H, E] in ``qkv``; state [slots, H, D, E].
+    Per token, with unit q (times q_scale) and k, g = exp(-exp(a_log) *
+    softplus(decay + dt_bias)):
+      S <- g S;  u = sigmoid(beta) (v - S^T k);  S <- S + k u^T;  o = S^T q.
+    ``conv`` = (conv_w, ring): decode rows, whose q, k, v are first convolved
+    as by short_conv, over the columns from q's on.  With ``chunks`` = (tiles,
+    chunk_cu) of DELTA_CHUNK tokens the rows go through the matrix cores."""
+    if _on_gpu(qkv):
+        mod = _require_gated()
+        args = (qkv, beta, decay, gate, p.a_log, p.dt_bias, p.norm, state,
+                slots, cu_seqlens, starts, out, offs, p.kv_heads, p.silu,
+                p.q_scale, p.unit_eps, p.norm_eps)
+        if chunks is not None and state.shape[2] <= mod.CHUNK_MAX_DIM:
+            assert mod.CHUNK == DELTA_CHUNK
+            mod.gated_chunk(*args, *chunks)
+        else:
+            mod.gated_step(*args, *(conv or (None, None)))
+        return
+    if conv is not None:
+        n = slots.numel()
+        width = conv[0].shape[1]
+        x = reference.short_conv(
+            qkv[:, offs[0]:offs[0] + width], *conv,
+            torch.arange(n + 1, dtype=torch.int32), starts, slots)
+        qkv, offs = x, [o - offs[0] for o in offs]
+    reference.gated_delta(p, qkv, offs, beta, decay, gate, state, slots,
+                          cu_seqlens, starts, out)

@@ -12,37 +12,17 @@
 //   O  = R S + tril(R K^T) V - tril(R B^T) P
 //   S' = e^{c_15} S + (e^{c_15} K)^T V - (e^{c_15} B)^T P
 // delta_prep forms everything that does not need S, one workgroup per chunk
-// and head; delta_scan walks a sequence's chunks with 16 value columns of S in
-// each wave's registers; delta_out applies the head norm and the output gate.
+// and head; delta_scan.h walks the chunks and applies the head norm and gate.
 // Missing tokens of a last chunk have u = k = r = 0 and no decay.
-#include "mfma_util.h"
+#include "delta_scan.h"
 #include "mix_args.h"
-#include "vec_io.h"
 
 namespace {
-
-constexpr int C = 16;                   // tokens per chunk
-constexpr int SP = C + 4;               // row pitch of [.][16] arrays
-
-// one chunk-head's record in the workspace, in floats: the image that the scan
-// keeps in LDS, row pitches included
-template <int DP> struct Rec {
-  static constexpr int PP = DP + 4;               // pitch of [16][DP] arrays
-  static constexpr int TU = 0;                    // [16][DP]
-  static constexpr int R = TU + C * PP;           // [16][DP]
-  static constexpr int KT = R + C * PP;           // [DP][16]
-  static constexpr int BT = KT + DP * SP;         // [DP][16], negated
-  static constexpr int TM = BT + DP * SP;         // [16][16]
-  static constexpr int QK = TM + C * SP;          // [16][16]
-  static constexpr int QB = QK + C * SP;          // [16][16], negated
-  static constexpr int DC = QB + C * SP;          // [DP]
-  static constexpr int SIZE = DC + DP;
-};
 
 template <typename T, int DP>
 __global__ __launch_bounds__(256) void delta_prep_kernel(
     const DeltaArgs p, const int* __restrict__ tiles, float* __restrict__ ws) {
-  typedef Rec<DP> W;
+  typedef Rec<DP, true> W;
   constexpr int PP = W::PP;
   constexpr int GR = 256 / DP;          // token groups in the staging step
   constexpr int TPG = C / GR;           // tokens per group
@@ -205,248 +185,26 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(
   }
 }
 
-// grid (heads, seqs, column groups).  A workgroup is NC column groups of 16
-// value columns by KS parts of the key rows: wave (kp, cg) keeps its rows of
-// its columns of S.  With KS = 2 the parts' shares of P and O meet in LDS.
-// A record's loads fly under two chunks' MFMAs and land in the other half of
-// LDS.
-template <typename T, int DP, int KS, int NC>
-__global__ __launch_bounds__(KS * NC * 64) void delta_scan_kernel(
-    const DeltaArgs p, const int* __restrict__ chunk_cu,
-    const float* __restrict__ ws, float* __restrict__ o) {
-  typedef Rec<DP> W;
-  constexpr int PP = W::PP, NT = KS * NC * 64, TT = DP / 16 / KS;
-  constexpr int V4 = W::SIZE / 4, PER = (V4 + NT - 1) / NT;
-  extern __shared__ __attribute__((aligned(16))) float smem[];
-  f32x4* xch = reinterpret_cast<f32x4*>(smem + 2 * W::SIZE);  // [2][KS*NC*64]
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int gl = lane & 15, gs = lane >> 4;
-  const int cg = wave % NC, kp = wave / NC;
-  const int head = blockIdx.x, seq = blockIdx.y;
-  const int D = p.dim, HD = p.heads * D;
-  const int vcol = (blockIdx.z * NC + cg) * 16 + gl;
-  const bool vlive = vcol < D;
-  const int vc = min(vcol, D - 1);
-  const int row0 = p.cu[seq], len = p.cu[seq + 1] - row0;
-  const int ch0 = chunk_cu[seq], nch = chunk_cu[seq + 1] - ch0;
-  const bool fresh = p.starts[seq] == 0;
-  float* S = p.state + ((size_t)p.slots[seq] * p.heads + head) * D * D;
-  const int k0 = kp * TT * 16;                  // this wave's key rows
-
-  f32x4 s[TT];
-#pragma unroll
-  for (int t = 0; t < TT; ++t)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int kr = k0 + t * 16 + gs * 4 + r;
-      s[t][r] = !fresh && vlive && kr < D ? S[(size_t)kr * D + vcol] : 0.f;
-    }
-
-  f32x4 stage[2][PER];
-  float v[4], vn[2][4];
-#define DC_FETCH(c, h)                                                        \
-  do {                                                                        \
-    const f32x4* src = reinterpret_cast<const f32x4*>(                        \
-        ws + ((size_t)(ch0 + (c)) * p.heads + head) * W::SIZE);               \
-    _Pragma("unroll") for (int i = 0; i < PER; ++i)                           \
-      stage[h][i] = src[min(tid + i * NT, V4 - 1)];                           \
-    _Pragma("unroll") for (int r = 0; r < 4; ++r) {                           \
-      const int t = (c) * C + gs * 4 + r;                                     \
-      vn[h][r] = to_f(((const T*)p.proj)[                                     \
-          (size_t)(row0 + min(t, len - 1)) * p.proj_stride + p.off_v +        \
-          head * D + vc]);                                                    \
-      if (t >= len || !vlive) vn[h][r] = 0.f;                                 \
-    }                                                                         \
-  } while (0)
-#define DC_LAND(half)                                                         \
-  do {                                                                        \
-    f32x4* dst = reinterpret_cast<f32x4*>(smem + (half) * W::SIZE);           \
-    _Pragma("unroll") for (int i = 0; i < PER; ++i)                           \
-      if (tid + i * NT < V4) dst[tid + i * NT] = stage[half][i];              \
-    _Pragma("unroll") for (int r = 0; r < 4; ++r) v[r] = vn[half][r];         \
-  } while (0)
-  DC_FETCH(0, 0);
-  DC_LAND(0);
-  DC_FETCH(min(1, nch - 1), 1);
-  __syncthreads();
-  for (int cc = 0; cc < nch; cc += 2)
-#pragma unroll
-  for (int h = 0; h < 2; ++h) {
-    const int c = cc + h;
-    if (c >= nch) break;
-    const float* rec = smem + h * W::SIZE;
-    // always: a skipped load would make the waits below drain every load
-    DC_FETCH(min(c + 2, nch - 1), h);
-
-    // P and O over the old state, two products side by side
-    f32x4 pa = {0.f, 0.f, 0.f, 0.f}, oa = pa;
-    if (kp == 0) {
-      float x[4], y[4];
-      load_vec<4>(rec + W::TM + gl * SP + gs * 4, x);
-      load_vec<4>(rec + W::QK + gl * SP + gs * 4, y);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        pa = mfma_f32_k4(x[r], v[r], pa);
-        oa = mfma_f32_k4(y[r], v[r], oa);
-      }
-    }
-#pragma unroll
-    for (int t = 0; t < TT; ++t) {
-      float x[4], y[4];
-      load_vec<4>(rec + W::TU + gl * PP + k0 + t * 16 + gs * 4, x);
-      load_vec<4>(rec + W::R + gl * PP + k0 + t * 16 + gs * 4, y);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        pa = mfma_f32_k4(x[r], s[t][r], pa);
-        oa = mfma_f32_k4(y[r], s[t][r], oa);
-      }
-    }
-    if constexpr (KS == 2) {
-      xch[wave * 64 + lane] = pa;
-      if (kp == 1) xch[(KS * NC + cg) * 64 + lane] = oa;
-    }
-    // the decay and k v^T parts do not wait for P
-#pragma unroll
-    for (int t = 0; t < TT; ++t) {
-      float x[4], d[4];
-      load_vec<4>(rec + W::DC + k0 + t * 16 + gs * 4, d);
-      load_vec<4>(rec + W::KT + (k0 + t * 16 + gl) * SP + gs * 4, x);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) s[t][r] *= d[r];
-#pragma unroll
-      for (int r = 0; r < 4; ++r) s[t] = mfma_f32_k4(x[r], v[r], s[t]);
-    }
-    if constexpr (KS == 2) {
-      __syncthreads();
-      const f32x4 p0 = xch[cg * 64 + lane], p1 = xch[(NC + cg) * 64 + lane];
-      pa = p0 + p1;
-      if (kp == 0) oa += xch[(KS * NC + cg) * 64 + lane];
-    }
-#pragma unroll
-    for (int t = 0; t < TT; ++t) {
-      float y[4];
-      load_vec<4>(rec + W::BT + (k0 + t * 16 + gl) * SP + gs * 4, y);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) s[t] = mfma_f32_k4(y[r], pa[r], s[t]);
-    }
-    if (kp == 0) {
-      float y[4];
-      load_vec<4>(rec + W::QB + gl * SP + gs * 4, y);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) oa = mfma_f32_k4(y[r], pa[r], oa);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = c * C + gs * 4 + r;
-        if (t < len && vlive)
-          o[(size_t)(row0 + t) * HD + head * D + vcol] = oa[r];
-      }
-    }
-    DC_LAND(1 - h);
-    __syncthreads();
-  }
-#undef DC_FETCH
-#undef DC_LAND
-#pragma unroll
-  for (int t = 0; t < TT; ++t)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int kr = k0 + t * 16 + gs * 4 + r;
-      if (vlive && kr < D) S[(size_t)kr * D + vcol] = s[t][r];
-    }
-}
-
-// out = o / rms(o) * norm_w * sigmoid(g).  VEC: dim is 4 * LPI for a power of
-// two LPI, and LPI lanes take a row of a head; else one wave does.
-template <typename T, int LPI>
-__global__ __launch_bounds__(256) void delta_out_vec_kernel(
-    const DeltaArgs p, const float* __restrict__ o, const long items) {
-  const int lane = threadIdx.x & 63;
-  const long item = (blockIdx.x * 4L + (threadIdx.x >> 6)) * (64 / LPI) +
-                    lane / LPI;
-  const int d = (lane % LPI) * 4;
-  const long it = item < items ? item : items - 1;
-  const int head = (int)(it % p.heads);
-  const long row = it / p.heads;
-  float x[4], w[4];
-  load_vec<4>(o + it * (LPI * 4) + d, x);
-  float ss = 0.f;
-#pragma unroll
-  for (int r = 0; r < 4; ++r) ss += x[r] * x[r];
-#pragma unroll
-  for (int off = LPI / 2; off >= 1; off >>= 1) ss += __shfl_xor(ss, off, 64);
-  const float inv = 1.f / sqrtf(ss / (LPI * 4) + p.norm_eps);
-  const int col = head * LPI * 4 + d;
-  load_vec<4>(p.norm_w + col, w);
-  if (item >= items) return;
-  const T* g = (const T*)p.proj + row * p.proj_stride + p.off_g + col;
-  T* out = (T*)p.out + row * p.out_stride + col;
-  if constexpr (sizeof(T) == 2) {
-    union { uint2 u; __hip_bfloat16 e[4]; } gv, ov;
-    gv.u = *reinterpret_cast<const uint2*>(g);
-#pragma unroll
-    for (int r = 0; r < 4; ++r)
-      ov.e[r] = f2bf(x[r] * inv * w[r] * sigmoid_f(bf2f(gv.e[r])));
-    *reinterpret_cast<uint2*>(out) = ov.u;
-  } else {
-    float gv[4];
-    load_vec<4>((const float*)g, gv);
-#pragma unroll
-    for (int r = 0; r < 4; ++r) gv[r] = x[r] * inv * w[r] * sigmoid_f(gv[r]);
-    store_vec<4>((float*)out, gv);
-  }
-}
-
-template <typename T>
-__global__ __launch_bounds__(256) void delta_out_kernel(
-    const DeltaArgs p, const float* __restrict__ o, const long items) {
-  const long item = blockIdx.x * 4L + (threadIdx.x >> 6);
-  const int lane = threadIdx.x & 63;
-  if (item >= items) return;
-  const int head = (int)(item % p.heads);
-  const long row = item / p.heads;
-  const int D = p.dim;
-  const float* src = o + item * D;
-  float ss = 0.f;
-  for (int d = lane; d < D; d += 64) ss += src[d] * src[d];
-  const float inv = 1.f / sqrtf(wave_sum(ss) / D + p.norm_eps);
-  const T* g = (const T*)p.proj + row * p.proj_stride + p.off_g + head * D;
-  T* out = (T*)p.out + row * p.out_stride + head * D;
-  for (int d = lane; d < D; d += 64)
-    out[d] = from_f<T>(src[d] * inv * p.norm_w[head * D + d] *
-                       sigmoid_f(to_f(g[d])));
-}
-
 template <typename T, int DP, int KS, int NC>
 void delta_chunk_t(const DeltaArgs& p, const int* tiles, const int* chunk_cu,
                    float* ws, float* o, int n_tiles, int seqs, long rows,
                    hipStream_t s) {
-  constexpr int NT = KS * NC * 64;
-  const int zs = (p.dim + NC * 16 - 1) / (NC * 16);
-  const size_t lds = 2 * Rec<DP>::SIZE * sizeof(float) +
-                     (KS == 2 ? (size_t)(KS + 1) * NC * 64 * 16 : 0);
-  static bool once = false;
-  if (!once) {
-    (void)hipFuncSetAttribute((const void*)delta_scan_kernel<T, DP, KS, NC>,
-                              hipFuncAttributeMaxDynamicSharedMemorySize,
-                              (int)lds);
-    once = true;
-  }
   delta_prep_kernel<T, DP><<<dim3(n_tiles, p.heads), 256, 0, s>>>(p, tiles,
                                                                   ws);
-  delta_scan_kernel<T, DP, KS, NC><<<dim3(p.heads, seqs, zs), NT, lds, s>>>(
-      p, chunk_cu, ws, o);
-  const long items = rows * p.heads;
-  const bool vec = p.dim == DP && p.proj_stride % 4 == 0 &&
-                   p.out_stride % 4 == 0 && p.off_g % 4 == 0 &&
-                   ((uintptr_t)p.proj & 15) == 0 &&
-                   ((uintptr_t)p.out & 15) == 0;
-  if (vec) {
-    const long per = 4L * (64 / (DP / 4));
-    delta_out_vec_kernel<T, DP / 4>
-        <<<(int)((items + per - 1) / per), 256, 0, s>>>(p, o, items);
-  } else {
-    delta_out_kernel<T><<<(int)((items + 3) / 4), 256, 0, s>>>(p, o, items);
-  }
+  DeltaScanArgs sa{};
+  sa.v = (const T*)p.proj + p.off_v;
+  sa.state = p.state; sa.slots = p.slots; sa.cu = p.cu; sa.starts = p.starts;
+  sa.chunk_cu = chunk_cu; sa.ws = ws; sa.o = o;
+  sa.v_row = p.proj_stride;
+  sa.heads = p.heads; sa.dk = sa.dv = p.dim;
+  delta_scan<T, DP, KS, NC, true>(sa, seqs, s);
+  DeltaOutArgs oa{};
+  oa.o = o; oa.gate = (const T*)p.proj + p.off_g; oa.norm_w = p.norm_w;
+  oa.out = p.out;
+  oa.g_row = p.proj_stride; oa.o_row = p.out_stride;
+  oa.heads = p.heads; oa.dv = oa.w_head = p.dim;
+  oa.eps = p.norm_eps;
+  delta_out<T>(oa, rows, s);
 }
 
 template <typename T>
@@ -470,8 +228,8 @@ int delta_chunk_tokens() { return C; }
 
 // floats of workspace per chunk and head
 long delta_chunk_record(int dim) {
-  return dim <= 32 ? Rec<32>::SIZE : dim <= 64 ? Rec<64>::SIZE
-                                               : Rec<128>::SIZE;
+  return dim <= 32 ? Rec<32, true>::SIZE
+       : dim <= 64 ? Rec<64, true>::SIZE : Rec<128, true>::SIZE;
 }
 
 void launch_delta_chunk(const DeltaArgs* p, const int* tiles,

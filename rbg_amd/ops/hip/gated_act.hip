@@ -1,5 +1,5 @@
-// Elementwise gates in bf16 or f32: gelu_tanh(gate) * up, and tanh of a low-rank
-// projection.  Inputs and outputs are column slices of the
+// Elementwise gates in bf16 or f32: gelu_tanh(gate) * up, silu(gate) * up with
+// or without biases, and tanh of a low-rank projection.  Inputs and outputs are column slices of the
 // fused projection buffers (row strides), so no copy stands between a GEMM and
 // its gate, and the products land in the operand of the layer's output GEMM.
 #include "vec_io.h"
@@ -11,22 +11,40 @@ DEV_INLINE float gelu_tanh_f(float z) {
   return 0.5f * z * (1.f + tanhf(c * (z + 0.044715f * z * z * z)));
 }
 
-template <typename T, int V>
-__global__ void gelu_mul_kernel(T* __restrict__ out, const long out_stride,
-                                const T* __restrict__ x, const int inter,
-                                const long total) {
+struct GluArgs {
+  void* out;              // [rows, out_row]
+  const void* gate;       // + row*x_row
+  const void* up;         // + row*x_row
+  const float* gate_bias; // [inter], or null (both)
+  const float* up_bias;
+  long out_row, x_row;
+  int inter;
+};
+
+template <typename T, int V, bool SILU>
+__global__ void glu_kernel(const GluArgs p, const long total) {
   const long step = (long)gridDim.x * blockDim.x;
-  const int nv = inter / V;
+  const int nv = p.inter / V;
   for (long i = blockIdx.x * (long)blockDim.x + threadIdx.x; i < total;
        i += step) {
     const long row = i / nv;
     const int c = (int)(i % nv) * V;
     float g[V], u[V];
-    load_vec<V>(x + row * 2 * inter + c, g);
-    load_vec<V>(x + row * 2 * inter + inter + c, u);
+    load_vec<V>((const T*)p.gate + row * p.x_row + c, g);
+    load_vec<V>((const T*)p.up + row * p.x_row + c, u);
+    if (p.gate_bias != nullptr) {
+      float b[V];
+      load_vec<V>(p.gate_bias + c, b);
 #pragma unroll
-    for (int j = 0; j < V; ++j) u[j] *= gelu_tanh_f(g[j]);
-    store_vec<V>(out + row * out_stride + c, u);
+      for (int j = 0; j < V; ++j) g[j] += b[j];
+      load_vec<V>(p.up_bias + c, b);
+#pragma unroll
+      for (int j = 0; j < V; ++j) u[j] += b[j];
+    }
+#pragma unroll
+    for (int j = 0; j < V; ++j)
+      u[j] *= SILU ? g[j] * sigmoid_f(g[j]) : gelu_tanh_f(g[j]);
+    store_vec<V>((T*)p.out + row * p.out_row + c, u);
   }
 }
 
@@ -46,29 +64,38 @@ int blocks_for(long total) {
 
 bool aligned16(const void* p) { return ((uintptr_t)p & 15) == 0; }
 
-template <typename T>
-void gelu_mul_t(void* out, long os, const void* x, long rows, int inter,
-                hipStream_t s) {
-  const bool vec = inter % 8 == 0 && os % 8 == 0 && aligned16(out);
-  const long total = rows * (inter / (vec ? 8 : 1));
+template <typename T, bool SILU>
+void glu_t(const GluArgs& p, long rows, hipStream_t s) {
+  const bool vec = p.inter % 8 == 0 && p.out_row % 8 == 0 &&
+                   p.x_row % 8 == 0 && aligned16(p.out) &&
+                   aligned16(p.gate) && aligned16(p.up) &&
+                   aligned16(p.gate_bias) && aligned16(p.up_bias);
+  const long total = rows * (p.inter / (vec ? 8 : 1));
   int b = blocks_for(total);
   if (b > 16384) b = 16384;
-  if (vec)
-    gelu_mul_kernel<T, 8><<<b, 256, 0, s>>>((T*)out, os, (const T*)x, inter,
-                                            total);
-  else
-    gelu_mul_kernel<T, 1><<<b, 256, 0, s>>>((T*)out, os, (const T*)x, inter,
-                                            total);
+  if (vec) {
+    glu_kernel<T, 8, SILU><<<b, 256, 0, s>>>(p, total);
+  } else {
+    glu_kernel<T, 1, SILU><<<b, 256, 0, s>>>(p, total);
+  }
 }
 
 }  // namespace
 
 extern "C" {
 
-void launch_gelu_mul(void* out, long out_stride, const void* x, long rows,
-                     int inter, int f32, hipStream_t s) {
-  if (f32) gelu_mul_t<float>(out, out_stride, x, rows, inter, s);
-  else gelu_mul_t<__hip_bfloat16>(out, out_stride, x, rows, inter, s);
+// out = act(gate + gate_bias) * (up + up_bias); act: silu or gelu_tanh
+void launch_glu(void* out, long out_row, const void* gate, const void* up,
+                long x_row, const float* gate_bias, const float* up_bias,
+                long rows, int inter, int silu, int f32, hipStream_t s) {
+  const GluArgs p{out, gate, up, gate_bias, up_bias, out_row, x_row, inter};
+  if (f32) {
+    if (silu) glu_t<float, true>(p, rows, s);
+    else glu_t<float, false>(p, rows, s);
+  } else {
+    if (silu) glu_t<__hip_bfloat16, true>(p, rows, s);
+    else glu_t<__hip_bfloat16, false>(p, rows, s);
+  }
 }
 
 void launch_tanh_rows(void* out, const void* x, long stride, long rows,

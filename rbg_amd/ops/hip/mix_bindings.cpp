@@ -13,7 +13,8 @@ void launch_stream_norm(float*, const void*, const float*, const float*, void*,
 void launch_causal_conv(void*, const void*, const float*, void*, const int*,
                         const int*, const int*, const int*, int, int, int, int,
                         int, hipStream_t);
-void launch_gelu_mul(void*, long, const void*, long, int, int, hipStream_t);
+void launch_glu(void*, long, const void*, const void*, long, const float*,
+                const float*, long, int, int, int, hipStream_t);
 void launch_tanh_rows(void*, const void*, long, long, int, int, hipStream_t);
 void launch_delta_step(const DeltaArgs*, int, int, hipStream_t);
 void launch_latent_store(void*, void*, const void*, long, const float*,
@@ -124,9 +125,11 @@ void gelu_mul(Tensor x, Tensor out) {
   same_dtype(x, out, "gelu_mul");
   TORCH_CHECK(x.is_contiguous() && x.size(1) == 2 * out.size(1) &&
               x.size(0) == out.size(0), "x must be [T, 2*ff] of out's rows");
+  const int64_t F = out.size(1);
   if (x.size(0))
-    launch_gelu_mul(out.data_ptr(), out.stride(0), x.data_ptr(), x.size(0),
-                    (int)out.size(1), is_f32(x), current_stream());
+    launch_glu(out.data_ptr(), out.stride(0), x.data_ptr(),
+               (const char*)x.data_ptr() + F * x.element_size(), 2 * F, nullptr,
+               nullptr, x.size(0), (int)F, 0, is_f32(x), current_stream());
 }
 
 Tensor tanh_rows(Tensor x) {

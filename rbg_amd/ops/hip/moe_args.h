@@ -4,7 +4,7 @@
 
 struct PagedAttnArgs {
   const void* q;          // + row*q_row + head*q_head
-  const void* k;          // [pages, kv_heads, page_size, d]
+  const void* k;          // [pages, kv_heads, page_size, maps*d]
   const void* v;          // [pages, kv_heads, page_size, dv]
   void* out;              // + row*o_row + head*dv
   const int* tables;      // [seqs, max_pages]
@@ -13,19 +13,24 @@ struct PagedAttnArgs {
                           //   the first
   const int* row_info;    // prompts: [rows, 2] = sequence, position
   const int* blocks;      // prompts: [n_blocks, 2] = sequence, first query
-  float* part_o;          // decode: [splits, seqs, heads, dv]  (splits > 1)
-  float* part_ml;         //         [splits, seqs, heads, 2]
+  float* part_o;          // decode: [splits, seqs, heads*maps, dv] when
+  float* part_ml;         //         splits > 1 or maps == 2; [.., 2]
+  const float* lam;       // maps == 2: [1] what the second map counts
   long q_row, q_head, o_row;
   int rows, heads, kv_heads, d, dv, page_size, max_pages, n_blocks, splits;
   int page_shift;         // log2(page_size); prompt and decode forms only
   float scale, softcap;   // softcap 0: none
   int sink;               // one key of score 0 without a value
+  int window;             // keys seen, this one included; 0: all before
+  int maps;               // 2: a head's q and k are two of size d, and its
+                          //   output (o1 - lam o2) / rms * out_scale
+  float out_scale, out_eps;
 };
 
 struct RopePagedArgs {
   void* proj;             // [rows, stride]
-  const float* bias;      // [width]
-  const float* cos_sin;   // [positions, rot] = [cos | sin]
+  const float* bias;      // [width], or null
+  const float* cos_sin;   // [positions, rot] = [cos | sin]; null: rot is 0
   const int* positions;   // [rows]
   const int* slots;       // [rows]
   void* k;                // [pages, kv_heads, page_size, d], or null
@@ -46,14 +51,17 @@ struct MoeRouteArgs {
   int* count;             // [1] tiles used
   int* part;              // [blocks, experts] of moe_route_blocks
   int tokens, experts, groups, keep, top, tile;
+  int softmax;            // choice by logit + correction, weights by softmax
+                          //   over the chosen; else sigmoids
 };
 
 struct MoeGemmArgs {
   const void* x;          // [.., k] rows
   const void* w;          // [experts, n, k]
-  void* out;              // [pairs, n]
+  void* out;              // [pairs, n], swiglu: [pairs, n / 2]
   const int* rows;        // gather: row -> row of x; null: the same
   const int* tiles;
   const int* count;
   int max_tiles, tile, n, k, relu2;
+  int swiglu;             // silu(gate) * up; w's rows go gate, gate, up, up
 };

@@ -132,17 +132,19 @@ void check_pages(const Tensor& k, const Tensor& v, const Tensor& like) {
 }
 
 // offs: columns of q, k, v, or of q alone (nothing is stored then)
-void rope_store_paged(Tensor proj, Tensor bias, Tensor cos_sin,
+void rope_store_paged(Tensor proj, OptTensor bias, OptTensor cos_sin,
                       Tensor positions, Tensor slots, int64_t heads,
                       int64_t dim, Tensor k, Tensor v,
                       std::vector<int64_t> offs) {
   check_rows(proj, "proj");
   check_pages(k, v, proj);
   const int64_t T = proj.size(0), N = proj.size(1);
-  check_f32(bias, "bias", N);
-  TORCH_CHECK(cos_sin.dim() == 2 && cos_sin.size(1) % 2 == 0 &&
-              cos_sin.size(1) <= dim, "cos_sin [positions, rotated dims]");
-  check_f32(cos_sin, "cos_sin", cos_sin.numel());
+  if (bias) check_f32(*bias, "bias", N);
+  if (cos_sin) {
+    TORCH_CHECK(cos_sin->dim() == 2 && cos_sin->size(1) % 2 == 0 &&
+                cos_sin->size(1) <= dim, "cos_sin [positions, rotated dims]");
+    check_f32(*cos_sin, "cos_sin", cos_sin->numel());
+  }
   TORCH_CHECK(k.size(3) == dim, "key size");
   TORCH_CHECK(offs.size() == 1 || offs.size() == 3, "columns of q or q, k, v");
   const int64_t G = k.size(1), DV = v.size(3);
@@ -157,34 +159,43 @@ void rope_store_paged(Tensor proj, Tensor bias, Tensor cos_sin,
     p.off_v = (int)offs[2];
   }
   p.proj = proj.data_ptr();
-  p.bias = bias.data_ptr<float>();
-  p.cos_sin = cos_sin.data_ptr<float>();
+  p.bias = bias ? bias->data_ptr<float>() : nullptr;
+  p.cos_sin = cos_sin ? cos_sin->data_ptr<float>() : nullptr;
   p.positions = i32(positions, "positions", T);
   p.slots = i32(slots, "slots", T);
   p.stride = proj.stride(0);
   p.off_q = (int)offs[0];
-  p.rows = (int)T; p.heads = (int)heads; p.kv_heads = (int)G;
-  p.d = (int)dim; p.dv = (int)DV; p.rot = (int)cos_sin.size(1);
+  // queries that neither shift nor turn stay as they are
+  p.rows = (int)T; p.heads = bias || cos_sin ? (int)heads : 0;
+  p.kv_heads = (int)G;
+  p.d = (int)dim; p.dv = (int)DV;
+  p.rot = cos_sin ? (int)cos_sin->size(1) : 0;
   p.page_size = (int)k.size(2);
-  p.table_rows = (int)cos_sin.size(0);
+  p.table_rows = cos_sin ? (int)cos_sin->size(0) : 0;
   const bool vec = mult8({dim, DV, p.rot / 2, p.stride, p.off_q, p.off_k,
                           p.off_v}) && aligned(proj, 16) && aligned(k, 16) &&
                    aligned(v, 16);
-  if (T) launch_rope_paged(&p, is_f32(proj), vec, current_stream());
+  if (T && (p.heads || p.k)) launch_rope_paged(&p, is_f32(proj), vec, current_stream());
 }
 
 // fields that prompts and decode share; returns whether the matrix-core forms
 // take the sizes
 bool paged_args(PagedAttnArgs& p, const Tensor& q, const Tensor& k,
                 const Tensor& v, const Tensor& tables, const Tensor& out,
-                double scale, double softcap, bool sink) {
+                double scale, double softcap, bool sink, int64_t window,
+                const OptTensor& lam, double out_scale, double out_eps) {
   check_heads(q, "q");
   check_pages(k, v, q);
   check_rows(out, "out");
   same_dtype(q, out, "attn out");
-  const int64_t R = q.size(0), H = q.size(1), D = q.size(2), DV = v.size(3);
+  const int64_t M = lam ? 2 : 1;
+  const int64_t R = q.size(0), H = q.size(1), D = q.size(2) / M,
+                DV = v.size(3);
   const int64_t G = k.size(1), PS = k.size(2);
-  TORCH_CHECK(k.size(3) == D && G > 0 && H % G == 0, "key heads or size");
+  TORCH_CHECK(k.size(3) == q.size(2) && q.size(2) % M == 0 && G > 0 &&
+              H % G == 0, "key heads or size");
+  TORCH_CHECK(window >= 0 && window < (1ll << 31), "window");
+  if (lam) check_f32(*lam, "lam", 1);
   TORCH_CHECK(out.size(0) == R && out.size(1) == H * DV, "out shape");
   TORCH_CHECK(D <= 1024 && DV <= 1024, "head size above 1024");
   TORCH_CHECK(tables.dim() == 2, "tables [seqs, pages]");
@@ -198,7 +209,10 @@ bool paged_args(PagedAttnArgs& p, const Tensor& q, const Tensor& k,
   while ((1 << (p.page_shift + 1)) <= PS) ++p.page_shift;
   p.splits = 1;
   p.scale = (float)scale; p.softcap = (float)softcap; p.sink = sink;
-  return !is_f32(q) && D <= 256 && DV <= 256 && PS % 16 == 0 &&
+  p.window = (int)window; p.maps = (int)M;
+  p.lam = lam ? lam->data_ptr<float>() : nullptr;
+  p.out_scale = (float)out_scale; p.out_eps = (float)out_eps;
+  return !is_f32(q) && D * M <= 256 && DV <= 256 && PS % 16 == 0 &&
          (1 << p.page_shift) == PS && mult8({D, DV, p.q_row, p.q_head}) &&
          p.o_row % 4 == 0 && aligned(q, 16) && aligned(k, 16) &&
          aligned(v, 16) && aligned(out, 8);
@@ -206,9 +220,11 @@ bool paged_args(PagedAttnArgs& p, const Tensor& q, const Tensor& k,
 
 void paged_prefill(Tensor q, Tensor k, Tensor v, Tensor tables,
                    Tensor seq_info, Tensor row_info, Tensor blocks, Tensor out,
-                   double scale, double softcap, bool sink) {
+                   double scale, double softcap, bool sink, int64_t window,
+                   OptTensor lam, double out_scale, double out_eps) {
   PagedAttnArgs p{};
-  const bool tiled = paged_args(p, q, k, v, tables, out, scale, softcap, sink);
+  const bool tiled = paged_args(p, q, k, v, tables, out, scale, softcap, sink,
+                                window, lam, out_scale, out_eps);
   if (!p.rows) return;
   if (tiled) {
     TORCH_CHECK(paged_block_rows() == 128, "block size");
@@ -227,9 +243,11 @@ void paged_prefill(Tensor q, Tensor k, Tensor v, Tensor tables,
 
 void paged_decode(Tensor q, Tensor k, Tensor v, Tensor tables, Tensor ctx,
                   Tensor out, double scale, double softcap, bool sink,
-                  int64_t splits) {
+                  int64_t window, OptTensor lam, double out_scale,
+                  double out_eps, int64_t splits) {
   PagedAttnArgs p{};
-  const bool tiled = paged_args(p, q, k, v, tables, out, scale, softcap, sink);
+  const bool tiled = paged_args(p, q, k, v, tables, out, scale, softcap, sink,
+                                window, lam, out_scale, out_eps);
   TORCH_CHECK(tables.size(0) == q.size(0), "one table per row");
   if (!p.rows) return;
   p.ctx = i32(ctx, "ctx", p.rows);
@@ -239,10 +257,10 @@ void paged_decode(Tensor q, Tensor k, Tensor v, Tensor tables, Tensor ctx,
   }
   p.splits = (int)(splits < 1 ? 1 : splits > 64 ? 64 : splits);
   Tensor po, pml;
-  if (p.splits > 1) {
+  if (p.splits > 1 || p.maps > 1) {
     auto f32 = q.options().dtype(torch::kFloat32);
-    po = torch::empty({p.splits, p.rows, p.heads, p.dv}, f32);
-    pml = torch::empty({p.splits, p.rows, p.heads, 2}, f32);
+    po = torch::empty({p.splits, p.rows, p.heads * p.maps, p.dv}, f32);
+    pml = torch::empty({p.splits, p.rows, p.heads * p.maps, 2}, f32);
     p.part_o = po.data_ptr<float>();
     p.part_ml = pml.data_ptr<float>();
   }
@@ -271,7 +289,8 @@ int64_t most_tiles(int64_t pairs, int64_t experts, int64_t tile) {
 
 // weights [T, top], inv, rows [T * top], tiles [most, 3], count [1]
 std::vector<Tensor> moe_route(Tensor logits, Tensor correction, int64_t groups,
-                              int64_t keep, int64_t top, int64_t tile) {
+                              int64_t keep, int64_t top, int64_t tile,
+                              bool softmax) {
   TORCH_CHECK(logits.dim() == 2, "logits [T, E]");
   const int64_t T = logits.size(0), E = logits.size(1), P = T * top;
   check_f32(logits, "logits", T * E);
@@ -301,12 +320,14 @@ std::vector<Tensor> moe_route(Tensor logits, Tensor correction, int64_t groups,
   }
   p.tokens = (int)T; p.experts = (int)E; p.groups = (int)groups;
   p.keep = (int)keep; p.top = (int)top; p.tile = (int)tile;
+  p.softmax = softmax;
   if (T) launch_moe_route(&p, current_stream());
   return {weights, inv, rows, tiles, count};
 }
 
 Tensor expert_linear(Tensor x, Tensor w, OptTensor rows, Tensor tiles,
-                     Tensor count, int64_t pairs, int64_t tile, bool relu2) {
+                     Tensor count, int64_t pairs, int64_t tile, bool relu2,
+                     bool swiglu) {
   check_rows(x, "x");
   TORCH_CHECK(w.is_cuda() && w.dim() == 3 && w.is_contiguous() &&
               x.is_contiguous(), "w [E, N, K] and x must be contiguous");
@@ -316,7 +337,8 @@ Tensor expert_linear(Tensor x, Tensor w, OptTensor rows, Tensor tiles,
   TORCH_CHECK(rows || x.size(0) == pairs, "one row of x per pair");
   TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 3 &&
               tiles.size(0) == most_tiles(pairs, E, tile), "tiles shape");
-  auto out = torch::empty({pairs, N}, x.options());
+  TORCH_CHECK(!swiglu || (!relu2 && N % 4 == 0), "swiglu rows");
+  auto out = torch::empty({pairs, swiglu ? N / 2 : N}, x.options());
   MoeGemmArgs p{};
   p.x = x.data_ptr(); p.w = w.data_ptr(); p.out = out.data_ptr();
   p.rows = rows ? i32(*rows, "rows", pairs) : nullptr;
@@ -324,6 +346,7 @@ Tensor expert_linear(Tensor x, Tensor w, OptTensor rows, Tensor tiles,
   p.count = i32(count, "count", 1);
   p.max_tiles = (int)tiles.size(0); p.tile = (int)tile;
   p.n = (int)N; p.k = (int)K; p.relu2 = relu2;
+  p.swiglu = swiglu;
   const bool vec = !is_f32(x) && mult8({N, K}) && aligned(x, 16) &&
                    aligned(w, 16);
   TORCH_CHECK(tile <= (vec ? 128 : 16), "tile too large for these sizes");

@@ -14,6 +14,7 @@
 //           the MFMAs, waves split K and meet in LDS: batches whose experts do
 //           not fill the chip otherwise.
 //   rows    any sizes, bf16 or f32: a thread per column, up to 16 rows at once.
+// A squared relu, or silu(gate) * up of interleaved rows, rides on the way out.
 #include "lds_stream.h"
 #include "moe_args.h"
 #include "vec_io.h"
@@ -25,9 +26,19 @@ DEV_INLINE float relu2_f(float x) {
   return x * x;
 }
 
+DEV_INLINE float swiglu_f(float g, float u) { return g * sigmoid_f(g) * u; }
+
 // four neighbouring columns of one row
 DEV_INLINE void put4(const MoeGemmArgs& p, const size_t row, const int n,
                      f32x4 v) {
+  if (p.swiglu) {                               // gate, gate, up, up
+    union { uint32_t u; __hip_bfloat16 e[2]; } o;
+    o.e[0] = f2bf(swiglu_f(v[0], v[2]));
+    o.e[1] = f2bf(swiglu_f(v[1], v[3]));
+    *reinterpret_cast<uint32_t*>((__hip_bfloat16*)p.out + row * (p.n / 2) +
+                                 n / 2) = o.u;
+    return;
+  }
   union { uint2 u; __hip_bfloat16 e[4]; } o;
 #pragma unroll
   for (int r = 0; r < 4; ++r) o.e[r] = f2bf(p.relu2 ? relu2_f(v[r]) : v[r]);
@@ -240,32 +251,49 @@ __global__ __launch_bounds__(SW * 64) void moe_skinny_kernel(
   if (gl < rows && n < p.n) put4(p, row0 + gl, n, acc);
 }
 
-template <typename T>
+// GLU: a thread per column of the result, from two rows of w
+template <typename T, bool GLU>
 __global__ __launch_bounds__(256) void moe_rows_kernel(const MoeGemmArgs p) {
   if ((int)blockIdx.y >= *p.count) return;
   const int* tile = p.tiles + (size_t)blockIdx.y * 3;
   const int expert = tile[0], row0 = tile[1], rows = tile[2];
-  const int n = blockIdx.x * 256 + threadIdx.x;
-  if (n >= p.n) return;
+  const int c = blockIdx.x * 256 + threadIdx.x, cols = GLU ? p.n / 2 : p.n;
+  if (c >= cols) return;
+  const int n = GLU ? c / 2 * 4 + c % 2 : c;
   const T* w = (const T*)p.w + ((size_t)expert * p.n + n) * p.k;
   const T* x[16];
-  float acc[16];
+  float acc[16], up[GLU ? 16 : 1];
 #pragma unroll
   for (int r = 0; r < 16; ++r) {
     const int at = row0 + min(r, rows - 1);
     x[r] = (const T*)p.x + (size_t)(p.rows != nullptr ? p.rows[at] : at) * p.k;
     acc[r] = 0.f;
+    if (GLU) up[r] = 0.f;
   }
   for (int k = 0; k < p.k; ++k) {
-    const float wv = to_f(w[k]);
+    const float wv = to_f(w[k]), wu = GLU ? to_f(w[2 * (size_t)p.k + k]) : 0.f;
 #pragma unroll
-    for (int r = 0; r < 16; ++r) acc[r] += wv * to_f(x[r][k]);
+    for (int r = 0; r < 16; ++r) {
+      const float xv = to_f(x[r][k]);
+      acc[r] += wv * xv;
+      if (GLU) up[r] += wu * xv;
+    }
   }
 #pragma unroll
   for (int r = 0; r < 16; ++r)
     if (r < rows)
-      ((T*)p.out)[(size_t)(row0 + r) * p.n + n] =
-          from_f<T>(p.relu2 ? relu2_f(acc[r]) : acc[r]);
+      ((T*)p.out)[(size_t)(row0 + r) * cols + c] = from_f<T>(
+          GLU ? swiglu_f(acc[r], up[r]) : p.relu2 ? relu2_f(acc[r]) : acc[r]);
+}
+
+template <typename T>
+void moe_rows(const MoeGemmArgs& p, hipStream_t s) {
+  const dim3 grid(((p.swiglu ? p.n / 2 : p.n) + 255) / 256, p.max_tiles);
+  if (p.swiglu) {
+    moe_rows_kernel<T, true><<<grid, 256, 0, s>>>(p);
+  } else {
+    moe_rows_kernel<T, false><<<grid, 256, 0, s>>>(p);
+  }
 }
 
 }  // namespace
@@ -273,12 +301,8 @@ __global__ __launch_bounds__(256) void moe_rows_kernel(const MoeGemmArgs p) {
 extern "C" void launch_moe_gemm(const MoeGemmArgs* p, int f32, int vec,
                                 hipStream_t s) {
   if (!vec) {                                   // tile <= 16
-    const dim3 grid((p->n + 255) / 256, p->max_tiles);
-    if (f32) {
-      moe_rows_kernel<float><<<grid, 256, 0, s>>>(*p);
-    } else {
-      moe_rows_kernel<__hip_bfloat16><<<grid, 256, 0, s>>>(*p);
-    }
+    if (f32) moe_rows<float>(*p, s);
+    else moe_rows<__hip_bfloat16>(*p, s);
   } else if (p->tile <= 16) {
     moe_skinny_kernel<<<dim3((p->n + 15) / 16, p->max_tiles), SW * 64, 0,
                         s>>>(*p);

@@ -2,8 +2,10 @@
 //
 //   logits   x W^T with f32 sums.  W rows are MFMA A fragments: lanes are tokens,
 //            registers experts.
-//   choose   one wave per token: sigmoid, correction, the two best of each group
-//            of neighbours, the best groups, the best experts of those.  Ranks
+//   choose   one wave per token: sigmoid (or the logit itself), correction, the
+//            two best of each group of neighbours, the best groups, the best
+//            experts of those; weights are the sigmoids, or a softmax over the
+//            chosen.  Ranks
 //            are counted, not sorted: an expert's rank is the number of experts
 //            ahead of it in the order (score, index), which is total, so every
 //            place is filled exactly once whatever the scores are.
@@ -140,7 +142,8 @@ DEV_INLINE void choose(const MoeRouteArgs& p, const int token, float* choice,
   float* group = choice + ep;
   for (int e = lane; e < ep; e += 64)           // NaN becomes the least score
     choice[e] = e < p.experts
-        ? fmaxf(sigmoid_exact(z[e]) + p.correction[e], -3e38f) : -INFINITY;
+        ? fmaxf((p.softmax ? z[e] : sigmoid_exact(z[e])) + p.correction[e],
+                -3e38f) : -INFINITY;
   wave_fence();
   const int size = p.experts / p.groups;
   if (p.keep < p.groups) {
@@ -163,13 +166,31 @@ DEV_INLINE void choose(const MoeRouteArgs& p, const int token, float* choice,
         for (int i = 0; i < size; ++i) choice[g * size + i] = -INFINITY;
     wave_fence();
   }
+  float most = -INFINITY, sum = 0.f;
+  if (p.softmax) {
+    for (int e = lane; e < p.experts; e += 64) most = fmaxf(most, choice[e]);
+    most = wave_max(most);
+  }
   for (int e = lane; e < p.experts; e += 64) {
     const float mine = choice[e];
     if (mine == -INFINITY) continue;
     const int rank = rank_of(choice, ep, mine, e);
     if (rank < p.top) {
+      const float w = p.softmax ? expf(mine - most) : sigmoid_exact(z[e]);
       p.ids[(size_t)token * p.top + rank] = e;
-      p.weights[(size_t)token * p.top + rank] = sigmoid_exact(z[e]);
+      p.weights[(size_t)token * p.top + rank] = w;
+      sum += w;
+    }
+  }
+  if (p.softmax) {
+    // each lane divides the weights that it wrote itself
+    const float inv = 1.f / wave_sum(sum);
+    for (int e = lane; e < p.experts; e += 64) {
+      const float mine = choice[e];
+      if (mine == -INFINITY) continue;
+      const int rank = rank_of(choice, ep, mine, e);
+      if (rank < p.top)
+        p.weights[(size_t)token * p.top + rank] = expf(mine - most) * inv;
     }
   }
   wave_fence();

@@ -1,7 +1,13 @@
 // Causal attention over paged keys and values (gfx950): grouped heads, key and
-// value sizes of their own, soft-capped scores and a silent key of score zero
-// (a sink).  Pages are [page, kv head, row, size]: a head's 16 rows are one
-// contiguous piece.
+// value sizes of their own, soft-capped scores, a silent key of score zero (a
+// sink), a sliding window, and differential heads.  Pages are [page, kv head,
+// row, size]: a head's 16 rows are one contiguous piece.
+//
+// A differential head (MAPS 2) has two queries and two keys side by side, whose
+// softmaxes weigh the same values; its output is o1 - lam o2, divided by its
+// root mean square.  Prompts keep both maps' sums in one wave, so values are read
+// once; decode takes the maps as two query heads whose queries are zero in each
+// other's half of the key.
 //
 //   prompt   128 query rows of one head per workgroup over 64-key tiles.  S^T =
 //            K Q^T, so a query is a lane column and the softmax registers are
@@ -14,6 +20,8 @@
 //            straight into MFMA operands, value rows through a wave's own LDS
 //            strip.  The waves meet at the end, the splits in a second kernel.
 //   rows     one wave per (query row, head), any sizes, bf16 or f32.
+//
+// A window starts the walk over keys at the first one that a row sees.
 //
 // A soft cap bounds the scores; when its exponentials fit f32 with room (BOUND),
 // nothing has to be subtracted, and the running maximum and every rescaling go.
@@ -52,14 +60,19 @@ constexpr float BOUND_LOG2 = 100.f;
 
 constexpr int KT = 64;
 
-template <int DK, int DV, int NW, int QT, bool BOUND>
+// A wave keeps QT sums: of QT query tiles, or (MAPS 2) of one tile's two maps.
+template <int DK, int DV, int NW, int QT, bool BOUND, int MAPS = 1>
 __global__ __launch_bounds__(NW * 64, (DK + DV) > 256 ? 1 : 2)
 void paged_prefill_kernel(const PagedAttnArgs p) {
-  constexpr int KP = DK + 16, VP = DV + 16;   // 8 banks per row
-  constexpr int ROWS = NW * QT * 16;          // 128
+  static_assert(MAPS == 1 || (MAPS == 2 && QT == 2 && !BOUND), "maps");
+  constexpr int DKM = DK * MAPS;              // a key row, maps side by side
+  constexpr int KP = DKM + 16, VP = DV + 16;  // 8 banks per row
+  constexpr int WR = QT / MAPS * 16;          // query rows of a wave
+  constexpr int ROWS = NW * WR;               // 128
   constexpr int NT = NW * 64;
-  constexpr int KPC = KT * DK / 8 / NT, VPC = KT * DV / 8 / NT;
-  static_assert(KPC * NT * 8 == KT * DK && VPC * NT * 8 == KT * DV, "tile");
+  constexpr int KPC = KT * DKM / 8 / NT, VPC = (KT * DV / 8 + NT - 1) / NT;
+  constexpr bool VFULL = VPC * NT * 8 == KT * DV;
+  static_assert(KPC * NT * 8 == KT * DKM, "tile");
   __shared__ __hip_bfloat16 ks[KT * KP];
   __shared__ __hip_bfloat16 vs[KT * VP];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -80,19 +93,20 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
 
   const __hip_bfloat16* q = (const __hip_bfloat16*)p.q + head * p.q_head;
   const __hip_bfloat16* k = (const __hip_bfloat16*)p.k +
-                            (size_t)kvh * p.page_size * p.d;
+                            (size_t)kvh * p.page_size * p.d * MAPS;
   const __hip_bfloat16* v = (const __hip_bfloat16*)p.v +
                             (size_t)kvh * p.page_size * p.dv;
-  const size_t k_page = (size_t)p.kv_heads * p.page_size * p.d;
+  const size_t k_page = (size_t)p.kv_heads * p.page_size * p.d * MAPS;
   const size_t v_page = (size_t)p.kv_heads * p.page_size * p.dv;
 
   mf_bf8 qf[QT][DK / 32];
   int qpos[QT];
 #pragma unroll
   for (int t = 0; t < QT; ++t) {
-    const int r = t0 + (wave * QT + t) * 16 + gl;
+    const int r = t0 + wave * WR + t / MAPS * 16 + gl;
     qpos[t] = qoff + r;                       // may lie past the end: unused
-    const __hip_bfloat16* qr = q + (size_t)(qrow0 + min(r, qlen - 1)) * p.q_row;
+    const __hip_bfloat16* qr = q + (size_t)(qrow0 + min(r, qlen - 1)) * p.q_row +
+                               t % MAPS * p.d;
 #pragma unroll
     for (int s = 0; s < DK / 32; ++s) {
       const int d = s * 32 + gs * 8;
@@ -101,15 +115,19 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
     }
   }
   const int last = min(qoff + t0 + ROWS - 1, klen - 1);
-  const int whi = min(qoff + t0 + (wave + 1) * QT * 16 - 1, klen - 1);
+  const int whi = min(qoff + t0 + (wave + 1) * WR - 1, klen - 1);
   const int kt1 = last / KT;
+  // keys before a window; a bounded score's form has none
+  const int behind = !BOUND && p.window > 0 ? p.window : 1 << 30;
+  const int wlo = qoff + t0 + wave * WR - behind + 1;
+  const int kt0 = max(qoff + t0 - behind + 1, 0) / KT;
 
   // keys past the end repeat the last one, so every row read is a written one
   int kpg[KPC], vpg[VPC];
   auto pages = [&](int kt) {
 #pragma unroll
     for (int i = 0; i < KPC; ++i)
-      kpg[i] = table[min(kt * KT + (tid + i * NT) / (DK / 8), klen - 1) >>
+      kpg[i] = table[min(kt * KT + (tid + i * NT) / (DKM / 8), klen - 1) >>
                      p.page_shift];
 #pragma unroll
     for (int i = 0; i < VPC; ++i)
@@ -121,10 +139,12 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
   auto fetch = [&](int kt) {
 #pragma unroll
     for (int i = 0; i < KPC; ++i) {
-      const int e = tid + i * NT, c = (e % (DK / 8)) * 8;
-      const int at = min(kt * KT + e / (DK / 8), klen - 1) & (p.page_size - 1);
+      const int e = tid + i * NT, cm = (e % (DKM / 8)) * 8;
+      const int map = MAPS == 1 ? 0 : cm / DK, c = cm - map * DK;
+      const int at = min(kt * KT + e / (DKM / 8), klen - 1) &
+                     (p.page_size - 1);
       kr[i] = c < p.d ? *reinterpret_cast<const u32x4*>(
-                            k + kpg[i] * k_page + at * p.d + c)
+                            k + kpg[i] * k_page + (at * MAPS + map) * p.d + c)
                       : zero4;
     }
 #pragma unroll
@@ -139,13 +159,15 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
   auto land = [&]() {
 #pragma unroll
     for (int i = 0; i < KPC; ++i) {
-      const int e = tid + i * NT, key = e / (DK / 8), c = (e % (DK / 8)) * 8;
+      const int e = tid + i * NT, key = e / (DKM / 8);
+      const int c = (e % (DKM / 8)) * 8;
       *reinterpret_cast<u32x4*>(&ks[key * KP + c]) = kr[i];
     }
 #pragma unroll
     for (int i = 0; i < VPC; ++i) {
       const int e = tid + i * NT, key = e / (DV / 8), c = (e % (DV / 8)) * 8;
-      *reinterpret_cast<u32x4*>(&vs[key * VP + c]) = vr[i];
+      if (VFULL || e < KT * DV / 8)
+        *reinterpret_cast<u32x4*>(&vs[key * VP + c]) = vr[i];
     }
   };
 
@@ -159,10 +181,10 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
     for (int d = 0; d < DV / 16; ++d) acc[t][d] = {0.f, 0.f, 0.f, 0.f};
   }
   const ScoreMap score(p);
-  pages(0);
-  fetch(0);
-  pages(min(1, kt1));
-  for (int kt = 0; kt <= kt1; ++kt) {
+  pages(kt0);
+  fetch(kt0);
+  pages(min(kt0 + 1, kt1));
+  for (int kt = kt0; kt <= kt1; ++kt) {
     __syncthreads();                          // the tile before is read
     land();
     __syncthreads();
@@ -171,7 +193,8 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
       pages(min(kt + 2, kt1));
     }
     const int k0 = kt * KT;
-    if (k0 > whi) continue;                   // barriers stay uniform
+    // barriers stay uniform
+    if (k0 > whi || k0 + KT - 1 < wlo) continue;
 
     f32x4 s[QT][4];
 #pragma unroll
@@ -181,16 +204,19 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
 #pragma unroll
     for (int c = 0; c < 4; ++c)
 #pragma unroll
-      for (int st = 0; st < DK / 32; ++st) {
-        const mf_bf8 kf = frag8(&ks[(c * 16 + gl) * KP + st * 32 + gs * 8]);
+      for (int st = 0; st < DK / 32; ++st)
 #pragma unroll
-        for (int t = 0; t < QT; ++t)
-          s[t][c] = mfma_bf16_k32(kf, qf[t][st], s[t][c]);
-      }
+        for (int map = 0; map < MAPS; ++map) {
+          const mf_bf8 kf = frag8(
+              &ks[(c * 16 + gl) * KP + map * DK + st * 32 + gs * 8]);
+#pragma unroll
+          for (int t = map; t < QT; t += MAPS)
+            s[t][c] = mfma_bf16_k32(kf, qf[t][st], s[t][c]);
+        }
     mf_bf8 ph[QT][2], pl[QT][2];
 #pragma unroll
     for (int t = 0; t < QT; ++t) {
-      const int hi = qpos[t];
+      const int hi = qpos[t], lo = hi - behind;
       float mn = 0.f;
       if (!BOUND) {
         float mx = MASKED;
@@ -199,7 +225,8 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
             const int j = k0 + c * 16 + gs * 4 + r;
-            const float x = j <= hi ? score(s[t][c][r]) : MASKED;
+            const float x =
+                j <= hi && j > lo ? score(s[t][c][r]) : MASKED;
             s[t][c][r] = x;
             mx = fmaxf(mx, x);
           }
@@ -219,7 +246,8 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
         for (int r = 0; r < 4; ++r) {
           const int j = k0 + c * 16 + gs * 4 + r;
           const float x = BOUND ? score(s[t][c][r]) : s[t][c][r] - mn;
-          const float e = j <= hi ? exp2_fast(x) : 0.f;
+          const float e =
+              j <= hi && (BOUND || j > lo) ? exp2_fast(x) : 0.f;
           sum += e;
           __bf16 h, lw;
           split_bf16(e, h, lw);
@@ -245,15 +273,33 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
       }
   }
 
+  float sums[QT];
 #pragma unroll
   for (int t = 0; t < QT; ++t) {
-    float sum = l[t];
-    sum += __shfl_xor(sum, 16, 64);
-    sum += __shfl_xor(sum, 32, 64);
-    if (p.sink) sum += exp2_fast(-m[t]);
-    const int r = t0 + (wave * QT + t) * 16 + gl;
+    sums[t] = l[t];
+    sums[t] += __shfl_xor(sums[t], 16, 64);
+    sums[t] += __shfl_xor(sums[t], 32, 64);
+    if (p.sink) sums[t] += exp2_fast(-m[t]);
+  }
+  if constexpr (MAPS == 2) {
+    // the difference of the maps, over its root mean square, in acc[0]
+    const float f1 = 1.f / sums[0], f2 = p.lam[0] / sums[1];
+    float ss = 0.f;
+#pragma unroll
+    for (int d = 0; d < DV / 16; ++d) {
+      acc[0][d] = acc[0][d] * f1 - acc[1][d] * f2;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss += acc[0][d][e] * acc[0][d][e];
+    }
+    ss += __shfl_xor(ss, 16, 64);
+    ss += __shfl_xor(ss, 32, 64);
+    sums[0] = sqrtf(ss / p.dv + p.out_eps) / p.out_scale;
+  }
+#pragma unroll
+  for (int t = 0; t < QT / MAPS; ++t) {
+    const int r = t0 + wave * WR + t * 16 + gl;
     if (r >= qlen) continue;
-    const float inv = 1.f / sum;
+    const float inv = 1.f / sums[t];
     __hip_bfloat16* o = (__hip_bfloat16*)p.out + (size_t)(qrow0 + r) * p.o_row +
                         (size_t)head * p.dv;
 #pragma unroll
@@ -270,7 +316,8 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
 
 constexpr int DW = 4;                         // waves of a decode workgroup
 
-template <int DK, int DV, bool BOUND>
+// DK: a key row, maps side by side
+template <int DK, int DV, bool BOUND, int MAPS = 1>
 __global__ __launch_bounds__(DW * 64, (DK + DV) > 256 ? 1 : 2)
 void paged_decode_kernel(const PagedAttnArgs p) {
   constexpr int VP = DV + 16, VL = DV / 16;   // VL 16-byte loads of 32 rows
@@ -283,30 +330,37 @@ void paged_decode_kernel(const PagedAttnArgs p) {
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int gl = lane & 15, gs = lane >> 4;
   const int split = blockIdx.x, seq = blockIdx.y;
-  const int ratio = p.heads / p.kv_heads, tiles = (ratio + 15) / 16;
+  // (head, map) pairs of a kv head, 16 at a time
+  const int ratio = p.heads / p.kv_heads * MAPS, tiles = (ratio + 15) / 16;
   const int kvh = blockIdx.z / tiles, r0 = (blockIdx.z % tiles) * 16;
   const int h0 = kvh * ratio + r0, nh = min(16, ratio - r0);
+  const int kd = p.d * MAPS;
   const int pos = p.ctx[seq] - 1;
-  const int steps = (pos + DW * 32) / (DW * 32);
+  const int lo = !BOUND && p.window > 0 ? max(pos - p.window + 1, 0) : 0;
+  const int first = lo / (DW * 32);
+  const int steps = pos / (DW * 32) + 1 - first;
   const int per = (steps + p.splits - 1) / p.splits;
-  const int s_beg = split * per, s_end = min(s_beg + per, steps);
+  const int s_beg = first + split * per;
+  const int s_end = min(s_beg + per, first + steps);
   const int* table = p.tables + (size_t)seq * p.max_pages;
-  const size_t k_page = (size_t)p.kv_heads * p.page_size * p.d;
+  const size_t k_page = (size_t)p.kv_heads * p.page_size * kd;
   const size_t v_page = (size_t)p.kv_heads * p.page_size * p.dv;
   const __hip_bfloat16* k = (const __hip_bfloat16*)p.k +
-                            (size_t)kvh * p.page_size * p.d;
+                            (size_t)kvh * p.page_size * kd;
   const __hip_bfloat16* v = (const __hip_bfloat16*)p.v +
                             (size_t)kvh * p.page_size * p.dv;
   __hip_bfloat16* vs = (__hip_bfloat16*)(smem + wave * PER);
 
+  const int qh = h0 + min(gl, nh - 1);
   const __hip_bfloat16* q = (const __hip_bfloat16*)p.q +
-      (size_t)seq * p.q_row + (size_t)(h0 + min(gl, nh - 1)) * p.q_head;
+      (size_t)seq * p.q_row + (size_t)(qh / MAPS) * p.q_head;
+  const int q_lo = qh % MAPS * p.d;           // its map's part of the key
   mf_bf8 qf[DK / 32];
 #pragma unroll
   for (int s = 0; s < DK / 32; ++s) {
     const int d = s * 32 + gs * 8;
     mf_bf8 z = {};
-    qf[s] = d < p.d ? frag8(q + d) : z;
+    qf[s] = d >= q_lo && d < q_lo + p.d ? frag8(q + d) : z;
   }
   float m = BOUND || p.sink ? 0.f : MASKED, l = 0.f;
   f32x4 acc[DV / 16];
@@ -329,13 +383,13 @@ void paged_decode_kernel(const PagedAttnArgs p) {
     at1 = b & (p.page_size - 1);
   };
   auto fetch = [&]() {
-    const __hip_bfloat16* k0 = k + pg0 * k_page + (at0 + gl) * p.d;
-    const __hip_bfloat16* k1 = k + pg1 * k_page + (at1 + gl) * p.d;
+    const __hip_bfloat16* k0 = k + pg0 * k_page + (at0 + gl) * kd;
+    const __hip_bfloat16* k1 = k + pg1 * k_page + (at1 + gl) * kd;
 #pragma unroll
     for (int s = 0; s < DK / 32; ++s) {
       const int d = s * 32 + gs * 8;
-      kr[0][s] = d < p.d ? frag8(k0 + d) : zero8;
-      kr[1][s] = d < p.d ? frag8(k1 + d) : zero8;
+      kr[0][s] = d < kd ? frag8(k0 + d) : zero8;
+      kr[1][s] = d < kd ? frag8(k1 + d) : zero8;
     }
     const __hip_bfloat16* v0 = v + pg0 * v_page + at0 * p.dv;
     const __hip_bfloat16* v1 = v + pg1 * v_page + at1 * p.dv;
@@ -383,7 +437,7 @@ void paged_decode_kernel(const PagedAttnArgs p) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int j = j0 + c * 16 + gs * 4 + r;
-          const float x = j <= pos ? score(s[c][r]) : MASKED;
+          const float x = j <= pos && j >= lo ? score(s[c][r]) : MASKED;
           s[c][r] = x;
           mx = fmaxf(mx, x);
         }
@@ -403,7 +457,8 @@ void paged_decode_kernel(const PagedAttnArgs p) {
       for (int r = 0; r < 4; ++r) {
         const int j = j0 + c * 16 + gs * 4 + r;
         const float x = BOUND ? score(s[c][r]) : s[c][r] - mn;
-        const float e = j <= pos ? exp2_fast(x) : 0.f;
+        const float e =
+            j <= pos && (BOUND || j >= lo) ? exp2_fast(x) : 0.f;
         l += e;
         __bf16 h, lw;
         split_bf16(e, h, lw);
@@ -442,9 +497,10 @@ void paged_decode_kernel(const PagedAttnArgs p) {
   for (int d = 0; d < DV / 16; ++d) sums[d * 64 + lane] = acc[d] * mine;
   __syncthreads();
   if (gl >= nh) return;
-  const size_t row = (size_t)seq * p.heads + h0 + gl;
-  const size_t part = (size_t)split * p.rows * p.heads + row;
-  if (p.splits > 1 && wave == 0 && gs == 0) {
+  const size_t row = (size_t)seq * p.heads * MAPS + h0 + gl;
+  const size_t part = (size_t)split * p.rows * p.heads * MAPS + row;
+  const bool parts = MAPS > 1 || p.splits > 1;
+  if (parts && wave == 0 && gs == 0) {
     p.part_ml[part * 2] = M;
     p.part_ml[part * 2 + 1] = L;
   }
@@ -456,7 +512,7 @@ void paged_decode_kernel(const PagedAttnArgs p) {
 #pragma unroll
     for (int w = 0; w < DW; ++w)
       o += ((const f32x4*)(smem + w * PER))[d * 64 + lane];
-    if (p.splits > 1) {
+    if (parts) {
       *reinterpret_cast<f32x4*>(&p.part_o[part * p.dv + c]) = o;
     } else {
       union { uint2 u; __hip_bfloat16 e[4]; } ov;
@@ -497,8 +553,50 @@ __global__ __launch_bounds__(64) void paged_combine_kernel(
   }
 }
 
+// The same of a differential head's two maps, then their difference over its
+// root mean square.  dv <= 256
+__global__ __launch_bounds__(64) void paged_difference_kernel(
+    const PagedAttnArgs p) {
+  __shared__ float f[2][64];                  // splits <= 64
+  const size_t row = blockIdx.x;              // seq * heads + head
+  const size_t rows = (size_t)p.rows * p.heads * 2;
+  const int tid = threadIdx.x;
+  const bool on = tid < p.splits;
+#pragma unroll
+  for (int map = 0; map < 2; ++map) {
+    const size_t at = tid * rows + row * 2 + map;
+    const float m = on ? p.part_ml[at * 2] : MASKED;
+    const float l = on ? p.part_ml[at * 2 + 1] : 0.f;
+    const float M = p.sink ? fmaxf(wave_max(m), 0.f) : wave_max(m);
+    const float w = on ? exp2_fast(m - M) : 0.f;
+    f[map][tid] = w / (wave_sum(l * w) + (p.sink ? exp2_fast(-M) : 0.f)) *
+                  (map ? -p.lam[0] : 1.f);
+  }
+  __syncthreads();
+  const int d = tid * 4;
+  f32x4 o = {0.f, 0.f, 0.f, 0.f};
+  if (d < p.dv) {
+#pragma unroll 4
+    for (int s = 0; s < p.splits; ++s) {
+      const float* at = &p.part_o[(s * rows + row * 2) * p.dv + d];
+      o += *reinterpret_cast<const f32x4*>(at) * f[0][s];
+      o += *reinterpret_cast<const f32x4*>(at + p.dv) * f[1][s];
+    }
+  }
+  const float ss = wave_sum(o[0] * o[0] + o[1] * o[1] + o[2] * o[2] +
+                            o[3] * o[3]);
+  const float inv = p.out_scale / sqrtf(ss / p.dv + p.out_eps);
+  if (d >= p.dv) return;
+  union { uint2 u; __hip_bfloat16 e[4]; } ov;
+#pragma unroll
+  for (int r = 0; r < 4; ++r) ov.e[r] = f2bf(o[r] * inv);
+  *reinterpret_cast<uint2*>((__hip_bfloat16*)p.out +
+                            (row / p.heads) * p.o_row +
+                            (row % p.heads) * p.dv + d) = ov.u;
+}
+
 // NACC: value dimensions per lane (dv <= 64 * NACC)
-template <typename T, int NACC>
+template <typename T, int NACC, int MAPS>
 __global__ __launch_bounds__(256) void paged_rows_kernel(
     const PagedAttnArgs p) {
   extern __shared__ float rows_smem[];
@@ -507,66 +605,89 @@ __global__ __launch_bounds__(256) void paged_rows_kernel(
   if (item >= (long)p.rows * p.heads) return;       // whole wave leaves
   const int row = (int)(item / p.heads), head = (int)(item % p.heads);
   const int kvh = head / (p.heads / p.kv_heads);
-  float* q = rows_smem + wave * (p.d + 64);
-  float* pr = q + p.d;
+  const int kd = p.d * MAPS;
+  float* q = rows_smem + wave * (kd + 64 * MAPS);
+  float* pr = q + kd;
   const T* qp = (const T*)p.q + row * p.q_row + head * p.q_head;
-  for (int i = lane; i < p.d; i += 64) q[i] = to_f(qp[i]);
+  for (int i = lane; i < kd; i += 64) q[i] = to_f(qp[i]);
   __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
   __builtin_amdgcn_wave_barrier();
   const int seq = p.ctx != nullptr ? row : p.row_info[row * 2];
   const int pos = p.ctx != nullptr ? p.ctx[row] - 1 : p.row_info[row * 2 + 1];
+  const int lo = p.window > 0 ? max(pos - p.window + 1, 0) : 0;
   const int* table = p.tables + (size_t)seq * p.max_pages;
   auto key_row = [&](int j) -> size_t {
     return ((size_t)table[j / p.page_size] * p.kv_heads + kvh) * p.page_size +
            j % p.page_size;
   };
-  float m = p.sink ? 0.f : -INFINITY, l = p.sink ? 1.f : 0.f, acc[NACC];
+  float m[MAPS], l[MAPS], acc[MAPS][NACC];
 #pragma unroll
-  for (int i = 0; i < NACC; ++i) acc[i] = 0.f;
+  for (int a = 0; a < MAPS; ++a) {
+    m[a] = p.sink ? 0.f : -INFINITY;
+    l[a] = p.sink ? 1.f : 0.f;
+#pragma unroll
+    for (int i = 0; i < NACC; ++i) acc[a][i] = 0.f;
+  }
 
-  for (int j0 = 0; j0 <= pos; j0 += 64) {
+  for (int j0 = lo; j0 <= pos; j0 += 64) {
     const int j = j0 + lane;
-    float s = -INFINITY;
-    if (j <= pos) {
-      const T* kr = (const T*)p.k + key_row(j) * p.d;
-      float dot = 0.f;
-      for (int i = 0; i < p.d; ++i) dot += q[i] * to_f(kr[i]);
-      s = dot * p.scale;
-      if (p.softcap > 0.f) s = p.softcap * tanhf(s / p.softcap);
+#pragma unroll
+    for (int a = 0; a < MAPS; ++a) {
+      float s = -INFINITY;
+      if (j <= pos) {
+        const T* kr = (const T*)p.k + key_row(j) * kd + a * p.d;
+        float dot = 0.f;
+        for (int i = 0; i < p.d; ++i) dot += q[a * p.d + i] * to_f(kr[i]);
+        s = dot * p.scale;
+        if (p.softcap > 0.f) s = p.softcap * tanhf(s / p.softcap);
+      }
+      const float mn = fmaxf(m[a], wave_max(s));
+      const float e = expf(s - mn);
+      const float corr = expf(m[a] - mn);
+      l[a] = l[a] * corr + wave_sum(e);
+      m[a] = mn;
+      pr[a * 64 + lane] = e;
+#pragma unroll
+      for (int i = 0; i < NACC; ++i) acc[a][i] *= corr;
     }
-    const float mn = fmaxf(m, wave_max(s));
-    const float e = expf(s - mn);
-    const float corr = expf(m - mn);
-    l = l * corr + wave_sum(e);
-    m = mn;
-    pr[lane] = e;
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
     __builtin_amdgcn_wave_barrier();
-#pragma unroll
-    for (int i = 0; i < NACC; ++i) acc[i] *= corr;
     const int n = min(64, pos - j0 + 1);
     for (int t = 0; t < n; ++t) {
       const T* vr = (const T*)p.v + key_row(j0 + t) * p.dv;
-      const float w = pr[t];
 #pragma unroll
       for (int i = 0; i < NACC; ++i) {
         const int d = i * 64 + lane;
-        if (d < p.dv) acc[i] += w * to_f(vr[d]);
+        const float x = d < p.dv ? to_f(vr[d]) : 0.f;
+#pragma unroll
+        for (int a = 0; a < MAPS; ++a) acc[a][i] += pr[a * 64 + t] * x;
       }
     }
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
     __builtin_amdgcn_wave_barrier();
   }
   T* op = (T*)p.out + row * p.o_row + (size_t)head * p.dv;
+  float f = 1.f;
+#pragma unroll
+  for (int i = 0; i < NACC; ++i) acc[0][i] /= l[0];
+  if constexpr (MAPS == 2) {
+    float ss = 0.f;                             // dimensions past dv are zero
+#pragma unroll
+    for (int i = 0; i < NACC; ++i) {
+      acc[0][i] -= p.lam[0] * (acc[1][i] / l[1]);
+      ss += acc[0][i] * acc[0][i];
+    }
+    f = p.out_scale / sqrtf(wave_sum(ss) / p.dv + p.out_eps);
+  }
 #pragma unroll
   for (int i = 0; i < NACC; ++i) {
     const int d = i * 64 + lane;
-    if (d < p.dv) op[d] = from_f<T>(acc[i] / l);
+    if (d < p.dv) op[d] = from_f<T>(acc[0][i] * f);
   }
 }
 
 bool bounded(const PagedAttnArgs& p) {
-  return p.softcap > 0.f && p.softcap * LOG2E <= BOUND_LOG2;
+  return p.softcap > 0.f && p.softcap * LOG2E <= BOUND_LOG2 && p.window == 0;
 }
 
 template <int DK>
@@ -586,13 +707,28 @@ void prefill_dv(const PagedAttnArgs& p, hipStream_t s) {
 #undef PP_GO
 }
 
+// two maps: a wave's two sums are one query tile's
 template <int DK>
+void prefill_maps(const PagedAttnArgs& p, hipStream_t s) {
+  const int grid = 8 * ((p.n_blocks * p.heads + 7) / 8);
+#define PP_GO(DV)                                                             \
+  paged_prefill_kernel<DK, DV, 8, 2, false, 2><<<grid, 512, 0, s>>>(p)
+  if (p.dv <= 64) PP_GO(64);
+  else if (p.dv <= 96) PP_GO(96);
+  else if (p.dv <= 128) PP_GO(128);
+  else PP_GO(256);
+#undef PP_GO
+}
+
+template <int DK, int MAPS = 1>
 void decode_dv(const PagedAttnArgs& p, hipStream_t s) {
-  const int tiles = (p.heads / p.kv_heads + 15) / 16;
+  const int tiles = (p.heads / p.kv_heads * MAPS + 15) / 16;
   const dim3 grid(p.splits, p.rows, p.kv_heads * tiles);
 #define PD_GO(DV)                                                             \
   do {                                                                        \
-    if (bounded(p))                                                           \
+    if constexpr (MAPS > 1)                                                   \
+      paged_decode_kernel<DK, DV, false, MAPS><<<grid, DW * 64, 0, s>>>(p);   \
+    else if (bounded(p))                                                      \
       paged_decode_kernel<DK, DV, true><<<grid, DW * 64, 0, s>>>(p);          \
     else                                                                      \
       paged_decode_kernel<DK, DV, false><<<grid, DW * 64, 0, s>>>(p);         \
@@ -607,8 +743,15 @@ void decode_dv(const PagedAttnArgs& p, hipStream_t s) {
 template <typename T>
 void paged_rows_t(const PagedAttnArgs& p, hipStream_t s) {
   const int grid = (int)(((long)p.rows * p.heads + 3) / 4);
-  const size_t lds = sizeof(float) * 4 * (p.d + 64);
-#define PR_GO(N) paged_rows_kernel<T, N><<<grid, 256, lds, s>>>(p)
+  const size_t lds = sizeof(float) * 4 * p.maps * (p.d + 64);
+#define PR_GO(N)                                                              \
+  do {                                                                        \
+    if (p.maps == 2) {                                                        \
+      paged_rows_kernel<T, N, 2><<<grid, 256, lds, s>>>(p);                   \
+    } else {                                                                  \
+      paged_rows_kernel<T, N, 1><<<grid, 256, lds, s>>>(p);                   \
+    }                                                                         \
+  } while (0)
   if (p.dv <= 64) PR_GO(1);
   else if (p.dv <= 128) PR_GO(2);
   else if (p.dv <= 256) PR_GO(4);
@@ -624,12 +767,24 @@ extern "C" {
 int paged_block_rows() { return 128; }        // query rows per prompt block
 
 void launch_paged_prefill(const PagedAttnArgs* p, hipStream_t s) {
+  if (p->maps == 2) {
+    if (p->d <= 64) prefill_maps<64>(*p, s);
+    else prefill_maps<128>(*p, s);
+    return;
+  }
   if (p->d <= 64) prefill_dv<64>(*p, s);
   else if (p->d <= 128) prefill_dv<128>(*p, s);
   else prefill_dv<256>(*p, s);
 }
 
 void launch_paged_decode(const PagedAttnArgs* p, hipStream_t s) {
+  if (p->maps == 2) {
+    if (p->d <= 32) decode_dv<64, 2>(*p, s);
+    else if (p->d <= 64) decode_dv<128, 2>(*p, s);
+    else decode_dv<256, 2>(*p, s);
+    paged_difference_kernel<<<p->rows * p->heads, 64, 0, s>>>(*p);
+    return;
+  }
   if (p->d <= 64) decode_dv<64>(*p, s);
   else if (p->d <= 128) decode_dv<128>(*p, s);
   else decode_dv<256>(*p, s);

@@ -1,12 +1,22 @@
 // What stands between the fused query/key/value projection and attention over
-// pages: biases, rotary positions on the leading dimensions of queries and keys
-// (rotate-half pairs, any rotated size), and the paged store of keys and values,
+// pages: biases (or none), rotary positions on the leading dimensions of queries and keys
+// (rotate-half pairs, any rotated size, or none), and the paged store of keys and values,
 // in 32-bit registers and one pass.  A thread takes V pairs, or V dimensions
 // that do not rotate, of one head (a unit).
 #include "moe_args.h"
 #include "vec_io.h"
 
 namespace {
+
+template <int V>
+DEV_INLINE void load_bias(const float* b, const int at, float* o) {
+  if (b != nullptr) {
+    load_vec<V>(b + at, o);
+  } else {
+#pragma unroll
+    for (int j = 0; j < V; ++j) o[j] = 0.f;
+  }
+}
 
 // R neighbouring rows, one unit of the row: the biases are read once, the rows'
 // loads are all in flight together
@@ -38,7 +48,7 @@ __global__ __launch_bounds__(256) void rope_paged_kernel(
     const int vu = p.dv / V, head = u / vu, d = (u % vu) * V;
     const int col = p.off_v + head * p.dv + d;
     float x[R][V], b[V];
-    load_vec<V>(p.bias + col, b);
+    load_bias<V>(p.bias, col, b);
 #pragma unroll
     for (int r = 0; r < R; ++r) load_vec<V>(y[r] + col, x[r]);
 #pragma unroll
@@ -63,7 +73,7 @@ __global__ __launch_bounds__(256) void rope_paged_kernel(
   if (e >= pair_u) {                    // dimensions that do not rotate
     const int d = p.rot + (e - pair_u) * V;
     float x[R][V], b[V];
-    load_vec<V>(p.bias + col + d, b);
+    load_bias<V>(p.bias, col + d, b);
 #pragma unroll
     for (int r = 0; r < R; ++r) load_vec<V>(y[r] + col + d, x[r]);
 #pragma unroll
@@ -76,8 +86,8 @@ __global__ __launch_bounds__(256) void rope_paged_kernel(
   }
   const int d = e * V;
   float ba[V], bb[V];
-  load_vec<V>(p.bias + col + d, ba);
-  load_vec<V>(p.bias + col + half + d, bb);
+  load_bias<V>(p.bias, col + d, ba);
+  load_bias<V>(p.bias, col + half + d, bb);
   float a[R][V], b[R][V], c[R][V], s[R][V];
 #pragma unroll
   for (int r = 0; r < R; ++r) {

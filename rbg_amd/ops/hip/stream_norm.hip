@@ -1,5 +1,5 @@
-// f32 residual stream: embedding, residual add, grouped RMS norm under one or
-// two weights, and the causal input convolution.
+// f32 residual stream: residual add, grouped RMS norm under one or two weights,
+// and the causal input convolution.
 //
 // The stream x [T, W] stays f32 end to end; what the projections read is
 // written in the activation dtype (bf16 or f32).  One workgroup per token row:
@@ -14,21 +14,6 @@
 namespace {
 
 constexpr int NT = 256;
-
-template <typename T, int V>
-__global__ __launch_bounds__(NT) void embed_stream_kernel(
-    float* __restrict__ x, const T* __restrict__ table,
-    const long* __restrict__ tokens, const float scale, const int width) {
-  const T* src = table + (size_t)tokens[blockIdx.x] * width;
-  float* dst = x + (size_t)blockIdx.x * width;
-  for (int i = threadIdx.x * V; i < width; i += NT * V) {
-    float v[V];
-    load_vec<V>(src + i, v);
-#pragma unroll
-    for (int j = 0; j < V; ++j) v[j] *= scale;
-    store_vec<V>(dst + i, v);
-  }
-}
 
 // CONV: n1 becomes n1 + conv(n1) with the history of state slot slots[row]
 // (all zeros at position 0), and the history moves on by one token.
@@ -234,17 +219,6 @@ void stream_norm_t(float* x, const void* delta, const float* w1,
 }  // namespace
 
 extern "C" {
-
-void launch_embed_stream(float* x, const void* table, const long* tokens,
-                         float scale, int n, int width, int f32,
-                         hipStream_t s) {
-#define EM_GO(T, V) embed_stream_kernel<T, V><<<n, NT, 0, s>>>(               \
-      x, (const T*)table, tokens, scale, width)
-  const bool vec = width % 8 == 0;
-  if (f32) { if (vec) EM_GO(float, 8); else EM_GO(float, 1); }
-  else { if (vec) EM_GO(__hip_bfloat16, 8); else EM_GO(__hip_bfloat16, 1); }
-#undef EM_GO
-}
 
 void launch_stream_norm(float* x, const void* delta, const float* w1,
                         const float* w2, void* n1, void* n2, int tokens,

@@ -303,18 +303,22 @@ def sandwich_norm(x, rows, route, wb, w, eps, dtype):
 
 def rope_store_paged(proj, bias, cos_sin, positions, slots, heads, dim, k, v,
                      offs):
-    y = proj.float() + bias
-    half = cos_sin.shape[1] // 2
-    cs = cos_sin[positions.long()].unsqueeze(1)
-    cos, sin = cs[..., :half], cs[..., half:]
+    y = proj.float() if bias is None else proj.float() + bias
+    half = 0 if cos_sin is None else cos_sin.shape[1] // 2
+    if half:
+        cs = cos_sin[positions.long()].unsqueeze(1)
+        cos, sin = cs[..., :half], cs[..., half:]
 
     def turn(at, n):
         t = y[:, at:at + n * dim].view(-1, n, dim)
+        if not half:
+            return t
         a, b = t[..., :half], t[..., half:2 * half]
         return torch.cat([a * cos - b * sin, b * cos + a * sin,
                           t[..., 2 * half:]], dim=-1)
-    proj[:, offs[0]:offs[0] + heads * dim] = \
-        turn(offs[0], heads).flatten(1).to(proj.dtype)
+    if half or bias is not None:
+        proj[:, offs[0]:offs[0] + heads * dim] = \
+            turn(offs[0], heads).flatten(1).to(proj.dtype)
     if len(offs) == 1:
         return
     ps, kvh, vdim = k.shape[2], k.shape[1], v.shape[3]
@@ -324,37 +328,44 @@ def rope_store_paged(proj, bias, cos_sin, positions, slots, heads, dim, k, v,
         -1, kvh, vdim).to(v.dtype)
 
 
-def paged_rows(q, k, v, tables, row_info, out, scale, softcap, sink):
+def paged_rows(q, k, v, tables, row_info, out, scale, softcap, sink, window=0,
+               diff=None):
     """Each row of q [R, H, D] against the keys of its sequence up to its
     position; row_info [R, 2] = (row of tables, position)."""
     ps, kvh = k.shape[2], k.shape[1]
-    per = q.shape[1] // kvh
+    per, maps = q.shape[1] // kvh, 1 if diff is None else 2
     for r, (seq, pos) in enumerate(row_info.tolist()):
-        j = torch.arange(pos + 1)
+        j = torch.arange(max(0, pos + 1 - window) if window else 0, pos + 1)
         pages, at = tables[seq].long()[j // ps], j % ps
-        ks = k[pages, :, at].float()                # [keys, kvh, D]
-        qs = q[r].float().view(kvh, per, -1)
-        s = torch.einsum("gpd,kgd->gpk", qs, ks) * scale
+        ks = k[pages, :, at].float().view(len(j), kvh, maps, -1)
+        qs = q[r].float().view(kvh, per, maps, -1)
+        s = torch.einsum("gpmd,kgmd->gpmk", qs, ks) * scale
         if softcap > 0:
             s = softcap * torch.tanh(s / softcap)
         if sink:                                    # a key without a value
             s = torch.cat([s, torch.zeros_like(s[..., :1])], dim=-1)
-        p = torch.softmax(s, dim=-1)[..., :pos + 1]
-        o = torch.einsum("gpk,kgd->gpd", p, v[pages, :, at].float())
+        p = torch.softmax(s, dim=-1)[..., :len(j)]
+        o = torch.einsum("gpmk,kgd->gpmd", p, v[pages, :, at].float())
+        if diff is None:
+            o = o[:, :, 0]
+        else:
+            o = _rms(o[:, :, 0] - diff.lam * o[:, :, 1], diff.scale, diff.eps)
         out[r] = o.reshape(-1).to(out.dtype)
 
 
-def moe_choose(logits, correction, groups, keep, top):
+def moe_choose(logits, correction, groups, keep, top, softmax=False):
     """(experts, weights) of each token, [T, top]."""
     T, E = logits.shape
-    s = torch.sigmoid(logits)
+    s = logits if softmax else torch.sigmoid(logits)
     choice = (s + correction).view(T, groups, E // groups)
     best = choice.topk(min(2, E // groups), dim=-1).values.sum(-1)
     kept = torch.zeros(T, groups, dtype=torch.bool)
     kept.scatter_(1, best.topk(keep, dim=-1).indices, True)
     choice = choice.masked_fill(~kept.unsqueeze(-1), float("-inf"))
-    ids = choice.view(T, E).topk(top, dim=-1).indices
-    return ids, s.gather(1, ids)
+    chosen = choice.view(T, E).topk(top, dim=-1)
+    if softmax:
+        return chosen.indices, torch.softmax(chosen.values, dim=-1)
+    return chosen.indices, s.gather(1, chosen.indices)
 
 
 def moe_tiles(ids, experts, tile):
@@ -372,10 +383,86 @@ def moe_tiles(ids, experts, tile):
             torch.tensor(tiles, dtype=torch.int32).view(-1, 3))
 
 
-def expert_linear(x, w, route, gather, relu2):
-    out = x.new_empty((route.rows.numel(), w.shape[1]))
+def expert_linear(x, w, route, gather, relu2, swiglu=False):
+    out = x.new_empty((route.rows.numel(), w.shape[1] // (2 if swiglu else 1)))
     for e, at, n in route.tiles.tolist():
         rows = x[route.rows[at:at + n].long()] if gather else x[at:at + n]
         y = rows.float() @ w[e].float().T
-        out[at:at + n] = (torch.relu(y).pow(2) if relu2 else y).to(x.dtype)
+        if relu2:
+            y = torch.relu(y).pow(2)
+        elif swiglu:                    # columns gate, gate, up, up
+            y = y.unflatten(1, (-1, 2, 2))
+            y = (torch.nn.functional.silu(y[:, :, 0]) * y[:, :, 1]).flatten(1)
+        out[at:at + n] = y.to(x.dtype)
     return out
+
+
+# -- gated branches, gated delta rule -------------------------------------------
+
+
+def gate_norm(x, branches, w, eps, dtype):
+    for b in branches:
+        y = b.rows.float() if b.route is None else moe_combine(b.rows, b.route)
+        if b.bias is not None:
+            y = y + b.bias
+        x += y * b.scale * torch.sigmoid(b.logits.float() + b.gate_bias)
+    return None if w is None else _rms(x, w, eps).to(dtype)
+
+
+def silu_glu(gate, up, gate_bias, up_bias, out):
+    g, u = gate.float(), up.float()
+    if gate_bias is not None:
+        g, u = g + gate_bias, u + up_bias
+    out.copy_((torch.nn.functional.silu(g) * u).to(out.dtype))
+
+
+def short_conv(x, conv_w, ring, cu_seqlens, starts, slots):
+    taps = conv_w.shape[0]
+    out = x.new_empty(x.shape)
+    cu = cu_seqlens.tolist()
+    for b, slot in enumerate(slots.tolist()):
+        start, rows = int(starts[b]), x[cu[b]:cu[b + 1]].float()
+        hist = [ring[slot, p % taps].float() if p >= 0 else
+                torch.zeros_like(conv_w[0])
+                for p in range(start - taps + 1, start)]
+        ext = torch.cat([torch.stack(hist), rows]) if hist else rows
+        y = sum(conv_w[j] * ext[j:j + rows.shape[0]] for j in range(taps))
+        out[cu[b]:cu[b + 1]] = torch.nn.functional.silu(y).to(x.dtype)
+        for t in range(max(0, rows.shape[0] - taps + 1), rows.shape[0]):
+            ring[slot, (start + t) % taps] = rows[t].to(ring.dtype)
+    return out
+
+
+def gated_delta(p, qkv, offs, beta, decay, gate, state, slots, cu_seqlens,
+                starts, out):
+    H, D, E = state.shape[1:]
+    G = p.kv_heads
+
+    def heads(at, n, size):
+        return qkv[:, at:at + n * size].float().view(-1, n, size)
+
+    def unit(t):
+        t = t * torch.rsqrt(t.pow(2).sum(-1, keepdim=True) + p.unit_eps)
+        return t.repeat_interleave(H // G, dim=1)
+    q = unit(heads(offs[0], G, D)) * p.q_scale
+    k = unit(heads(offs[1], G, D))
+    v = heads(offs[2], H, E)
+    per = p.dt_bias.numel() // H        # 1, or D
+    rate = torch.exp(p.a_log).view(H, 1)
+    g = torch.exp(-rate * torch.nn.functional.softplus(
+        decay.float() + p.dt_bias, threshold=30).view(-1, H, per))
+    beta = torch.sigmoid(beta.float()).unsqueeze(-1)
+    z = gate.float()
+    z = torch.nn.functional.silu(z) if p.silu else torch.sigmoid(z)
+    cu = (cu_seqlens.tolist() if cu_seqlens is not None
+          else list(range(slots.numel() + 1)))
+    for b, slot in enumerate(slots.tolist()):
+        S = state[slot]
+        if int(starts[b]) == 0:
+            S.zero_()
+        for t in range(cu[b], cu[b + 1]):
+            S.mul_(g[t].unsqueeze(-1))
+            u = beta[t] * (v[t] - torch.einsum("hkv,hk->hv", S, k[t]))
+            S.add_(k[t].unsqueeze(-1) * u.unsqueeze(1))
+            o = _rms(torch.einsum("hkv,hk->hv", S, q[t]), p.norm, p.norm_eps)
+            out[t] = (o.reshape(-1) * z[t]).to(out.dtype)

@@ -40,6 +40,7 @@ HIP_SOURCES = {
     ],
     # f32-stream norms and the token mixers (delta rule, latents)
     "_hip_mix": [
+        "embed.hip",
         "stream_norm.hip",
         "gated_act.hip",
         "delta_rule.hip",
@@ -61,18 +62,33 @@ HIP_SOURCES = {
         "skinny_gemm.hip",
         "moe_bindings.cpp",
     ],
+    # gated delta rule, short convolution, gated norms and linear units
+    "_hip_gated": [
+        "embed.hip",
+        "gate_norm.hip",
+        "gated_act.hip",
+        "short_conv.hip",
+        "gated_delta.hip",
+        "gated_delta_chunk.hip",
+        "skinny_gemm.hip",
+        "gated_bindings.cpp",
+    ],
 }
 
 HIP_HEADERS = {
     "_hip_ops": ["common.h", "gemm_bindings.h"],
-    "_hip_mix": ["bind_util.h", "common.h", "gemm_bindings.h", "mfma_util.h",
-                 "mix_args.h", "vec_io.h"],
-    "_hip_moe": ["bind_util.h", "common.h", "gemm_bindings.h", "lds_stream.h",
-                 "mfma_util.h", "moe_args.h", "vec_io.h"],
+    "_hip_mix": ["bind_util.h", "common.h", "delta_scan.h", "gemm_bindings.h",
+                 "mfma_util.h", "mix_args.h", "vec_io.h"],
+    "_hip_moe": ["bind_util.h", "common.h", "expert_rows.h", "gemm_bindings.h",
+                 "lds_stream.h", "mfma_util.h", "moe_args.h", "vec_io.h"],
+    "_hip_gated": ["bind_util.h", "common.h", "delta_scan.h", "expert_rows.h",
+                   "gated_args.h", "gated_delta.h", "gemm_bindings.h",
+                   "mfma_util.h", "vec_io.h"],
 }
 
-# model architecture -> the extension with its kernels (default: _hip_ops)
-EXTENSION_OF = {"Bitatar": "_hip_mix", "Notadra": "_hip_moe"}
+# model architecture -> the extensions with its kernels (default: _hip_ops)
+EXTENSIONS_OF = {"Bitatar": ("_hip_mix",), "Notadra": ("_hip_moe",),
+                 "Gogalix": ("_hip_gated", "_hip_moe")}
 
 
 def source_hash(name: str) -> str:
@@ -116,11 +132,13 @@ def build(names: Optional[Iterable[str]] = None, clean: bool = False) -> None:
             f.write(source_hash(name))
 
 
-def ensure(name: str) -> None:
-    """Build one extension if it is missing or stale (one builder at a time)."""
-    if is_built(name) and not is_stale(name):
+def ensure(*names: str) -> None:
+    """Build extensions that are missing or stale (one builder at a time)."""
+    def due():
+        return [n for n in names if not is_built(n) or is_stale(n)]
+    if not due():
         return
     with open(os.path.join(ROOT, ".build.lock"), "w") as lock:
         fcntl.flock(lock, fcntl.LOCK_EX)
-        if not is_built(name) or is_stale(name):
-            build([name])
+        if due():
+            build(due())
