@@ -27,10 +27,13 @@ SIZES = {
 
 
 def pair(size: str, family: str = "bitatar") -> List[ModelConfig]:
-    """The family's model and the Llama of equal size."""
+    """The family's model and the one of equal size it is compared to."""
     if family == "notadra":
         from .notadra_bench import notadra_pair
         return notadra_pair(size)
+    if family == "gogalix":
+        from .gogalix_bench import gogalix_set
+        return gogalix_set(size)
     w, ff, heads, kvh, layers, rank, window, dh, dd = SIZES[size]
     return [
         BitatarConfig.stacked(
@@ -140,6 +143,9 @@ def run_kernels(size: str, batches=(1, 8, 32, 128), ctx: int = 2048,
     if family == "notadra":
         from .notadra_bench import notadra_kernels
         return notadra_kernels(size, batches, ctx, prompts)
+    if family == "gogalix":
+        from .gogalix_bench import gogalix_kernels
+        return gogalix_kernels(size, batches, ctx, prompts)
     import math
 
     from .. import ops

@@ -12,8 +12,9 @@
 // which is what delta_scan.h walks.  Every exponent there is at most zero; only
 // A and Q have factors of both signs when the matrix cores form them, e^{c_t -
 // c_7} and e^{c_7 - c_s}.  A chunk whose decays span more than RANGE forms A and
-// Q pair by pair instead, so that any decay is exact.  One decay per head
-// factors out of A and Q altogether.
+// Q from running products instead, so that any decay keeps its precision.  One
+// decay per head factors out of A and Q altogether.  Sums of log decays are taken
+// over the tokens they span, never as differences of longer ones.
 // Missing tokens of a last chunk have q = k = beta = 0 and no decay.
 #include "delta_scan.h"
 #include "gated_delta.h"
@@ -31,11 +32,15 @@ __global__ __launch_bounds__(256) void gated_prep_kernel(
   constexpr int GR = 256 / DP;          // token groups in the staging step
   constexpr int TPG = C / GR;           // tokens per group
   constexpr int NWV = (DP + 63) / 64;   // waves that share a token's channels
-  __shared__ __attribute__((aligned(16))) float qs[C * PP], ks[C * PP],
-      cs[CHANNEL ? C * PP : C];
+  // CHANNEL: kx = k e^{c_t - c_7}, qx = q e^{c_t - c_7}, ky = k e^{c_7 - c_t};
+  // in a wide chunk k, q and the decay factors.  Else kx = k, qx = q.
+  __shared__ __attribute__((aligned(16))) float kx[C * PP], qx[C * PP],
+      ky[CHANNEL ? C * PP : 4];
   __shared__ __attribute__((aligned(16))) float ls[C * SP], ts[C * SP];
+  __shared__ float fs[CHANNEL ? 1 : C * SP];    // e^{c_t - c_s} of the head
   __shared__ f32x4 half[2][64];
-  __shared__ float csum[GR][DP], nk[C][NWV], nq[C][NWV], bs[C];
+  __shared__ float csum[GR][DP], nk[C][NWV], nq[C][NWV], bs[C], lws[C];
+  __shared__ float mid[DP];                     // e^{c_7}
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int gl = lane & 15, gs = lane >> 4;
   const int tile = blockIdx.x, head = blockIdx.y;
@@ -46,13 +51,13 @@ __global__ __launch_bounds__(256) void gated_prep_kernel(
   const int D = p.dim;
   float* rec = ws + ((size_t)tile * p.heads + head) * W::SIZE;
 
-  // ---- channels x tokens: unit vectors and cumulative decays -------------
+  // ---- channels x tokens: unit vectors and decays -------------------------
   const int ch = tid % DP, grp = tid / DP;
   const bool live = ch < D;
   const int cc = min(ch, D - 1);
   const float rate = expf(p.a_log[head]);
   const float bias = p.dt_bias[CHANNEL ? head * D + cc : head];
-  float lw[TPG], kv[TPG], qv[TPG];
+  float lw[TPG], kv[TPG], qv[TPG], sum = 0.f;
 #pragma unroll
   for (int i = 0; i < TPG; ++i) {
     const int t = grp * TPG + i;
@@ -75,86 +80,118 @@ __global__ __launch_bounds__(256) void gated_prep_kernel(
       nk[t][ch >> 6] = sk;
       nq[t][ch >> 6] = sq;
     }
-    if (i) lw[i] += lw[i - 1];          // running within the group
+    if (ch == 0) lws[t] = lw[i];
+    sum += lw[i];
   }
-  csum[grp][ch] = lw[TPG - 1];
+  csum[grp][ch] = sum;
   if (tid < C)
     bs[tid] = tid < n ? sigmoid_f(to_f(((const T*)p.beta)[
         (size_t)(row0 + tid) * p.beta_row + head])) : 0.f;
   __syncthreads();
-  float base = 0.f, tot = 0.f;
+  float before = 0.f, after = 0.f, c7 = 0.f, tot = 0.f;
 #pragma unroll
   for (int g = 0; g < GR; ++g) {
-    if (g < grp) base += csum[g][ch];
+    if (g < grp) before += csum[g][ch];
+    if (g > grp) after += csum[g][ch];
+    if (g < GR / 2) c7 += csum[g][ch];
     tot += csum[g][ch];
+  }
+  bool wide = false;
+  if (CHANNEL) wide = __syncthreads_or(tot < -RANGE);
+  float bt[TPG];
+#pragma unroll
+  for (int i = TPG - 1; i >= 0; --i) {          // sums of what comes after
+    bt[i] = __expf(after);
+    after += lw[i];
   }
 #pragma unroll
   for (int i = 0; i < TPG; ++i) {
-    const int t = grp * TPG + i;
+    const int t = grp * TPG + i, at = t * PP + ch;
     float sk = 0.f, sq = 0.f;
 #pragma unroll
     for (int w = 0; w < NWV; ++w) {
       sk += nk[t][w];
       sq += nq[t][w];
     }
-    ks[t * PP + ch] = kv[i] / sqrtf(sk + p.unit_eps);
-    qs[t * PP + ch] = qv[i] * (p.q_scale / sqrtf(sq + p.unit_eps));
-    if (CHANNEL) cs[t * PP + ch] = base + lw[i];
-    else if (ch == 0) cs[t] = base + lw[i];
+    const float k = kv[i] / sqrtf(sk + p.unit_eps);
+    const float q = qv[i] * (p.q_scale / sqrtf(sq + p.unit_eps));
+    before += lw[i];                            // now c_t
+    rec[W::R + at] = q * __expf(before);
+    bt[i] *= -k;
+    if (CHANNEL) {
+      const float e = wide ? 1.f : __expf(before - c7);
+      kx[at] = k * e;
+      qx[at] = q * e;
+      ky[at] = wide ? __expf(lw[i]) : k * __expf(c7 - before);
+    } else {
+      kx[at] = k;
+      qx[at] = q;
+    }
   }
-  if (grp == 0) rec[W::DC + ch] = __expf(tot);
-  // the barrier that publishes the vectors also asks every channel
-  const bool wide = __syncthreads_or(CHANNEL && tot < -RANGE);
+  store_vec<TPG>(rec + W::BT + ch * SP + grp * TPG, bt);
+  if (grp == 0) {
+    rec[W::DC + ch] = __expf(tot);
+    mid[ch] = wide ? 1.f : __expf(c7);
+  }
+  if (!CHANNEL) {
+    const int t = tid >> 4, s = tid & 15;
+    float x = 0.f;
+    for (int j = s + 1; j <= t; ++j) x += lws[j];
+    fs[t * SP + s] = s <= t ? __expf(x) : 0.f;
+  }
+  __syncthreads();
 
-  // ---- A and Q -----------------------------------------------------------
-  // beta_t A_ts into ls, -Q_ts into the record
-  auto put = [&](bool is_q, int t, int s, float x) {
-    if (!CHANNEL && s <= t) x *= __expf(cs[t] - cs[s]);
-    if (is_q) rec[W::QB + t * SP + s] = s <= t ? -x : 0.f;
-    else ls[t * SP + s] = s < t ? bs[t] * x : 0.f;
+  // ---- A and Q: beta_t A_ts into ls, -Q_ts into the record ------------------
+  auto put_a = [&](int t, int s, float x) {
+    ls[t * SP + s] = s < t ? bs[t] * x : 0.f;
+  };
+  auto put_q = [&](int t, int s, float x) {
+    rec[W::QB + t * SP + s] = s <= t ? -x : 0.f;
   };
   if (CHANNEL && wide) {
-    const int t = tid >> 4, s = tid & 15;
-    float a = 0.f, q = 0.f;
-    if (s <= t) {
-      for (int d = 0; d < DP; d += 4) {
-        float kt[4], k2[4], qt[4], ct[4], c2[4];
-        load_vec<4>(ks + t * PP + d, kt);
-        load_vec<4>(ks + s * PP + d, k2);
-        load_vec<4>(qs + t * PP + d, qt);
-        load_vec<4>(cs + t * PP + d, ct);
-        load_vec<4>(cs + s * PP + d, c2);
+    // a thread follows one s through its share of the channels
+    const int s = tid >> 4, part = tid & 15;
+    float a[C], q[C];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const float x = k2[r] * __expf(ct[r] - c2[r]);
-          a += kt[r] * x;
-          q += qt[r] * x;
-        }
+    for (int t = 0; t < C; ++t) a[t] = q[t] = 0.f;
+    for (int d = part; d < DP; d += 16) {
+      float f = kx[s * PP + d];
+#pragma unroll
+      for (int t = 0; t < C; ++t) {
+        if (t < s) continue;
+        if (t > s) f *= ky[t * PP + d];
+        a[t] += f * kx[t * PP + d];
+        q[t] += f * qx[t * PP + d];
       }
     }
-    put(false, t, s, a);
-    put(true, t, s, q);
+#pragma unroll
+    for (int t = 0; t < C; ++t) {
+      const float x = group16_sum(a[t]), y = group16_sum(q[t]);
+      if (part == t) {
+        put_a(t, s, x);
+        put_q(t, s, y);
+      }
+    }
+    __syncthreads();
+    if (tid < DP) {                             // kx = k e^{c_t}
+      float f = 1.f;
+      for (int t = 0; t < C; ++t) {
+        f *= ky[t * PP + tid];
+        kx[t * PP + tid] *= f;
+      }
+    }
   } else {
     // waves 0, 1: A and Q over the first half of the channels; 2, 3: the other
     const bool is_q = wave & 1;
     const int d0 = (wave >> 1) * (DP / 2);
-    const float* a = is_q ? qs : ks;
+    const float* a = is_q ? qx : kx;
+    const float* b = CHANNEL ? ky : kx;
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll 4
     for (int d = d0; d < d0 + DP / 2; d += 16) {
       float x[4], y[4];
       load_vec<4>(a + gl * PP + d + gs * 4, x);
-      load_vec<4>(ks + gl * PP + d + gs * 4, y);
-      if constexpr (CHANNEL) {
-        float c[4], m[4];
-        load_vec<4>(cs + gl * PP + d + gs * 4, c);
-        load_vec<4>(cs + (C / 2 - 1) * PP + d + gs * 4, m);
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          x[r] *= __expf(c[r] - m[r]);
-          y[r] *= __expf(m[r] - c[r]);
-        }
-      }
+      load_vec<4>(b + gl * PP + d + gs * 4, y);
 #pragma unroll
       for (int r = 0; r < 4; ++r) acc = mfma_f32_k4(x[r], y[r], acc);
     }
@@ -163,46 +200,31 @@ __global__ __launch_bounds__(256) void gated_prep_kernel(
     if (wave < 2) {
       acc += half[wave][lane];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) put(is_q, gs * 4 + r, gl, acc[r]);
+      for (int r = 0; r < 4; ++r) {
+        const int t = gs * 4 + r;
+        const float x = CHANNEL ? acc[r] : acc[r] * fs[t * SP + gl];
+        if (is_q) put_q(t, gl, x);
+        else put_a(t, gl, x);
+      }
     }
   }
   __syncthreads();
 
-  // ---- wave 0: T, a lane per column; the others write out ------------------
-  if (wave == 0) {
-    if (lane < C) {
-      float tc[C];
-      const float b = bs[lane];
-      const float e = CHANNEL ? 1.f : __expf(cs[lane]);
+  // ---- T, a lane per column -------------------------------------------------
+  if (wave == 0 && lane < C) {
+    float tc[C], c = 0.f;
+    const float b = bs[lane];
+    if (!CHANNEL)
+      for (int j = 0; j <= lane; ++j) c += lws[j];
+    const float e = CHANNEL ? 1.f : __expf(c);
 #pragma unroll
-      for (int t = 0; t < C; ++t) {
-        float x = t == lane ? 1.f : 0.f;
+    for (int t = 0; t < C; ++t) {
+      float x = t == lane ? 1.f : 0.f;
 #pragma unroll
-        for (int s = 0; s < t; ++s) x -= ls[t * SP + s] * tc[s];
-        tc[t] = x;
-        ts[t * SP + lane] = x * b * e;            // times k e^c below
-        rec[W::TM + t * SP + lane] = -x * b;
-      }
-    }
-  } else {
-    for (int i = (tid - 64) * 4; i < C * DP; i += 192 * 4) {
-      const int t = i / DP, at = t * PP + i % DP;
-      float q[4], c[4];
-      load_vec<4>(qs + at, q);
-      if (CHANNEL) load_vec<4>(cs + at, c);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) q[r] *= __expf(CHANNEL ? c[r] : cs[t]);
-      store_vec<4>(rec + W::R + at, q);
-    }
-    for (int i = tid - 64; i < DP * 4; i += 192) {
-      const int d = i >> 2, t = (i & 3) * 4;      // 4 tokens of a channel
-      const float last = CHANNEL ? cs[(C - 1) * PP + d] : cs[C - 1];
-      float x[4];
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        x[r] = -ks[(t + r) * PP + d] *
-               __expf(last - (CHANNEL ? cs[(t + r) * PP + d] : cs[t + r]));
-      store_vec<4>(rec + W::BT + d * SP + t, x);
+      for (int s = 0; s < t; ++s) x -= ls[t * SP + s] * tc[s];
+      tc[t] = x;
+      ts[t * SP + lane] = x * b * e;            // times k e^c below
+      rec[W::TM + t * SP + lane] = -x * b;
     }
   }
   __syncthreads();
@@ -213,14 +235,12 @@ __global__ __launch_bounds__(256) void gated_prep_kernel(
   for (int d = wave * 16; d < DP; d += 64) {
     f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int at = (gs * 4 + r) * PP + d + gl;
-      acc = mfma_f32_k4(tf[r], CHANNEL ? ks[at] * __expf(cs[at]) : ks[at],
-                        acc);
-    }
+    for (int r = 0; r < 4; ++r)
+      acc = mfma_f32_k4(tf[r], kx[(gs * 4 + r) * PP + d + gl], acc);
+    const float m = CHANNEL ? mid[d + gl] : 1.f;
 #pragma unroll
     for (int r = 0; r < 4; ++r)
-      rec[W::TU + (gs * 4 + r) * PP + d + gl] = acc[r];
+      rec[W::TU + (gs * 4 + r) * PP + d + gl] = acc[r] * m;
   }
 }
 

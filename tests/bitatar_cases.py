@@ -88,8 +88,7 @@ def save(folder, cfg, w):
         json.dump(cfg, f)
     meta, blobs, at = {}, [], 0
     for name, t in w.items():
-        raw = t.contiguous().view(torch.uint8).numpy().tobytes() \
-            if t.dim() else b""
+        raw = t.contiguous().view(-1).view(torch.uint8).numpy().tobytes()
         meta[name] = {"dtype": _TAGS[t.dtype], "shape": list(t.shape),
                       "data_offsets": [at, at + len(raw)]}
         blobs.append(raw)
