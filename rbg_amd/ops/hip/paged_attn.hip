@@ -61,33 +61,45 @@ constexpr float BOUND_LOG2 = 100.f;
 constexpr int KT = 64;
 
 // A wave keeps QT sums: of QT query tiles, or (MAPS 2) of one tile's two maps.
+// SPLIT (MAPS 2, QT 1): one tile's two maps are a pair of waves, which meet in
+// LDS at the end.
 template <int DK, int DV, int NW, int QT, bool BOUND, int MAPS = 1>
 __global__ __launch_bounds__(NW * 64, (DK + DV) > 256 ? 1 : 2)
 void paged_prefill_kernel(const PagedAttnArgs p) {
-  static_assert(MAPS == 1 || (MAPS == 2 && QT == 2 && !BOUND), "maps");
+  static_assert(MAPS == 1 || (MAPS == 2 && QT <= 2 && !BOUND), "maps");
+  constexpr bool SPLIT = MAPS == 2 && QT == 1;
   constexpr int DKM = DK * MAPS;              // a key row, maps side by side
   constexpr int KP = DKM + 16, VP = DV + 16;  // 8 banks per row
-  constexpr int WR = QT / MAPS * 16;          // query rows of a wave
-  constexpr int ROWS = NW * WR;               // 128
+  constexpr int SM = SPLIT ? 1 : MAPS;        // maps of a wave
+  constexpr int WR = QT / SM * 16;            // query rows of a wave
+  constexpr int ROWS = SPLIT ? NW / 2 * WR : NW * WR;   // or SUB pieces of 128
+  constexpr int SUB = 128 / ROWS;
   constexpr int NT = NW * 64;
   constexpr int KPC = KT * DKM / 8 / NT, VPC = (KT * DV / 8 + NT - 1) / NT;
   constexpr bool VFULL = VPC * NT * 8 == KT * DV;
   static_assert(KPC * NT * 8 == KT * DKM, "tile");
-  __shared__ __hip_bfloat16 ks[KT * KP];
-  __shared__ __hip_bfloat16 vs[KT * VP];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  constexpr int TILE = KT * (KP + VP), MEET = SPLIT ? NW / 2 * DV * 32 : 0;
+  __shared__ __attribute__((aligned(16)))
+  __hip_bfloat16 ks[TILE > MEET ? TILE : MEET];
+  __hip_bfloat16* vs = ks + KT * KP;
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int own = SPLIT ? (tid >> 6) & 1 : 0; // SPLIT: the wave's map
+  const int wave = SPLIT ? tid >> 7 : tid >> 6;
   const int gl = lane & 15, gs = lane >> 4;
 
   // workgroups go round the 8 XCDs: give each XCD whole heads, so that the
   // query tiles of a head (and of its neighbours with the same keys) share L2
-  const int items = p.n_blocks * p.heads, per = (items + 7) / 8;
+  const int nb = p.n_blocks * SUB;
+  const int items = nb * p.heads, per = (items + 7) / 8;
   const int work = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
   if ((blockIdx.x >> 3) >= per || work >= items) return;
-  const int head = work / p.n_blocks, kvh = head / (p.heads / p.kv_heads);
-  const int* bi = p.blocks + (p.n_blocks - 1 - work % p.n_blocks) * 2;
+  const int head = work / nb, kvh = head / (p.heads / p.kv_heads);
+  const int piece = nb - 1 - work % nb;
+  const int* bi = p.blocks + piece / SUB * 2;
   const int* si = p.seq_info + bi[0] * 3;
   const int qrow0 = si[0], qlen = si[1], qoff = si[2];
-  const int t0 = bi[1];                       // first query of the block
+  const int t0 = bi[1] + piece % SUB * ROWS;  // first query of the piece
+  if (SUB > 1 && t0 >= qlen) return;
   const int klen = qoff + qlen;
   const int* table = p.tables + (size_t)bi[0] * p.max_pages;
 
@@ -103,10 +115,10 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
   int qpos[QT];
 #pragma unroll
   for (int t = 0; t < QT; ++t) {
-    const int r = t0 + wave * WR + t / MAPS * 16 + gl;
+    const int r = t0 + wave * WR + t / SM * 16 + gl;
     qpos[t] = qoff + r;                       // may lie past the end: unused
     const __hip_bfloat16* qr = q + (size_t)(qrow0 + min(r, qlen - 1)) * p.q_row +
-                               t % MAPS * p.d;
+                               (own + t % SM) * p.d;
 #pragma unroll
     for (int s = 0; s < DK / 32; ++s) {
       const int d = s * 32 + gs * 8;
@@ -206,11 +218,11 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
 #pragma unroll
       for (int st = 0; st < DK / 32; ++st)
 #pragma unroll
-        for (int map = 0; map < MAPS; ++map) {
+        for (int map = 0; map < SM; ++map) {
           const mf_bf8 kf = frag8(
-              &ks[(c * 16 + gl) * KP + map * DK + st * 32 + gs * 8]);
+              &ks[(c * 16 + gl) * KP + (own + map) * DK + st * 32 + gs * 8]);
 #pragma unroll
-          for (int t = map; t < QT; t += MAPS)
+          for (int t = map; t < QT; t += SM)
             s[t][c] = mfma_bf16_k32(kf, qf[t][st], s[t][c]);
         }
     mf_bf8 ph[QT][2], pl[QT][2];
@@ -283,11 +295,26 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
   }
   if constexpr (MAPS == 2) {
     // the difference of the maps, over its root mean square, in acc[0]
-    const float f1 = 1.f / sums[0], f2 = p.lam[0] / sums[1];
+    float f1 = 1.f / sums[0], f2 = p.lam[0];
+    f32x4* meet = (f32x4*)ks + wave * DV * 4 + lane;
+    if constexpr (SPLIT) {
+      __syncthreads();                        // keys and values are read
+      if (own) {
+#pragma unroll
+        for (int d = 0; d < DV / 16; ++d) meet[d * 64] = acc[0][d] * f1;
+      }
+      __syncthreads();
+      if (own) return;
+    } else {
+      f2 /= sums[1];
+    }
     float ss = 0.f;
 #pragma unroll
     for (int d = 0; d < DV / 16; ++d) {
-      acc[0][d] = acc[0][d] * f1 - acc[1][d] * f2;
+      f32x4 other;
+      if constexpr (SPLIT) other = meet[d * 64];
+      else other = acc[QT - 1][d];
+      acc[0][d] = acc[0][d] * f1 - other * f2;
 #pragma unroll
       for (int e = 0; e < 4; ++e) ss += acc[0][d][e] * acc[0][d][e];
     }
@@ -296,7 +323,7 @@ void paged_prefill_kernel(const PagedAttnArgs p) {
     sums[0] = sqrtf(ss / p.dv + p.out_eps) / p.out_scale;
   }
 #pragma unroll
-  for (int t = 0; t < QT / MAPS; ++t) {
+  for (int t = 0; t < QT / SM; ++t) {
     const int r = t0 + wave * WR + t * 16 + gl;
     if (r >= qlen) continue;
     const float inv = 1.f / sums[t];
@@ -707,16 +734,19 @@ void prefill_dv(const PagedAttnArgs& p, hipStream_t s) {
 #undef PP_GO
 }
 
-// two maps: a wave's two sums are one query tile's
+// two maps: a wave's two sums are one query tile's; sums of 256 values take a
+// wave each
 template <int DK>
 void prefill_maps(const PagedAttnArgs& p, hipStream_t s) {
-  const int grid = 8 * ((p.n_blocks * p.heads + 7) / 8);
-#define PP_GO(DV)                                                             \
-  paged_prefill_kernel<DK, DV, 8, 2, false, 2><<<grid, 512, 0, s>>>(p)
-  if (p.dv <= 64) PP_GO(64);
-  else if (p.dv <= 96) PP_GO(96);
-  else if (p.dv <= 128) PP_GO(128);
-  else PP_GO(256);
+#define PP_GO(DV, QT)                                                         \
+  do {                                                                        \
+    const int grid = 8 * ((p.n_blocks * (2 / QT) * p.heads + 7) / 8);         \
+    paged_prefill_kernel<DK, DV, 8, QT, false, 2><<<grid, 512, 0, s>>>(p);    \
+  } while (0)
+  if (p.dv <= 64) PP_GO(64, 2);
+  else if (p.dv <= 96) PP_GO(96, 2);
+  else if (p.dv <= 128) PP_GO(128, 2);
+  else PP_GO(256, 1);
 #undef PP_GO
 }
 
