@@ -122,12 +122,16 @@ def linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     # measured policy (profiles/sg_micro7_b*.json): the custom kernel wins
     # on narrow-N shapes (o/down, N<=4096) at any decode batch, on mid-N
     # (qkv, 6144) only up to M=64, and never on wide-N (gate_up 28672,
-    # where hipBLASLt already streams at ~6 TB/s)
+    # where hipBLASLt already streams at ~6 TB/s).  Between them, for a few
+    # rows, hipBLASLt takes up to 2.7 times as long (18432 x 2048: 58 us
+    # against 22) and is nowhere ahead by more than a tenth
     if (SKINNY_GEMM and _on_gpu(x) and x.dim() == 2 and
             x.dtype == torch.bfloat16 and x.shape[0] <= 128 and
             w.shape[0] % 32 == 0 and x.shape[1] % 512 == 0 and
             (w.shape[0] <= 4608 or
-             (x.shape[0] <= 64 and w.shape[0] <= 8192))):
+             (x.shape[0] <= 64 and w.shape[0] <= 8192) or
+             (x.shape[0] <= 16 and w.shape[0] <= 24576 and
+              x.shape[1] <= 4096))):
         # linked into every extension: a process has the one its model needs
         return (_hip or _mix or _gated or _require_moe()).skinny_gemm(
             x if x.is_contiguous() else x.contiguous(), w)

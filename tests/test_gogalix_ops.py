@@ -287,7 +287,7 @@ def test_one_key_is_kept_and_written_over(where):
 #            H   G   D    DV
 DIFF_SIZES = [(4, 2, 32, 32), (3, 3, 8, 16), (8, 1, 64, 80), (2, 2, 128, 128),
               (10, 1, 40, 96), (2, 1, 16, 256), (20, 1, 16, 8), (2, 1, 10, 36),
-              (2, 1, 136, 24)]
+              (2, 1, 136, 24), (2, 1, 128, 256)]
 
 
 def diff_case(where, H, G, D, DV, n, scale, window, seed=0):
