@@ -8,57 +8,34 @@ as the implementation.
 """
 from __future__ import annotations
 
+import importlib
 from dataclasses import dataclass
-from typing import Optional
+from typing import Any, Dict, Optional
 
 import torch
 
+from ..utils import hip_build
 from . import reference
 
-_hip = None
-_hip_err: Exception | None = None
-try:
-    from . import _hip_ops as _hip   # type: ignore[attr-defined]
-except Exception as e:  # noqa: BLE001
-    _hip_err = e
+# Extension modules by name, loaded as far as they are built; a process needs
+# those that its model runs on (utils/hip_build.py EXTENSIONS_OF).
+EXTENSIONS: Dict[str, Any] = {}
+_errors: Dict[str, Exception] = {}
+for _name in hip_build.HIP_SOURCES:
+    try:
+        EXTENSIONS[_name] = importlib.import_module("." + _name, __name__)
+    except Exception as e:  # noqa: BLE001
+        _errors[_name] = e
 
+_hip = EXTENSIONS.get("_hip_ops")
 HAVE_HIP = _hip is not None
-
-_mix = None
-_mix_err: Exception | None = None
-try:
-    from . import _hip_mix as _mix   # type: ignore[attr-defined]
-except Exception as e:  # noqa: BLE001
-    _mix_err = e
-
-HAVE_MIX = _mix is not None
-
-_moe = None
-_moe_err: Exception | None = None
-try:
-    from . import _hip_moe as _moe   # type: ignore[attr-defined]
-except Exception as e:  # noqa: BLE001
-    _moe_err = e
-
-HAVE_MOE = _moe is not None
-
-_gated = None
-_gated_err: Exception | None = None
-try:
-    from . import _hip_gated as _gated   # type: ignore[attr-defined]
-except Exception as e:  # noqa: BLE001
-    _gated_err = e
-
-HAVE_GATED = _gated is not None
 
 
 def _check_stale() -> None:
     """Fail loudly on a GPU box if a shipped .so predates its kernel sources
     (stale-binary guard; the stamps are written by utils/hip_build.py)."""
-    from ..utils import hip_build
-    for name, mod in (("_hip_ops", _hip), ("_hip_mix", _mix),
-                      ("_hip_moe", _moe), ("_hip_gated", _gated)):
-        if mod is not None and hip_build.is_stale(name):
+    for name in EXTENSIONS:
+        if hip_build.is_stale(name):
             raise RuntimeError(
                 f"rbg_amd HIP extension {name} is STALE: kernel sources "
                 "changed after the last build.  Rebuild in-tree: "
@@ -66,45 +43,44 @@ def _check_stale() -> None:
                 "--inplace")
 
 
-if (HAVE_HIP or HAVE_MIX or HAVE_MOE or HAVE_GATED) and \
-        torch.cuda.is_available():
+if EXTENSIONS and torch.cuda.is_available():
     _check_stale()
 
 
+def require(*names: str):
+    """The first of these extensions that is built."""
+    for name in names:
+        if name in EXTENSIONS:
+            return EXTENSIONS[name]
+    errors = "; ".join(f"{n}: {_errors[n]!r}" for n in names)
+    raise RuntimeError(
+        f"rbg_amd HIP extension {' or '.join(names)} is not built but a GPU "
+        "tensor was passed.  Build it in-tree: PYTORCH_ROCM_ARCH=gfx950 "
+        f"python setup.py build_ext --inplace (import error: {errors})")
+
+
 def _require_hip():
-    if _hip is None:
-        raise RuntimeError(
-            "rbg_amd HIP extension is not built but a GPU tensor was passed. "
-            "Build it in-tree: PYTORCH_ROCM_ARCH=gfx950 python setup.py "
-            f"build_ext --inplace (import error: {_hip_err!r})")
-    return _hip
+    return require("_hip_ops")
 
 
 def _require_mix():
-    if _mix is None:
-        raise RuntimeError(
-            "rbg_amd HIP extension _hip_mix is not built but a GPU tensor was "
-            "passed.  Build it in-tree: PYTORCH_ROCM_ARCH=gfx950 python "
-            f"setup.py build_ext --inplace (import error: {_mix_err!r})")
-    return _mix
+    return require("_hip_mix")
+
+
+def _require_latent():
+    return require("_hip_latent")
 
 
 def _require_moe():
-    if _moe is None:
-        raise RuntimeError(
-            "rbg_amd HIP extension _hip_moe is not built but a GPU tensor was "
-            "passed.  Build it in-tree: PYTORCH_ROCM_ARCH=gfx950 python "
-            f"setup.py build_ext --inplace (import error: {_moe_err!r})")
-    return _moe
+    return require("_hip_moe")
+
+
+def _require_experts():
+    return require("_hip_experts")
 
 
 def _require_gated():
-    if _gated is None:
-        raise RuntimeError(
-            "rbg_amd HIP extension _hip_gated is not built but a GPU tensor "
-            "was passed.  Build it in-tree: PYTORCH_ROCM_ARCH=gfx950 python "
-            f"setup.py build_ext --inplace (import error: {_gated_err!r})")
-    return _gated
+    return require("_hip_gated")
 
 
 def _on_gpu(t: torch.Tensor) -> bool:
@@ -132,8 +108,9 @@ def linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
              (x.shape[0] <= 64 and w.shape[0] <= 8192) or
              (x.shape[0] <= 16 and w.shape[0] <= 24576 and
               x.shape[1] <= 4096))):
-        # linked into every extension: a process has the one its model needs
-        return (_hip or _mix or _gated or _require_moe()).skinny_gemm(
+        # one of these is there whatever the model
+        return require("_hip_ops", "_hip_mix", "_hip_gated",
+                       "_hip_moe").skinny_gemm(
             x if x.is_contiguous() else x.contiguous(), w)
     return torch.nn.functional.linear(x, w)
 
@@ -237,7 +214,7 @@ def embed_stream(tokens, table, scale: float) -> torch.Tensor:
     """f32 stream [T, W] = table[tokens] * scale."""
     if _on_gpu(table):
         # linked into both extensions of designs that scale
-        return (_mix or _require_gated()).embed_stream(tokens, table, scale)
+        return require("_hip_mix", "_hip_gated").embed_stream(tokens, table, scale)
     return reference.embed_stream(tokens, table, scale)
 
 
@@ -335,7 +312,7 @@ def delta_rule(proj, z, w2, w0, a_bias, norm_w, state, slots, cu_seqlens,
 def latent_store(x, w, cache, slots, eps: float) -> torch.Tensor:
     """c = rms_norm(x) * w, written to the paged latents; returns c."""
     if _on_gpu(x):
-        return _require_mix().latent_store(x, w, cache, slots, eps)
+        return _require_latent().latent_store(x, w, cache, slots, eps)
     return reference.latent_store(x, w, cache, slots, eps)
 
 
@@ -345,7 +322,7 @@ def window_attention(q, k, v, gate, out, view, scale: float,
     [T, H, D], v [T, H, Dv]; ``view`` locates each query among the keys
     (engine/batch.py WindowView).  out = o * sigmoid(gate)."""
     if _on_gpu(q):
-        _require_mix().window_attention(q, k, v, gate, out, view.row_info,
+        _require_latent().window_attention(q, k, v, gate, out, view.row_info,
                                         view.seq_info, view.blocks, scale,
                                         window)
         return
@@ -372,7 +349,7 @@ def latent_decode(q, cache, block_tables, context_lens, scale: float,
         keys = block_tables.shape[1] * cache.shape[1]
         splits = pick_latent_splits(q.shape[0], q.shape[1],
                                     min(keys, window) if window else keys)
-        return _require_mix().latent_decode(q, cache, block_tables,
+        return _require_latent().latent_decode(q, cache, block_tables,
                                             context_lens, scale, window,
                                             splits)
     return reference.latent_decode(q, cache, block_tables, context_lens,
@@ -385,7 +362,7 @@ def head_linear(x, w, gate=None, out=None) -> torch.Tensor:
     if out is None:
         out = x.new_empty((x.shape[0], w.shape[0] * w.shape[1]))
     if _on_gpu(x):
-        _require_mix().head_linear(x, w, gate, out)
+        _require_latent().head_linear(x, w, gate, out)
     else:
         reference.head_linear(x, w, gate, out)
     return out
@@ -436,7 +413,7 @@ def sandwich_norm(x, pending, w, eps: float, dtype):
 def moe_combine(y, route) -> torch.Tensor:
     """Weighed sums of each token's expert rows, in y's dtype."""
     if _on_gpu(y):
-        return _require_moe().moe_combine(y, route.inv, route.weights)
+        return _require_experts().moe_combine(y, route.inv, route.weights)
     return reference.moe_combine(y, route).to(y.dtype)
 
 
@@ -520,7 +497,7 @@ def paged_decode(q, k, v, tables, context_lens, out, scale: float,
 def router_logits(x, w) -> torch.Tensor:
     """x W^T in 32-bit, [T, experts] f32."""
     if _on_gpu(x):
-        return _require_moe().router_logits(x, w)
+        return _require_experts().router_logits(x, w)
     return x.float() @ w.float().T
 
 
@@ -544,7 +521,7 @@ def moe_route(logits, correction, groups: int, keep: int, top: int,
     choice is by logit + correction, the weights are the softmax of the
     chosen."""
     if _on_gpu(logits):
-        weights, inv, rows, tiles, count = _require_moe().moe_route(
+        weights, inv, rows, tiles, count = _require_experts().moe_route(
             logits, correction, groups, keep, top, tile, softmax)
         return Routing(top, tile, weights, inv, rows, tiles, count)
     ids, weights = reference.moe_choose(logits, correction, groups, keep, top,
@@ -567,7 +544,7 @@ def expert_linear(x, w, route, gather: bool = False, relu2: bool = False,
     x's rows by token, ``relu2`` applies max(0, .)^2, ``swiglu`` takes w's rows
     as interleave_glu lays them and gives silu(gate) * up, [.., N / 2]."""
     if _on_gpu(x):
-        return _require_moe().expert_linear(
+        return _require_experts().expert_linear(
             x, w, route.rows if gather else None, route.tiles, route.count,
             route.rows.numel(), route.tile, relu2, swiglu)
     return reference.expert_linear(x, w, route, gather, relu2, swiglu)

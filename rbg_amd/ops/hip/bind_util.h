@@ -64,4 +64,14 @@ using OptTensor = c10::optional<torch::Tensor>;
   return ((uintptr_t)t.data_ptr() % bytes) == 0;
 }
 
+// y [tokens * top, width] in expert order, as inv and weights [tokens, top] say
+[[maybe_unused]] void check_experts(const Tensor& y, const Tensor& inv, const Tensor& weights,
+                   int64_t tokens) {
+  TORCH_CHECK(weights.dim() == 2 && weights.size(0) == tokens,
+              "weights [tokens, top]");
+  check_f32(weights, "weights", weights.numel());
+  TORCH_CHECK(y.size(0) == weights.numel() && inv.numel() == weights.numel(),
+              "one row per (token, choice)");
+}
+
 }  // namespace

@@ -9,7 +9,7 @@
 // rows and its registers four neighbouring columns.  f32 (and sizes that are
 // not multiples of 8): one thread per output.
 #include "mfma_util.h"
-#include "mix_args.h"
+#include "latent_args.h"
 #include "vec_io.h"
 
 namespace {

@@ -8,7 +8,7 @@
 //                 the value dimensions.  Contiguous keys/values (expanded per
 //                 head, prefill) or the paged latents themselves as both key
 //                 and value (query absorbed into the latent space, decode).
-#include "mix_args.h"
+#include "latent_args.h"
 #include "vec_io.h"
 
 namespace {

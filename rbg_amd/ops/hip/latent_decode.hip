@@ -14,7 +14,7 @@
 // but the sum of the weights.  Splits of the keys meet in latent_combine.  The
 // second tile of 16 heads finds the latents in L2.
 #include "mfma_util.h"
-#include "mix_args.h"
+#include "latent_args.h"
 
 namespace {
 

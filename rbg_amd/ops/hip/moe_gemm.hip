@@ -16,7 +16,7 @@
 //   rows    any sizes, bf16 or f32: a thread per column, up to 16 rows at once.
 // A squared relu, or silu(gate) * up of interleaved rows, rides on the way out.
 #include "lds_stream.h"
-#include "moe_args.h"
+#include "expert_args.h"
 #include "vec_io.h"
 
 namespace {

@@ -14,7 +14,7 @@
 //            with the choice for small batches; for prompts the counting and the
 //            permutation are spread over blocks of tokens.
 #include "lds_stream.h"
-#include "moe_args.h"
+#include "expert_args.h"
 #include "vec_io.h"
 
 namespace {

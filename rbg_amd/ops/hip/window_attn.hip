@@ -14,7 +14,7 @@
 // current tile's MFMAs.  Row pitch is dim + 16 elements: 8 banks per row, which
 // keeps both read patterns conflict-free.
 #include "mfma_util.h"
-#include "mix_args.h"
+#include "latent_args.h"
 #include "vec_io.h"
 
 namespace {

@@ -38,27 +38,36 @@ HIP_SOURCES = {
         "allreduce.hip",
         "bindings.cpp",
     ],
-    # f32-stream norms and the token mixers (delta rule, latents)
+    # f32-stream norms, gates and the generalized delta rule
     "_hip_mix": [
         "embed.hip",
         "stream_norm.hip",
         "gated_act.hip",
         "delta_rule.hip",
         "delta_chunk.hip",
+        "skinny_gemm.hip",
+        "mix_bindings.cpp",
+    ],
+    # latent attention
+    "_hip_latent": [
         "latent_attn.hip",
         "latent_decode.hip",
         "window_attn.hip",
         "head_linear.hip",
-        "skinny_gemm.hip",
-        "mix_bindings.cpp",
+        "latent_bindings.cpp",
     ],
-    # sandwich norms, paged attention of any sizes, sparse experts
+    # mixtures of experts
+    "_hip_experts": [
+        "moe_route.hip",
+        "moe_gemm.hip",
+        "moe_combine.hip",
+        "expert_bindings.cpp",
+    ],
+    # sandwich norms, paged attention of any sizes
     "_hip_moe": [
         "sandwich_norm.hip",
         "rope_paged.hip",
         "paged_attn.hip",
-        "moe_route.hip",
-        "moe_gemm.hip",
         "skinny_gemm.hip",
         "moe_bindings.cpp",
     ],
@@ -79,16 +88,22 @@ HIP_HEADERS = {
     "_hip_ops": ["common.h", "gemm_bindings.h"],
     "_hip_mix": ["bind_util.h", "common.h", "delta_scan.h", "gemm_bindings.h",
                  "mfma_util.h", "mix_args.h", "vec_io.h"],
+    "_hip_latent": ["bind_util.h", "common.h", "latent_args.h", "mfma_util.h",
+                    "vec_io.h"],
+    "_hip_experts": ["bind_util.h", "common.h", "expert_args.h",
+                     "expert_rows.h", "lds_stream.h", "mfma_util.h",
+                     "vec_io.h"],
     "_hip_moe": ["bind_util.h", "common.h", "expert_rows.h", "gemm_bindings.h",
-                 "lds_stream.h", "mfma_util.h", "moe_args.h", "vec_io.h"],
+                 "mfma_util.h", "moe_args.h", "vec_io.h"],
     "_hip_gated": ["bind_util.h", "common.h", "delta_scan.h", "expert_rows.h",
                    "gated_args.h", "gated_delta.h", "gemm_bindings.h",
                    "mfma_util.h", "vec_io.h"],
 }
 
 # model architecture -> the extensions with its kernels (default: _hip_ops)
-EXTENSIONS_OF = {"Bitatar": ("_hip_mix",), "Notadra": ("_hip_moe",),
-                 "Gogalix": ("_hip_gated", "_hip_moe")}
+EXTENSIONS_OF = {"Bitatar": ("_hip_mix", "_hip_latent"),
+                 "Notadra": ("_hip_moe", "_hip_experts"),
+                 "Gogalix": ("_hip_gated", "_hip_moe", "_hip_experts")}
 
 
 def source_hash(name: str) -> str:

@@ -394,7 +394,7 @@ def test_latent_decode_splits(splits):
     cache = seen(rnd(30, ps, rank), where)
     q = seen(rnd(2, H, rank, seed=1), where)
     bt = i32([list(range(1, 11)), list(range(11, 21))], where)
-    o = ops._require_mix().latent_decode(
+    o = ops._require_latent().latent_decode(
         put(q, where), put(cache, where), bt, i32([150, 3], where), 0.1,
         window, splits)
     for b, c in enumerate([150, 3]):

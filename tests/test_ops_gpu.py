@@ -23,7 +23,7 @@ def dev():
 
 def test_hip_extension_loaded(dev):
     # on a GPU box the native extension must be the path that runs
-    assert ops.HAVE_HIP, f"HIP extension missing: {ops._hip_err!r}"
+    ops.require("_hip_ops")
 
 
 def test_mfma_fragment_layout(dev):
