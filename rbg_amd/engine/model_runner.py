@@ -129,7 +129,7 @@ class ModelRunner:
         hidden_in = None
         if not self.pp.first:
             hidden_in = self.pp.recv_prev(
-                (cu[-1], self.cfg.model.hidden_size),
+                (cu[-1], self.model.stream_width),
                 self.model.stream_dtype, self.device)
         hidden = self.model.forward(self._join(tokens), batch, self.cache,
                                     hidden=hidden_in)
@@ -255,7 +255,7 @@ class ModelRunner:
         hidden_in = None
         if not self.pp.first:
             hidden_in = self.pp.recv_prev(
-                (n, self.cfg.model.hidden_size),
+                (n, self.model.stream_width),
                 self.model.stream_dtype, self.device)
         hidden = self.model.forward(state["tokens"], batch, self.cache,
                                     hidden=hidden_in)

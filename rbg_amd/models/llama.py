@@ -293,6 +293,7 @@ class LlamaForCausalLM(nn.Module):
         self.device = device
         dtype = torch.bfloat16
         self.dtype = self.stream_dtype = dtype
+        self.stream_width = cfg.hidden_size
 
         # Per-tensor generators keyed by (base_seed, tag): weights are
         # identical for every TP degree (full-then-shard) AND every PP

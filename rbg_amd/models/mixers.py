@@ -150,15 +150,23 @@ class GeneralDelta(nn.Module):
 
 
 class LatentAttention(nn.Module):
-    """Softmax attention over a cached low-rank latent, without positions,
-    through a sliding window, with an output gate.
+    """Softmax attention over a cached low-rank latent, through a sliding window,
+    with an output gate (``gated``).
+
+    With ``rotary`` ("interleaved" or "halves", how pairs lie) the spec's
+    rot_dim last dims of a head's query meet one rotated key part that all
+    heads share and that is cached behind the latent.  ``q_latent``: queries
+    come from a normed latent of their own.  ``sink``: a learned logit per head
+    that has no key and no value.
 
     Prefill expands the visible latents to per-head keys and values; decode
     folds the key expansion into the query and the value expansion into the
     output, so that it streams only the latents."""
 
     def __init__(self, spec: Dict[str, Any], width: int, eps: float,
-                 src: WeightSource, prefix: str, tp, dtype: torch.dtype):
+                 src: WeightSource, prefix: str, tp, dtype: torch.dtype,
+                 gated: bool = True, rotary: Optional[str] = None,
+                 q_latent: bool = False, sink: bool = False):
         super().__init__()
         heads = int(spec["heads"])
         assert heads % tp.size == 0, "TP degree must divide head counts"
@@ -166,61 +174,110 @@ class LatentAttention(nn.Module):
         self.dim, self.vdim = int(spec["dim"]), int(spec["vdim"])
         self.rank = int(spec["kv_rank"])
         self.scale = float(spec["scale"])
+        self.rot = self.cos_sin = None  # the table is set with the cache
+        self.rot_dim = 0
+        if rotary is not None:
+            self.rot, self.rot_dim = spec["rot"], int(spec["rot_dim"])
+            if int(self.rot["dims"]) != self.rot_dim:
+                raise ValueError(f"{self.rot['dims']} rotated dimensions in a "
+                                 f"part of {self.rot_dim}")
+        self.interleaved = rotary == "interleaved"
         mask = spec.get("mask") or {}
         self.window = int(mask.get("size") or 0)     # 0: everything before
         self.eps, self.dtype = eps, dtype
-        qk, vo = heads * self.dim, heads * self.vdim
+        f32 = torch.float32
+        qk, vo = heads * (self.dim + self.rot_dim), heads * self.vdim
 
         def lin(name, shape):
             return src.take(prefix + name, shape)
-        self.proj = FusedProjection([
-            ("q", shard(lin("q", (qk, width)), tp)),
-            ("dkv", lin("dkv", (self.rank, width))),
-            ("g", shard(lin("g", (vo, width)), tp))], dtype)
+        self.uq: Optional[nn.Parameter] = None
+        if q_latent:
+            q_rank = int(spec["q_rank"])
+            parts = [("dq", lin("dq", (q_rank, width)))]
+            self.uq = param(shard(lin("uq", (qk, q_rank)), tp), dtype)
+            self.q_norm = param(src.take(prefix + "dq.norm", (q_rank,),
+                                         "ones"), f32)
+        else:
+            parts = [("q", shard(lin("q", (qk, width)), tp))]
+        parts.append(("dkv", lin("dkv", (self.rank + self.rot_dim, width))))
+        self.gated = gated
+        if gated:
+            parts.append(("g", shard(lin("g", (vo, width)), tp)))
+        self.proj = FusedProjection(parts, dtype)
         self.c_norm = param(src.take(prefix + "dkv.norm", (self.rank,),
-                                     "ones"), torch.float32)
-        uk = shard(lin("uk", (qk, self.rank)), tp)
+                                     "ones"), f32)
+        uk = shard(lin("uk", (heads * self.dim, self.rank)), tp)
         uv = shard(lin("uv", (vo, self.rank)), tp)
         # prefill: one expansion GEMM.  decode: per-head maps [n, k]
         self.expand = FusedProjection([("k", uk), ("v", uv)], dtype)
         self.uk_t = param(uk.reshape(self.heads, self.dim, self.rank)
                           .transpose(1, 2), dtype)
         self.uv = param(uv.reshape(self.heads, self.vdim, self.rank), dtype)
+        self.sink: Optional[nn.Parameter] = None
+        if sink:
+            self.sink = param(shard(src.take(prefix + "sink", (heads,),
+                                             "normal"), tp), f32)
         self.w_out = shard(lin("o", (width, vo)), tp, dim=1)
         self.out_dim = self.heads * self.vdim
 
     def cache_spec(self) -> LayerCacheSpec:
-        return LayerCacheSpec(latent_rank=self.rank)
+        return LayerCacheSpec(latent_rank=self.rank + self.rot_dim)
 
     def forward(self, h: torch.Tensor, out: torch.Tensor, batch: ForwardBatch,
                 cache: StateCache, layer: int) -> None:
         y = self.proj(h)
         latents = cache.latents(layer)
-        c = ops.latent_store(self.proj.slice(y, "dkv"), self.c_norm, latents,
-                             batch.slot_mapping, self.eps)
+        rot = None
+        if self.rot is not None:
+            rot = ops.Rotary(self.cos_sin, batch.positions, self.interleaved)
+        low = self.proj.slice(y, "dkv")
+        if self.uq is None:
+            c = ops.latent_store(low, self.c_norm, latents,
+                                 batch.slot_mapping, self.eps, rot)
+            q = self.proj.slice(y, "q")
+        else:
+            c, cq = ops.latent_store(
+                low, self.c_norm, latents, batch.slot_mapping, self.eps, rot,
+                second=(self.proj.slice(y, "dq"), self.q_norm))
+            q = ops.linear(cq, self.uq)
+        q = q.unflatten(1, (self.heads, self.dim + self.rot_dim))
+        g = self.proj.slice(y, "g") if self.gated else None
         nd = y.shape[0] if batch.mode == "decode" else batch.num_decode
-        if nd:
-            self._decode(y[:nd], out[:nd], batch, latents)
-        if nd < y.shape[0]:
-            self._prefill(y[nd:], c[nd:], out[nd:], batch, latents)
 
-    def _prefill(self, y, c, out, batch, latents) -> None:
+        def run(step, part, *args):
+            step(q[part], None if g is None else g[part],
+                 None if rot is None else rot.rows(part), out[part], batch,
+                 latents, *args)
+        if nd:
+            run(self._decode, slice(0, nd))
+        if nd < y.shape[0]:
+            run(self._prefill, slice(nd, None), c[nd:])
+
+    def _prefill(self, q, g, rot, out, batch, latents, c) -> None:
         view = batch.layout.window_view(self.window)
         if view.slots is not None:
-            c = latents.view(-1, self.rank)[view.slots]
-        kv = self.expand(c)
+            c = latents.view(-1, latents.shape[-1])[view.slots]
+        kv = self.expand(c[:, :self.rank])
         k = self.expand.slice(kv, "k").unflatten(1, (self.heads, self.dim))
         v = self.expand.slice(kv, "v").unflatten(1, (self.heads, self.vdim))
-        q = self.proj.slice(y, "q").unflatten(1, (self.heads, self.dim))
-        ops.window_attention(q, k, v, self.proj.slice(y, "g"), out, view,
-                             self.scale, self.window)
+        shared = None
+        if rot is not None:
+            ops.rotate_rows(q[..., self.dim:], rot)
+            shared = c[:, self.rank:]
+        ops.window_attention(q, k, v, g, out, view, self.scale, self.window,
+                             shared, self.sink)
 
-    def _decode(self, y, out, batch, latents) -> None:
-        q = self.proj.slice(y, "q").unflatten(1, (self.heads, self.dim))
-        q = ops.head_linear(q, self.uk_t).unflatten(1, (self.heads, self.rank))
+    def _decode(self, q, g, rot, out, batch, latents) -> None:
+        if rot is None:
+            q = ops.head_linear(q, self.uk_t).unflatten(
+                1, (self.heads, self.rank))
+        else:
+            q = ops.head_linear(q[..., :self.dim], self.uk_t,
+                                tail=q[..., self.dim:], rot=rot)
         o = ops.latent_decode(q, latents, batch.block_tables,
-                              batch.context_lens, self.scale, self.window)
-        ops.head_linear(o, self.uv, gate=self.proj.slice(y, "g"), out=out)
+                              batch.context_lens, self.scale, self.window,
+                              self.rank, self.sink)
+        ops.head_linear(o, self.uv, gate=g, out=out)
 
 
 class GatedGelu(nn.Module):
@@ -553,6 +610,20 @@ class GatedSilu(nn.Module):
         return ops.linear(act, self.down), None
 
 
+def glu_stack(prefixes: List[str], ff: int, width: int, src: WeightSource, tp,
+              dtype: torch.dtype) -> Tuple[nn.Parameter, nn.Parameter]:
+    """Gated feed-forwards of equal size as ops.expert_linear takes them: gate
+    and up interleaved, and down."""
+    def take(name, shape, dim):
+        # columns up to a multiple of 8: a gate of zero meets zeros in down
+        return pad8(shard(src.take(name, shape), tp, dim), dim)
+    up = [ops.interleave_glu(take(p + "gate", (ff, width), 0),
+                             take(p + "up", (ff, width), 0))
+          for p in prefixes]
+    down = [take(p + "down", (width, ff), 1) for p in prefixes]
+    return param(torch.stack(up), dtype), param(torch.stack(down), dtype)
+
+
 class GluExperts(nn.Module):
     """Mixture of small gated feed-forwards down(silu(gate x) * up x); the
     largest router logits are chosen and weighed by their softmax.
@@ -571,17 +642,8 @@ class GluExperts(nn.Module):
         if not 1 <= self.top <= n:
             raise ValueError(f"router: {n} experts, {self.top} chosen")
 
-        def take(e, name, shape, dim):
-            # columns up to a multiple of 8: silu(0) * 0 meets zeros in down
-            return pad8(shard(src.take(f"{prefix}e{e}.{name}", shape), tp,
-                              dim), dim)
-
-        def glu(e):
-            return ops.interleave_glu(take(e, "gate", (ff, width), 0),
-                                      take(e, "up", (ff, width), 0))
-        self.up = param(torch.stack([glu(e) for e in range(n)]), dtype)
-        self.down = param(torch.stack([take(e, "down", (width, ff), 1)
-                                       for e in range(n)]), dtype)
+        self.up, self.down = glu_stack(
+            [f"{prefix}e{e}." for e in range(n)], ff, width, src, tp, dtype)
         self.router = param(src.take(prefix + "router", (n, width)), dtype)
         self.router_b = param(src.take(prefix + "router.b", (n,), "zeros"),
                               torch.float32)
@@ -596,3 +658,75 @@ class GluExperts(nn.Module):
                               softmax=True)
         a = ops.expert_linear(h, self.up, route, gather=True, swiglu=True)
         return ops.expert_linear(a, self.down, route), route
+
+
+class ClampedGlu(nn.Module):
+    """down(g * sigmoid(1.702 g) * (u + 1)), g = min(gate x, limit) and u = up x
+    within +-limit."""
+
+    def __init__(self, spec: Dict[str, Any], width: int, src: WeightSource,
+                 prefix: str, tp, dtype: torch.dtype):
+        super().__init__()
+        ff, self.limit = int(spec["ff"]), float(spec["limit"])
+        assert ff % tp.size == 0, "TP degree must divide the feed-forward"
+        self.proj = FusedProjection(
+            [(n, pad8(shard(src.take(prefix + n, (ff, width)), tp)))
+             for n in ("gate", "up")], dtype)
+        self.down = param(pad8(shard(src.take(prefix + "down", (width, ff)),
+                                     tp, dim=1), 1), dtype)
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        y = self.proj(x)
+        act = y.new_empty((y.shape[0], self.down.shape[1]))
+        ops.clamped_glu(self.proj.slice(y, "gate"), self.proj.slice(y, "up"),
+                        self.limit, act)
+        return ops.linear(act, self.down)
+
+
+class ClampedExperts(nn.Module):
+    """Mixture of clamped gated feed-forwards (ClampedGlu): scores are a softmax
+    over all experts, the choice adds a correction to them, weights are the
+    chosen ones' shares of their scores times a constant.  The last
+    ``identity`` experts of the router have no weights and return their input;
+    a ``shared`` expert runs for every token.
+
+    Tensor parallelism shards every expert's inner columns."""
+
+    def __init__(self, spec: Dict[str, Any], width: int, src: WeightSource,
+                 prefix: str, tp, dtype: torch.dtype):
+        super().__init__()
+        r, ff = spec["router"], int(spec["expert"]["ff"])
+        assert ff % tp.size == 0, "TP degree must divide the feed-forward"
+        n, self.top = int(r["experts"]), int(r["top"])
+        self.identity = int(r.get("identity") or 0)
+        every = n + self.identity
+        if n < 1 or not 1 <= self.top <= every:
+            raise ValueError(f"router: {n} experts and {self.identity} "
+                             f"identity experts, {self.top} chosen")
+        self.share = float(r["scale"])
+        self.limit = float(spec["expert"]["limit"])
+        self.up, self.down = glu_stack(
+            [f"{prefix}e{e}." for e in range(n)], ff, width, src, tp, dtype)
+        self.router = param(src.take(prefix + "router", (every, width)), dtype)
+        self.correction = param(src.take(prefix + "correction", (every,),
+                                         "zeros"), torch.float32)
+        self.shared: Optional[ClampedGlu] = None
+        if spec.get("shared"):
+            self.shared = ClampedGlu(spec["shared"], width, src,
+                                     prefix + "shared.", tp, dtype)
+        # pairs that get a row, per choice
+        self.rows_per_choice = n / every
+
+    def forward(self, h: torch.Tensor):
+        """The shared expert's rows (or None), the chosen experts' outputs, one
+        row per (token, choice) in expert order, and the routing that weighs
+        and finds them."""
+        logits = ops.router_logits(h, self.router)
+        route = ops.moe_route(
+            logits, self.correction, 1, 1, self.top,
+            ops.expert_tile(h, self.up, self.top * self.rows_per_choice),
+            share=self.share, identity=self.identity)
+        a = ops.expert_linear(h, self.up, route, gather=True, swiglu=True,
+                              limit=self.limit)
+        y = ops.expert_linear(a, self.down, route)
+        return None if self.shared is None else self.shared(h), y, route

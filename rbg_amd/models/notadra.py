@@ -17,7 +17,6 @@ to an earlier layer's keys and values instead of its own.  On the GPU a layer is
 """
 from __future__ import annotations
 
-import json
 from dataclasses import dataclass, field
 from typing import Any, Dict, List, NamedTuple, Optional
 
@@ -30,7 +29,7 @@ from ..engine.config import EngineConfig, ModelConfig
 from ..engine.state_cache import StateCache
 from .llama import TPContext
 from .mixers import PagedAttention, SparseExperts, param
-from .rotary import rotary_table
+from .rotary import assign_tables
 from .stream_model import StreamForCausalLM
 from .weights import WeightSource
 
@@ -184,13 +183,8 @@ class NotadraForCausalLM(StreamForCausalLM):
                 for n in ("norm2", "norm2b")}
 
     def make_cache(self, cfg: EngineConfig) -> StateCache:
-        tables: Dict[str, torch.Tensor] = {}
-        for layer in self.layers:
-            key = json.dumps(layer.mixer.rot, sort_keys=True)
-            if key not in tables:
-                tables[key] = rotary_table(layer.mixer.rot, cfg.max_seq_len,
-                                           self.device)
-            layer.mixer.cos_sin = tables[key]
+        assign_tables((layer.mixer for layer in self.layers), cfg.max_seq_len,
+                      self.device)
         return super().make_cache(cfg)
 
     def embed_rows(self, tokens: torch.Tensor,

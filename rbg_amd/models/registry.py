@@ -6,7 +6,7 @@ import os
 from typing import Callable, Dict
 
 from ..engine.config import ModelConfig
-from . import bitatar, gogalix, llama, notadra
+from . import bitatar, danipel, gogalix, llama, notadra
 
 # architecture -> model class
 MODELS: Dict[str, type] = {
@@ -14,6 +14,7 @@ MODELS: Dict[str, type] = {
     "Bitatar": bitatar.BitatarForCausalLM,
     "Notadra": notadra.NotadraForCausalLM,
     "Gogalix": gogalix.GogalixForCausalLM,
+    "Danipel": danipel.DanipelForCausalLM,
 }
 
 # architecture of a config.json -> its reader
@@ -21,6 +22,7 @@ CONFIG_READERS: Dict[str, Callable[..., ModelConfig]] = {
     "Bitatar": bitatar.BitatarConfig.from_json,
     "Notadra": notadra.NotadraConfig.from_json,
     "Gogalix": gogalix.GogalixConfig.from_json,
+    "Danipel": danipel.DanipelConfig.from_json,
 }
 
 
@@ -41,7 +43,7 @@ def resolve_model(name: str) -> ModelConfig:
     """A preset's name, or a model folder."""
     if os.path.isdir(name):
         return load_config(name)
-    for family in (bitatar, notadra, gogalix):
+    for family in (bitatar, notadra, gogalix, danipel):
         cfg = family.preset(name)
         if cfg is not None:
             return cfg

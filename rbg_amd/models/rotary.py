@@ -8,8 +8,9 @@ frequency, those that turn less than ``slow`` times are slowed down by
 """
 from __future__ import annotations
 
+import json
 import math
-from typing import Any, Dict, Tuple
+from typing import Any, Dict, Iterable, Tuple
 
 import torch
 
@@ -44,3 +45,17 @@ def rotary_table(rot: Dict[str, Any], positions: int,
     angle = torch.outer(torch.arange(positions, dtype=torch.float64), freq)
     return (torch.cat([angle.cos(), angle.sin()], dim=1) * mult).float().to(
         device)
+
+
+def assign_tables(mixers: Iterable, positions: int,
+                  device: torch.device) -> None:
+    """Gives every mixer with a rotation (``rot``) its table (``cos_sin``); one
+    per distinct rotation."""
+    tables: Dict[str, torch.Tensor] = {}
+    for mixer in mixers:
+        if mixer.rot is None:
+            continue
+        key = json.dumps(mixer.rot, sort_keys=True)
+        if key not in tables:
+            tables[key] = rotary_table(mixer.rot, positions, device)
+        mixer.cos_sin = tables[key]

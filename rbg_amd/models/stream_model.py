@@ -100,6 +100,11 @@ class StreamForCausalLM(nn.Module):
                           [layer.cache_spec() for layer in self.layers],
                           self.dtype)
 
+    @property
+    def stream_width(self) -> int:
+        """Columns of what one pipeline stage hands to the next."""
+        return self.cfg.hidden_size
+
     def decode_splits(self, batch_size: int, max_seq_len: int) -> int:
         return 0                        # per layer, from its sizes
 

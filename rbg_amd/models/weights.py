@@ -100,6 +100,8 @@ class RandomSource(WeightSource):
             return t.fill_(1.0)
         if init == "zeros":
             return t.zero_()
+        if init == "eye":
+            return t.copy_(torch.eye(*shape))
         scale = 1.0
         if init == "linear":
             scale = 1.0 / math.sqrt(shape[-1])

@@ -75,6 +75,10 @@ def _require_moe():
     return require("_hip_moe")
 
 
+def _require_hyper():
+    return require("_hip_hyper")
+
+
 def _require_experts():
     return require("_hip_experts")
 
@@ -109,8 +113,8 @@ def linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
              (x.shape[0] <= 16 and w.shape[0] <= 24576 and
               x.shape[1] <= 4096))):
         # one of these is there whatever the model
-        return require("_hip_ops", "_hip_mix", "_hip_gated",
-                       "_hip_moe").skinny_gemm(
+        return require("_hip_ops", "_hip_mix", "_hip_gated", "_hip_moe",
+                       "_hip_hyper").skinny_gemm(
             x if x.is_contiguous() else x.contiguous(), w)
     return torch.nn.functional.linear(x, w)
 
@@ -210,12 +214,14 @@ build_cos_sin_table = reference.build_cos_sin_table
 # -- f32 residual stream ----------------------------------------------------
 
 
-def embed_stream(tokens, table, scale: float) -> torch.Tensor:
-    """f32 stream [T, W] = table[tokens] * scale."""
+def embed_stream(tokens, table, scale: float, copies: int = 1) -> torch.Tensor:
+    """f32 stream [T, W] = table[tokens] * scale; [T, copies * W] of equal
+    streams."""
     if _on_gpu(table):
-        # linked into both extensions of designs that scale
-        return require("_hip_mix", "_hip_gated").embed_stream(tokens, table, scale)
-    return reference.embed_stream(tokens, table, scale)
+        # linked into every extension of designs that scale
+        return require("_hip_mix", "_hip_gated", "_hip_hyper").embed_stream(
+            tokens, table, scale, copies)
+    return reference.embed_stream(tokens, table, scale, copies)
 
 
 def stream_norm(x, delta, w1, w2, groups: int, eps: float, dtype):
@@ -264,9 +270,18 @@ def causal_conv(x, conv_w, conv_state, tiles, cu_seqlens, starts, slots):
 def gelu_mul(x, out) -> None:
     """out (may be a column slice) = gelu_tanh(x[:, :F]) * x[:, F:]."""
     if _on_gpu(x):
-        _require_mix().gelu_mul(x, out)
+        require("_hip_mix", "_hip_hyper").gelu_mul(x, out)
         return
     reference.gelu_mul(x, out)
+
+
+def clamped_glu(gate, up, limit: float, out) -> None:
+    """out = g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = up within
+    +-limit; gate and up are column slices of one buffer."""
+    if _on_gpu(gate):
+        _require_hyper().clamped_glu(gate, up, limit, out)
+        return
+    reference.clamped_glu(gate, up, limit, out)
 
 
 def tanh_rows(x) -> torch.Tensor:
@@ -309,25 +324,65 @@ def delta_rule(proj, z, w2, w0, a_bias, norm_w, state, slots, cu_seqlens,
 # -- latent attention -----------------------------------------------------------
 
 
-def latent_store(x, w, cache, slots, eps: float) -> torch.Tensor:
-    """c = rms_norm(x) * w, written to the paged latents; returns c."""
+@dataclass
+class Rotary:
+    """Rotary positions of a step's rows: table [positions, dims] = [cos | sin]
+    (models/rotary.py); pairs are neighbours (interleaved) or half the dims
+    apart."""
+    table: torch.Tensor
+    positions: torch.Tensor     # [T] int32
+    interleaved: bool
+
+    def rows(self, part: slice) -> "Rotary":
+        return Rotary(self.table, self.positions[part], self.interleaved)
+
+    @property
+    def dims(self) -> int:
+        return self.table.shape[1]
+
+
+def _rotary(rot: Optional[Rotary]):
+    return (None, None, False) if rot is None else (rot.table, rot.positions,
+                                                    rot.interleaved)
+
+
+def latent_store(x, w, cache, slots, eps: float,
+                 rot: Optional[Rotary] = None, second=None):
+    """c = rms_norm(x) * w, written to the paged latents; returns c.  With
+    ``rot`` x's last columns are no latent but a key part: rotated, it follows
+    in the cache and in c.  ``second`` = (x2, w2), another latent of the same
+    rows: its norm is returned beside c."""
     if _on_gpu(x):
-        return _require_latent().latent_store(x, w, cache, slots, eps)
-    return reference.latent_store(x, w, cache, slots, eps)
+        out = _require_latent().latent_store(x, w, cache, slots, eps,
+                                             *_rotary(rot),
+                                             *(second or (None, None)))
+    else:
+        out = reference.latent_store(x, w, cache, slots, eps, rot, second)
+    return out[0] if second is None else out
 
 
-def window_attention(q, k, v, gate, out, view, scale: float,
-                     window: int) -> None:
+def rotate_rows(x, rot: Rotary) -> None:
+    """Rotates x [T, H, rot.dims] in place."""
+    if _on_gpu(x):
+        _require_latent().rotate_rows(x, *_rotary(rot))
+        return
+    x.copy_(reference.rotate(x, rot))
+
+
+def window_attention(q, k, v, gate, out, view, scale: float, window: int,
+                     shared=None, sink=None) -> None:
     """Causal attention over the last ``window`` positions (0: all), q/k
     [T, H, D], v [T, H, Dv]; ``view`` locates each query among the keys
-    (engine/batch.py WindowView).  out = o * sigmoid(gate)."""
+    (engine/batch.py WindowView).  out = o * sigmoid(gate).  ``shared`` [T, D2]
+    are the last dims of every head's key (k then has the others); ``sink`` [H]
+    f32 is a logit per head without key and value."""
     if _on_gpu(q):
         _require_latent().window_attention(q, k, v, gate, out, view.row_info,
-                                        view.seq_info, view.blocks, scale,
-                                        window)
+                                           view.seq_info, view.blocks, scale,
+                                           window, shared, sink)
         return
     reference.window_attention(q, k, v, gate, out, view.row_info, scale,
-                               window)
+                               window, shared, sink)
 
 
 def pick_latent_splits(num_seqs: int, num_heads: int, max_keys: int) -> int:
@@ -342,30 +397,39 @@ def pick_latent_splits(num_seqs: int, num_heads: int, max_keys: int) -> int:
 
 
 def latent_decode(q, cache, block_tables, context_lens, scale: float,
-                  window: int) -> torch.Tensor:
-    """q [S, H, rank] absorbed queries against the paged latents (key and
-    value at once); returns [S, H, rank]."""
+                  window: int, rank: int = 0, sink=None) -> torch.Tensor:
+    """q [S, H, D] absorbed queries against the paged latents [.., D], whose
+    first ``rank`` columns (0: all) are the value; returns [S, H, rank].
+    ``sink`` as in window_attention."""
+    rank = rank or q.shape[2]
     if _on_gpu(q):
         keys = block_tables.shape[1] * cache.shape[1]
         splits = pick_latent_splits(q.shape[0], q.shape[1],
                                     min(keys, window) if window else keys)
         return _require_latent().latent_decode(q, cache, block_tables,
-                                            context_lens, scale, window,
-                                            splits)
+                                               context_lens, scale, window,
+                                               splits, rank, sink)
     return reference.latent_decode(q, cache, block_tables, context_lens,
-                                   scale, window)
+                                   scale, window, rank, sink)
 
 
-def head_linear(x, w, gate=None, out=None) -> torch.Tensor:
-    """out[s, h*n + j] = sum_k x[s, h, k] w[h, j, k], times sigmoid(gate);
-    ``out`` [S, H*n] may be a column slice."""
+def head_linear(x, w, gate=None, out=None, tail=None,
+                rot: Optional[Rotary] = None) -> torch.Tensor:
+    """out[s, h, j] = sum_k x[s, h, k] w[h, j, k], times sigmoid(gate); ``out``
+    [S, H * n] may be a column slice.  With ``tail`` [S, H, rot.dims] each head
+    of out ends in its rotation: out [S, H, n + dims]."""
+    heads, n = w.shape[0], w.shape[1]
+    full = n + (rot.dims if rot is not None else 0)
     if out is None:
-        out = x.new_empty((x.shape[0], w.shape[0] * w.shape[1]))
+        out = x.new_empty((x.shape[0], heads * full))
+    o = out.unflatten(1, (heads, full))
     if _on_gpu(x):
-        _require_latent().head_linear(x, w, gate, out)
+        _require_latent().head_linear(x, w, gate, o, tail, *_rotary(rot))
     else:
-        reference.head_linear(x, w, gate, out)
-    return out
+        reference.head_linear(x, w, gate, o[..., :n])
+        if rot is not None:
+            o[..., n:] = reference.rotate(tail, rot)
+    return out if rot is None else o
 
 
 # -- sandwich norms, paged attention, sparse experts ---------------------------
@@ -501,8 +565,9 @@ def router_logits(x, w) -> torch.Tensor:
     return x.float() @ w.float().T
 
 
-def expert_tile(x, w, top: int) -> int:
-    """Rows per tile that suit x [T, K] through experts w [E, N, K]."""
+def expert_tile(x, w, top: float) -> int:
+    """Rows per tile that suit x [T, K] through experts w [E, N, K], ``top`` of
+    them a token on average."""
     pairs = x.shape[0] * top
     rows = pairs / w.shape[0]                   # per expert, on average
     if (not _on_gpu(x) or x.dtype == torch.float32 or w.shape[1] % 8 or
@@ -514,20 +579,27 @@ def expert_tile(x, w, top: int) -> int:
 
 
 def moe_route(logits, correction, groups: int, keep: int, top: int,
-              tile: int, softmax: bool = False) -> Routing:
+              tile: int, softmax: bool = False, share: Optional[float] = None,
+              identity: int = 0) -> Routing:
     """Chooses the ``top`` experts of each token by sigmoid(logit) + correction
     among the ``keep`` groups with the largest sums of their two best, and lays
     the pairs out by expert.  Weights are the sigmoids.  ``softmax``: the
     choice is by logit + correction, the weights are the softmax of the
-    chosen."""
+    chosen.  ``share``: the scores are the softmax of all, the weights the
+    chosen ones' shares of their scores times ``share``.  The last ``identity``
+    experts return their input: their pairs are weighed but get no row."""
     if _on_gpu(logits):
-        weights, inv, rows, tiles, count = _require_experts().moe_route(
-            logits, correction, groups, keep, top, tile, softmax)
+        mod = _require_experts()
+        mode = (mod.ROUTE_SHARE if share is not None else
+                mod.ROUTE_CHOSEN if softmax else mod.ROUTE_SIGMOID)
+        weights, inv, rows, tiles, count = mod.moe_route(
+            logits, correction, groups, keep, top, tile, mode, identity,
+            1.0 if share is None else share)
         return Routing(top, tile, weights, inv, rows, tiles, count)
     ids, weights = reference.moe_choose(logits, correction, groups, keep, top,
-                                        softmax)
-    return Routing(top, tile, weights,
-                   *reference.moe_tiles(ids, logits.shape[1], tile))
+                                        softmax, share)
+    return Routing(top, tile, weights, *reference.moe_tiles(
+        ids, logits.shape[1] - identity, tile))
 
 
 def interleave_glu(gate, up) -> torch.Tensor:
@@ -539,15 +611,61 @@ def interleave_glu(gate, up) -> torch.Tensor:
 
 
 def expert_linear(x, w, route, gather: bool = False, relu2: bool = False,
-                  swiglu: bool = False) -> torch.Tensor:
+                  swiglu: bool = False,
+                  limit: Optional[float] = None) -> torch.Tensor:
     """Rows in expert order times their expert's w [E, N, K]; ``gather`` takes
     x's rows by token, ``relu2`` applies max(0, .)^2, ``swiglu`` takes w's rows
-    as interleave_glu lays them and gives silu(gate) * up, [.., N / 2]."""
+    as interleave_glu lays them and gives silu(gate) * up, [.., N / 2]; with
+    ``limit`` it is clamped_glu."""
     if _on_gpu(x):
-        return _require_experts().expert_linear(
+        mod = _require_experts()
+        act = (mod.EXPERT_RELU2 if relu2 else mod.EXPERT_NONE if not swiglu
+               else mod.EXPERT_SILU_GLU if limit is None else
+               mod.EXPERT_CLAMPED_GLU)
+        return mod.expert_linear(
             x, w, route.rows if gather else None, route.tiles, route.count,
-            route.rows.numel(), route.tile, relu2, swiglu)
-    return reference.expert_linear(x, w, route, gather, relu2, swiglu)
+            route.rows.numel(), route.tile, act, limit or 0.0)
+    return reference.expert_linear(x, w, route, gather, relu2, swiglu, limit)
+
+
+# -- hyper-connections -----------------------------------------------------------
+
+
+@dataclass
+class TanhNorm:
+    """Dynamic tanh: tanh(alpha * x) * w + b, no statistics of the row."""
+    alpha: torch.Tensor         # [1] f32
+    w: torch.Tensor             # [W] f32
+    b: torch.Tensor             # [W] f32
+
+
+@dataclass
+class Stir:
+    """A sublayer's output on its way into the streams: x_t becomes
+    sum_s mix[s, t] x_s + mult * out[t] * y, y = rows plus, with a routing, the
+    weighed sum of the token's expert rows (``self_rows``: of experts that
+    return their input)."""
+    conn: torch.Tensor          # [S * S + S] f32 = mix[from, to] | out
+    mult: float
+    rows: Optional[torch.Tensor] = None         # [T, W]
+    experts: Optional[torch.Tensor] = None      # [T * top, W]
+    route: Optional[Routing] = None
+    self_rows: Optional[torch.Tensor] = None    # [T, W]
+
+
+def hyper_norm(x, streams: int, stir: Optional[Stir], read,
+               norm: Optional[TanhNorm], dtype):
+    """x [T, streams * W] f32 takes what is pending (in place); returns the
+    norm of sum_s read[s] x_s in ``dtype`` (None without a norm)."""
+    if _on_gpu(x):
+        s = stir or Stir(None, 1.0)
+        n = norm or TanhNorm(None, None, None)
+        return _require_hyper().hyper_norm(
+            x, streams, s.conn, s.rows, s.experts,
+            s.route.inv if s.route else None,
+            s.route.weights if s.route else None, s.self_rows, s.mult, read,
+            n.w, n.b, n.alpha, dtype == torch.float32)
+    return reference.hyper_norm(x, streams, stir, read, norm, dtype)
 
 
 # -- gated branches, gated delta rule -------------------------------------------

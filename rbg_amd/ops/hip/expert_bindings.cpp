@@ -50,10 +50,11 @@ int64_t most_tiles(int64_t pairs, int64_t experts, int64_t tile) {
   return std::min(pairs, experts) + pairs / tile;
 }
 
-// weights [T, top], inv, rows [T * top], tiles [most, 3], count [1]
+// weights [T, top], inv, rows [T * top], tiles [most, 3], count [1]; the last
+// `identity` of the experts return their input and get no rows
 std::vector<Tensor> moe_route(Tensor logits, Tensor correction, int64_t groups,
                               int64_t keep, int64_t top, int64_t tile,
-                              bool softmax) {
+                              int64_t mode, int64_t identity, double scale) {
   TORCH_CHECK(logits.dim() == 2, "logits [T, E]");
   const int64_t T = logits.size(0), E = logits.size(1), P = T * top;
   check_f32(logits, "logits", T * E);
@@ -62,11 +63,14 @@ std::vector<Tensor> moe_route(Tensor logits, Tensor correction, int64_t groups,
   TORCH_CHECK(groups > 0 && E % groups == 0 && keep > 0 && keep <= groups &&
               top > 0 && top <= keep * (E / groups) && tile > 0,
               "groups, keep or top out of range");
+  TORCH_CHECK(mode >= ROUTE_SIGMOID && mode <= ROUTE_SHARE, "route mode");
+  TORCH_CHECK(identity >= 0 && identity < E, "identity experts");
+  const int64_t real = E - identity;
   auto i = logits.options().dtype(torch::kInt32);
   auto weights = torch::empty({T, top}, logits.options());
   auto ids = torch::empty({T, top}, i), inv = torch::empty({P}, i),
        rows = torch::empty({P}, i),
-       tiles = torch::empty({most_tiles(P, E, tile), 3}, i),
+       tiles = torch::empty({most_tiles(P, real, tile), 3}, i),
        count = torch::empty({1}, i);
   MoeRouteArgs p{};
   p.logits = logits.data_ptr<float>();
@@ -83,14 +87,14 @@ std::vector<Tensor> moe_route(Tensor logits, Tensor correction, int64_t groups,
   }
   p.tokens = (int)T; p.experts = (int)E; p.groups = (int)groups;
   p.keep = (int)keep; p.top = (int)top; p.tile = (int)tile;
-  p.softmax = softmax;
+  p.real = (int)real; p.mode = (int)mode; p.scale = (float)scale;
   if (T) launch_moe_route(&p, current_stream());
   return {weights, inv, rows, tiles, count};
 }
 
 Tensor expert_linear(Tensor x, Tensor w, OptTensor rows, Tensor tiles,
-                     Tensor count, int64_t pairs, int64_t tile, bool relu2,
-                     bool swiglu) {
+                     Tensor count, int64_t pairs, int64_t tile, int64_t act,
+                     double limit) {
   check_rows(x, "x");
   TORCH_CHECK(w.is_cuda() && w.dim() == 3 && w.is_contiguous() &&
               x.is_contiguous(), "w [E, N, K] and x must be contiguous");
@@ -100,16 +104,18 @@ Tensor expert_linear(Tensor x, Tensor w, OptTensor rows, Tensor tiles,
   TORCH_CHECK(rows || x.size(0) == pairs, "one row of x per pair");
   TORCH_CHECK(tiles.dim() == 2 && tiles.size(1) == 3 &&
               tiles.size(0) == most_tiles(pairs, E, tile), "tiles shape");
-  TORCH_CHECK(!swiglu || (!relu2 && N % 4 == 0), "swiglu rows");
-  auto out = torch::empty({pairs, swiglu ? N / 2 : N}, x.options());
+  TORCH_CHECK(act >= EXPERT_NONE && act <= EXPERT_CLAMPED_GLU, "activation");
+  const bool glu = act >= EXPERT_SILU_GLU;
+  TORCH_CHECK(!glu || N % 4 == 0, "gate and up rows");
+  auto out = torch::empty({pairs, glu ? N / 2 : N}, x.options());
   MoeGemmArgs p{};
   p.x = x.data_ptr(); p.w = w.data_ptr(); p.out = out.data_ptr();
   p.rows = rows ? i32(*rows, "rows", pairs) : nullptr;
   p.tiles = i32(tiles, "tiles", 0);
   p.count = i32(count, "count", 1);
   p.max_tiles = (int)tiles.size(0); p.tile = (int)tile;
-  p.n = (int)N; p.k = (int)K; p.relu2 = relu2;
-  p.swiglu = swiglu;
+  p.n = (int)N; p.k = (int)K;
+  p.act = (int)act; p.limit = (float)limit;
   const bool vec = !is_f32(x) && mult8({N, K}) && aligned(x, 16) &&
                    aligned(w, 16);
   TORCH_CHECK(tile <= (vec ? 128 : 16), "tile too large for these sizes");
@@ -127,4 +133,11 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("router_logits", &router_logits, "x W^T with f32 sums and result");
   m.def("moe_route", &moe_route, "choice of experts and pairs by expert");
   m.def("expert_linear", &expert_linear, "grouped products by expert");
+  m.attr("ROUTE_SIGMOID") = (int)ROUTE_SIGMOID;
+  m.attr("ROUTE_CHOSEN") = (int)ROUTE_CHOSEN;
+  m.attr("ROUTE_SHARE") = (int)ROUTE_SHARE;
+  m.attr("EXPERT_NONE") = (int)EXPERT_NONE;
+  m.attr("EXPERT_RELU2") = (int)EXPERT_RELU2;
+  m.attr("EXPERT_SILU_GLU") = (int)EXPERT_SILU_GLU;
+  m.attr("EXPERT_CLAMPED_GLU") = (int)EXPERT_CLAMPED_GLU;
 }

@@ -2,6 +2,28 @@
 #pragma once
 #include "vec_io.h"
 
+// o += the weighed sum of one token's `top` expert rows.  A choice whose inv is
+// negative has no row: its expert returns its own input, row `self` of the token
+// (null: such choices are left out, as are expert rows when y is null).
+template <typename T, int V>
+DEV_INLINE void add_expert_rows(const T* __restrict__ y,
+                                const int* __restrict__ inv,
+                                const float* __restrict__ wts, const int top,
+                                const T* __restrict__ self, const size_t token,
+                                const int width, const int i, float* o) {
+#pragma unroll 4
+  for (int t = 0; t < top; ++t) {
+    const int at = inv[token * top + t];
+    const T* src = at < 0 ? self : y;
+    if (src == nullptr) continue;
+    float r[V];
+    load_vec<V>(src + (at < 0 ? token : (size_t)at) * width + i, r);
+    const float w = wts[token * top + t];
+#pragma unroll
+    for (int j = 0; j < V; ++j) o[j] += w * r[j];
+  }
+}
+
 // y of one token: its row, or the weighed sum of its `top` expert rows
 template <typename T, int V>
 DEV_INLINE void branch_row(const T* __restrict__ y, const int* __restrict__ inv,
@@ -14,12 +36,5 @@ DEV_INLINE void branch_row(const T* __restrict__ y, const int* __restrict__ inv,
   }
 #pragma unroll
   for (int j = 0; j < V; ++j) o[j] = 0.f;
-#pragma unroll 4
-  for (int t = 0; t < top; ++t) {
-    float r[V];
-    load_vec<V>(y + (size_t)inv[token * top + t] * width + i, r);
-    const float w = wts[token * top + t];
-#pragma unroll
-    for (int j = 0; j < V; ++j) o[j] += w * r[j];
-  }
+  add_expert_rows<T, V>(y, inv, wts, top, nullptr, token, width, i, o);
 }

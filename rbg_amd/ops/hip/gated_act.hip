@@ -1,7 +1,8 @@
 // Elementwise gates in bf16 or f32: gelu_tanh(gate) * up, silu(gate) * up with
-// or without biases, and tanh of a low-rank projection.  Inputs and outputs are column slices of the
-// fused projection buffers (row strides), so no copy stands between a GEMM and
-// its gate, and the products land in the operand of the layer's output GEMM.
+// or without biases, clamped units, and tanh of a low-rank projection.  Inputs and
+// outputs are column slices of the fused projection buffers (row strides), so no
+// copy stands between a GEMM and its gate, and the products land in the operand of the layer's output GEMM.
+#include "act.h"
 #include "vec_io.h"
 
 namespace {
@@ -19,9 +20,10 @@ struct GluArgs {
   const float* up_bias;
   long out_row, x_row;
   int inter;
+  float limit;            // clamped units
 };
 
-template <typename T, int V, bool SILU>
+template <typename T, int V, int ACT>
 __global__ void glu_kernel(const GluArgs p, const long total) {
   const long step = (long)gridDim.x * blockDim.x;
   const int nv = p.inter / V;
@@ -43,7 +45,9 @@ __global__ void glu_kernel(const GluArgs p, const long total) {
     }
 #pragma unroll
     for (int j = 0; j < V; ++j)
-      u[j] *= SILU ? g[j] * sigmoid_f(g[j]) : gelu_tanh_f(g[j]);
+      u[j] = ACT == GLU_GELU   ? gelu_tanh_f(g[j]) * u[j]
+             : ACT == GLU_SILU ? g[j] * sigmoid_f(g[j]) * u[j]
+                               : clamped_glu_f(g[j], u[j], p.limit);
     store_vec<V>((T*)p.out + row * p.out_row + c, u);
   }
 }
@@ -64,7 +68,7 @@ int blocks_for(long total) {
 
 bool aligned16(const void* p) { return ((uintptr_t)p & 15) == 0; }
 
-template <typename T, bool SILU>
+template <typename T, int ACT>
 void glu_t(const GluArgs& p, long rows, hipStream_t s) {
   const bool vec = p.inter % 8 == 0 && p.out_row % 8 == 0 &&
                    p.x_row % 8 == 0 && aligned16(p.out) &&
@@ -74,9 +78,9 @@ void glu_t(const GluArgs& p, long rows, hipStream_t s) {
   int b = blocks_for(total);
   if (b > 16384) b = 16384;
   if (vec) {
-    glu_kernel<T, 8, SILU><<<b, 256, 0, s>>>(p, total);
+    glu_kernel<T, 8, ACT><<<b, 256, 0, s>>>(p, total);
   } else {
-    glu_kernel<T, 1, SILU><<<b, 256, 0, s>>>(p, total);
+    glu_kernel<T, 1, ACT><<<b, 256, 0, s>>>(p, total);
   }
 }
 
@@ -84,18 +88,23 @@ void glu_t(const GluArgs& p, long rows, hipStream_t s) {
 
 extern "C" {
 
-// out = act(gate + gate_bias) * (up + up_bias); act: silu or gelu_tanh
+// out = act(gate + gate_bias) * (up + up_bias); act: GLU_GELU or GLU_SILU.
+// GLU_CLAMPED: clamped_glu_f of the two, with `limit`.
 void launch_glu(void* out, long out_row, const void* gate, const void* up,
                 long x_row, const float* gate_bias, const float* up_bias,
-                long rows, int inter, int silu, int f32, hipStream_t s) {
-  const GluArgs p{out, gate, up, gate_bias, up_bias, out_row, x_row, inter};
-  if (f32) {
-    if (silu) glu_t<float, true>(p, rows, s);
-    else glu_t<float, false>(p, rows, s);
-  } else {
-    if (silu) glu_t<__hip_bfloat16, true>(p, rows, s);
-    else glu_t<__hip_bfloat16, false>(p, rows, s);
-  }
+                long rows, int inter, int act, float limit, int f32,
+                hipStream_t s) {
+  const GluArgs p{out,     gate,  up,    gate_bias, up_bias,
+                  out_row, x_row, inter, limit};
+#define GLU_T(ACT)                                                            \
+  do {                                                                        \
+    if (f32) glu_t<float, ACT>(p, rows, s);                                   \
+    else glu_t<__hip_bfloat16, ACT>(p, rows, s);                              \
+  } while (0)
+  if (act == GLU_GELU) GLU_T(GLU_GELU);
+  else if (act == GLU_SILU) GLU_T(GLU_SILU);
+  else GLU_T(GLU_CLAMPED);
+#undef GLU_T
 }
 
 void launch_tanh_rows(void* out, const void* x, long stride, long rows,

@@ -2,16 +2,14 @@
 // and gated linear units (bf16 or f32 activations).  Shapes, strides and dtypes
 // are checked here, before launch.
 #include "bind_util.h"
+#include "embed_bindings.h"
 #include "gated_args.h"
 #include "gemm_bindings.h"
+#include "glu_bindings.h"
 
 extern "C" {
-void launch_embed_stream(float*, const void*, const long*, float, int, int,
-                         int, hipStream_t);
 int gate_norm_max_width(int);
 void launch_gate_norm(const GateNormArgs*, int, int, hipStream_t);
-void launch_glu(void*, long, const void*, const void*, long, const float*,
-                const float*, long, int, int, int, hipStream_t);
 void launch_short_conv(const ShortConvArgs*, int, int, hipStream_t);
 void launch_gated_step(const GatedDeltaArgs*, int, int, hipStream_t);
 int gated_chunk_tokens();
@@ -22,21 +20,6 @@ void launch_gated_chunk(const GatedDeltaArgs*, const int*, const int*, float*,
 }
 
 namespace {
-
-Tensor embed_stream(Tensor tokens, Tensor table, double scale) {
-  check_rows(table, "table");
-  TORCH_CHECK(table.is_contiguous() && tokens.is_cuda() &&
-              tokens.scalar_type() == torch::kInt64 && tokens.is_contiguous(),
-              "tokens must be int64 on GPU, table contiguous");
-  auto x = torch::empty({tokens.numel(), table.size(1)},
-                        table.options().dtype(torch::kFloat32));
-  if (tokens.numel())
-    launch_embed_stream(x.data_ptr<float>(), table.data_ptr(),
-                        (const long*)tokens.data_ptr<int64_t>(), (float)scale,
-                        (int)tokens.numel(), (int)table.size(1),
-                        is_f32(table), current_stream());
-  return x;
-}
 
 // one branch: (rows, inv, weights, logits, gate_bias, scale, bias)
 using Branch = std::tuple<Tensor, OptTensor, OptTensor, Tensor, Tensor, Tensor,
@@ -105,28 +88,10 @@ OptTensor gate_norm(Tensor x, std::vector<Branch> branches, OptTensor w,
   return out;
 }
 
-// out = silu(gate + gate_bias) * (up + up_bias); gate, up: slices of one buffer
+// out = silu(gate + gate_bias) * (up + up_bias)
 void silu_glu(Tensor gate, Tensor up, OptTensor gate_bias, OptTensor up_bias,
               Tensor out) {
-  check_rows(gate, "gate");
-  check_rows(up, "up");
-  check_rows(out, "out");
-  same_dtype(gate, up, "up");
-  same_dtype(gate, out, "glu out");
-  const int64_t T = gate.size(0), F = gate.size(1);
-  TORCH_CHECK(up.size(0) == T && up.size(1) == F && out.size(0) == T &&
-              out.size(1) == F && up.stride(0) == gate.stride(0),
-              "gate, up and out must have one shape, gate and up one stride");
-  TORCH_CHECK(gate_bias.has_value() == up_bias.has_value(), "both biases");
-  if (gate_bias) {
-    check_f32(*gate_bias, "gate_bias", F);
-    check_f32(*up_bias, "up_bias", F);
-  }
-  if (T && F)
-    launch_glu(out.data_ptr(), out.stride(0), gate.data_ptr(), up.data_ptr(),
-               gate.stride(0), gate_bias ? gate_bias->data_ptr<float>() : nullptr,
-               up_bias ? up_bias->data_ptr<float>() : nullptr, T, (int)F, 1,
-               is_f32(gate), current_stream());
+  glu_slices(gate, up, gate_bias, up_bias, out, GLU_SILU, 0.0);
 }
 
 void check_ring(const Tensor& ring, const Tensor& conv_w, const Tensor& like,

@@ -1,6 +1,8 @@
 // Per-head linear maps of a decode batch: every head multiplies its own weight
 // [n, k] (the absorbed key and value expansions of latent attention), with an
-// optional sigmoid output gate, straight into a column slice.
+// optional sigmoid output gate, straight into a column slice.  Behind a head's
+// columns may follow the rotated dims of its query: the absorbed query of latent
+// attention is then ready.
 //
 // Decode-shaped: few rows, so the time is the weights' stream.  bf16: a wave
 // owns 16 output columns of a head for 16 * MT rows; weight rows are MFMA A
@@ -8,11 +10,25 @@
 // exactly one wave), the rows are B fragments from L2.  The result's lanes are
 // rows and its registers four neighbouring columns.  f32 (and sizes that are
 // not multiples of 8): one thread per output.
-#include "mfma_util.h"
 #include "latent_args.h"
+#include "mfma_util.h"
+#include "rotary.h"
 #include "vec_io.h"
 
 namespace {
+
+// rows [s0, s1) of a head's tail; the workgroup's threads together
+template <typename T>
+DEV_INLINE void rotate_tail(const HeadLinearArgs& p, const int head,
+                            const int s0, const int s1) {
+  const int half = p.rot.dims / 2;
+  for (int e = threadIdx.x; e < (s1 - s0) * half; e += blockDim.x) {
+    const int s = s0 + e / half;
+    rotate_pair(p.rot, rotary_row(p.rot, s), e % half,
+                (const T*)p.tail + (size_t)s * p.t_row + head * p.t_head,
+                (T*)p.out + (size_t)s * p.o_row + head * p.o_head + p.n);
+  }
+}
 
 template <int MT>
 __global__ __launch_bounds__(256) void head_linear_kernel(
@@ -22,6 +38,10 @@ __global__ __launch_bounds__(256) void head_linear_kernel(
   const int head = blockIdx.y;
   const int n0 = (blockIdx.x * 4 + wave) * 16;
   const int s0 = blockIdx.z * 16 * MT;
+  if (blockIdx.x * 64 >= p.n) {                 // the workgroup behind the last
+    rotate_tail<__hip_bfloat16>(p, head, s0, min(s0 + 16 * MT, p.rows));
+    return;
+  }
   if (n0 >= p.n) return;
   const __hip_bfloat16* w = (const __hip_bfloat16*)p.w +
       ((size_t)head * p.n + min(n0 + gl, p.n - 1)) * p.k;
@@ -55,18 +75,18 @@ __global__ __launch_bounds__(256) void head_linear_kernel(
     if (p.pack) {                       // four columns as one 8-byte access
       const int n = n0 + gs * 4;
       if (n >= p.n) continue;
-      const size_t col = (size_t)head * p.n + n;
       union { uint2 u; __hip_bfloat16 e[4]; } ov, gv;
       if (p.gate != nullptr)
         gv.u = *reinterpret_cast<const uint2*>(
-            (const __hip_bfloat16*)p.gate + (size_t)s * p.g_row + col);
+            (const __hip_bfloat16*)p.gate + (size_t)s * p.g_row +
+            (size_t)head * p.n + n);
 #pragma unroll
       for (int r = 0; r < 4; ++r)
         ov.e[r] = f2bf(p.gate != nullptr
                            ? acc[t][r] * sigmoid_f(bf2f(gv.e[r]))
                            : acc[t][r]);
       *reinterpret_cast<uint2*>((__hip_bfloat16*)p.out + (size_t)s * p.o_row +
-                                col) = ov.u;
+                                head * p.o_head + n) = ov.u;
       continue;
     }
 #pragma unroll
@@ -77,7 +97,7 @@ __global__ __launch_bounds__(256) void head_linear_kernel(
       if (p.gate != nullptr)
         o *= sigmoid_f(bf2f(((const __hip_bfloat16*)p.gate)[
             (size_t)s * p.g_row + (size_t)head * p.n + n]));
-      ((__hip_bfloat16*)p.out)[(size_t)s * p.o_row + (size_t)head * p.n + n] =
+      ((__hip_bfloat16*)p.out)[(size_t)s * p.o_row + head * p.o_head + n] =
           f2bf(o);
     }
   }
@@ -87,6 +107,12 @@ template <typename T>
 __global__ __launch_bounds__(256) void head_linear_rows_kernel(
     const HeadLinearArgs p, const long total) {
   const long i = blockIdx.x * 256L + threadIdx.x;
+  const long main = (total + 255) / 256;
+  if (blockIdx.x >= main) {                     // one (row, head) each
+    const int at = (int)(blockIdx.x - main), s = at / p.heads;
+    rotate_tail<T>(p, at % p.heads, s, s + 1);
+    return;
+  }
   if (i >= total) return;
   const int n = (int)(i % p.n), head = (int)(i / p.n % p.heads);
   const long s = i / ((long)p.n * p.heads);
@@ -94,10 +120,10 @@ __global__ __launch_bounds__(256) void head_linear_rows_kernel(
   const T* x = (const T*)p.x + s * p.x_row + head * p.x_head;
   float o = 0.f;
   for (int k = 0; k < p.k; ++k) o += to_f(x[k]) * to_f(w[k]);
-  const long col = (long)head * p.n + n;
   if (p.gate != nullptr)
-    o *= sigmoid_f(to_f(((const T*)p.gate)[s * p.g_row + col]));
-  ((T*)p.out)[s * p.o_row + col] = from_f<T>(o);
+    o *= sigmoid_f(
+        to_f(((const T*)p.gate)[s * p.g_row + (long)head * p.n + n]));
+  ((T*)p.out)[s * p.o_row + head * p.o_head + n] = from_f<T>(o);
 }
 
 }  // namespace
@@ -105,14 +131,15 @@ __global__ __launch_bounds__(256) void head_linear_rows_kernel(
 extern "C" void launch_head_linear(const HeadLinearArgs* p, int f32, int vec,
                                    hipStream_t s) {
   const long total = (long)p->rows * p->heads * p->n;
+  const bool tail = p->rot.dims > 0;
+  const int grid = (int)((total + 255) / 256) +
+                   (tail ? p->rows * p->heads : 0);
   if (f32) {
-    head_linear_rows_kernel<float>
-        <<<(int)((total + 255) / 256), 256, 0, s>>>(*p, total);
+    head_linear_rows_kernel<float><<<grid, 256, 0, s>>>(*p, total);
   } else if (!vec) {
-    head_linear_rows_kernel<__hip_bfloat16>
-        <<<(int)((total + 255) / 256), 256, 0, s>>>(*p, total);
+    head_linear_rows_kernel<__hip_bfloat16><<<grid, 256, 0, s>>>(*p, total);
   } else {
-    const int nb = (p->n + 63) / 64;
+    const int nb = (p->n + 63) / 64 + (tail ? 1 : 0);
     if (p->rows <= 16) {
       head_linear_kernel<1><<<dim3(nb, p->heads, 1), 256, 0, s>>>(*p);
     } else if (p->rows <= 32) {

@@ -1,28 +1,38 @@
 // Latent attention (gfx950): the normed latent is the only cached row, and a
 // query sees the last `window` positions (window 0: all of them).
 //
-//   latent_store  c = rms_norm(down-projection) * w, written to the paged pool
-//                 and to a contiguous buffer for this step's expansion
+//   latent_store  c = rms_norm(down-projection) * w, and behind it a rotated key
+//                 part that all heads share, written to the paged pool and to a
+//                 contiguous buffer for this step's expansion; a second latent
+//                 (of queries) may be normed in the same launch
+//   rotate        the rotated part of a step's queries, in place
 //   attn_rows     one wave per (query row, head), any head sizes, bf16 or f32:
 //                 keys 64 at a time, a lane scores a key, then the lanes hold
 //                 the value dimensions.  Contiguous keys/values (expanded per
 //                 head, prefill) or the paged latents themselves as both key
 //                 and value (query absorbed into the latent space, decode).
 #include "latent_args.h"
+#include "rotary.h"
 #include "vec_io.h"
 
 namespace {
 
+// blockIdx.y 0: the latent and its key part; 1: the second latent
 template <typename T, int V>
 __global__ __launch_bounds__(256) void latent_store_kernel(
-    T* __restrict__ c, T* __restrict__ cache, const T* __restrict__ x,
-    const long x_stride, const float* __restrict__ w,
-    const int* __restrict__ slots, const int rows, const int rank,
-    const float eps) {
+    const LatentStoreArgs p) {
   const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
   const int lane = threadIdx.x & 63;
-  if (row >= rows) return;
-  const T* src = x + (size_t)row * x_stride;
+  if (row >= p.rows) return;
+  const bool second = blockIdx.y == 1;
+  const int rank = second ? p.rank2 : p.rank;
+  const T* src = second ? (const T*)p.x2 + (size_t)row * p.x2_row
+                        : (const T*)p.x + (size_t)row * p.x_row;
+  const float* w = second ? p.w2 : p.w;
+  const int wide = second ? rank : rank + p.rot.dims;
+  T* c = (second ? (T*)p.c2 : (T*)p.c) + (size_t)row * wide;
+  const int slot = second ? -1 : p.slots[row];
+  T* kept = slot >= 0 ? (T*)p.cache + (size_t)slot * wide : nullptr;
   float ss = 0.f;
   for (int i = lane * V; i < rank; i += 64 * V) {
     float v[V];
@@ -30,17 +40,73 @@ __global__ __launch_bounds__(256) void latent_store_kernel(
 #pragma unroll
     for (int j = 0; j < V; ++j) ss += v[j] * v[j];
   }
-  const float inv = 1.f / sqrtf(wave_sum(ss) / rank + eps);
-  const int slot = slots[row];
+  const float inv = 1.f / sqrtf(wave_sum(ss) / rank + p.eps);
   for (int i = lane * V; i < rank; i += 64 * V) {
     float v[V], wv[V];
     load_vec<V>(src + i, v);
     load_vec<V>(w + i, wv);
 #pragma unroll
     for (int j = 0; j < V; ++j) v[j] = v[j] * inv * wv[j];
-    if (slot >= 0) store_vec<V>(cache + (size_t)slot * rank + i, v);
-    if (c != nullptr) store_vec<V>(c + (size_t)row * rank + i, v);
+    if (kept != nullptr) store_vec<V>(kept + i, v);
+    store_vec<V>(c + i, v);
   }
+  if (second || p.rot.dims == 0) return;
+  const float* cs = rotary_row(p.rot, row);
+  for (int i = lane; i < p.rot.dims / 2; i += 64) {
+    rotate_pair(p.rot, cs, i, src + rank, c + rank);
+    if (kept != nullptr) rotate_pair(p.rot, cs, i, src + rank, kept + rank);
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void rotate_kernel(const RotateArgs p,
+                                                     const long total) {
+  const long item = blockIdx.x * 256l + threadIdx.x;
+  if (item >= total) return;
+  const int half = p.rot.dims / 2, i = (int)(item % half);
+  const int head = (int)(item / half % p.heads);
+  const int row = (int)(item / ((long)half * p.heads));
+  T* x = (T*)p.x + row * p.x_row + head * p.x_head;
+  rotate_pair(p.rot, rotary_row(p.rot, row), i, x, x);
+}
+
+// 8 neighbouring elements a thread (twice 8 when the halves are paired)
+__global__ __launch_bounds__(256) void rotate_vec_kernel(const RotateArgs p,
+                                                         const long total) {
+  const long item = blockIdx.x * 256l + threadIdx.x;
+  if (item >= total) return;
+  const int dims = p.rot.dims, half = dims / 2;
+  const int per = p.rot.interleaved ? dims / 8 : half / 8;
+  const int i = (int)(item % per) * 8;
+  const int head = (int)(item / per % p.heads);
+  const int row = (int)(item / ((long)per * p.heads));
+  __hip_bfloat16* x =
+      (__hip_bfloat16*)p.x + row * p.x_row + head * p.x_head + i;
+  const float* cs = rotary_row(p.rot, row);
+  float a[8], o[8];
+  load_vec<8>(x, a);
+  if (p.rot.interleaved) {
+    float c[4], s[4];
+    load_vec<4>(cs + i / 2, c);
+    load_vec<4>(cs + half + i / 2, s);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      o[2 * j] = a[2 * j] * c[j] - a[2 * j + 1] * s[j];
+      o[2 * j + 1] = a[2 * j + 1] * c[j] + a[2 * j] * s[j];
+    }
+    store_vec<8>(x, o);
+    return;
+  }
+  float b[8], c[8], s[8];
+  load_vec<8>(x + half, b);
+  load_vec<8>(cs + i, c);
+  load_vec<8>(cs + half + i, s);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) o[j] = a[j] * c[j] - b[j] * s[j];
+  store_vec<8>(x, o);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) o[j] = b[j] * c[j] + a[j] * s[j];
+  store_vec<8>(x + half, o);
 }
 
 // NACC: value dimensions per lane (dv <= 64 * NACC)
@@ -72,8 +138,13 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnRowsArgs p) {
   };
   const int lo = p.window > 0 ? max(0, pos - p.window + 1) : 0;
   const T* kp = (const T*)p.k + head * p.k_head;
+  const T* k2 = (const T*)p.k2;
   const T* vp = (const T*)p.v + head * p.v_head;
   float m = -INFINITY, l = 0.f, acc[NACC];
+  if (p.sink != nullptr) {
+    m = p.sink[head];
+    l = 1.f;
+  }
 #pragma unroll
   for (int i = 0; i < NACC; ++i) acc[i] = 0.f;
 
@@ -81,9 +152,14 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnRowsArgs p) {
     const int j = j0 + lane;
     float s = -INFINITY;
     if (j <= pos) {
-      const T* kr = kp + key_row(j) * p.k_row;
+      const long at = key_row(j);
+      const T* kr = kp + at * p.k_row;
       float dot = 0.f;
-      for (int i = 0; i < p.d; ++i) dot += q[i] * to_f(kr[i]);
+      for (int i = 0; i < p.d1; ++i) dot += q[i] * to_f(kr[i]);
+      if (k2 != nullptr) {
+        kr = k2 + at * p.k2_row - p.d1;
+        for (int i = p.d1; i < p.d; ++i) dot += q[i] * to_f(kr[i]);
+      }
       s = dot * p.scale;
     }
     const float mn = fmaxf(m, wave_max(s));
@@ -139,17 +215,27 @@ void attn_rows_t(const AttnRowsArgs& p, hipStream_t s) {
 
 extern "C" {
 
-void launch_latent_store(void* c, void* cache, const void* x, long x_stride,
-                         const float* w, const int* slots, int rows, int rank,
-                         float eps, int f32, hipStream_t s) {
-  const int grid = (rows + 3) / 4;
-  const bool vec = rank % 8 == 0 && x_stride % 8 == 0 &&
-                   ((uintptr_t)x & 15) == 0;
-#define LS_GO(T, V) latent_store_kernel<T, V><<<grid, 256, 0, s>>>(           \
-      (T*)c, (T*)cache, (const T*)x, x_stride, w, slots, rows, rank, eps)
+void launch_latent_store(const LatentStoreArgs* p, int f32, int vec,
+                         hipStream_t s) {
+  const dim3 grid((p->rows + 3) / 4, p->x2 != nullptr ? 2 : 1);
+#define LS_GO(T, V) latent_store_kernel<T, V><<<grid, 256, 0, s>>>(*p)
   if (f32) { if (vec) LS_GO(float, 8); else LS_GO(float, 1); }
   else { if (vec) LS_GO(__hip_bfloat16, 8); else LS_GO(__hip_bfloat16, 1); }
 #undef LS_GO
+}
+
+void launch_rotate(const RotateArgs* p, int f32, int vec, hipStream_t s) {
+  const int half = p->rot.dims / 2;
+  const long per = !vec ? half : p->rot.interleaved ? half / 4 : half / 8;
+  const long total = (long)p->rows * p->heads * per;
+  const int grid = (int)((total + 255) / 256);
+  if (vec) {
+    rotate_vec_kernel<<<grid, 256, 0, s>>>(*p, total);
+  } else if (f32) {
+    rotate_kernel<float><<<grid, 256, 0, s>>>(*p, total);
+  } else {
+    rotate_kernel<__hip_bfloat16><<<grid, 256, 0, s>>>(*p, total);
+  }
 }
 
 void launch_attn_rows(const AttnRowsArgs* p, int f32, hipStream_t s) {

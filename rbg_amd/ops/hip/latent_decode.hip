@@ -1,5 +1,6 @@
 // Decode attention over paged latents (gfx950, bf16): absorbed queries, one
-// token per sequence, the latent as key and value at once, window-limited.
+// token per sequence, the latent as key and value at once, window-limited.  A key
+// may be longer than its value (a rotated part behind the latent).
 //
 // A workgroup takes one sequence, 16 heads and one split of the visible keys,
 // 64 keys a step (4 chunks of 16: a chunk is part of one page, so contiguous):
@@ -20,11 +21,12 @@ namespace {
 
 constexpr int NW = 4;
 
-template <int RK>
+// RK: value columns, DK: key columns
+template <int RK, int DK>
 __global__ __launch_bounds__(NW * 64, 2) void latent_decode_kernel(
     const LatentDecodeArgs p) {
-  constexpr int PITCH = RK + 16;              // 8 banks per row
-  constexpr int LPC = 16 * RK / 8 / 64;       // 16-byte loads per chunk
+  constexpr int PITCH = DK + 16;              // 8 banks per row
+  constexpr int LPC = 16 * DK / 8 / 64;       // 16-byte loads per chunk
   constexpr int DT = RK / 16 / NW;            // 16-column tiles per wave
   static_assert(DT >= 1 && LPC >= 1, "rank tile too small");
   extern __shared__ __attribute__((aligned(16))) char smem[];
@@ -47,20 +49,24 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_decode_kernel(
   const int* table = p.tables + (size_t)seq * p.max_pages;
   const __hip_bfloat16* cache = (const __hip_bfloat16*)p.cache;
   const int cpp = p.page_size >> 4;           // chunks per page
-  const bool full = p.rank == RK;
+  const bool full = p.d == DK;
 
   const int head = min(h0 + gl, p.heads - 1);
   const __hip_bfloat16* q = (const __hip_bfloat16*)p.q +
                             (size_t)seq * p.q_row + (size_t)head * p.q_head;
-  mf_bf8 qf[RK / 32];
+  mf_bf8 qf[DK / 32];
 #pragma unroll
-  for (int s = 0; s < RK / 32; ++s) {
+  for (int s = 0; s < DK / 32; ++s) {
     const int d = s * 32 + gs * 8;
     mf_bf8 z = {};
-    qf[s] = d < p.rank ? frag8(q + d) : z;
+    qf[s] = d < p.d ? frag8(q + d) : z;
   }
 
   float m = MASKED, l = 0.f;
+  if (p.sink != nullptr && split == 0) {      // counts once
+    m = p.sink[head] * LOG2E;
+    l = wave == 0 && gs == 0 ? 1.f : 0.f;
+  }
   f32x4 acc[DT];
 #pragma unroll
   for (int d = 0; d < DT; ++d) acc[d] = {0.f, 0.f, 0.f, 0.f};
@@ -74,11 +80,11 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_decode_kernel(
     const int cc = min((c), c_end - 1);                                       \
     const __hip_bfloat16* src =                                               \
         cache + ((size_t)table[cc / cpp] * p.page_size + (cc % cpp) * 16) *   \
-                    p.rank;                                                   \
+                    p.d;                                                      \
     _Pragma("unroll") for (int i = 0; i < LPC; ++i) {                         \
-      const int e = i * 64 + lane, key = e / (RK / 8), d = (e % (RK / 8)) * 8;\
-      reg[i] = full || d < p.rank                                             \
-          ? *reinterpret_cast<const u32x4*>(src + key * p.rank + d) : zero4;  \
+      const int e = i * 64 + lane, key = e / (DK / 8), d = (e % (DK / 8)) * 8;\
+      reg[i] = full || d < p.d                                                \
+          ? *reinterpret_cast<const u32x4*>(src + key * p.d + d) : zero4;     \
     }                                                                         \
   } while (0)
 
@@ -91,7 +97,7 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_decode_kernel(
     const int c_hi = min(pos, c_end * 16 - 1);
 #pragma unroll
     for (int i = 0; i < LPC; ++i) {
-      const int e = i * 64 + lane, key = e / (RK / 8), d = (e % (RK / 8)) * 8;
+      const int e = i * 64 + lane, key = e / (DK / 8), d = (e % (DK / 8)) * 8;
       const int j = c * 16 + key;
       *reinterpret_cast<u32x4*>(&mine[key * PITCH + d]) =
           j >= lo && j <= c_hi ? reg[i] : zero4;
@@ -99,7 +105,7 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_decode_kernel(
     if (c0 + NW < c_end) LD_FETCH(c + NW);
     f32x4 s = {0.f, 0.f, 0.f, 0.f}, s2 = s;
 #pragma unroll
-    for (int st = 0; st < RK / 32; st += 2) {
+    for (int st = 0; st < DK / 32; st += 2) {
       s = mfma_bf16_k32(frag8(&mine[gl * PITCH + st * 32 + gs * 8]), qf[st],
                         s);
       s2 = mfma_bf16_k32(frag8(&mine[gl * PITCH + st * 32 + 32 + gs * 8]),
@@ -231,33 +237,49 @@ __global__ __launch_bounds__(128) void latent_combine_kernel(
   }
 }
 
-template <int RK>
-void latent_decode_t(const LatentDecodeArgs& p, hipStream_t s) {
-  const size_t lds = (size_t)64 * (RK + 16) * 2 + 2 * 256 * 8 + NW * 16 * 4;
+template <int RK, int DK>
+void latent_decode_go(const LatentDecodeArgs& p, hipStream_t s) {
+  const size_t lds = (size_t)64 * (DK + 16) * 2 + 2 * 256 * 8 + NW * 16 * 4;
   static bool once = false;
   if (!once) {
-    (void)hipFuncSetAttribute((const void*)latent_decode_kernel<RK>,
+    (void)hipFuncSetAttribute((const void*)latent_decode_kernel<RK, DK>,
                               hipFuncAttributeMaxDynamicSharedMemorySize,
                               (int)lds);
     once = true;
   }
   const dim3 grid(p.splits, p.seqs, (p.heads + 15) / 16);
-  latent_decode_kernel<RK><<<grid, NW * 64, lds, s>>>(p);
+  latent_decode_kernel<RK, DK><<<grid, NW * 64, lds, s>>>(p);
+}
+
+template <int RK>
+void latent_decode_t(const LatentDecodeArgs& p, hipStream_t s) {
+  if (p.d <= RK) latent_decode_go<RK, RK>(p, s);
+  else if (p.d <= RK + 64) latent_decode_go<RK, RK + 64>(p, s);
+  else latent_decode_go<RK, RK + 128>(p, s);
+}
+
+int value_columns(int rank) {
+  return rank <= 64 ? 64 : rank <= 128 ? 128 : rank <= 256 ? 256 : 512;
 }
 
 }  // namespace
 
-extern "C" void launch_latent_decode(const LatentDecodeArgs* p,
-                                     hipStream_t s) {
-  if (p->rank <= 64) {
-    latent_decode_t<64>(*p, s);
-  } else if (p->rank <= 128) {
-    latent_decode_t<128>(*p, s);
-  } else if (p->rank <= 256) {
-    latent_decode_t<256>(*p, s);
-  } else {
-    latent_decode_t<512>(*p, s);
+extern "C" {
+
+// whether there is a form for these sizes
+int latent_decode_fits(int d, int rank) {
+  return rank <= 512 && d >= rank && d <= value_columns(rank) + 128;
+}
+
+void launch_latent_decode(const LatentDecodeArgs* p, hipStream_t s) {
+  switch (value_columns(p->rank)) {
+    case 64: latent_decode_t<64>(*p, s); break;
+    case 128: latent_decode_t<128>(*p, s); break;
+    case 256: latent_decode_t<256>(*p, s); break;
+    default: latent_decode_t<512>(*p, s); break;
   }
   if (p->splits > 1)
     latent_combine_kernel<<<p->seqs * p->heads, 128, 0, s>>>(*p);
 }
+
+}  // extern "C"

@@ -1,20 +1,18 @@
 // PyTorch bindings for the f32-stream and token-mixer kernels (bf16 or f32
 // activations).  Shapes, strides and dtypes are checked here, before launch.
 #include "bind_util.h"
+#include "embed_bindings.h"
 #include "gemm_bindings.h"
+#include "glu_bindings.h"
 #include "mix_args.h"
 
 extern "C" {
-void launch_embed_stream(float*, const void*, const long*, float, int, int,
-                         int, hipStream_t);
 void launch_stream_norm(float*, const void*, const float*, const float*, void*,
                         void*, int, int, int, float, const float*, void*,
                         const int*, const int*, int, int, hipStream_t);
 void launch_causal_conv(void*, const void*, const float*, void*, const int*,
                         const int*, const int*, const int*, int, int, int, int,
                         int, hipStream_t);
-void launch_glu(void*, long, const void*, const void*, long, const float*,
-                const float*, long, int, int, int, hipStream_t);
 void launch_tanh_rows(void*, const void*, long, long, int, int, hipStream_t);
 void launch_delta_step(const DeltaArgs*, int, int, hipStream_t);
 int delta_chunk_tokens();
@@ -24,21 +22,6 @@ void launch_delta_chunk(const DeltaArgs*, const int*, const int*, float*,
 }
 
 namespace {
-
-Tensor embed_stream(Tensor tokens, Tensor table, double scale) {
-  check_rows(table, "table");
-  TORCH_CHECK(table.is_contiguous() && tokens.is_cuda() &&
-              tokens.scalar_type() == torch::kInt64 && tokens.is_contiguous(),
-              "tokens must be int64 on GPU, table contiguous");
-  auto x = torch::empty({tokens.numel(), table.size(1)},
-                        table.options().dtype(torch::kFloat32));
-  if (tokens.numel())
-    launch_embed_stream(x.data_ptr<float>(), table.data_ptr(),
-                        (const long*)tokens.data_ptr<int64_t>(), (float)scale,
-                        (int)tokens.numel(), (int)table.size(1),
-                        is_f32(table), current_stream());
-  return x;
-}
 
 // x += delta; n1, n2 = grouped norms of x under w1, w2 (w2 optional).  With
 // conv arguments n1 becomes the convolved mixer input of a decode step.
@@ -110,19 +93,6 @@ Tensor causal_conv(Tensor x, Tensor conv_w, Tensor state, Tensor tiles,
                        i32(slots, "slots", B), (int)tiles.size(0), (int)tile,
                        (int)W, (int)taps, is_f32(x), current_stream());
   return out;
-}
-
-void gelu_mul(Tensor x, Tensor out) {
-  check_rows(x, "x");
-  check_rows(out, "out");
-  same_dtype(x, out, "gelu_mul");
-  TORCH_CHECK(x.is_contiguous() && x.size(1) == 2 * out.size(1) &&
-              x.size(0) == out.size(0), "x must be [T, 2*ff] of out's rows");
-  const int64_t F = out.size(1);
-  if (x.size(0))
-    launch_glu(out.data_ptr(), out.stride(0), x.data_ptr(),
-               (const char*)x.data_ptr() + F * x.element_size(), 2 * F, nullptr,
-               nullptr, x.size(0), (int)F, 0, is_f32(x), current_stream());
 }
 
 Tensor tanh_rows(Tensor x) {

@@ -14,9 +14,10 @@
 //           the MFMAs, waves split K and meet in LDS: batches whose experts do
 //           not fill the chip otherwise.
 //   rows    any sizes, bf16 or f32: a thread per column, up to 16 rows at once.
-// A squared relu, or silu(gate) * up of interleaved rows, rides on the way out.
+// A squared relu, or a gated unit of interleaved rows, rides on the way out.
 #include "lds_stream.h"
 #include "expert_args.h"
+#include "act.h"
 #include "vec_io.h"
 
 namespace {
@@ -26,22 +27,27 @@ DEV_INLINE float relu2_f(float x) {
   return x * x;
 }
 
-DEV_INLINE float swiglu_f(float g, float u) { return g * sigmoid_f(g) * u; }
+DEV_INLINE bool gated(const MoeGemmArgs& p) { return p.act >= EXPERT_SILU_GLU; }
+
+DEV_INLINE float glu_f(const MoeGemmArgs& p, float g, float u) {
+  return p.act == EXPERT_CLAMPED_GLU ? clamped_glu_f(g, u, p.limit)
+                                     : silu_glu_f(g, u);
+}
 
 // four neighbouring columns of one row
 DEV_INLINE void put4(const MoeGemmArgs& p, const size_t row, const int n,
                      f32x4 v) {
-  if (p.swiglu) {                               // gate, gate, up, up
+  if (gated(p)) {                               // gate, gate, up, up
     union { uint32_t u; __hip_bfloat16 e[2]; } o;
-    o.e[0] = f2bf(swiglu_f(v[0], v[2]));
-    o.e[1] = f2bf(swiglu_f(v[1], v[3]));
+    o.e[0] = f2bf(glu_f(p, v[0], v[2]));
+    o.e[1] = f2bf(glu_f(p, v[1], v[3]));
     *reinterpret_cast<uint32_t*>((__hip_bfloat16*)p.out + row * (p.n / 2) +
                                  n / 2) = o.u;
     return;
   }
   union { uint2 u; __hip_bfloat16 e[4]; } o;
 #pragma unroll
-  for (int r = 0; r < 4; ++r) o.e[r] = f2bf(p.relu2 ? relu2_f(v[r]) : v[r]);
+  for (int r = 0; r < 4; ++r) o.e[r] = f2bf(p.act == EXPERT_RELU2 ? relu2_f(v[r]) : v[r]);
   *reinterpret_cast<uint2*>((__hip_bfloat16*)p.out + row * p.n + n) = o.u;
 }
 
@@ -283,13 +289,16 @@ __global__ __launch_bounds__(256) void moe_rows_kernel(const MoeGemmArgs p) {
   for (int r = 0; r < 16; ++r)
     if (r < rows)
       ((T*)p.out)[(size_t)(row0 + r) * cols + c] = from_f<T>(
-          GLU ? swiglu_f(acc[r], up[r]) : p.relu2 ? relu2_f(acc[r]) : acc[r]);
+          GLU                       ? glu_f(p, acc[r], up[r])
+          : p.act == EXPERT_RELU2 ? relu2_f(acc[r])
+                                  : acc[r]);
 }
 
 template <typename T>
 void moe_rows(const MoeGemmArgs& p, hipStream_t s) {
-  const dim3 grid(((p.swiglu ? p.n / 2 : p.n) + 255) / 256, p.max_tiles);
-  if (p.swiglu) {
+  const bool glu = p.act >= EXPERT_SILU_GLU;
+  const dim3 grid(((glu ? p.n / 2 : p.n) + 255) / 256, p.max_tiles);
+  if (glu) {
     moe_rows_kernel<T, true><<<grid, 256, 0, s>>>(p);
   } else {
     moe_rows_kernel<T, false><<<grid, 256, 0, s>>>(p);

@@ -2,17 +2,16 @@
 //
 //   logits   x W^T with f32 sums.  W rows are MFMA A fragments: lanes are tokens,
 //            registers experts.
-//   choose   one wave per token: sigmoid (or the logit itself), correction, the
+//   choose   one wave per token: sigmoid, logit or softmax, correction, the
 //            two best of each group of neighbours, the best groups, the best
-//            experts of those; weights are the sigmoids, or a softmax over the
-//            chosen.  Ranks
-//            are counted, not sorted: an expert's rank is the number of experts
+//            experts of those; weights by the rule's mode.  Ranks are counted, not sorted: an expert's rank is the number of experts
 //            ahead of it in the order (score, index), which is total, so every
 //            place is filled exactly once whatever the scores are.
 //   lay out  pairs (token, choice) counted per expert, offsets by a scan, tiles
 //            of one expert each, and the permutation: one workgroup, together
 //            with the choice for small batches; for prompts the counting and the
-//            permutation are spread over blocks of tokens.
+//            permutation are spread over blocks of tokens.  Experts from `real`
+//            on have no weights: their pairs are weighed, but get no row.
 #include "lds_stream.h"
 #include "expert_args.h"
 #include "vec_io.h"
@@ -140,10 +139,21 @@ DEV_INLINE void choose(const MoeRouteArgs& p, const int token, float* choice,
   const float* z = p.logits + (size_t)token * p.experts;
   const int ep = (p.experts + 3) & ~3, gp = (p.groups + 3) & ~3;
   float* group = choice + ep;
+  float most = -INFINITY, sum = 0.f;
+  if (p.mode == ROUTE_SHARE) {                  // softmax over all
+    for (int e = lane; e < p.experts; e += 64) most = fmaxf(most, z[e]);
+    most = wave_max(most);
+    for (int e = lane; e < p.experts; e += 64) sum += expf(z[e] - most);
+    sum = wave_sum(sum);
+  }
+  auto score = [&](int e) {
+    return p.mode == ROUTE_SHARE    ? expf(z[e] - most) / sum
+           : p.mode == ROUTE_CHOSEN ? z[e]
+                                    : sigmoid_exact(z[e]);
+  };
   for (int e = lane; e < ep; e += 64)           // NaN becomes the least score
     choice[e] = e < p.experts
-        ? fmaxf((p.softmax ? z[e] : sigmoid_exact(z[e])) + p.correction[e],
-                -3e38f) : -INFINITY;
+        ? fmaxf(score(e) + p.correction[e], -3e38f) : -INFINITY;
   wave_fence();
   const int size = p.experts / p.groups;
   if (p.keep < p.groups) {
@@ -166,31 +176,36 @@ DEV_INLINE void choose(const MoeRouteArgs& p, const int token, float* choice,
         for (int i = 0; i < size; ++i) choice[g * size + i] = -INFINITY;
     wave_fence();
   }
-  float most = -INFINITY, sum = 0.f;
-  if (p.softmax) {
+  if (p.mode == ROUTE_CHOSEN) {
     for (int e = lane; e < p.experts; e += 64) most = fmaxf(most, choice[e]);
     most = wave_max(most);
   }
+  auto weight = [&](int e) {
+    return p.mode == ROUTE_CHOSEN ? expf(choice[e] - most) : score(e);
+  };
+  float total = 0.f;
   for (int e = lane; e < p.experts; e += 64) {
     const float mine = choice[e];
     if (mine == -INFINITY) continue;
     const int rank = rank_of(choice, ep, mine, e);
     if (rank < p.top) {
-      const float w = p.softmax ? expf(mine - most) : sigmoid_exact(z[e]);
+      const float w = weight(e);
       p.ids[(size_t)token * p.top + rank] = e;
       p.weights[(size_t)token * p.top + rank] = w;
-      sum += w;
+      total += w;
     }
   }
-  if (p.softmax) {
+  if (p.mode != ROUTE_SIGMOID) {
     // each lane divides the weights that it wrote itself
-    const float inv = 1.f / wave_sum(sum);
+    total = wave_sum(total);
+    const float inv = p.mode == ROUTE_SHARE ? p.scale / (total + 1e-20f)
+                                            : 1.f / total;
     for (int e = lane; e < p.experts; e += 64) {
       const float mine = choice[e];
       if (mine == -INFINITY) continue;
       const int rank = rank_of(choice, ep, mine, e);
       if (rank < p.top)
-        p.weights[(size_t)token * p.top + rank] = expf(mine - most) * inv;
+        p.weights[(size_t)token * p.top + rank] = weight(e) * inv;
     }
   }
   wave_fence();
@@ -254,7 +269,7 @@ DEV_INLINE void count_pairs(const MoeRouteArgs& p, int* count, int lo, int hi) {
   __syncthreads();
 #pragma unroll 4
   for (int i = lo + threadIdx.x; i < hi; i += NT)
-    atomicAdd(&count[p.ids[i]], 1);
+    if (p.ids[i] < p.real) atomicAdd(&count[p.ids[i]], 1);
   __syncthreads();
 }
 
@@ -263,9 +278,10 @@ DEV_INLINE void place_pairs(const MoeRouteArgs& p, int* cursor, int lo,
                             int hi) {
 #pragma unroll 4
   for (int i = lo + threadIdx.x; i < hi; i += NT) {
-    const int at = atomicAdd(&cursor[p.ids[i]], 1);
+    const int e = p.ids[i];
+    const int at = e < p.real ? atomicAdd(&cursor[e], 1) : -1;
     p.inv[i] = at;
-    p.rows[at] = i / p.top;
+    if (at >= 0) p.rows[at] = i / p.top;
   }
 }
 

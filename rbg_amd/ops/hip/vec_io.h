@@ -22,6 +22,11 @@ DEV_INLINE void load_vec(const __hip_bfloat16* p, float* o) {
     t.u = *reinterpret_cast<const uint4*>(p);
 #pragma unroll
     for (int j = 0; j < 8; ++j) o[j] = bf2f(t.e[j]);
+  } else if constexpr (V == 4) {
+    union { uint2 u; __hip_bfloat16 e[4]; } t;
+    t.u = *reinterpret_cast<const uint2*>(p);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o[j] = bf2f(t.e[j]);
   } else {
 #pragma unroll
     for (int j = 0; j < V; ++j) o[j] = bf2f(p[j]);
@@ -49,6 +54,11 @@ DEV_INLINE void store_vec(__hip_bfloat16* p, const float* o) {
 #pragma unroll
     for (int j = 0; j < 8; ++j) t.e[j] = f2bf(o[j]);
     *reinterpret_cast<uint4*>(p) = t.u;
+  } else if constexpr (V == 4) {
+    union { uint2 u; __hip_bfloat16 e[4]; } t;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) t.e[j] = f2bf(o[j]);
+    *reinterpret_cast<uint2*>(p) = t.u;
   } else {
 #pragma unroll
     for (int j = 0; j < V; ++j) p[j] = f2bf(o[j]);

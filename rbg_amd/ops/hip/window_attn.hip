@@ -1,6 +1,6 @@
 // Causal window attention over contiguous keys and values (gfx950, bf16):
 // varlen prefill of any head sizes up to 256, with an optional sigmoid output
-// gate.  A query at position i sees keys j with 0 <= i - j < window.
+// gate, an optional key part that all heads share, and an optional sink per head.  A query at position i sees keys j with 0 <= i - j < window.
 //
 // A workgroup takes 128 query rows of one head (NW waves x QT x 16) and walks the
 // 64-key tiles between its first row's window edge and its last row.  Per tile
@@ -22,7 +22,7 @@ namespace {
 constexpr int KT = 64;
 
 template <int DK, int DV, int NW, int QT>
-__global__ __launch_bounds__(NW * 64, (DK + DV) > 256 ? 1 : 2)
+__global__ __launch_bounds__(NW * 64, (DK + DV) > 320 ? 1 : 2)
 void window_attn_kernel(const WindowAttnArgs p) {
   constexpr int KP = DK + 16, VP = DV + 16;
   constexpr int ROWS = NW * QT * 16;          // 128
@@ -47,6 +47,7 @@ void window_attn_kernel(const WindowAttnArgs p) {
 
   const __hip_bfloat16* q = (const __hip_bfloat16*)p.q + head * p.q_head;
   const __hip_bfloat16* k = (const __hip_bfloat16*)p.k + head * p.k_head;
+  const __hip_bfloat16* k2 = (const __hip_bfloat16*)p.k2 - p.d1;
   const __hip_bfloat16* v = (const __hip_bfloat16*)p.v + head * p.v_head;
 
   // Q as B operand: column = query, 8 dims per lane
@@ -78,8 +79,9 @@ void window_attn_kernel(const WindowAttnArgs p) {
     for (int i = 0; i < KPC; ++i) {
       const int e = tid + i * NT, key = e / (DK / 8), c = (e % (DK / 8)) * 8;
       const size_t row = krow0 + min(kt * KT + key, klen - 1);
-      kr[i] = c < p.d ? *reinterpret_cast<const u32x4*>(k + row * p.k_row + c)
-                      : zero4;
+      const __hip_bfloat16* src =
+          c < p.d1 ? k + row * p.k_row : k2 + row * p.k2_row;
+      kr[i] = c < p.d ? *reinterpret_cast<const u32x4*>(src + c) : zero4;
     }
 #pragma unroll
     for (int i = 0; i < VPC; ++i) {
@@ -106,8 +108,9 @@ void window_attn_kernel(const WindowAttnArgs p) {
   f32x4 acc[QT][DV / 16];
 #pragma unroll
   for (int t = 0; t < QT; ++t) {
-    m[t] = MASKED;
-    l[t] = 0.f;
+    // a sink is the first maximum and one more term of the sum
+    m[t] = p.sink != nullptr ? p.sink[head] * LOG2E : MASKED;
+    l[t] = p.sink != nullptr && gs == 0 ? 1.f : 0.f;
 #pragma unroll
     for (int d = 0; d < DV / 16; ++d) acc[t][d] = {0.f, 0.f, 0.f, 0.f};
   }
@@ -245,6 +248,7 @@ int window_attn_rows() { return 128; }        // query rows per block
 void launch_window_attn(const WindowAttnArgs* p, hipStream_t s) {
   if (p->d <= 64) go_dv<64>(*p, s);
   else if (p->d <= 128) go_dv<128>(*p, s);
+  else if (p->d <= 192) go_dv<192>(*p, s);
   else go_dv<256>(*p, s);
 }
 

@@ -164,8 +164,8 @@ def prefill_block_info(cu_seqlens: torch.Tensor, qtile: int = 64,
 # -- f32 residual stream, delta rule, latent attention ------------------------
 
 
-def embed_stream(tokens, table, scale):
-    return table[tokens.long()].float() * scale
+def embed_stream(tokens, table, scale, copies=1):
+    return (table[tokens.long()].float() * scale).repeat(1, copies)
 
 
 def stream_norm(x, delta, w1, w2, groups, eps, dtype):
@@ -201,6 +201,15 @@ def gelu_mul(x, out):
     out.copy_((act * up).to(x.dtype))
 
 
+def clamped_glu_act(g, u, limit):
+    g = g.clamp(max=limit)
+    return g * torch.sigmoid(1.702 * g) * (u.clamp(-limit, limit) + 1)
+
+
+def clamped_glu(gate, up, limit, out):
+    out.copy_(clamped_glu_act(gate.float(), up.float(), limit).to(out.dtype))
+
+
 def delta_rule(proj, z, w2, w0, a_bias, norm_w, state, slots, cu_seqlens,
                starts, out, offs, decay_scale, unit_eps, norm_eps):
     H, D = state.shape[1:3]
@@ -230,47 +239,78 @@ def delta_rule(proj, z, w2, w0, a_bias, norm_w, state, slots, cu_seqlens,
             out[t] = o.to(out.dtype)
 
 
-def latent_store(x, w, cache, slots, eps):
+def rotate(x, rot):
+    """x [T, .., dims] by its rows' positions, in f32."""
+    half = rot.dims // 2
+    cs = rot.table[rot.positions.long()]
+    cs = cs.view(cs.shape[0], *[1] * (x.dim() - 2), rot.dims)
+    cos, sin = cs[..., :half], cs[..., half:]
     xf = x.float()
-    c = (xf / torch.sqrt(xf.pow(2).mean(-1, keepdim=True) + eps) * w)
-    c = c.to(x.dtype)
+    if rot.interleaved:
+        u, v = xf[..., ::2], xf[..., 1::2]
+        y = torch.stack([u * cos - v * sin, v * cos + u * sin], dim=-1)
+        return y.flatten(-2).to(x.dtype)
+    u, v = xf[..., :half], xf[..., half:]
+    return torch.cat([u * cos - v * sin, v * cos + u * sin],
+                     dim=-1).to(x.dtype)
+
+
+def latent_store(x, w, cache, slots, eps, rot=None, second=None):
+    n = w.numel()
+    c = _rms(x[:, :n].float(), w, eps).to(x.dtype)
+    if rot is not None:
+        c = torch.cat([c, rotate(x[:, n:], rot)], dim=1)
     cache.view(-1, cache.shape[-1])[slots.long()] = c
-    return c
+    if second is None:
+        return [c]
+    return [c, _rms(second[0].float(), second[1], eps).to(x.dtype)]
 
 
-def window_attention(q, k, v, gate, out, row_info, scale, window):
+def window_attention(q, k, v, gate, out, row_info, scale, window, shared=None,
+                     sink=None):
     T, H, _ = q.shape
+    if shared is not None:
+        k = torch.cat([k, shared.unsqueeze(1).expand(-1, H, -1)], dim=-1)
     for t, (base, pos) in enumerate(row_info.tolist()):
         lo = max(0, pos - window + 1) if window > 0 else 0
         ks = k[base + lo:base + pos + 1].float()
         s = torch.einsum("hd,khd->hk", q[t].float(), ks) * scale
-        o = torch.einsum("hk,khd->hd", torch.softmax(s, dim=-1),
+        o = torch.einsum("hk,khd->hd", _softmax(s, sink),
                          v[base + lo:base + pos + 1].float()).reshape(-1)
         if gate is not None:
             o = o * torch.sigmoid(gate[t].float())
         out[t] = o.to(out.dtype)
 
 
-def latent_decode(q, cache, block_tables, context_lens, scale, window):
-    S, H, R = q.shape
-    out = torch.empty_like(q)
+def _softmax(s, sink):
+    """Over the last dim of s [H, keys], with a logit per head that counts in
+    the sum alone."""
+    if sink is None:
+        return torch.softmax(s, dim=-1)
+    return torch.softmax(torch.cat([s, sink.view(-1, 1)], dim=-1),
+                         dim=-1)[:, :-1]
+
+
+def latent_decode(q, cache, block_tables, context_lens, scale, window, rank,
+                  sink=None):
+    S, H, D = q.shape
+    out = q.new_empty((S, H, rank))
     ps = cache.shape[1]
-    flat = cache.view(-1, R)
+    flat = cache.view(-1, D)
     for s in range(S):
         ctx = int(context_lens[s])
         lo = max(0, ctx - window) if window > 0 else 0
         j = torch.arange(lo, ctx)
         c = flat[block_tables[s].long()[j // ps] * ps + j % ps].float()
-        p = torch.softmax(q[s].float() @ c.T * scale, dim=-1)
-        out[s] = (p @ c).to(q.dtype)
+        p = _softmax(q[s].float() @ c.T * scale, sink)
+        out[s] = (p @ c[:, :rank]).to(q.dtype)
     return out
 
 
 def head_linear(x, w, gate, out):
     y = torch.einsum("shk,hjk->shj", x.float(), w.float())
-    y = y.reshape(out.shape)
     if gate is not None:
-        y = y * torch.sigmoid(gate.float())
+        y = y * torch.sigmoid(gate.float()).view(y.shape)
     out.copy_(y.to(out.dtype))
 
 
@@ -289,8 +329,11 @@ def _rms(x, w, eps):
 
 
 def moe_combine(y, route):
-    """f32 sums of each token's weighed expert rows."""
-    rows = y.float()[route.inv.long()].view(-1, route.top, y.shape[1])
+    """f32 sums of each token's weighed expert rows (a pair without a row
+    counts nothing)."""
+    inv = route.inv.long()
+    rows = y.float()[inv.clamp(min=0)] * (inv >= 0).unsqueeze(1)
+    rows = rows.view(-1, route.top, y.shape[1])
     return (rows * route.weights.unsqueeze(-1)).sum(1)
 
 
@@ -353,10 +396,12 @@ def paged_rows(q, k, v, tables, row_info, out, scale, softcap, sink, window=0,
         out[r] = o.reshape(-1).to(out.dtype)
 
 
-def moe_choose(logits, correction, groups, keep, top, softmax=False):
+def moe_choose(logits, correction, groups, keep, top, softmax=False,
+               share=None):
     """(experts, weights) of each token, [T, top]."""
     T, E = logits.shape
-    s = logits if softmax else torch.sigmoid(logits)
+    s = (torch.softmax(logits, dim=-1) if share is not None else
+         logits if softmax else torch.sigmoid(logits))
     choice = (s + correction).view(T, groups, E // groups)
     best = choice.topk(min(2, E // groups), dim=-1).values.sum(-1)
     kept = torch.zeros(T, groups, dtype=torch.bool)
@@ -365,25 +410,31 @@ def moe_choose(logits, correction, groups, keep, top, softmax=False):
     chosen = choice.view(T, E).topk(top, dim=-1)
     if softmax:
         return chosen.indices, torch.softmax(chosen.values, dim=-1)
-    return chosen.indices, s.gather(1, chosen.indices)
+    w = s.gather(1, chosen.indices)
+    if share is not None:
+        w = w / (w.sum(-1, keepdim=True) + 1e-20) * share
+    return chosen.indices, w
 
 
 def moe_tiles(ids, experts, tile):
     """Pairs in expert order: (inverse permutation, their tokens, tiles [n, 3]
-    = (expert, first row, rows))."""
+    = (expert, first row, rows)).  Pairs of experts from ``experts`` on have no
+    row: -1."""
     flat = ids.reshape(-1)
     order = torch.sort(flat, stable=True).indices
     inv = torch.empty_like(order)
     inv[order] = torch.arange(order.numel())
     tiles, at = [], 0
-    for e, n in enumerate(torch.bincount(flat, minlength=experts).tolist()):
+    inv[flat >= experts] = -1
+    counts = torch.bincount(flat, minlength=experts).tolist()
+    for e, n in enumerate(counts[:experts]):
         tiles += [(e, at + i, min(tile, n - i)) for i in range(0, n, tile)]
         at += n
     return (inv.int(), (order // ids.shape[1]).int(),
             torch.tensor(tiles, dtype=torch.int32).view(-1, 3))
 
 
-def expert_linear(x, w, route, gather, relu2, swiglu=False):
+def expert_linear(x, w, route, gather, relu2, swiglu=False, limit=None):
     out = x.new_empty((route.rows.numel(), w.shape[1] // (2 if swiglu else 1)))
     for e, at, n in route.tiles.tolist():
         rows = x[route.rows[at:at + n].long()] if gather else x[at:at + n]
@@ -392,9 +443,35 @@ def expert_linear(x, w, route, gather, relu2, swiglu=False):
             y = torch.relu(y).pow(2)
         elif swiglu:                    # columns gate, gate, up, up
             y = y.unflatten(1, (-1, 2, 2))
-            y = (torch.nn.functional.silu(y[:, :, 0]) * y[:, :, 1]).flatten(1)
+            g, u = y[:, :, 0], y[:, :, 1]
+            y = (torch.nn.functional.silu(g) * u if limit is None else
+                 clamped_glu_act(g, u, limit)).flatten(1)
         out[at:at + n] = y.to(x.dtype)
     return out
+
+
+# -- hyper-connections -----------------------------------------------------------
+
+
+def hyper_norm(x, streams, stir, read, norm, dtype):
+    xs = x.view(x.shape[0], streams, -1)
+    if stir is not None:
+        y = 0.0 if stir.rows is None else stir.rows.float()
+        if stir.route is not None:
+            if stir.experts is not None:
+                y = y + moe_combine(stir.experts, stir.route)
+            if stir.self_rows is not None:
+                none = (stir.route.inv < 0).view(-1, stir.route.top)
+                y = y + (stir.route.weights * none).sum(
+                    1, keepdim=True) * stir.self_rows.float()
+        mix = stir.conn[:streams * streams].view(streams, streams)
+        out = stir.conn[streams * streams:] * stir.mult
+        new = torch.einsum("st,nsw->ntw", mix, xs)
+        xs.copy_(new + out.view(1, -1, 1) * y.unsqueeze(1))
+    if norm is None:
+        return None
+    u = torch.einsum("s,nsw->nw", read, xs)
+    return (torch.tanh(norm.alpha * u) * norm.w + norm.b).to(dtype)
 
 
 # -- gated branches, gated delta rule -------------------------------------------

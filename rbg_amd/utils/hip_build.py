@@ -71,6 +71,14 @@ HIP_SOURCES = {
         "skinny_gemm.hip",
         "moe_bindings.cpp",
     ],
+    # hyper-connections, tanh norms, gated linear units
+    "_hip_hyper": [
+        "embed.hip",
+        "hyper_norm.hip",
+        "gated_act.hip",
+        "skinny_gemm.hip",
+        "hyper_bindings.cpp",
+    ],
     # gated delta rule, short convolution, gated norms and linear units
     "_hip_gated": [
         "embed.hip",
@@ -86,24 +94,30 @@ HIP_SOURCES = {
 
 HIP_HEADERS = {
     "_hip_ops": ["common.h", "gemm_bindings.h"],
-    "_hip_mix": ["bind_util.h", "common.h", "delta_scan.h", "gemm_bindings.h",
-                 "mfma_util.h", "mix_args.h", "vec_io.h"],
+    "_hip_mix": ["act.h", "act_kinds.h", "bind_util.h", "common.h",
+                 "delta_scan.h", "embed_bindings.h", "gemm_bindings.h",
+                 "glu_bindings.h", "mfma_util.h", "mix_args.h", "vec_io.h"],
     "_hip_latent": ["bind_util.h", "common.h", "latent_args.h", "mfma_util.h",
-                    "vec_io.h"],
-    "_hip_experts": ["bind_util.h", "common.h", "expert_args.h",
-                     "expert_rows.h", "lds_stream.h", "mfma_util.h",
-                     "vec_io.h"],
+                    "rotary.h", "vec_io.h"],
+    "_hip_experts": ["act.h", "act_kinds.h", "bind_util.h", "common.h",
+                     "expert_args.h", "expert_rows.h", "lds_stream.h",
+                     "mfma_util.h", "vec_io.h"],
     "_hip_moe": ["bind_util.h", "common.h", "expert_rows.h", "gemm_bindings.h",
                  "mfma_util.h", "moe_args.h", "vec_io.h"],
-    "_hip_gated": ["bind_util.h", "common.h", "delta_scan.h", "expert_rows.h",
+    "_hip_hyper": ["act.h", "act_kinds.h", "bind_util.h", "common.h",
+                   "embed_bindings.h", "expert_rows.h", "gemm_bindings.h",
+                   "glu_bindings.h", "hyper_args.h", "vec_io.h"],
+    "_hip_gated": ["act.h", "act_kinds.h", "bind_util.h", "common.h",
+                   "delta_scan.h", "embed_bindings.h", "expert_rows.h",
                    "gated_args.h", "gated_delta.h", "gemm_bindings.h",
-                   "mfma_util.h", "vec_io.h"],
+                   "glu_bindings.h", "mfma_util.h", "vec_io.h"],
 }
 
 # model architecture -> the extensions with its kernels (default: _hip_ops)
 EXTENSIONS_OF = {"Bitatar": ("_hip_mix", "_hip_latent"),
                  "Notadra": ("_hip_moe", "_hip_experts"),
-                 "Gogalix": ("_hip_gated", "_hip_moe", "_hip_experts")}
+                 "Gogalix": ("_hip_gated", "_hip_moe", "_hip_experts"),
+                 "Danipel": ("_hip_hyper", "_hip_latent", "_hip_experts")}
 
 
 def source_hash(name: str) -> str:
