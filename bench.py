@@ -51,11 +51,12 @@ def parse_args():
                         "tp/pp: all ranks form one sharded engine")
     p.add_argument("--eager", action="store_true",
                    help="disable hipGraph capture")
-    p.add_argument("--compare", choices=["bitatar", "notadra", "gogalix"],
+    p.add_argument("--compare", choices=["bitatar", "notadra", "gogalix", "danipel"],
                    default=None,
                    help="instead: prefill/decode throughput of this family "
-                        "beside Llama (gogalix: Bitatar) at equal size, one "
-                        "GPU, one JSON line per workload (--sizes, --batches, "
+                        "beside Llama (gogalix: Bitatar; danipel: Bitatar, "
+                        "with experts Gogalix) at equal size, one GPU, one "
+                        "JSON line per workload (--sizes, --batches, "
                         "--seq-len)")
     p.add_argument("--sizes", default="2k,4k", help="with --compare")
     p.add_argument("--batches", default="1,32", help="with --compare")

@@ -34,6 +34,9 @@ def pair(size: str, family: str = "bitatar") -> List[ModelConfig]:
     if family == "gogalix":
         from .gogalix_bench import gogalix_set
         return gogalix_set(size)
+    if family == "danipel":
+        from .danipel_bench import danipel_set
+        return danipel_set(size)
     w, ff, heads, kvh, layers, rank, window, dh, dd = SIZES[size]
     return [
         BitatarConfig.stacked(
@@ -146,6 +149,9 @@ def run_kernels(size: str, batches=(1, 8, 32, 128), ctx: int = 2048,
     if family == "gogalix":
         from .gogalix_bench import gogalix_kernels
         return gogalix_kernels(size, batches, ctx, prompts)
+    if family == "danipel":
+        from .danipel_bench import danipel_kernels
+        return danipel_kernels(size, batches, ctx, prompts)
     import math
 
     from .. import ops

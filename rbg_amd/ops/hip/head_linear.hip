@@ -17,12 +17,13 @@
 
 namespace {
 
-// rows [s0, s1) of a head's tail; the workgroup's threads together
+// rows [s0, s1) of a head's tail, pairs from `at` on in steps of `step`
 template <typename T>
 DEV_INLINE void rotate_tail(const HeadLinearArgs& p, const int head,
-                            const int s0, const int s1) {
+                            const int s0, const int s1, const int at,
+                            const int step) {
   const int half = p.rot.dims / 2;
-  for (int e = threadIdx.x; e < (s1 - s0) * half; e += blockDim.x) {
+  for (int e = at; e < (s1 - s0) * half; e += step) {
     const int s = s0 + e / half;
     rotate_pair(p.rot, rotary_row(p.rot, s), e % half,
                 (const T*)p.tail + (size_t)s * p.t_row + head * p.t_head,
@@ -38,8 +39,11 @@ __global__ __launch_bounds__(256) void head_linear_kernel(
   const int head = blockIdx.y;
   const int n0 = (blockIdx.x * 4 + wave) * 16;
   const int s0 = blockIdx.z * 16 * MT;
-  if (blockIdx.x * 64 >= p.n) {                 // the workgroup behind the last
-    rotate_tail<__hip_bfloat16>(p, head, s0, min(s0 + 16 * MT, p.rows));
+  const int nb = (p.n + 63) / 64;
+  if ((int)blockIdx.x >= nb) {                  // workgroups behind the last
+    rotate_tail<__hip_bfloat16>(p, head, s0, min(s0 + 16 * MT, p.rows),
+                                (blockIdx.x - nb) * 256 + threadIdx.x,
+                                (gridDim.x - nb) * 256);
     return;
   }
   if (n0 >= p.n) return;
@@ -54,18 +58,24 @@ __global__ __launch_bounds__(256) void head_linear_kernel(
   f32x4 acc[MT];
 #pragma unroll
   for (int t = 0; t < MT; ++t) acc[t] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-  for (int k0 = 0; k0 < p.k; k0 += 32) {
-    const int k = k0 + gs * 8;
-    // unconditional clamped loads: a guard would serialise them
-    const int kc = min(k, p.k - 8);
-    mf_bf8 wf = frag8(w + kc);
+  constexpr int UN = 4;                         // 32-k steps in flight
+  for (int k0 = 0; k0 < p.k; k0 += 32 * UN) {
+    // unconditional clamped loads, all before the first product: a guard would
+    // serialise them
+    mf_bf8 wf[UN], xf[UN][MT];
     const mf_bf8 z = {};
-    wf = k < p.k ? wf : z;
 #pragma unroll
-    for (int t = 0; t < MT; ++t) {
-      const mf_bf8 xf = frag8(x[t] + kc);
-      acc[t] = mfma_bf16_k32(wf, xf, acc[t]);
+    for (int u = 0; u < UN; ++u) {
+      const int kc = min(k0 + u * 32 + gs * 8, p.k - 8);
+      wf[u] = frag8(w + kc);
+#pragma unroll
+      for (int t = 0; t < MT; ++t) xf[u][t] = frag8(x[t] + kc);
+    }
+#pragma unroll
+    for (int u = 0; u < UN; ++u) {
+      const mf_bf8 wu = k0 + u * 32 + gs * 8 < p.k ? wf[u] : z;
+#pragma unroll
+      for (int t = 0; t < MT; ++t) acc[t] = mfma_bf16_k32(wu, xf[u][t], acc[t]);
     }
   }
 #pragma unroll
@@ -110,7 +120,7 @@ __global__ __launch_bounds__(256) void head_linear_rows_kernel(
   const long main = (total + 255) / 256;
   if (blockIdx.x >= main) {                     // one (row, head) each
     const int at = (int)(blockIdx.x - main), s = at / p.heads;
-    rotate_tail<T>(p, at % p.heads, s, s + 1);
+    rotate_tail<T>(p, at % p.heads, s, s + 1, threadIdx.x, 256);
     return;
   }
   if (i >= total) return;
@@ -139,7 +149,10 @@ extern "C" void launch_head_linear(const HeadLinearArgs* p, int f32, int vec,
   } else if (!vec) {
     head_linear_rows_kernel<__hip_bfloat16><<<grid, 256, 0, s>>>(*p, total);
   } else {
-    const int nb = (p->n + 63) / 64 + (tail ? 1 : 0);
+    // one pair of the tail a thread
+    const int most = p->rows <= 16 ? 16 : p->rows <= 32 ? 32 : 64;
+    const int nb = (p->n + 63) / 64 +
+        (tail ? (min(p->rows, most) * (p->rot.dims / 2) + 255) / 256 : 0);
     if (p->rows <= 16) {
       head_linear_kernel<1><<<dim3(nb, p->heads, 1), 256, 0, s>>>(*p);
     } else if (p->rows <= 32) {

@@ -26,7 +26,9 @@ template <int RK, int DK>
 __global__ __launch_bounds__(NW * 64, 2) void latent_decode_kernel(
     const LatentDecodeArgs p) {
   constexpr int PITCH = DK + 16;              // 8 banks per row
-  constexpr int LPC = 16 * DK / 8 / 64;       // 16-byte loads per chunk
+  // 16-byte loads per chunk: whole value rows, then what the keys have more
+  constexpr int LPV = 16 * RK / 8 / 64, LPC = 16 * DK / 8 / 64;
+  constexpr int VL = RK / 8, XL = DK > RK ? (DK - RK) / 8 : 1;
   constexpr int DT = RK / 16 / NW;            // 16-column tiles per wave
   static_assert(DT >= 1 && LPC >= 1, "rank tile too small");
   extern __shared__ __attribute__((aligned(16))) char smem[];
@@ -74,21 +76,28 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_decode_kernel(
 
   u32x4 reg[LPC];
   const u32x4 zero4 = {0, 0, 0, 0};
+  // load i of a chunk brings key k(i), columns d(i) ..; both are one lane's
+  // constant plus one of i, so that addresses are too
+  const int vk = lane / VL, vd = lane % VL * 8;
+  const int xk = lane / XL, xd = RK + lane % XL * 8;
+  auto key_of = [&](int i) {
+    return i < LPV ? vk + i * (64 / VL)
+                   : xk + (i - LPV) * (64 / XL);
+  };
+  auto dim_of = [&](int i) { return i < LPV ? vd : xd; };
   // a chunk past the end re-reads the last one, as zeros
-#define LD_FETCH(c)                                                           \
-  do {                                                                        \
-    const int cc = min((c), c_end - 1);                                       \
-    const __hip_bfloat16* src =                                               \
-        cache + ((size_t)table[cc / cpp] * p.page_size + (cc % cpp) * 16) *   \
-                    p.d;                                                      \
-    _Pragma("unroll") for (int i = 0; i < LPC; ++i) {                         \
-      const int e = i * 64 + lane, key = e / (DK / 8), d = (e % (DK / 8)) * 8;\
-      reg[i] = full || d < p.d                                                \
-          ? *reinterpret_cast<const u32x4*>(src + key * p.d + d) : zero4;     \
-    }                                                                         \
-  } while (0)
+  auto fetch = [&](const int c) {
+    const int cc = min(c, c_end - 1);
+    const __hip_bfloat16* src =
+        cache + ((size_t)table[cc / cpp] * p.page_size + (cc % cpp) * 16) * p.d;
+#pragma unroll
+    for (int i = 0; i < LPC; ++i)
+      reg[i] = full || dim_of(i) < p.d
+          ? *reinterpret_cast<const u32x4*>(src + key_of(i) * p.d + dim_of(i))
+          : zero4;
+  };
 
-  if (c_beg < c_end) LD_FETCH(c_beg + wave);
+  if (c_beg < c_end) fetch(c_beg + wave);
   for (int c0 = c_beg; c0 < c_end; c0 += NW) {
     const int c = c0 + wave;
     __hip_bfloat16* mine = cs + wave * 16 * PITCH;
@@ -97,12 +106,11 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_decode_kernel(
     const int c_hi = min(pos, c_end * 16 - 1);
 #pragma unroll
     for (int i = 0; i < LPC; ++i) {
-      const int e = i * 64 + lane, key = e / (DK / 8), d = (e % (DK / 8)) * 8;
-      const int j = c * 16 + key;
-      *reinterpret_cast<u32x4*>(&mine[key * PITCH + d]) =
+      const int j = c * 16 + key_of(i);
+      *reinterpret_cast<u32x4*>(&mine[key_of(i) * PITCH + dim_of(i)]) =
           j >= lo && j <= c_hi ? reg[i] : zero4;
     }
-    if (c0 + NW < c_end) LD_FETCH(c + NW);
+    if (c0 + NW < c_end) fetch(c + NW);
     f32x4 s = {0.f, 0.f, 0.f, 0.f}, s2 = s;
 #pragma unroll
     for (int st = 0; st < DK / 32; st += 2) {
@@ -168,7 +176,6 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_decode_kernel(
     }
     __syncthreads();                          // LDS is free again
   }
-#undef LD_FETCH
 
   // sum of the weights over lane groups and waves
   l += __shfl_xor(l, 16, 64);

@@ -113,9 +113,11 @@ DEV_INLINE void wave_fence() {
 
 DEV_INLINE float sigmoid_exact(float z) { return 1.f / (1.f + expf(-z)); }
 
-// LDS floats of one wave's choice: experts and groups, padded to whole quads
-__host__ __device__ inline int choice_floats(int experts, int groups) {
-  return ((experts + 3) & ~3) + ((groups + 3) & ~3);
+// LDS floats of one wave's choice: experts and groups, padded to whole quads, and
+// the chosen's numbers and weights
+__host__ __device__ inline int choice_floats(const MoeRouteArgs& p) {
+  return ((p.experts + 3) & ~3) + ((p.groups + 3) & ~3) +
+         2 * ((p.top + 3) & ~3);
 }
 
 // how many of the n values (padded with -inf) are ahead of value `mine` at `at`
@@ -139,15 +141,18 @@ DEV_INLINE void choose(const MoeRouteArgs& p, const int token, float* choice,
   const float* z = p.logits + (size_t)token * p.experts;
   const int ep = (p.experts + 3) & ~3, gp = (p.groups + 3) & ~3;
   float* group = choice + ep;
-  float most = -INFINITY, sum = 0.f;
+  float* won = group + gp;                      // by rank
+  int* who = (int*)(won + ((p.top + 3) & ~3));
+  float most = -INFINITY, part = 1.f;
   if (p.mode == ROUTE_SHARE) {                  // softmax over all
     for (int e = lane; e < p.experts; e += 64) most = fmaxf(most, z[e]);
     most = wave_max(most);
+    float sum = 0.f;
     for (int e = lane; e < p.experts; e += 64) sum += expf(z[e] - most);
-    sum = wave_sum(sum);
+    part = 1.f / wave_sum(sum);
   }
   auto score = [&](int e) {
-    return p.mode == ROUTE_SHARE    ? expf(z[e] - most) / sum
+    return p.mode == ROUTE_SHARE    ? expf(z[e] - most) * part
            : p.mode == ROUTE_CHOSEN ? z[e]
                                     : sigmoid_exact(z[e]);
   };
@@ -183,30 +188,26 @@ DEV_INLINE void choose(const MoeRouteArgs& p, const int token, float* choice,
   auto weight = [&](int e) {
     return p.mode == ROUTE_CHOSEN ? expf(choice[e] - most) : score(e);
   };
-  float total = 0.f;
   for (int e = lane; e < p.experts; e += 64) {
     const float mine = choice[e];
     if (mine == -INFINITY) continue;
     const int rank = rank_of(choice, ep, mine, e);
     if (rank < p.top) {
-      const float w = weight(e);
-      p.ids[(size_t)token * p.top + rank] = e;
-      p.weights[(size_t)token * p.top + rank] = w;
-      total += w;
+      won[rank] = weight(e);
+      who[rank] = e;
     }
   }
+  wave_fence();
+  float scale = 1.f;
   if (p.mode != ROUTE_SIGMOID) {
-    // each lane divides the weights that it wrote itself
+    float total = 0.f;
+    for (int r = lane; r < p.top; r += 64) total += won[r];
     total = wave_sum(total);
-    const float inv = p.mode == ROUTE_SHARE ? p.scale / (total + 1e-20f)
-                                            : 1.f / total;
-    for (int e = lane; e < p.experts; e += 64) {
-      const float mine = choice[e];
-      if (mine == -INFINITY) continue;
-      const int rank = rank_of(choice, ep, mine, e);
-      if (rank < p.top)
-        p.weights[(size_t)token * p.top + rank] = weight(e) * inv;
-    }
+    scale = p.mode == ROUTE_SHARE ? p.scale / (total + 1e-20f) : 1.f / total;
+  }
+  for (int r = lane; r < p.top; r += 64) {
+    p.ids[(size_t)token * p.top + r] = who[r];
+    p.weights[(size_t)token * p.top + r] = won[r] * scale;
   }
   wave_fence();
 }
@@ -290,7 +291,7 @@ template <int NT>
 __global__ __launch_bounds__(NT) void route_small_kernel(const MoeRouteArgs p) {
   extern __shared__ float route_smem[];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  float* mine = route_smem + wave * choice_floats(p.experts, p.groups);
+  float* mine = route_smem + wave * choice_floats(p);
   for (int t = wave; t < p.tokens; t += NT / 64) choose(p, t, mine, lane);
   __threadfence_block();
   __syncthreads();
@@ -306,7 +307,7 @@ __global__ __launch_bounds__(256) void choose_kernel(const MoeRouteArgs p) {
   extern __shared__ float route_smem[];
   const int wave = threadIdx.x >> 6, t = blockIdx.x * 4 + wave;
   if (t < p.tokens)                             // whole waves
-    choose(p, t, route_smem + wave * choice_floats(p.experts, p.groups),
+    choose(p, t, route_smem + wave * choice_floats(p),
            threadIdx.x & 63);
 }
 
@@ -329,7 +330,7 @@ __global__ __launch_bounds__(NT) void choose_count_kernel(
     const MoeRouteArgs p) {
   extern __shared__ float route_smem[];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  float* mine = route_smem + wave * choice_floats(p.experts, p.groups);
+  float* mine = route_smem + wave * choice_floats(p);
   const int lo = blockIdx.x * BT, hi = min(lo + BT, p.tokens);
   for (int t = lo + wave; t < hi; t += NT / 64) choose(p, t, mine, lane);
   __threadfence_block();
@@ -434,7 +435,7 @@ int moe_route_blocks(int tokens) {
 
 void launch_moe_route(const MoeRouteArgs* p, hipStream_t s) {
   const int blocks = moe_route_blocks(p->tokens);
-  const size_t own = sizeof(float) * choice_floats(p->experts, p->groups);
+  const size_t own = sizeof(float) * choice_floats(*p);
   const size_t lay = sizeof(int) * (2 * p->experts + 32);
   if (blocks > 0) {
     if (own * 16 <= 65536) {

@@ -97,8 +97,8 @@ HIP_HEADERS = {
     "_hip_mix": ["act.h", "act_kinds.h", "bind_util.h", "common.h",
                  "delta_scan.h", "embed_bindings.h", "gemm_bindings.h",
                  "glu_bindings.h", "mfma_util.h", "mix_args.h", "vec_io.h"],
-    "_hip_latent": ["bind_util.h", "common.h", "latent_args.h", "mfma_util.h",
-                    "rotary.h", "vec_io.h"],
+    "_hip_latent": ["bind_util.h", "common.h", "latent_args.h", "lds_stream.h",
+                    "mfma_util.h", "rotary.h", "vec_io.h"],
     "_hip_experts": ["act.h", "act_kinds.h", "bind_util.h", "common.h",
                      "expert_args.h", "expert_rows.h", "lds_stream.h",
                      "mfma_util.h", "vec_io.h"],

@@ -396,7 +396,7 @@ def test_latent_decode_splits(splits):
     bt = i32([list(range(1, 11)), list(range(11, 21))], where)
     o = ops._require_latent().latent_decode(
         put(q, where), put(cache, where), bt, i32([150, 3], where), 0.1,
-        window, splits)
+        window, splits, rank, None)
     for b, c in enumerate([150, 3]):
         keys = cache[1 + 10 * b:11 + 10 * b].reshape(-1, rank)
         keys = keys[max(0, c - window):c]
