@@ -11,16 +11,26 @@ DEV_INLINE void add_expert_rows(const T* __restrict__ y,
                                 const float* __restrict__ wts, const int top,
                                 const T* __restrict__ self, const size_t token,
                                 const int width, const int i, float* o) {
-#pragma unroll 4
-  for (int t = 0; t < top; ++t) {
-    const int at = inv[token * top + t];
-    const T* src = at < 0 ? self : y;
-    if (src == nullptr) continue;
-    float r[V];
-    load_vec<V>(src + (at < 0 ? token : (size_t)at) * width + i, r);
-    const float w = wts[token * top + t];
+  constexpr int UN = 4;                         // rows in flight
+  for (int t0 = 0; t0 < top; t0 += UN) {
+    float r[UN][V], w[UN];
+    bool on[UN];
 #pragma unroll
-    for (int j = 0; j < V; ++j) o[j] += w * r[j];
+    for (int u = 0; u < UN; ++u) {
+      const size_t at = token * top + min(t0 + u, top - 1);
+      const int row = inv[at];
+      const T* src = row < 0 ? self : y;
+      on[u] = t0 + u < top && src != nullptr;
+      w[u] = wts[at];
+      if (src != nullptr)
+        load_vec<V>(src + (row < 0 ? token : (size_t)row) * width + i, r[u]);
+    }
+#pragma unroll
+    for (int u = 0; u < UN; ++u)
+      if (on[u]) {
+#pragma unroll
+        for (int j = 0; j < V; ++j) o[j] += w[u] * r[u][j];
+      }
   }
 }
 

@@ -17,7 +17,25 @@
 
 namespace {
 
-// rows [s0, s1) of a head's tail, pairs from `at` on in steps of `step`
+// rows [s0, s1) of a head's tail, pieces (pairs) from `at` on in steps of `step`
+__host__ DEV_INLINE int tail_pieces(const HeadLinearArgs& p) {
+  return p.tail_vec ? rotary_vecs(p.rot) : p.rot.dims / 2;
+}
+
+DEV_INLINE void rotate_tail_vec(const HeadLinearArgs& p, const int head,
+                                const int s0, const int s1, const int at,
+                                const int step) {
+  const int per = rotary_vecs(p.rot);
+  for (int e = at; e < (s1 - s0) * per; e += step) {
+    const int s = s0 + e / per;
+    rotate_vec(p.rot, rotary_row(p.rot, s), e % per,
+               (const __hip_bfloat16*)p.tail + (size_t)s * p.t_row +
+                   head * p.t_head,
+               (__hip_bfloat16*)p.out + (size_t)s * p.o_row +
+                   head * p.o_head + p.n);
+  }
+}
+
 template <typename T>
 DEV_INLINE void rotate_tail(const HeadLinearArgs& p, const int head,
                             const int s0, const int s1, const int at,
@@ -41,9 +59,11 @@ __global__ __launch_bounds__(256) void head_linear_kernel(
   const int s0 = blockIdx.z * 16 * MT;
   const int nb = (p.n + 63) / 64;
   if ((int)blockIdx.x >= nb) {                  // workgroups behind the last
-    rotate_tail<__hip_bfloat16>(p, head, s0, min(s0 + 16 * MT, p.rows),
-                                (blockIdx.x - nb) * 256 + threadIdx.x,
-                                (gridDim.x - nb) * 256);
+    const int s1 = min(s0 + 16 * MT, p.rows);
+    const int at = (blockIdx.x - nb) * 256 + threadIdx.x;
+    const int step = (gridDim.x - nb) * 256;
+    if (p.tail_vec) rotate_tail_vec(p, head, s0, s1, at, step);
+    else rotate_tail<__hip_bfloat16>(p, head, s0, s1, at, step);
     return;
   }
   if (n0 >= p.n) return;
@@ -149,10 +169,10 @@ extern "C" void launch_head_linear(const HeadLinearArgs* p, int f32, int vec,
   } else if (!vec) {
     head_linear_rows_kernel<__hip_bfloat16><<<grid, 256, 0, s>>>(*p, total);
   } else {
-    // one pair of the tail a thread
+    // one piece of the tail a thread
     const int most = p->rows <= 16 ? 16 : p->rows <= 32 ? 32 : 64;
     const int nb = (p->n + 63) / 64 +
-        (tail ? (min(p->rows, most) * (p->rot.dims / 2) + 255) / 256 : 0);
+        (tail ? (min(p->rows, most) * tail_pieces(*p) + 255) / 256 : 0);
     if (p->rows <= 16) {
       head_linear_kernel<1><<<dim3(nb, p->heads, 1), 256, 0, s>>>(*p);
     } else if (p->rows <= 32) {

@@ -95,4 +95,5 @@ struct HeadLinearArgs {
   long x_row, x_head, g_row, t_row, t_head, o_row, o_head;
   int rows, heads, n, k;
   int pack;               // out (and gate) allow 8-byte accesses
+  int tail_vec;           // tail and its place in out allow 16-byte accesses
 };

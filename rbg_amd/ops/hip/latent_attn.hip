@@ -70,43 +70,15 @@ __global__ __launch_bounds__(256) void rotate_kernel(const RotateArgs p,
   rotate_pair(p.rot, rotary_row(p.rot, row), i, x, x);
 }
 
-// 8 neighbouring elements a thread (twice 8 when the halves are paired)
 __global__ __launch_bounds__(256) void rotate_vec_kernel(const RotateArgs p,
                                                          const long total) {
   const long item = blockIdx.x * 256l + threadIdx.x;
   if (item >= total) return;
-  const int dims = p.rot.dims, half = dims / 2;
-  const int per = p.rot.interleaved ? dims / 8 : half / 8;
-  const int i = (int)(item % per) * 8;
+  const int per = rotary_vecs(p.rot);
   const int head = (int)(item / per % p.heads);
   const int row = (int)(item / ((long)per * p.heads));
-  __hip_bfloat16* x =
-      (__hip_bfloat16*)p.x + row * p.x_row + head * p.x_head + i;
-  const float* cs = rotary_row(p.rot, row);
-  float a[8], o[8];
-  load_vec<8>(x, a);
-  if (p.rot.interleaved) {
-    float c[4], s[4];
-    load_vec<4>(cs + i / 2, c);
-    load_vec<4>(cs + half + i / 2, s);
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      o[2 * j] = a[2 * j] * c[j] - a[2 * j + 1] * s[j];
-      o[2 * j + 1] = a[2 * j + 1] * c[j] + a[2 * j] * s[j];
-    }
-    store_vec<8>(x, o);
-    return;
-  }
-  float b[8], c[8], s[8];
-  load_vec<8>(x + half, b);
-  load_vec<8>(cs + i, c);
-  load_vec<8>(cs + half + i, s);
-#pragma unroll
-  for (int j = 0; j < 8; ++j) o[j] = a[j] * c[j] - b[j] * s[j];
-  store_vec<8>(x, o);
-#pragma unroll
-  for (int j = 0; j < 8; ++j) o[j] = b[j] * c[j] + a[j] * s[j];
-  store_vec<8>(x + half, o);
+  __hip_bfloat16* x = (__hip_bfloat16*)p.x + row * p.x_row + head * p.x_head;
+  rotate_vec(p.rot, rotary_row(p.rot, row), (int)(item % per), x, x);
 }
 
 // NACC: value dimensions per lane (dv <= 64 * NACC)
@@ -225,8 +197,7 @@ void launch_latent_store(const LatentStoreArgs* p, int f32, int vec,
 }
 
 void launch_rotate(const RotateArgs* p, int f32, int vec, hipStream_t s) {
-  const int half = p->rot.dims / 2;
-  const long per = !vec ? half : p->rot.interleaved ? half / 4 : half / 8;
+  const long per = vec ? rotary_vecs(p->rot) : p->rot.dims / 2;
   const long total = (long)p->rows * p->heads * per;
   const int grid = (int)((total + 255) / 256);
   if (vec) {

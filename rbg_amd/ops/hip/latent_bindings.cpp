@@ -270,6 +270,10 @@ void head_linear(Tensor x, Tensor w, OptTensor gate, Tensor out,
   p.pack = N % 4 == 0 && p.o_row % 4 == 0 && p.o_head % 4 == 0 &&
            aligned(out, 8) &&
            (!gate || (p.g_row % 4 == 0 && aligned(*gate, 8)));
+  p.tail_vec = tail && !is_f32(x) && aligned(*tail, 16) && aligned(out, 16) &&
+               aligned(*table, 16) &&
+               mult8({N, p.t_row, p.t_head, p.o_row, p.o_head}) &&
+               p.rot.dims % (interleaved ? 8 : 16) == 0;
   const bool vec = mult8({K, p.x_row, p.x_head}) && aligned(x, 16) &&
                    aligned(w, 16);
   if (R) launch_head_linear(&p, is_f32(x), vec, current_stream());

@@ -113,10 +113,10 @@ DEV_INLINE void wave_fence() {
 
 DEV_INLINE float sigmoid_exact(float z) { return 1.f / (1.f + expf(-z)); }
 
-// LDS floats of one wave's choice: experts and groups, padded to whole quads, and
-// the chosen's numbers and weights
+// LDS floats of one wave's choice: experts (twice) and groups, padded to whole
+// quads, and the chosen's numbers and weights
 __host__ __device__ inline int choice_floats(const MoeRouteArgs& p) {
-  return ((p.experts + 3) & ~3) + ((p.groups + 3) & ~3) +
+  return 2 * ((p.experts + 3) & ~3) + ((p.groups + 3) & ~3) +
          2 * ((p.top + 3) & ~3);
 }
 
@@ -140,25 +140,32 @@ DEV_INLINE void choose(const MoeRouteArgs& p, const int token, float* choice,
                        const int lane) {
   const float* z = p.logits + (size_t)token * p.experts;
   const int ep = (p.experts + 3) & ~3, gp = (p.groups + 3) & ~3;
-  float* group = choice + ep;
+  float* score = choice + ep;
+  float* group = score + ep;
   float* won = group + gp;                      // by rank
   int* who = (int*)(won + ((p.top + 3) & ~3));
-  float most = -INFINITY, part = 1.f;
+  float most = -INFINITY;
+  for (int e = lane; e < p.experts; e += 64) {
+    score[e] = z[e];
+    choice[e] = p.correction[e];
+    most = fmaxf(most, score[e]);
+  }
   if (p.mode == ROUTE_SHARE) {                  // softmax over all
-    for (int e = lane; e < p.experts; e += 64) most = fmaxf(most, z[e]);
     most = wave_max(most);
     float sum = 0.f;
-    for (int e = lane; e < p.experts; e += 64) sum += expf(z[e] - most);
-    part = 1.f / wave_sum(sum);
+    for (int e = lane; e < p.experts; e += 64) {
+      score[e] = expf(score[e] - most);
+      sum += score[e];
+    }
+    const float part = 1.f / wave_sum(sum);
+    for (int e = lane; e < p.experts; e += 64) score[e] *= part;
+  } else if (p.mode == ROUTE_SIGMOID) {
+    for (int e = lane; e < p.experts; e += 64)
+      score[e] = sigmoid_exact(score[e]);
   }
-  auto score = [&](int e) {
-    return p.mode == ROUTE_SHARE    ? expf(z[e] - most) * part
-           : p.mode == ROUTE_CHOSEN ? z[e]
-                                    : sigmoid_exact(z[e]);
-  };
   for (int e = lane; e < ep; e += 64)           // NaN becomes the least score
-    choice[e] = e < p.experts
-        ? fmaxf(score(e) + p.correction[e], -3e38f) : -INFINITY;
+    choice[e] = e < p.experts ? fmaxf(score[e] + choice[e], -3e38f)
+                              : -INFINITY;
   wave_fence();
   const int size = p.experts / p.groups;
   if (p.keep < p.groups) {
@@ -182,18 +189,16 @@ DEV_INLINE void choose(const MoeRouteArgs& p, const int token, float* choice,
     wave_fence();
   }
   if (p.mode == ROUTE_CHOSEN) {
+    most = -INFINITY;
     for (int e = lane; e < p.experts; e += 64) most = fmaxf(most, choice[e]);
     most = wave_max(most);
   }
-  auto weight = [&](int e) {
-    return p.mode == ROUTE_CHOSEN ? expf(choice[e] - most) : score(e);
-  };
   for (int e = lane; e < p.experts; e += 64) {
     const float mine = choice[e];
     if (mine == -INFINITY) continue;
     const int rank = rank_of(choice, ep, mine, e);
     if (rank < p.top) {
-      won[rank] = weight(e);
+      won[rank] = p.mode == ROUTE_CHOSEN ? expf(mine - most) : score[e];
       who[rank] = e;
     }
   }
