@@ -51,7 +51,8 @@ def parse_args():
                         "tp/pp: all ranks form one sharded engine")
     p.add_argument("--eager", action="store_true",
                    help="disable hipGraph capture")
-    p.add_argument("--compare", choices=["bitatar", "notadra", "gogalix", "danipel"],
+    p.add_argument("--compare", choices=["bitatar", "notadra", "gogalix",
+                                         "danipel"],
                    default=None,
                    help="instead: prefill/decode throughput of this family "
                         "beside Llama (gogalix: Bitatar; danipel: Bitatar, "

@@ -60,7 +60,7 @@ def require(*names: str):
 
 
 def _require_hip():
-    return require("_hip_ops")
+    return _hip if _hip is not None else require("_hip_ops")
 
 
 def _require_mix():

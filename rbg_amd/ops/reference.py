@@ -332,7 +332,8 @@ def moe_combine(y, route):
     """f32 sums of each token's weighed expert rows (a pair without a row
     counts nothing)."""
     inv = route.inv.long()
-    rows = y.float()[inv.clamp(min=0)] * (inv >= 0).unsqueeze(1)
+    # rows that no pair has are never written
+    rows = y.float()[inv.clamp(min=0)].masked_fill((inv < 0).unsqueeze(1), 0)
     rows = rows.view(-1, route.top, y.shape[1])
     return (rows * route.weights.unsqueeze(-1)).sum(1)
 

@@ -126,6 +126,25 @@ def test_experts_into_the_streams(where, S, W, top, identity):
           where)
 
 
+@pytest.mark.parametrize("where", WHERE)
+def test_only_experts_without_rows(where):
+    """Nothing is read of expert rows that nobody wrote."""
+    T, W, S = 3, 40, 2
+    route = ops.moe_route(put(torch.tensor([[0.0, 9.0, 8.0]] * T), where, F32),
+                          put(torch.zeros(3), where, F32), 1, 1, 2, 16,
+                          share=1.0, identity=2)
+    assert (route.inv < 0).all()
+    y = torch.full((2 * T, W), float("nan"), device=where[0], dtype=where[1])
+    h = rnd(T, W)
+    x = torch.zeros(T, S * W, device=where[0])
+    conn = put(torch.cat([torch.eye(S).reshape(-1), torch.ones(S)]), where,
+               F32)
+    ops.hyper_norm(x, S, ops.Stir(conn, 1.0, None, y, route, put(h, where)),
+                   None, None, where[1])
+    close(x, seen(h, where).repeat(1, S), where, 1e-6)
+    assert ops.moe_combine(y, route).abs().max() == 0
+
+
 # -- rotation ----------------------------------------------------------------------
 
 
@@ -243,6 +262,32 @@ def test_attention_with_a_shared_key_part(where, sink, H, D, D2, DV):
                              put(s, where, F32) if sink else None)
         close(out, want[at:at + m], where)
         at += m
+
+
+@pytest.mark.parametrize("where", WHERE)
+@pytest.mark.parametrize("H,D,D2,DV", [(2, 128, 64, 128), (1, 64, 64, 64),
+                                       (3, 64, 0, 128), (1, 40, 8, 24)])
+def test_long_portions(where, H, D, D2, DV):
+    """Several query blocks and many key tiles, after a past that ends inside
+    a tile; a key of another tile stands out."""
+    n, past, scale = 463, 150, 0.5
+    q, k = rnd(n, H, D + D2, seed=D), rnd(n, H, D, seed=1)
+    k2, v = rnd(n, max(D2, 8), seed=2)[:, :D2], rnd(n, H, DV, seed=3)
+    full = torch.cat([k, k2.unsqueeze(1).expand(-1, H, -1)], dim=-1)
+    for first, pick in ((150, lambda i: 0), (151, lambda i: i - 64),
+                        (152, lambda i: i // 64 * 64 - 1), (153, lambda i: i),
+                        (154, lambda i: i // 64 * 64)):
+        stand_out(q, full, range(first, n, 9), pick, 12 / scale)
+    s = rnd(H, seed=4) + 2.0
+    q, k, k2, v = (seen(t, where) for t in (q, k, k2, v))
+    full = torch.cat([k, k2.unsqueeze(1).expand(-1, H, -1)], dim=-1)
+    want = oracle.causal_attention(q, full, v, scale, s.float().double())
+    lay = layout([past], [n], where)
+    out = torch.zeros(n - past, H * DV, device=where[0], dtype=where[1])
+    ops.window_attention(put(q[past:], where), put(k, where), put(v, where),
+                         None, out, lay.window_view(0), scale, 0,
+                         put(k2, where) if D2 else None, put(s, where, F32))
+    close(out, want.reshape(n, -1)[past:], where)
 
 
 @pytest.mark.parametrize("where", WHERE)
